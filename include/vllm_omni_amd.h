@@ -713,6 +713,73 @@ int mi_compute_slot_mapping(int64_t* slot_mapping, const int32_t* block_table,
                             int32_t block_table_stride, const int32_t* req_indices,
                             const int64_t* positions, int32_t num_tokens, int32_t block_size);
 
+/* ------------------------------------------------------------------------
+ * Decoders with a 32-bit residual stream, sublayers normed on both sides,
+ * latent attention without positions and gated-delta-rule layers (Dogulorn).
+ * dtype is MI_DTYPE_BF16 or MI_DTYPE_F32 (activations, weights, cache); the
+ * residual stream, recurrent state, A_log and dt_bias are always fp32.
+ * RMS norms here are x / sqrt(mean(x^2) + eps) * w, one rounding at the end.
+ * ---------------------------------------------------------------------- */
+/* x[row] += rms_norm(y[row]; w_post);  h[row] = rms_norm(x[row]; w_pre), or
+ * the cast of x[row] when w_pre == NULL; no h at all when h == NULL.
+ * y: rows of dtype (split == 0) or fp32 split-K partials [split][rows][width]
+ * (what mi_linear_partials leaves; y_stride unused). */
+int mi_residual_norm(void* x, const void* y, int32_t split, const void* w_post, const void* w_pre,
+                     void* h, float eps, int32_t rows, int32_t width, int64_t x_stride,
+                     int64_t y_stride, int64_t h_stride, int dtype, void* stream);
+/* x = table[id] * scale + pairs[(prev * mul_prev + id * mul_cur) % buckets]
+ * (position 0: pairs[buckets]);  h = rms_norm(x; w_pre).  The previous token
+ * is prev_ids[row], or last_token[slots[row]] where prev_ids is NULL or the
+ * entry is negative; a row with slots[row] >= 0 leaves its id in last_token. */
+int mi_pair_embed_norm(void* x, void* h, const void* table, const void* pairs, const void* w_pre,
+                       const int64_t* ids, const int64_t* prev_ids, const int32_t* slots,
+                       int64_t* last_token, const int64_t* positions, float scale,
+                       int64_t mul_prev, int64_t mul_cur, int64_t buckets, float eps, int32_t rows,
+                       int32_t width, int32_t vocab, int64_t x_stride, int64_t h_stride, int dtype,
+                       void* stream);
+/* out[row][j] = gelu_tanh(z[row][j]) * table[ids[row]][offset + j], j < dim */
+int mi_gelu_lookup_mul(void* out, const void* z, const void* table, const int64_t* ids,
+                       int32_t rows, int32_t dim, int64_t z_stride, int64_t table_stride,
+                       int64_t offset, int32_t vocab, int dtype, void* stream);
+/* g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1);
+ * a row of gate_up holds the ff gate values, then the ff up values */
+int mi_clamped_glu(void* out, const void* gate_up, int32_t rows, int32_t ff, int64_t gu_stride,
+                   int64_t out_stride, float alpha, float limit, int dtype, void* stream);
+/* x row: query latent (q_rank) | new cache latent (kv_rank, 0 = none); q_out
+ * [rows][q_rank] and the cache row at slot_mapping[row] (< 0: none) get the
+ * normed halves. */
+int mi_latent_norm_cache(const void* x, int64_t x_stride, const void* q_weight, int32_t q_rank,
+                         void* q_out, const void* c_weight, int32_t kv_rank, void* cache,
+                         const int64_t* slot_mapping, int32_t block_size,
+                         int64_t cache_block_stride, int64_t cache_token_stride, float eps,
+                         int32_t rows, int dtype, void* stream);
+/* y[row][head][0..n) = sum_k x[row][head][k] * w(head, n, k); w by its strides */
+int mi_head_gemm(void* y, const void* x, const void* w, int32_t rows, int32_t heads, int32_t n,
+                 int32_t k, int64_t y_row_stride, int64_t x_row_stride, int64_t w_head_stride,
+                 int64_t w_n_stride, int64_t w_k_stride, int dtype, void* stream);
+/* Absorbed latent attention of rows [row0, row0 + rows): q, out [.][heads][kv_rank];
+ * a row at position i sees cache rows max(0, i - window + 1) .. i of its request.
+ * Any sizes (kv_rank <= 2048); one workgroup per (row, head). */
+int mi_latent_attn_rows(void* out, const void* q, const void* cache, const int32_t* block_table,
+                        const int32_t* seq_lens, const int32_t* query_start_loc, int32_t row0,
+                        int32_t rows, int32_t num_reqs, int32_t heads, int32_t kv_rank,
+                        int32_t block_size, int32_t window, float scale,
+                        int64_t cache_block_stride, int64_t cache_token_stride,
+                        int64_t table_stride, int dtype, void* stream);
+/* Gated delta rule over requests [req0, req0 + num_reqs), token by token:
+ * proj rows [q | k | v | gate | b | a] (heads / kv_heads q-k sharing), short
+ * causal convolutions (conv_w [2 kv_heads dim + heads vdim][taps]) + silu, unit
+ * q / k, decayed state update and read-out, gated norm; out [rows][heads vdim].
+ * state [slots][heads][dim][vdim] fp32, ring [slots][taps][conv channels].
+ * update_ring: also leave multi-token portions' last rows in the ring (a
+ * one-token portion's row is always left there). */
+int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_w,
+                        const float* a_log, const float* dt_bias, const void* norm_w, float* state,
+                        void* ring, const int32_t* slots, const int32_t* query_start_loc,
+                        const int32_t* seq_lens, void* out, int32_t req0, int32_t num_reqs,
+                        int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps,
+                        float eps, int32_t update_ring, int dtype, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

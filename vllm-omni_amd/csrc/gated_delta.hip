@@ -1,0 +1,227 @@
+// Gated delta rule with per-channel short convolutions in front of it: the recurrent mixer of a decoder layer.
+//
+// Per v-head h (its q/k head is h / (heads / kv_heads)) and token:
+//   q, k, v   = silu(causal conv over time of the projections);  q, k made unit vectors, q times dim^-1/2
+//   S        <- g S,  u = beta (v - S^T k),  S <- S + k u^T,  o = S^T q        g = exp(-exp(A_log) softplus(a + dt_bias))
+//   out       = o / rms(o) * norm * silu(gate)
+// The projections of a row arrive as one row [q | k | v | gate | b | a].  Per request slot the state is S [dim][vdim]
+// fp32 per head and a ring of the last `taps` projection rows (row p % taps holds position p); a request whose first
+// token is position 0 starts from zeros whatever the slot holds, so slots need no clearing.
+//
+// Kernels:
+//   * gated_delta_step: one workgroup per (head, request), the state in registers, tokens one after the other: decode
+//     (HBM bound: the state is read and written once), and any shape the chunked pair does not build.
+//   * conv_ring_update: leaves a multi-token portion's last rows in the ring (after every reader of the old rows).
+#include "gated_delta.h"
+
+namespace mi {
+namespace {
+
+// LDS: q[D] k[D] v[V] red[2][groups * V]
+template <typename T, int VEC, int NT>
+__global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams p) {
+  scalar_cache_acquire();
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int R = 64 / VEC;   // rows of the state a thread can hold
+  const int h = blockIdx.x, r = p.req0 + blockIdx.y;
+  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
+  if (L <= 0) return;
+  const int start = p.seq_lens[r] - L;     // < 0: a padded row of a graph replay (scratch slot)
+  const int64_t slot = p.slots[r];
+  const int D = p.D, V = p.V, H = p.H, per = H / p.K, kh = h / per;
+  float* sq = lds;
+  float* sk = sq + D;
+  float* sv = sk + D;
+  const int lv = V / VEC, groups = NT / lv;
+  float* red0 = sv + V;
+  float* red1 = red0 + groups * V;
+  const int tid = threadIdx.x, g = tid / lv, c = (tid % lv) * VEC;
+  const bool on = g < groups;
+  float* S = p.state + ((slot * H + h) * D) * (int64_t)V;
+  const T* proj = reinterpret_cast<const T*>(p.proj);
+  const T* convw = reinterpret_cast<const T*>(p.convw);
+  T* ring = reinterpret_cast<T*>(p.ring) + slot * p.taps * (int64_t)p.CH;
+  float st[R][VEC];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int d = g + i * groups;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) st[i][j] = 0.f;
+    if (on && d < D && start > 0) {
+      if constexpr (VEC == 4) {
+        const float4 a = *reinterpret_cast<const float4*>(S + (int64_t)d * V + c);
+        st[i][0] = a.x, st[i][1] = a.y, st[i][2] = a.z, st[i][3] = a.w;
+      } else {
+        st[i][0] = S[(int64_t)d * V + c];
+      }
+    }
+  }
+  const float neg_a = -expf(p.a_log[h]), dtb = p.dt_bias[h];
+  const float qs = 1.0f / sqrtf((float)D);
+  for (int i = 0; i < L; ++i) {
+    const int64_t row = s0 + i;
+    const int pos = start + i;
+    const T* pr = proj + row * p.ld;
+    for (int n = tid; n < 2 * D + V; n += NT) {
+      const int ch = n < D ? kh * D + n : n < 2 * D ? p.K * D + kh * D + (n - D) : 2 * p.K * D + h * V + (n - 2 * D);
+      const float cur = Io<T>::ld(pr + ch);
+      float acc = cur * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1);
+      for (int b = 1; b < p.taps; ++b) {
+        if (pos - b < 0) break;
+        const float x = i >= b ? Io<T>::ld(pr - b * p.ld + ch) : Io<T>::ld(ring + (int64_t)((pos - b) % p.taps) * p.CH + ch);
+        acc += x * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1 - b);
+      }
+      lds[n] = silu_f(acc);
+      // one token: its row of the ring is nobody's to read this step (readers take the taps - 1 rows before it)
+      if (L == 1 && pos >= 0 && (n >= 2 * D || h % per == 0)) ring[(int64_t)(pos % p.taps) * p.CH + ch] = pr[ch];
+    }
+    __syncthreads();
+    float qq = 0.f, kk = 0.f;
+    for (int d = tid & 63; d < D; d += 64) qq += sq[d] * sq[d], kk += sk[d] * sk[d];
+    const float qn = qs / sqrtf(wave_allreduce_sum(qq) + 1e-6f), kn = 1.0f / sqrtf(wave_allreduce_sum(kk) + 1e-6f);
+    const float decay = expf(neg_a * softplus_f(Io<T>::ld(pr + p.off_a + h) + dtb));
+    const float beta = sigmoid_f(Io<T>::ld(pr + p.off_b + h));
+    float acc[VEC] = {};
+#pragma unroll
+    for (int n = 0; n < R; ++n) {
+      const int d = g + n * groups;
+      if (on && d < D) {
+        const float k = sk[d] * kn;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) st[n][j] *= decay, acc[j] += st[n][j] * k;
+      }
+    }
+    if (on)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) red0[g * V + c + j] = acc[j];
+    __syncthreads();
+    float u[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      float t = 0.f;
+      if (on)
+        for (int n = 0; n < groups; ++n) t += red0[n * V + c + j];
+      u[j] = on ? beta * (sv[c + j] - t) : 0.f;
+      acc[j] = 0.f;
+    }
+#pragma unroll
+    for (int n = 0; n < R; ++n) {
+      const int d = g + n * groups;
+      if (on && d < D) {
+        const float k = sk[d] * kn, q = sq[d] * qn;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) st[n][j] += k * u[j], acc[j] += st[n][j] * q;
+      }
+    }
+    if (on)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) red1[g * V + c + j] = acc[j];
+    __syncthreads();
+    if (tid < 64) {   // the read-out: norm over vdim, gate, store
+      float ss = 0.f;
+      for (int v = tid; v < V; v += 64) {
+        float t = 0.f;
+        for (int n = 0; n < groups; ++n) t += red1[n * V + v];
+        red1[v] = t;
+        ss += t * t;
+      }
+      const float inv = inv_rms(wave_allreduce_sum(ss), V, p.eps);
+      T* o = reinterpret_cast<T*>(p.out) + row * (int64_t)H * V + (int64_t)h * V;
+      for (int v = tid; v < V; v += 64)
+        Io<T>::st(o + v, red1[v] * inv * Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + v) *
+                             silu_f(Io<T>::ld(pr + p.off_g + h * V + v)));
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int d = g + i * groups;
+    if (on && d < D) {
+      if constexpr (VEC == 4) *reinterpret_cast<float4*>(S + (int64_t)d * V + c) = make_float4(st[i][0], st[i][1], st[i][2], st[i][3]);
+      else S[(int64_t)d * V + c] = st[i][0];
+    }
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void conv_ring_update_kernel(const DeltaParams p) {
+  scalar_cache_acquire();
+  const int r = p.req0 + blockIdx.y;
+  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
+  const int ch = blockIdx.x * 256 + threadIdx.x;
+  if (L <= 1 || ch >= p.CH) return;
+  const int start = p.seq_lens[r] - L;
+  T* ring = reinterpret_cast<T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
+  const T* proj = reinterpret_cast<const T*>(p.proj);
+  for (int i = max(0, L - p.taps); i < L; ++i)
+    if (start + i >= 0) ring[(int64_t)((start + i) % p.taps) * p.CH + ch] = proj[(s0 + i) * p.ld + ch];
+}
+
+template <typename T, int VEC, int NT>
+int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
+  const int groups = NT / (p.V / VEC);
+  const size_t lds = (size_t)(2 * p.D + p.V + 2 * groups * p.V) * sizeof(float);
+  auto kern = gated_delta_step_kernel<T, VEC, NT>;
+  if (lds > 65536) {
+    if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return MI_ERR_LAUNCH;
+  }
+  hipLaunchKernelGGL(kern, dim3(p.H, nreq), dim3(NT), lds, s, p);
+  return launch_status();
+}
+
+template <typename T>
+int step_dispatch(const DeltaParams& p, int nreq, hipStream_t s) {
+  const int vec = p.V % 4 == 0 ? 4 : 1;
+  const int lv = p.V / vec;
+  // a thread holds at most 64 state elements: the smallest workgroup whose rows fit
+  auto fits = [&](int nt) { const int gr = nt / lv; return gr > 0 && (p.D + gr - 1) / gr <= 64 / vec; };
+  if (vec == 4) {
+    if (fits(256)) return launch_step<T, 4, 256>(p, nreq, s);
+    if (fits(1024)) return launch_step<T, 4, 1024>(p, nreq, s);
+  } else {
+    if (fits(256)) return launch_step<T, 1, 256>(p, nreq, s);
+    if (fits(1024)) return launch_step<T, 1, 1024>(p, nreq, s);
+  }
+  return MI_ERR_UNSUPPORTED;
+}
+
+}  // namespace
+}  // namespace mi
+
+using namespace mi;
+
+static int delta_fill(DeltaParams& p, const void* proj, int64_t ld, const void* convw, const float* a_log, const float* dt_bias,
+                      const void* norm_w, float* state, void* ring, const int32_t* slots, const int32_t* qsl,
+                      const int32_t* seq_lens, void* out, int32_t req0, int32_t nreq, int32_t H, int32_t K, int32_t D, int32_t V,
+                      int32_t taps, float eps) {
+  if (!proj || !convw || !a_log || !dt_bias || !norm_w || !state || !ring || !slots || !qsl || !seq_lens || !out)
+    return MI_ERR_INVALID_ARG;
+  if (req0 < 0 || nreq < 0 || H <= 0 || K <= 0 || D <= 0 || V <= 0 || taps <= 0 || H % K) return MI_ERR_INVALID_ARG;
+  const int CH = 2 * K * D + H * V;
+  if (ld < CH + H * V + 2 * H) return MI_ERR_INVALID_ARG;
+  p = DeltaParams{proj, convw, norm_w, ring, out, a_log, dt_bias, state, slots, qsl, seq_lens, ld, req0, H, K, D, V, taps, CH,
+                  CH, CH + H * V, CH + H * V + H, eps};
+  return MI_OK;
+}
+
+extern "C" int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_w, const float* a_log,
+                                   const float* dt_bias, const void* norm_w, float* state, void* ring, const int32_t* slots,
+                                   const int32_t* query_start_loc, const int32_t* seq_lens, void* out, int32_t req0,
+                                   int32_t num_reqs, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps,
+                                   float eps, int32_t update_ring, int dtype, void* stream) {
+  if (num_reqs == 0) return MI_OK;
+  DeltaParams p;
+  const int rc = delta_fill(p, proj, proj_stride, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
+                            out, req0, num_reqs, heads, kv_heads, dim, vdim, taps, eps);
+  if (rc != MI_OK) return rc;
+  hipStream_t s = (hipStream_t)stream;
+  int st;
+  if (dtype == MI_DTYPE_BF16) st = step_dispatch<uint16_t>(p, num_reqs, s);
+  else if (dtype == MI_DTYPE_F32) st = step_dispatch<float>(p, num_reqs, s);
+  else return MI_ERR_UNSUPPORTED;
+  if (st != MI_OK || !update_ring) return st;
+  const dim3 grid((p.CH + 255) / 256, num_reqs), block(256);
+  if (dtype == MI_DTYPE_BF16) hipLaunchKernelGGL((conv_ring_update_kernel<uint16_t>), grid, block, 0, s, p);
+  else hipLaunchKernelGGL((conv_ring_update_kernel<float>), grid, block, 0, s, p);
+  return launch_status();
+}

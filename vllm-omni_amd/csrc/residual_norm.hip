@@ -1,0 +1,287 @@
+// Row kernels of decoders whose residual stream is 32-bit and whose sublayers are normed on both sides
+// (x <- x + norm_b(f(norm_a(x)))), and the small gates of such decoders:
+//   * residual_norm:   post-norm of a sublayer's output + residual add + pre-norm (or plain cast) for the next one
+//   * pair_embed_norm: scaled token embedding + the row of the (previous, current) token pair + the first pre-norm
+//   * gelu_lookup_mul: gelu_tanh(z) * (a slice of a per-token table row)
+//   * clamped_glu:     g sigmoid(alpha g) (u + 1) on clamped g, u
+// One workgroup per row, the row stays in registers; fp32 arithmetic, one rounding to the output type.  All of them
+// stream: the bound is HBM (or launch latency at decode sizes).
+#include "row_io.h"
+
+namespace mi {
+namespace {
+
+struct ResidualNormParams {
+  float* x;
+  const void* y;        // T rows, or fp32 split-K partials [split][rows][width] (split >= 1)
+  const void* w_post;
+  const void* w_pre;    // nullptr: h = x cast
+  void* h;              // nullptr: no output
+  int64_t x_stride, y_stride, h_stride;
+  int rows, width, split;
+  float eps;
+};
+
+template <typename T, int VEC, int MAXC>
+__global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualNormParams p) {
+  scalar_cache_acquire();
+  __shared__ float smem[16];
+  const int64_t row = blockIdx.x;
+  float* xr = p.x + row * p.x_stride;
+  float y[MAXC][VEC], x[MAXC][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    Io<float>::ldv<VEC>(xr + c, x[k]);
+    if (p.split) {
+      const float* yp = reinterpret_cast<const float*>(p.y) + row * p.width + c;
+      Io<float>::ldv<VEC>(yp, y[k]);
+      for (int s = 1; s < p.split; ++s) {
+        float t[VEC];
+        Io<float>::ldv<VEC>(yp + (int64_t)s * p.rows * p.width, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[k][j] += t[j];
+      }
+    } else {
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.y) + row * p.y_stride + c, y[k]);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss += y[k][j] * y[k][j];
+  }
+  const float inv = inv_rms(wg_sum(ss, smem), p.width, p.eps);
+  ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float w[VEC];
+    Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.w_post) + c, w);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      x[k][j] += y[k][j] * inv * w[j];
+      ss += x[k][j] * x[k][j];
+    }
+    Io<float>::stv<VEC>(xr + c, x[k]);
+  }
+  if (p.h == nullptr) return;
+  const bool pre = p.w_pre != nullptr;
+  const float inv2 = pre ? inv_rms(wg_sum(ss, smem), p.width, p.eps) : 1.f;
+  T* hr = reinterpret_cast<T*>(p.h) + row * p.h_stride;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    if (pre) {
+      float w[VEC];
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.w_pre) + c, w);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] *= inv2 * w[j];
+    }
+    Io<T>::template stv<VEC>(hr + c, x[k]);
+  }
+}
+
+struct PairEmbedParams {
+  float* x;
+  void* h;
+  const void* table;       // [vocab, width]
+  const void* pairs;       // [buckets + 1, width]
+  const void* w_pre;
+  const int64_t* ids;
+  const int64_t* prev_ids;   // nullptr: every row takes the previous token from last_token[slot]
+  const int32_t* slots;      // per row: slot whose last_token this row leaves behind (< 0: none)
+  int64_t* last_token;
+  const int64_t* positions;
+  int64_t x_stride, h_stride, mul_prev, mul_cur, buckets;
+  int width, vocab;
+  float scale, eps;
+};
+
+template <typename T, int VEC, int MAXC>
+__global__ __launch_bounds__(256) void pair_embed_norm_kernel(const PairEmbedParams p) {
+  scalar_cache_acquire();
+  __shared__ float smem[16];
+  __shared__ int64_t s_prev;
+  const int64_t row = blockIdx.x;
+  const int64_t id = p.ids[row];
+  const int slot = p.slots[row];
+  if (threadIdx.x == 0) {
+    int64_t prev = p.prev_ids ? p.prev_ids[row] : -1;
+    if (prev < 0 && slot >= 0) prev = p.last_token[slot];
+    if (slot >= 0) p.last_token[slot] = id;
+    s_prev = prev < 0 ? 0 : prev;
+  }
+  __syncthreads();
+  const bool known = id >= 0 && id < p.vocab;   // an id outside the table reads as a zero row
+  const int64_t cur = known ? id : 0;
+  const int64_t pr = p.positions[row] <= 0 ? p.buckets : (s_prev * p.mul_prev + cur * p.mul_cur) % p.buckets;
+  const T* er = reinterpret_cast<const T*>(p.table) + cur * p.width;
+  const T* br = reinterpret_cast<const T*>(p.pairs) + pr * p.width;
+  float x[MAXC][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float b[VEC];
+    Io<T>::template ldv<VEC>(er + c, x[k]);
+    Io<T>::template ldv<VEC>(br + c, b);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      x[k][j] = known ? x[k][j] * p.scale + b[j] : 0.f;
+      ss += x[k][j] * x[k][j];
+    }
+    Io<float>::stv<VEC>(p.x + row * p.x_stride + c, x[k]);
+  }
+  const float inv = inv_rms(wg_sum(ss, smem), p.width, p.eps);
+  T* hr = reinterpret_cast<T*>(p.h) + row * p.h_stride;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float w[VEC];
+    Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.w_pre) + c, w);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[k][j] *= inv * w[j];
+    Io<T>::template stv<VEC>(hr + c, x[k]);
+  }
+}
+
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void gelu_lookup_mul_kernel(T* out, const T* z, const T* table, const int64_t* ids, int rows,
+                                                              int dim, int64_t z_stride, int64_t table_stride, int64_t offset,
+                                                              int vocab) {
+  scalar_cache_acquire();
+  const int per = dim / VEC;
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (int64_t)rows * per) return;
+  const int64_t row = i / per;
+  const int c = (int)(i % per) * VEC;
+  const int64_t id = ids[row];
+  float v[VEC], e[VEC];
+  Io<T>::template ldv<VEC>(z + row * z_stride + c, v);
+  const bool known = id >= 0 && id < vocab;
+  Io<T>::template ldv<VEC>(table + (known ? id : 0) * table_stride + offset + c, e);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) v[j] = known ? gelu_tanh_f(v[j]) * e[j] : 0.f;
+  Io<T>::template stv<VEC>(out + row * dim + c, v);
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(T* out, const T* gu, int rows, int ff, int64_t gu_stride,
+                                                          int64_t out_stride, float alpha, float limit) {
+  scalar_cache_acquire();
+  const int per = ff / VEC;
+  const int64_t n = (int64_t)rows * per;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+    const int64_t row = i / per;
+    const int c = (int)(i % per) * VEC;
+    float g[VEC], u[VEC];
+    Io<T>::template ldv<VEC>(gu + row * gu_stride + c, g);
+    Io<T>::template ldv<VEC>(gu + row * gu_stride + ff + c, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float a = fminf(g[j], limit);
+      g[j] = a * sigmoid_f(alpha * a) * (fminf(fmaxf(u[j], -limit), limit) + 1.0f);
+    }
+    Io<T>::template stv<VEC>(out + row * out_stride + c, g);
+  }
+}
+
+#define MI_ROW_DISPATCH(KERN, T, width, vec_ok, ...)                                         \
+  do {                                                                                       \
+    if (vec_ok) {                                                                            \
+      if ((width) <= 2048) hipLaunchKernelGGL((KERN<T, 8, 1>), grid, block, 0, s, __VA_ARGS__);      \
+      else if ((width) <= 4096) hipLaunchKernelGGL((KERN<T, 8, 2>), grid, block, 0, s, __VA_ARGS__); \
+      else if ((width) <= 8192) hipLaunchKernelGGL((KERN<T, 8, 4>), grid, block, 0, s, __VA_ARGS__); \
+      else if ((width) <= 16384) hipLaunchKernelGGL((KERN<T, 8, 8>), grid, block, 0, s, __VA_ARGS__); \
+      else return MI_ERR_UNSUPPORTED;                                                        \
+    } else {                                                                                 \
+      if ((width) <= 1024) hipLaunchKernelGGL((KERN<T, 1, 4>), grid, block, 0, s, __VA_ARGS__);      \
+      else if ((width) <= 8192) hipLaunchKernelGGL((KERN<T, 1, 32>), grid, block, 0, s, __VA_ARGS__); \
+      else return MI_ERR_UNSUPPORTED;                                                        \
+    }                                                                                        \
+  } while (0)
+
+}  // namespace
+}  // namespace mi
+
+using namespace mi;
+
+extern "C" int mi_residual_norm(void* x, const void* y, int32_t split, const void* w_post, const void* w_pre, void* h, float eps,
+                                int32_t rows, int32_t width, int64_t x_stride, int64_t y_stride, int64_t h_stride, int dtype,
+                                void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!x || !y || !w_post || rows < 0 || width <= 0 || split < 0) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  ResidualNormParams p{(float*)x, y, w_post, w_pre, h, x_stride, y_stride, h_stride, rows, width, split, eps};
+  const bool vec = width % 8 == 0 && x_stride % 8 == 0 && (split || y_stride % 8 == 0) && (!h || h_stride % 8 == 0) &&
+                   aligned16(x) && aligned16(y) && aligned16(w_post) && aligned16(w_pre) && aligned16(h);
+  const dim3 grid(rows), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(residual_norm_kernel, uint16_t, width, vec, p);
+  else MI_ROW_DISPATCH(residual_norm_kernel, float, width, vec, p);
+  return launch_status();
+}
+
+extern "C" int mi_pair_embed_norm(void* x, void* h, const void* table, const void* pairs, const void* w_pre, const int64_t* ids,
+                                  const int64_t* prev_ids, const int32_t* slots, int64_t* last_token, const int64_t* positions,
+                                  float scale, int64_t mul_prev, int64_t mul_cur, int64_t buckets, float eps, int32_t rows,
+                                  int32_t width, int32_t vocab, int64_t x_stride, int64_t h_stride, int dtype, void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!x || !h || !table || !pairs || !w_pre || !ids || !slots || !last_token || !positions) return MI_ERR_INVALID_ARG;
+  if (rows < 0 || width <= 0 || vocab <= 0 || buckets <= 0 || mul_prev < 0 || mul_cur < 0) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  PairEmbedParams p{(float*)x, h, table, pairs, w_pre, ids, prev_ids, slots, last_token, positions, x_stride, h_stride,
+                    mul_prev, mul_cur, buckets, width, vocab, scale, eps};
+  const bool vec = width % 8 == 0 && x_stride % 8 == 0 && h_stride % 8 == 0 && aligned16(x) && aligned16(h) &&
+                   aligned16(table) && aligned16(pairs) && aligned16(w_pre);
+  const dim3 grid(rows), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(pair_embed_norm_kernel, uint16_t, width, vec, p);
+  else MI_ROW_DISPATCH(pair_embed_norm_kernel, float, width, vec, p);
+  return launch_status();
+}
+
+extern "C" int mi_gelu_lookup_mul(void* out, const void* z, const void* table, const int64_t* ids, int32_t rows, int32_t dim,
+                                  int64_t z_stride, int64_t table_stride, int64_t offset, int32_t vocab, int dtype, void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!out || !z || !table || !ids || rows < 0 || dim <= 0 || vocab <= 0 || offset < 0) return MI_ERR_INVALID_ARG;
+  const bool vec = dim % 8 == 0 && z_stride % 8 == 0 && table_stride % 8 == 0 && offset % 8 == 0 && aligned16(out) &&
+                   aligned16(z) && aligned16(table);
+  const int64_t n = (int64_t)rows * (vec ? dim / 8 : dim);
+  const dim3 grid((unsigned)((n + 255) / 256)), block(256);
+  hipStream_t s = (hipStream_t)stream;
+#define MI_GL(T, V)                                                                                                     \
+  hipLaunchKernelGGL((gelu_lookup_mul_kernel<T, V>), grid, block, 0, s, (T*)out, (const T*)z, (const T*)table, ids, rows, dim, \
+                     z_stride, table_stride, offset, vocab)
+  if (dtype == MI_DTYPE_BF16) { if (vec) MI_GL(uint16_t, 8); else MI_GL(uint16_t, 1); }
+  else if (dtype == MI_DTYPE_F32) { if (vec) MI_GL(float, 8); else MI_GL(float, 1); }
+  else return MI_ERR_UNSUPPORTED;
+#undef MI_GL
+  return launch_status();
+}
+
+extern "C" int mi_clamped_glu(void* out, const void* gate_up, int32_t rows, int32_t ff, int64_t gu_stride, int64_t out_stride,
+                              float alpha, float limit, int dtype, void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!out || !gate_up || rows < 0 || ff <= 0) return MI_ERR_INVALID_ARG;
+  const bool vec = ff % 8 == 0 && gu_stride % 8 == 0 && out_stride % 8 == 0 && aligned16(out) && aligned16(gate_up);
+  const int64_t n = (int64_t)rows * (vec ? ff / 8 : ff);
+  const int64_t want = (n + 255) / 256;
+  const dim3 grid((unsigned)(want < 65536 ? want : 65536)), block(256);
+  hipStream_t s = (hipStream_t)stream;
+#define MI_CG(T, V) \
+  hipLaunchKernelGGL((clamped_glu_kernel<T, V>), grid, block, 0, s, (T*)out, (const T*)gate_up, rows, ff, gu_stride, out_stride, alpha, limit)
+  if (dtype == MI_DTYPE_BF16) { if (vec) MI_CG(uint16_t, 8); else MI_CG(uint16_t, 1); }
+  else if (dtype == MI_DTYPE_F32) { if (vec) MI_CG(float, 8); else MI_CG(float, 1); }
+  else return MI_ERR_UNSUPPORTED;
+#undef MI_CG
+  return launch_status();
+}

@@ -10,8 +10,10 @@ import os
 from ctypes import POINTER, c_char_p, c_float, c_int, c_int32, c_int64, c_uint64, c_void_p
 
 # VLLM_OMNI_AMD_LIB: an alternative build of the same ABI (kernel experiments: csrc/Makefile `make variant`)
-_LIB_PATH = os.environ.get("VLLM_OMNI_AMD_LIB") or os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib",
-                                                                "libvllm_omni_amd.so")
+_LIB_DIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib")
+_LIB_PATH = os.environ.get("VLLM_OMNI_AMD_LIB") or os.path.join(_LIB_DIR, "libvllm_omni_amd.so")
+# the subset built for models outside the talker family (csrc/Makefile `text`), used when the full library is not there
+_TEXT_LIB_PATH = os.path.join(_LIB_DIR, "libvllm_omni_amd_text.so")
 
 MI_DTYPE_F16, MI_DTYPE_BF16, MI_DTYPE_F32 = 0, 1, 2
 MI_OK = 0
@@ -125,6 +127,18 @@ SIGNATURES = {
     "mi_allreduce_status": (c_int, [_P]),
     "mi_allreduce_poll": (c_int, [_P]),
     "mi_allreduce_destroy": (c_int, [_P]),
+    "mi_residual_norm": (c_int, [_P, _P, c_int32, _P, _P, _P, c_float, c_int32, c_int32, c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_pair_embed_norm": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_float, c_int64, c_int64, c_int64, c_float, c_int32,
+                                   c_int32, c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_gelu_lookup_mul": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int64, c_int64, c_int64, c_int32, c_int, _P]),
+    "mi_clamped_glu": (c_int, [_P, _P, c_int32, c_int32, c_int64, c_int64, c_float, c_float, c_int, _P]),
+    "mi_latent_norm_cache": (c_int, [_P, c_int64, _P, c_int32, _P, _P, c_int32, _P, _P, c_int32, c_int64, c_int64, c_float, c_int32,
+                                     c_int, _P]),
+    "mi_head_gemm": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_latent_attn_rows": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float,
+                                    c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_gated_delta_step": (c_int, [_P, c_int64, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32,
+                                    c_int32, c_int32, c_float, c_int32, c_int, _P]),
     "mi_blockpool_create": (_P, [c_int32]),
     "mi_blockpool_destroy": (None, [_P]),
     "mi_blockpool_num_free": (c_int32, [_P]),
@@ -142,19 +156,33 @@ SIGNATURES = {
 }
 
 
+def _not_in_subset(name: str):
+    def missing(*_args):
+        raise RuntimeError(f"{name} is not part of {_TEXT_LIB_PATH}: build the full library with "
+                           "`python -c 'import __graft_entry__ as g; g.build()'`")
+
+    return missing
+
+
 def _load() -> ctypes.CDLL:
     # torch first: its wheel carries its own libamdhip64, and the process must end up with ONE HIP runtime — if this
     # library were loaded before torch it would pull in /opt/rocm's copy, and kernels registered with that runtime
     # fail to launch on torch's streams ("HIP kernel launch failed"; seen with build() + smoke() in one process)
     import torch  # noqa: F401
 
-    if not os.path.exists(_LIB_PATH):
+    path, subset = _LIB_PATH, False
+    if not os.path.exists(path) and os.path.dirname(path) == _LIB_DIR and os.path.exists(_TEXT_LIB_PATH):
+        path, subset = _TEXT_LIB_PATH, True
+    if not os.path.exists(path):
         raise ImportError(
-            f"{_LIB_PATH} is missing: build it with `python -c 'import __graft_entry__ as g; "
+            f"{path} is missing: build it with `python -c 'import __graft_entry__ as g; "
             "g.build()'` (hipcc --offload-arch=gfx950). There is no CPU fallback."
         )
-    lib = ctypes.CDLL(_LIB_PATH)
+    lib = ctypes.CDLL(path)
     for name, (res, args) in SIGNATURES.items():
+        if subset and not hasattr(lib, name):
+            setattr(lib, name, _not_in_subset(name))
+            continue
         fn = getattr(lib, name)  # AttributeError here == ABI drift, fail loudly
         fn.restype = res
         fn.argtypes = args
@@ -165,7 +193,7 @@ def _load() -> ctypes.CDLL:
 
 
 lib = _load()
-LIB_PATH = _LIB_PATH
+LIB_PATH = lib._name
 
 
 class MIError(RuntimeError):

@@ -105,6 +105,7 @@ def worker_config_from_vllm_config(vc: Any):
     engine_output_type), ``cache_config`` (block_size, gpu_memory_utilization, kv_cache_memory_bytes),
     ``parallel_config`` (tensor_parallel_size, world_size, data-parallel local rank), ``scheduler_config``
     (max_num_seqs, max_num_batched_tokens), ``device_config.device_type``."""
+    from .registry import config_from_hf
     from .worker import WorkerConfig
 
     mc, cc = vc.model_config, vc.cache_config
@@ -124,7 +125,7 @@ def worker_config_from_vllm_config(vc: Any):
     max_len = int(_get(mc, "max_model_len", 4096))
     max_seqs = int(_get(sc, "max_num_seqs", 256))
     return WorkerConfig(
-        model_config=talker_config_from_hf(mc.hf_config), dtype=torch_dtype(_get(mc, "dtype", "bfloat16")),
+        model_config=config_from_hf(mc.hf_config), dtype=torch_dtype(_get(mc, "dtype", "bfloat16")),
         tensor_parallel_size=tp, world_size=int(_get(pc, "world_size", tp)),
         gpu_memory_utilization=float(_get(cc, "gpu_memory_utilization", 0.9)),
         kv_cache_memory_bytes=_get(cc, "kv_cache_memory_bytes"), block_size=block_size,
@@ -236,4 +237,5 @@ def normalize_scheduler_output(so: Any) -> SchedulerOutput:
         finished_req_ids=set(_get(so, "finished_req_ids", set()) or set()),
         num_common_prefix_blocks=list(_get(so, "num_common_prefix_blocks", [0]) or [0]),
         new_block_ids_to_zero=_get(so, "new_block_ids_to_zero"),
+        preempted_req_ids=set(_get(so, "preempted_req_ids", set()) or set()),
         finished_requests_needing_kv_transfer=dict(_get(so, "finished_requests_needing_kv_transfer", {}) or {}))

@@ -602,9 +602,26 @@ class KVCacheSpec:
         return 2 * self.block_size * self.num_kv_heads * self.head_dim * torch.finfo(self.dtype).bits // 8
 
 
-def num_blocks_for_budget(available_bytes: int, num_layers: int, spec: KVCacheSpec) -> int:
-    """A15: how many blocks fit the KV budget (all layers share block ids)."""
-    return max(0, int(available_bytes) // (num_layers * spec.page_bytes))
+@dataclass
+class LatentCacheSpec:
+    """Geometry of one layer's paged latent cache: one row of ``rank`` values per token, shared by all heads."""
+
+    block_size: int
+    rank: int
+    dtype: torch.dtype
+
+    @property
+    def page_bytes(self) -> int:
+        return self.block_size * self.rank * torch.finfo(self.dtype).bits // 8
+
+
+def num_blocks_for_budget(available_bytes: int, num_layers: int, spec) -> int:
+    """A15: how many blocks fit the KV budget (all layers share block ids).  ``spec``: one geometry for ``num_layers``
+    layers, or a dict of the layers that have a cache, each with its own."""
+    per_block = sum(s.page_bytes for s in spec.values()) if isinstance(spec, dict) else num_layers * spec.page_bytes
+    if not per_block:      # no layer keeps a cache: the block table only counts tokens
+        return 1 << 20
+    return max(0, int(available_bytes) // per_block)
 
 
 def determine_available_memory(total_bytes: int, gpu_memory_utilization: float, used_by_process: int,
@@ -704,6 +721,11 @@ def allocate_kv_cache(num_layers: int, num_blocks: int, spec: KVCacheSpec, devic
         else:
             raise ValueError(f"unknown KV layout {layout!r}; expected one of {KV_LAYOUTS}")
     return out
+
+
+def allocate_latent_cache(num_blocks: int, spec: LatentCacheSpec, device) -> torch.Tensor:
+    """[num_blocks, block_size, rank]: a token's row is contiguous, a block's rows follow each other."""
+    return torch.zeros(num_blocks, spec.block_size, spec.rank, dtype=spec.dtype, device=device)
 
 
 def normalize_layer_kv(layer_kv):

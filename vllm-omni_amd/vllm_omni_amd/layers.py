@@ -50,6 +50,10 @@ class AttentionMetadata:
     # at `positions`: RoPE + KV append + attention run as ONE launch (ops.rope_cache_attend_block; the code predictor)
     single_block: bool = False
     uniform_position: Optional[int] = None   # with single_block: every sequence's new token sits at this position
+    # models that take token ids and keep recurrent state (state_cache.py)
+    state_rows: Optional[torch.Tensor] = None   # int32 [num_reqs], device: each request's state slot
+    prev_ids: Optional[torch.Tensor] = None     # int64 [num_tokens], device: the token before each row (< 0: in the slot); None: all in the slots
+    prev_slots: Optional[torch.Tensor] = None   # int32 [num_tokens], device: slot a row leaves its token in (a request's last row), else -1
 
 
 @dataclass

@@ -30,11 +30,13 @@ import torch.nn.functional as F
 
 from . import ops
 from .block_table import MultiGroupBlockTable
-from .kv_cache import KVCacheSpec, allocate_kv_cache, extract_request_kv
+from .kv_cache import KVCacheSpec, allocate_kv_cache, allocate_latent_cache, extract_request_kv
 from .layers import AttentionMetadata, set_forward_context
 from .sched_output import (EMPTY_MODEL_RUNNER_OUTPUT, CachedRequestData, NewRequestData, OmniModelRunnerOutput,
                            SamplingMetadata, SamplingParams, SchedulerOutput)
-from .talker import Qwen2_5OmniTalkerForConditionalGeneration, TalkerConfig
+from .registry import model_class_for
+from .state_cache import StateCache
+from .talker import Qwen2_5OmniTalkerForConditionalGeneration
 
 
 @dataclass
@@ -49,7 +51,7 @@ class CachedRequestState:
     additional_information: Optional[dict] = None
     sample_seed: int = 0                                  # Philox key of the request's draws
     seen_slot: int = -1                                   # row of the device seen-token bitmap, -1 = none
-    state_slot: int = -1                                  # row of the device per-request state (last talker hidden)
+    state_slot: int = -1                                  # row of the device per-request state (last talker hidden / recurrent state)
     reply_base: int = -1                                  # first row of the request's thinker_reply_part in the device pool
     reply_rows: int = 0                                   # rows it owns there
     reply_cursor: int = 0                                 # rows consumed so far (the reference's `q[1:]` queue, qwen2_5_omni.py:771-774)
@@ -386,8 +388,11 @@ class GPUARModelRunner:
         # so a request that hits the KV prefix cache still gets ALL its rows back (gpu_model_runner.py:79-85)
         self.enable_prefix_caching = bool(pick(enable_prefix_caching, wc and wc.enable_prefix_caching, False))
         self.omni_prefix_cache = None
-        if not isinstance(config, TalkerConfig):
-            raise TypeError(f"GPUARModelRunner needs a VllmConfig-shaped object or a TalkerConfig, got {type(config).__name__}")
+        try:
+            registered_cls = model_class_for(config)
+        except TypeError:
+            raise TypeError("GPUARModelRunner needs a VllmConfig-shaped object or the configuration of a registered model, "
+                            f"got {type(config).__name__}") from None
         self.config = config
         self.device = device
         self.dtype = dtype
@@ -407,7 +412,15 @@ class GPUARModelRunner:
         # codec token into all residual codebooks, the talker's input is the SUM of their embeddings + the text step
         self.code_predictor_config = code_predictor
         self.code_predictor = None
-        self.model_cls = model_cls or Qwen2_5OmniTalkerForConditionalGeneration
+        self.model_cls = model_cls or registered_cls
+        # the model embeds token ids itself and may keep recurrent state per request (state_cache.py); the talker's
+        # models take input rows instead
+        self._token_ids = bool(getattr(self.model_cls, "consumes_token_ids", False))
+        if self._token_ids:
+            max_reply_rows = 0
+            if code_predictor is not None:
+                raise ValueError("a code predictor needs a talker model")
+        self.state_cache: Optional[StateCache] = None
         self._generic_hooks = False      # set by load_model: drive the model's hooks per request (eager)
         self.parallel = get_parallel_state()
         self.model: Optional[Qwen2_5OmniTalkerForConditionalGeneration] = None
@@ -417,7 +430,7 @@ class GPUARModelRunner:
 
         # the step's small index arrays live in ONE pinned block / device block: one host->device copy per step
         # instead of one per array (block_table.StepArena); generous: 16 int64 arrays of the larger of tokens / requests
-        self._arena = StepArena(16 * 8 * (max(self.max_num_batched_tokens, max_num_reqs) + 64) + 64 * StepArena.ALIGN, device)
+        self._arena = StepArena(24 * 8 * (max(self.max_num_batched_tokens, max_num_reqs) + 64) + 64 * StepArena.ALIGN, device)
         self.input_batch = InputBatch(max_num_reqs, max_model_len, self.max_num_batched_tokens, block_size, device,
                                       arena=self._arena)
         self.execute_model_state: Optional[ExecuteModelState] = None
@@ -446,7 +459,12 @@ class GPUARModelRunner:
         self.logits_indices = ar.buffer(n, dtype=torch.int64)
         on_gpu = torch.device(dev).type == "cuda"
         e = self.config.embedding_size
-        self.inputs_embeds = torch.zeros(t, e, dtype=self.dtype, device=dev)
+        self.inputs_embeds = None if self._token_ids else torch.zeros(t, e, dtype=self.dtype, device=dev)
+        if self._token_ids:
+            self.input_ids = ar.buffer(t, dtype=torch.int64)
+            self.prev_ids = ar.buffer(t, dtype=torch.int64)
+            self.prev_slots = ar.buffer(t, dtype=torch.int32)
+            self.state_rows = ar.buffer(n, dtype=torch.int32)
         self.sampled_ids_gpu = torch.zeros(n, dtype=torch.int64, device=dev)
         # step outputs go device -> staging (same stream, ~2 us) -> pinned host on a side stream, through a ring of
         # OUT_SLOTS buffers so that the copy of step N can still be in flight while step N+1 runs
@@ -457,9 +475,11 @@ class GPUARModelRunner:
         hs = self.config.hidden_size
         k = self.OUT_SLOTS
         self._out_ids_cpu = [torch.zeros(n, dtype=torch.int64, pin_memory=on_gpu) for _ in range(k)]
-        self._out_hidden_cpu = [torch.zeros(t, hs, dtype=self.dtype, pin_memory=on_gpu) for _ in range(k)]
+        # (no hidden states leave a "text" stage: its ring of hidden rows has none)
+        th = 0 if self.engine_output_type == "text" else t
+        self._out_hidden_cpu = [torch.zeros(th, hs, dtype=self.dtype, pin_memory=on_gpu and th > 0) for _ in range(k)]
         self._out_ids_stage = [torch.zeros(n, dtype=torch.int64, device=dev) for _ in range(k)] if on_gpu else None
-        self._out_hidden_stage = [torch.zeros(t, hs, dtype=self.dtype, device=dev) for _ in range(k)] if on_gpu else None
+        self._out_hidden_stage = [torch.zeros(th, hs, dtype=self.dtype, device=dev) for _ in range(k)] if on_gpu else None
         self.copy_stream = torch.cuda.Stream(device=dev) if on_gpu else None
         self._out_done = [torch.cuda.Event() for _ in range(k)] if on_gpu else None
         self._out_inflight: list[Optional["AsyncOmniModelRunnerOutput"]] = [None] * k
@@ -520,13 +540,31 @@ class GPUARModelRunner:
     def get_model(self):
         return self.model
 
-    def get_kv_cache_spec(self) -> KVCacheSpec:
+    def get_kv_cache_spec(self):
+        """``KVCacheSpec`` of a uniform K/V stack, or {layer: spec} of a model whose layers differ."""
+        if self._token_ids:
+            return self.model.kv_cache_specs(self.block_size)
         a = self.model.language_model.model.layers[0].self_attn
         return KVCacheSpec(self.block_size, a.num_kv_heads, a.head_dim, self.dtype)
+
+    def state_bytes(self) -> int:
+        """Device bytes of the per-request state slots (0: the model keeps none)."""
+        if not self._token_ids:
+            return 0
+        return (self.max_num_reqs + 1) * sum(s.slot_bytes for s in self.model.state_specs())
 
     def initialize_kv_cache(self, num_blocks: int) -> None:
         spec = self.get_kv_cache_spec()
         self.num_gpu_blocks = num_blocks
+        if self._token_ids:
+            if self.enable_prefix_caching and self.model.is_recurrent:
+                raise ValueError("prefix caching re-uses KV blocks only: a model with recurrent layers cannot start behind them")
+            caches = {i: allocate_latent_cache(num_blocks, s, self.device) for i, s in spec.items()}
+            self.kv_caches = list(caches.values())
+            self.model.bind_kv_caches(caches)
+            self.state_cache = StateCache(self.max_num_reqs, self.device)
+            self.model.bind_states(self.state_cache.allocate(self.model.state_specs()))
+            return
         self.kv_caches = allocate_kv_cache(self.config.num_hidden_layers, num_blocks, spec, self.device, self.kv_layout)
         for layer, kv in zip(self.model.language_model.model.layers, self.kv_caches):
             layer.self_attn.attn.bind_kv_cache(kv)
@@ -555,6 +593,9 @@ class GPUARModelRunner:
         idx = torch.as_tensor(block_ids, dtype=torch.int64, device=self.device)
         for kv in self.kv_caches:
             from .kv_cache import normalize_layer_kv
+            if self._token_ids:
+                kv.index_fill_(0, idx, 0)
+                continue
             kb, vb = normalize_layer_kv(kv)
             kb.index_fill_(0, idx, 0)
             vb.index_fill_(0, idx, 0)
@@ -574,7 +615,10 @@ class GPUARModelRunner:
             if st is not None and st.reply_base >= 0:
                 self._reply_alloc.release(st.reply_base, st.reply_rows)
                 st.reply_base, st.reply_rows = -1, 0
+            self._release_state(st)
             ib.remove_request(rid)
+        for rid in so.preempted_req_ids:
+            self._release_state(self.requests.get(rid))
         if so.new_block_ids_to_zero:
             self._zero_block_ids(so.new_block_ids_to_zero)
         cached = so.scheduled_cached_reqs
@@ -616,6 +660,8 @@ class GPUARModelRunner:
             if self.code_predictor is not None:
                 st.state_slot = self._state_free.pop()
                 self._last_hidden[st.state_slot].zero_()
+            if self.state_cache is not None:
+                st.state_slot = self.state_cache.acquire()
             to_add.append(st)
 
         for i, rid in enumerate(cached.req_ids):
@@ -632,6 +678,10 @@ class GPUARModelRunner:
                 st.block_ids = tuple(list(b) for b in new_ids)
                 plen = len(st.prompt_token_ids) or (int(st.prompt_embeds.shape[0]) if st.prompt_embeds is not None else 0)
                 st.recompute_until = plen + len(st.output_token_ids)
+            if self.state_cache is not None and st.state_slot < 0:    # back from a preemption
+                st.state_slot = self.state_cache.acquire()
+            if cached.new_token_ids and cached.new_token_ids[i]:
+                self._extend_prompt(st, cached.new_token_ids[i])
             idx = ib.req_id_to_index.get(rid)
             if idx is None:
                 to_add.append(st)
@@ -659,6 +709,30 @@ class GPUARModelRunner:
                 if row is not None:
                     ib.reply_offset[row], ib.reply_end[row] = -1, 0
                     self._register_reply_part(st, row)
+
+    def _release_state(self, st: Optional[CachedRequestState]) -> None:
+        if self.state_cache is not None and st is not None and st.state_slot >= 0:
+            self.state_cache.release(st.state_slot)
+            st.state_slot = -1
+
+    def _extend_prompt(self, st: CachedRequestState, tokens: list[int]) -> None:
+        """``CachedRequestData.new_token_ids``: tokens from the request's computed position on that the scheduler got
+        from outside (a prompt that arrives in portions).  What the runner does not know yet extends the prompt; a
+        one-token portion then is a decode row like any other."""
+        known = len(st.prompt_token_ids) + len(st.output_token_ids)
+        new = list(tokens)[known - st.num_computed_tokens:]
+        if not new:
+            return
+        if st.output_token_ids or st.prompt_embeds is not None:
+            raise ValueError(f"request {st.req_id}: prompt tokens behind generated ones (or behind prompt embeddings)")
+        st.prompt_token_ids.extend(new)
+        ib = self.input_batch
+        row = ib.req_id_to_index.get(st.req_id)
+        if row is not None:
+            ib.num_prompt_tokens[row] = len(st.prompt_token_ids)
+            ib.decode_from[row] = len(st.prompt_token_ids) - 1
+            ib.last_token_ids_cpu[row] = st.prompt_token_ids[-1]
+            self._ids_on_device_for = None
 
     def _register_reply_part(self, st: CachedRequestState, row: int) -> None:
         """Move a request's ``thinker_reply_part`` rows (one consumed per decode step) into the device-resident
@@ -765,7 +839,59 @@ class GPUARModelRunner:
             num_actual_tokens=total, max_query_len=max_query_len, query_start_loc=self.query_start_loc.gpu[:n + 1],
             seq_lens=self.seq_lens.gpu[:n], max_seq_len=max_seq_len_bound, block_table=bt.block_table.gpu[:n],
             slot_mapping=bt.slot_mapping.gpu[:total], num_reqs=n, num_decodes=num_decodes,
-            decode_partition_size=0, decode_workspace=self._decode_ws)   # 0 = auto, per call
+            decode_partition_size=0, decode_workspace=self._decode_ws,   # 0 = auto, per call
+            **self._token_metadata(n, total, num_decodes))
+
+    def _token_metadata(self, n: int, total: int, num_decodes: int) -> dict:
+        if not self._token_ids:
+            return {}
+        rows = self.state_rows.gpu[:n]
+        if num_decodes == n == total:      # one row per request, the token before it is in its state slot
+            return {"state_rows": rows, "prev_slots": rows}
+        return {"state_rows": rows, "prev_ids": self.prev_ids.gpu[:total], "prev_slots": self.prev_slots.gpu[:total]}
+
+    def _commit_state_rows(self, n: int, padded: int = 0) -> None:
+        for i, rid in enumerate(self.input_batch.req_ids[:n]):
+            self.state_rows.np[i] = self.requests[rid].state_slot
+        m = max(n, padded)
+        self.state_rows.np[n:m] = self.state_cache.scratch_slot
+        self.state_rows.copy_to_gpu(m)
+
+    def _prepare_token_ids(self, n: int, total: int, num_sched: np.ndarray, num_decodes: int) -> None:
+        """Eager step of a model that takes token ids: the step's ids, the token in front of every row and the slot each
+        request's last row leaves its token in.  A pure-decode step reads the device's own last-token buffer instead."""
+        ib = self.input_batch
+        self._commit_state_rows(n)
+        if num_decodes == n == total:
+            if self._ids_on_device_for != tuple(ib.req_ids[:n]):
+                self.last_token_ids.np[:n] = ib.last_token_ids_cpu[:n]
+                self.last_token_ids.copy_to_gpu(n)
+            self._arena.flush()
+            return
+        ids, prev, slots = self.input_ids.np, self.prev_ids.np, self.prev_slots.np
+        slots[:total] = -1
+        t = 0
+        for i in range(n):
+            st = self.requests[ib.req_ids[i]]
+            k, c = int(num_sched[i]), int(ib.num_computed_tokens_cpu[i])
+            if i < num_decodes:
+                ids[t], prev[t] = ib.last_token_ids_cpu[i], -1
+            else:
+                pl = len(st.prompt_token_ids)
+                lo = max(c - 1, 0)
+                toks = st.prompt_token_ids[lo:c + k]
+                if c + k > pl:
+                    toks = toks + st.output_token_ids[max(lo - pl, 0):c + k - pl]
+                if len(toks) != c + k - lo:
+                    raise RuntimeError(f"request {st.req_id}: tokens {lo}..{c + k} scheduled, {len(toks)} known")
+                ids[t:t + k] = toks[-k:]
+                prev[t + 1:t + k] = toks[-k:-1]
+                prev[t] = toks[0] if c else -1
+            slots[t + k - 1] = st.state_slot
+            t += k
+        for b in (self.input_ids, self.prev_ids, self.prev_slots):
+            b.copy_to_gpu(total)
+        self._arena.flush()
 
     def _preprocess_embeds(self, n: int, total: int, num_sched: np.ndarray, num_decodes: int) -> None:
         """Fill ``self.inputs_embeds[:total]`` (the model's ``preprocess`` hook, batched)."""
@@ -914,6 +1040,8 @@ class GPUARModelRunner:
         self._cp_offset.copy_to_gpu(m)
 
     def _decode_embeds(self, nd: int) -> None:
+        if self._token_ids:      # the model's own first kernel embeds
+            return
         if self.code_predictor is not None:
             # talker_mtp (qwen3_omni.py:681-705): codes = code_predictor(last codec token, its embedding, last talker
             # hidden state); input = sum over the G codebook embeddings + the text step of the thinker's reply
@@ -938,8 +1066,12 @@ class GPUARModelRunner:
     def _forward(self, n: int, total: int, md: AttentionMetadata):
         """Model forward + logits + fused mask/argmax on the static buffers."""
         with set_forward_context(md):
-            hidden = self.model(input_ids=None, positions=self.positions.gpu[:total],
-                                inputs_embeds=self.inputs_embeds[:total])
+            if self._token_ids:
+                ids = self.last_token_ids.gpu[:n] if md.num_decodes == n == total else self.input_ids.gpu[:total]
+                hidden = self.model(input_ids=ids, positions=self.positions.gpu[:total])
+            else:
+                hidden = self.model(input_ids=None, positions=self.positions.gpu[:total],
+                                    inputs_embeds=self.inputs_embeds[:total])
         sample_h = hidden if total == n else hidden.index_select(0, self.logits_indices.gpu[:n])
         if self.code_predictor is not None:   # `last_talker_hidden` of the next step (talker_postprocess, qwen3_omni.py:634-640)
             self._last_hidden.index_copy_(0, self._state_rows.gpu[:n], sample_h)
@@ -983,6 +1115,8 @@ class GPUARModelRunner:
         saved = None
         if self.code_predictor is not None:
             saved = (self._last_hidden.clone(), self._cp_codes.clone())
+        if self.state_cache is not None:      # the warm-up runs must not advance live requests' recurrent state
+            self.state_rows.gpu[:n].fill_(self.state_cache.scratch_slot)
         # warm-up on a side stream (library handles, hipBLASLt heuristics), then capture
         s = torch.cuda.Stream(device=self.device)
         s.wait_stream(torch.cuda.current_stream())
@@ -1020,6 +1154,9 @@ class GPUARModelRunner:
         if saved is not None:
             self._last_hidden.copy_(saved[0])
             self._cp_codes.copy_(saved[1])
+        if self.state_cache is not None:
+            self.state_rows.copy_to_gpu(n)
+            self._arena.flush()
         self._graphs[n] = (g, {"hidden": hidden, "logits": logits, "ids": ids})
         return self._graphs[n]
 
@@ -1064,7 +1201,9 @@ class GPUARModelRunner:
             hidden, logits, ids = outs["hidden"], outs["logits"], outs["ids"]
         else:
             self._commit_inputs(n, total)
-            if self._generic_hooks:
+            if self._token_ids:
+                self._prepare_token_ids(n, total, num_sched, num_decodes)
+            elif self._generic_hooks:
                 self._preprocess_embeds_hooks(n, total, num_sched, num_decodes)
             else:
                 self._preprocess_embeds(n, total, num_sched, num_decodes)
@@ -1119,8 +1258,34 @@ class GPUARModelRunner:
             self.last_token_ids.np[:n] = ib.last_token_ids_cpu[:n]
             self.last_token_ids.copy_to_gpu(n)
         self.reply_idx.copy_to_gpu(max(n, padded))
+        if self._token_ids:
+            self._commit_state_rows(n, padded)
         self._commit_predictor_inputs(n, padded)
         self._arena.flush()   # one host->device copy for everything the replay reads
+
+    @torch.inference_mode()
+    def logits_at(self, wanted: dict[str, list[int]]) -> torch.Tensor:
+        """Between ``execute_model`` and ``sample_tokens``: logits (fp32) at the given places of the requests' portions of
+        this step, in the order of ``wanted``."""
+        st = self.execute_model_state
+        if st is None:
+            raise RuntimeError("State error: logits_at() called without a preceding execute_model().")
+        rows = []
+        for rid, places in wanted.items():
+            i = self.input_batch.req_id_to_index[rid]
+            lo, hi = int(st.query_start_loc_np[i]), int(st.query_start_loc_np[i + 1])
+            if any(not 0 <= p < hi - lo for p in places):
+                raise ValueError(f"request {rid}: a place outside its {hi - lo} tokens of this step")
+            rows.extend(lo + p for p in places)
+        idx = torch.as_tensor(rows, dtype=torch.int64, device=self.device)
+        return self.model.compute_logits(st.hidden_states.index_select(0, idx)).float()
+
+    def discard_step(self) -> None:
+        """End a step whose tokens come from outside: nothing is sampled."""
+        if self.execute_model_state is None:
+            raise RuntimeError("State error: discard_step() called without a preceding execute_model().")
+        self.execute_model_state = None
+        self._ids_on_device_for = None
 
     @torch.inference_mode()
     def sample_tokens(self, grammar_output=None, async_output: bool = False):
@@ -1282,6 +1447,8 @@ class GPUARModelRunner:
         decoded view of it (key_cache / value_cache lists, block_ids, metadata)."""
         from .kv_transfer import KVCacheTransferData, pack_request_kv
 
+        if self._token_ids:
+            raise ValueError("KV hand-off is built for K/V caches, not for latent caches and recurrent state")
         done = []
         on_gpu = torch.device(self.device).type == "cuda"
         for rid, info in finished.items():

@@ -1061,3 +1061,188 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gate_up: torch.Ten
         _p(out), _p(part), _p(row_of_pair), _p(w), _p(shared_out), _p(x), _p(shared_gate_weight), t, h, top_k,
         part.stride(0), out.stride(0), x.stride(0), shared_out.stride(0) if shared_out is not None else 0, dt, _stream()))
     return out
+
+
+# ------------------------------------------------- 32-bit residual stream, latent attention, gated delta rule
+def _rows(t: torch.Tensor) -> tuple[int, int]:
+    """(row stride, columns) of a 2-D tensor with contiguous rows"""
+    if t.dim() != 2 or t.stride(1) != 1:
+        raise ValueError("expected a 2-D tensor with contiguous rows")
+    return t.stride(0), t.shape[1]
+
+
+def _i32(*ts: Optional[torch.Tensor]) -> None:
+    for t in ts:
+        if t is not None and (t.dtype != torch.int32 or not t.is_contiguous()):
+            raise TypeError("expected a contiguous int32 tensor")
+
+
+def _i64(*ts: Optional[torch.Tensor]) -> None:
+    for t in ts:
+        if t is not None and (t.dtype != torch.int64 or not t.is_contiguous()):
+            raise TypeError("expected a contiguous int64 tensor")
+
+
+def residual_norm(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials"], w_post: torch.Tensor,
+                  w_pre: Optional[torch.Tensor], eps: float, want_h: bool = True) -> Optional[torch.Tensor]:
+    """``x += rms_norm(y; w_post)`` in place (x fp32 [T, W]); returns ``rms_norm(x; w_pre)``, or x cast to w_post's dtype
+    when ``w_pre`` is None.  ``y`` may be the split-K partials of the linear in front."""
+    part = isinstance(y, SplitKPartials)
+    if part:
+        y._live()
+        if y.bias is not None:
+            raise ValueError("residual_norm takes partials of a linear without bias")
+    src = y.part if part else y
+    _gpu(x, src, w_post, w_pre)
+    xs, width = _rows(x)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or w_post.numel() != width or (w_pre is not None and (w_pre.numel() != width or w_pre.dtype != w_post.dtype)):
+        raise ValueError("residual_norm: fp32 stream and weights of its width")
+    if part:
+        if (y.m, y.n) != (rows, width):
+            raise ValueError("partials of another shape")
+        ys = width
+    else:
+        ys, yw = _rows(y)
+        if y.shape[0] != rows or yw != width or y.dtype != w_post.dtype:
+            raise ValueError("sublayer output of another shape or dtype")
+    h = torch.empty(rows, width, dtype=w_post.dtype, device=x.device) if want_h else None
+    check("mi_residual_norm", lib.mi_residual_norm(
+        _p(x), _p(src), y.split if part else 0, _p(w_post), _p(w_pre), _p(h), float(eps), rows, width, xs, ys,
+        width, _dt(w_post.dtype), _stream()))
+    return h
+
+
+def pair_embed_norm(table: torch.Tensor, pairs: torch.Tensor, w_pre: torch.Tensor, ids: torch.Tensor,
+                    prev_ids: Optional[torch.Tensor], slots: torch.Tensor, last_token: torch.Tensor, positions: torch.Tensor,
+                    scale: float, mul_prev: int, mul_cur: int, eps: float) -> tuple[torch.Tensor, torch.Tensor]:
+    """Scaled token row + pair row (``pairs`` [buckets + 1, W]) -> (x fp32, rms_norm(x; w_pre))."""
+    _gpu(table, pairs, w_pre, ids, prev_ids, slots, last_token, positions)
+    _i64(ids, prev_ids, last_token, positions)
+    _i32(slots)
+    t, (vocab, width) = ids.shape[0], table.shape
+    if slots.numel() < t or positions.numel() < t or (prev_ids is not None and prev_ids.numel() < t):
+        raise ValueError("pair_embed_norm: index arrays shorter than the rows")
+    if pairs.shape[1] != width or w_pre.numel() != width or not (table.is_contiguous() and pairs.is_contiguous()):
+        raise ValueError("pair_embed_norm: tables of different widths")
+    x = torch.empty(t, width, dtype=torch.float32, device=table.device)
+    h = torch.empty(t, width, dtype=table.dtype, device=table.device)
+    check("mi_pair_embed_norm", lib.mi_pair_embed_norm(
+        _p(x), _p(h), _p(table), _p(pairs), _p(w_pre), _p(ids), _p(prev_ids), _p(slots), _p(last_token), _p(positions),
+        float(scale), int(mul_prev), int(mul_cur), pairs.shape[0] - 1, float(eps), t, width, vocab, width, width,
+        _dt(table.dtype), _stream()))
+    return x, h
+
+
+def gelu_lookup_mul(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, offset: int) -> torch.Tensor:
+    """``gelu_tanh(z) * table[ids, offset : offset + z.shape[1]]``"""
+    _gpu(z, table, ids)
+    _i64(ids)
+    zs, dim = _rows(z)
+    ts, cols = _rows(table)
+    if offset + dim > cols or ids.numel() < z.shape[0] or table.dtype != z.dtype:
+        raise ValueError("gelu_lookup_mul: slice outside the table, or dtypes differ")
+    out = torch.empty(z.shape[0], dim, dtype=z.dtype, device=z.device)
+    check("mi_gelu_lookup_mul", lib.mi_gelu_lookup_mul(_p(out), _p(z), _p(table), _p(ids), z.shape[0], dim, zs, ts, int(offset),
+                                                       table.shape[0], _dt(z.dtype), _stream()))
+    return out
+
+
+def clamped_glu(gate_up: torch.Tensor, alpha: float, limit: float) -> torch.Tensor:
+    """[T, 2 F] gate | up -> [T, F]: g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)"""
+    _gpu(gate_up)
+    gs, two = _rows(gate_up)
+    t, ff = gate_up.shape[0], two // 2
+    out = torch.empty(t, ff, dtype=gate_up.dtype, device=gate_up.device)
+    check("mi_clamped_glu", lib.mi_clamped_glu(_p(out), _p(gate_up), t, ff, gs, ff, float(alpha), float(limit),
+                                               _dt(gate_up.dtype), _stream()))
+    return out
+
+
+def latent_norm_cache(x: torch.Tensor, q_weight: torch.Tensor, c_weight: Optional[torch.Tensor], cache: Optional[torch.Tensor],
+                      slot_mapping: Optional[torch.Tensor], eps: float) -> torch.Tensor:
+    """Row = query latent | new cache latent: returns the normed query latent, writes the normed cache rows
+    (``cache`` [blocks, block_size, rank]) at their slots.  ``c_weight`` None: no cache half."""
+    _gpu(x, q_weight, c_weight, cache, slot_mapping)
+    xs, cols = _rows(x)
+    t, nq = x.shape[0], q_weight.numel()
+    nc = 0 if c_weight is None else c_weight.numel()
+    if cols < nq + nc or q_weight.dtype != x.dtype:
+        raise ValueError("latent_norm_cache: row shorter than its two halves")
+    bs = cb = ct = 0
+    if nc:
+        _i64(slot_mapping)
+        if cache.dim() != 3 or cache.shape[2] != nc or cache.stride(2) != 1 or cache.dtype != x.dtype or slot_mapping.numel() < t:
+            raise ValueError("latent_norm_cache: cache [blocks, block_size, rank] of x's dtype, one slot per row")
+        bs, cb, ct = cache.shape[1], cache.stride(0), cache.stride(1)
+    out = torch.empty(t, nq, dtype=x.dtype, device=x.device)
+    check("mi_latent_norm_cache", lib.mi_latent_norm_cache(
+        _p(x), xs, _p(q_weight), nq, _p(out), _p(c_weight), nc, _p(cache) if nc else None, _p(slot_mapping) if nc else None,
+        bs, cb, ct, float(eps), t, _dt(x.dtype), _stream()))
+    return out
+
+
+def head_gemm(x: torch.Tensor, w: torch.Tensor, transposed: bool = False) -> torch.Tensor:
+    """``y[t, h] = w[h] @ x[t, h]`` for x [T, H * K] and w [H, N, K] (``transposed``: w [H, K, N], used as w[h]^T)."""
+    _gpu(x, w)
+    xs, cols = _rows(x)
+    hh, a, b = w.shape
+    n, k = (b, a) if transposed else (a, b)
+    if cols != hh * k or w.dtype != x.dtype:
+        raise ValueError("head_gemm: x [T, heads * k] and w of one dtype")
+    y = torch.empty(x.shape[0], hh * n, dtype=x.dtype, device=x.device)
+    sn, sk = (w.stride(2), w.stride(1)) if transposed else (w.stride(1), w.stride(2))
+    check("mi_head_gemm", lib.mi_head_gemm(_p(y), _p(x), _p(w), x.shape[0], hh, n, k, hh * n, xs, w.stride(0), sn, sk,
+                                           _dt(x.dtype), _stream()))
+    return y
+
+
+def _latent_cache(cache: torch.Tensor, rank: int) -> tuple[int, int, int]:
+    if cache.dim() != 3 or cache.shape[2] != rank or cache.stride(2) != 1:
+        raise ValueError("latent cache must be [blocks, block_size, rank] with contiguous rows")
+    return cache.shape[1], cache.stride(0), cache.stride(1)
+
+
+def latent_attn_rows(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, seq_lens: torch.Tensor,
+                     query_start_loc: torch.Tensor, heads: int, window: int, scale: float, row0: int = 0,
+                     out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Absorbed latent attention of rows [row0, T) of ``q`` [T, heads * rank]; any sizes and dtypes."""
+    _gpu(q, cache, block_table, seq_lens, query_start_loc)
+    _i32(seq_lens, query_start_loc)
+    rank = q.shape[1] // heads
+    bs, cb, ct = _latent_cache(cache, rank)
+    if not q.is_contiguous() or cache.dtype != q.dtype or block_table.dtype != torch.int32 or block_table.stride(1) != 1:
+        raise ValueError("latent_attn_rows: contiguous q of the cache's dtype, int32 block table")
+    out = torch.empty_like(q) if out is None else out
+    check("mi_latent_attn_rows", lib.mi_latent_attn_rows(
+        _p(out), _p(q), _p(cache), _p(block_table), _p(seq_lens), _p(query_start_loc), row0, q.shape[0] - row0,
+        seq_lens.shape[0], heads, rank, bs, min(int(window), 2**31 - 1), float(scale), cb, ct, block_table.stride(0),
+        _dt(q.dtype), _stream()))
+    return out
+
+
+def gated_delta_step(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor,
+                     state: torch.Tensor, ring: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
+                     seq_lens: torch.Tensor, kv_heads: int, eps: float, out: torch.Tensor, req0: int, num_reqs: int,
+                     update_ring: bool = True) -> torch.Tensor:
+    """Gated delta rule of requests [req0, req0 + num_reqs), token by token.  ``state`` fp32 [slots, H, D, V], ``ring``
+    [slots, taps, channels]; ``out`` [T, H * V] receives the requests' rows."""
+    _gpu(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, out)
+    _i32(slots, query_start_loc, seq_lens)
+    ps, _ = _rows(proj)
+    _, hh, d, v = state.shape
+    taps, ch = ring.shape[1], ring.shape[2]
+    if not (state.is_contiguous() and ring.is_contiguous() and conv_w.is_contiguous() and out.is_contiguous()):
+        raise ValueError("gated_delta_step: contiguous state, ring, conv weights and output")
+    if state.dtype != torch.float32 or a_log.dtype != torch.float32 or dt_bias.dtype != torch.float32:
+        raise TypeError("recurrent state, A_log and dt_bias are fp32")
+    if ch != 2 * kv_heads * d + hh * v or tuple(conv_w.shape) != (ch, taps) or out.shape[1] != hh * v or norm_w.numel() != v:
+        raise ValueError("gated_delta_step: sizes do not fit")
+    if any(t.dtype != proj.dtype for t in (conv_w, norm_w, ring, out)):
+        raise TypeError("gated_delta_step: one activation dtype")
+    if req0 + num_reqs > seq_lens.shape[0] or slots.shape[0] < req0 + num_reqs or query_start_loc.shape[0] < req0 + num_reqs + 1:
+        raise ValueError("gated_delta_step: request range outside the metadata")
+    check("mi_gated_delta_step", lib.mi_gated_delta_step(
+        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
+        _p(seq_lens), _p(out), req0, num_reqs, hh, kv_heads, d, v, taps, float(eps), int(update_ring), _dt(proj.dtype), _stream()))
+    return out

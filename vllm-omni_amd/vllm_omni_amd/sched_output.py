@@ -151,6 +151,9 @@ class SchedulerOutput:
     finished_req_ids: set[str] = field(default_factory=set)
     num_common_prefix_blocks: list[int] = field(default_factory=lambda: [0])
     new_block_ids_to_zero: Optional[list[int]] = None
+    # requests preempted in this step: what the runner holds for them (state slots) is free again, their tokens are
+    # recomputed from position 0 when they resume
+    preempted_req_ids: set[str] = field(default_factory=set)
     # finished requests whose KV must be extracted before their blocks are reused
     # (OmniSchedulerOutput.finished_requests_needing_kv_transfer, core/sched/output.py:73-77)
     finished_requests_needing_kv_transfer: dict[str, dict] = field(default_factory=dict)

@@ -247,6 +247,12 @@ class StandaloneARScheduler:
                 new_blocks_of[req.request_id] = kv.get_block_ids(req.request_id)
                 budget -= n
 
+        return self._build_output(num_scheduled, new_blocks_of, scheduled_new, scheduled_resumed, scheduled_running,
+                                  preempted)
+
+    def _build_output(self, num_scheduled: dict[str, int], new_blocks_of: dict, scheduled_new: list, scheduled_resumed: list,
+                      scheduled_running: list, preempted: list, new_tokens: Optional[dict] = None) -> SchedulerOutput:
+        kv = self.kv_cache_manager
         total = sum(num_scheduled.values())
         assert total <= self.max_num_scheduled_tokens and len(self.running) <= self.max_num_running_reqs
         new_data = [NewRequestData(r.request_id, list(r.prompt_token_ids), r.sampling_params,
@@ -256,7 +262,7 @@ class StandaloneARScheduler:
         for r in scheduled_running + scheduled_resumed:
             rid = r.request_id
             cached.req_ids.append(rid)
-            cached.new_token_ids.append([])
+            cached.new_token_ids.append(list((new_tokens or {}).get(rid, ())))
             cached.new_block_ids.append(new_blocks_of.get(rid))
             cached.num_computed_tokens.append(r.num_computed_tokens)
             cached.num_output_tokens.append(r.num_output_tokens)
@@ -267,6 +273,7 @@ class StandaloneARScheduler:
         out = SchedulerOutput(scheduled_new_reqs=new_data, scheduled_cached_reqs=cached,
                               num_scheduled_tokens=num_scheduled, total_num_scheduled_tokens=total,
                               finished_req_ids=self.finished_req_ids, num_common_prefix_blocks=common,
+                              preempted_req_ids={r.request_id for r in preempted},
                               finished_requests_needing_kv_transfer=self.get_finished_requests_needing_kv_transfer())
         self.finished_req_ids = set()
         # upstream's `_update_after_schedule`: the tokens count as computed as soon as they are scheduled, so the next
@@ -274,6 +281,49 @@ class StandaloneARScheduler:
         for rid, n in num_scheduled.items():
             self.requests[rid].num_computed_tokens += n
         return out
+
+    def schedule_portions(self, portions: dict[str, list[int]]) -> SchedulerOutput:
+        """A step whose work is given: for every named request exactly these next tokens, all in one batch.  A name the
+        scheduler does not know yet is admitted; a running request that is not named keeps what it holds and sits the
+        step out.  Nothing is preempted: a pool or a batch too small for the step raises, with nothing scheduled."""
+        kv = self.kv_cache_manager
+        kv.new_step_starts()
+        fresh = [rid for rid in portions if rid not in self.requests]
+        if len(self.running) + len(fresh) > self.max_num_running_reqs:
+            raise RuntimeError(f"{len(self.running) + len(fresh)} live requests, at most {self.max_num_running_reqs}")
+        counts = {rid: len(t) for rid, t in portions.items()}
+        if min(counts.values(), default=1) < 1 or sum(counts.values()) > self.max_num_scheduled_tokens:
+            raise ValueError("a portion holds at least one token, a step at most "
+                             f"{self.max_num_scheduled_tokens} (this one: {sum(counts.values())})")
+        num_scheduled: dict[str, int] = {}
+        new_blocks_of: dict[str, Optional[tuple[list[int], ...]]] = {}
+        new, old = [], []
+        need = 0
+        for rid, n in counts.items():
+            req = self.requests.get(rid)
+            if req is not None and req.status != RequestStatus.RUNNING:
+                raise ValueError(f"request {rid} is not running")
+            have = len(kv.req_to_blocks.get(rid, ()))
+            need += max(0, -(-((req.num_computed_tokens if req else 0) + n) // self.block_size) - have)
+        if need > kv.block_pool.get_num_free_blocks():
+            raise RuntimeError(f"the step needs {need} KV blocks, {kv.block_pool.get_num_free_blocks()} are free")
+        for rid, n in counts.items():
+            req = self.requests.get(rid)
+            if req is None:
+                req = Request(rid, list(portions[rid]))
+                self.add_request(req)
+                self.waiting.remove(req)
+                self.running.append(req)
+                req.status = RequestStatus.RUNNING
+                new.append(req)
+            else:
+                req.prompt_token_ids = list(req.prompt_token_ids) + list(portions[rid])
+                old.append(req)
+            blocks = kv.allocate_slots(req, n)
+            assert blocks is not None
+            num_scheduled[rid] = n
+            new_blocks_of[rid] = blocks.get_block_ids() if blocks.blocks[0] else None
+        return self._build_output(num_scheduled, new_blocks_of, new, [], old, [], portions)
 
     # --------------------------------------------------------------- update_from_output
     def _should_transfer_kv_for_request(self, req_id: str) -> bool:

@@ -15,12 +15,11 @@ import torch
 from .distributed import init_distributed_environment
 from .kv_cache import determine_available_memory, get_process_gpu_memory, num_blocks_for_budget
 from .model_runner import GPUARModelRunner
-from .talker import TalkerConfig
 
 
 @dataclass
 class WorkerConfig:
-    model_config: TalkerConfig
+    model_config: object                      # configuration of a registered model (registry.py)
     dtype: torch.dtype = torch.bfloat16
     tensor_parallel_size: int = 1
     world_size: int = 1
@@ -160,7 +159,7 @@ class GPUARWorker:
 
     def determine_num_available_blocks(self) -> int:
         spec = self.get_kv_cache_spec()
-        return num_blocks_for_budget(self.determine_available_memory(), self.config.model_config.num_hidden_layers, spec)
+        return num_blocks_for_budget(self.determine_available_memory() - self.model_runner.state_bytes(), self.config.model_config.num_hidden_layers, spec)
 
     def initialize_cache(self, num_gpu_blocks: int) -> None:
         self.model_runner.initialize_kv_cache(num_gpu_blocks)
