@@ -134,6 +134,7 @@ class DogulornForCausalLM:
     """Takes token ids (and each request's state slot) from the step's metadata; returns final-normed hidden rows."""
 
     consumes_token_ids = True
+    extra_dtypes = (torch.float32,)      # runs in true 32-bit as well
     has_preprocess = False
     has_postprocess = False
     prefer_model_sampler = False

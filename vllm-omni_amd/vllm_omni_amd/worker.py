@@ -15,6 +15,7 @@ import torch
 from .distributed import init_distributed_environment
 from .kv_cache import determine_available_memory, get_process_gpu_memory, num_blocks_for_budget
 from .model_runner import GPUARModelRunner
+from .registry import model_class_for
 
 
 @dataclass
@@ -105,7 +106,9 @@ class GPUARWorker:
         torch.cuda.set_device(self.device)
         from .platform import MI355XOmniPlatform
 
-        MI355XOmniPlatform.check_if_supports_dtype(self.config.dtype)
+        # 32-bit is a property of the model's kernels, 16-bit types one of the platform
+        if self.config.dtype not in getattr(model_class_for(self.config.model_config), "extra_dtypes", ()):
+            MI355XOmniPlatform.check_if_supports_dtype(self.config.dtype)
         # distributed groups first, so communicator buffers are inside the memory snapshot
         init_distributed_environment(self.config.world_size, self.rank, self.config.tensor_parallel_size,
                                      backend=self.config.distributed_backend,
