@@ -766,6 +766,38 @@ int mi_latent_attn_rows(void* out, const void* q, const void* cache, const int32
                         int32_t block_size, int32_t window, float scale,
                         int64_t cache_block_stride, int64_t cache_token_stride,
                         int64_t table_stride, int dtype, void* stream);
+/* bf16, matrix cores.  mi_head_gemm_nt: w [heads][n][k]; k % 8 == 0, n % 4 == 0. */
+int mi_head_gemm_nt(void* y, const void* x, const void* w, int32_t rows, int32_t heads, int32_t n,
+                    int32_t k, int64_t y_row_stride, int64_t x_row_stride, int64_t w_head_stride,
+                    void* stream);
+/* Absorbed latent attention of one query per request (its newest token): q, out
+ * [num_reqs][heads][kv_rank], kv_rank <= 512 and a multiple of 8; seq_lens 0 (a
+ * padded row) gives zeros.  The launch depends on window and max_seq_len only. */
+int64_t mi_latent_decode_workspace_bytes(int32_t num_reqs, int32_t heads, int32_t kv_rank,
+                                         int32_t window, int32_t max_seq_len);
+int mi_latent_decode(void* out, const void* q, const void* cache, const int32_t* block_table,
+                     const int32_t* seq_lens, int32_t num_reqs, int32_t heads, int32_t kv_rank,
+                     int32_t block_size, int32_t window, int32_t max_seq_len, float scale,
+                     int64_t cache_block_stride, int64_t cache_token_stride, int64_t table_stride,
+                     void* workspace, int64_t workspace_bytes, void* stream);
+/* Dense context of prompt portions: request r's rows start at ctx_start[r] (a
+ * multiple of 64; ctx_start[num_reqs] == ctx_rows) and hold the cache rows of
+ * positions max(0, first query - window + 1) .. last query, then zeros. */
+int mi_latent_gather(void* ctx, const void* cache, const int32_t* ctx_start,
+                     const int32_t* block_table, const int32_t* seq_lens,
+                     const int32_t* query_start_loc, int32_t num_reqs, int32_t ctx_rows,
+                     int32_t kv_rank, int32_t block_size, int32_t window,
+                     int64_t cache_block_stride, int64_t cache_token_stride, int64_t table_stride,
+                     void* stream);
+/* Windowed attention of prompt portions over that context: k [ctx_rows][heads dim],
+ * vt [heads vdim][ctx_rows]; dim, vdim <= 256 and multiples of 8; query_start_loc
+ * indexes the rows of q and out. */
+int mi_latent_prefill(void* out, const void* q, const void* k, const void* vt,
+                      const int32_t* ctx_start, const int32_t* seq_lens,
+                      const int32_t* query_start_loc, int32_t num_reqs, int32_t max_query_len,
+                      int32_t heads, int32_t dim, int32_t vdim, int32_t window, float scale,
+                      int64_t out_stride, int64_t q_stride, int64_t k_stride, int64_t vt_stride,
+                      void* stream);
 /* Gated delta rule over requests [req0, req0 + num_reqs), token by token:
  * proj rows [q | k | v | gate | b | a] (heads / kv_heads q-k sharing), short
  * causal convolutions (conv_w [2 kv_heads dim + heads vdim][taps]) + silu, unit
@@ -779,6 +811,19 @@ int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_
                         const int32_t* seq_lens, void* out, int32_t req0, int32_t num_reqs,
                         int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps,
                         float eps, int32_t update_ring, int dtype, void* stream);
+/* The same for prompt portions, 64 tokens at a time on the fp32 matrix cores
+ * (dim, vdim <= 256): requests [req0, req0 + num_reqs) own rows [row0, row0 +
+ * rows); o_f32 [total rows][heads vdim] and the workspace are scratch. */
+int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads,
+                                               int32_t dim, int32_t vdim);
+int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w,
+                           const float* a_log, const float* dt_bias, const void* norm_w,
+                           float* state, void* ring, const int32_t* slots,
+                           const int32_t* query_start_loc, const int32_t* seq_lens, void* out,
+                           float* o_f32, int32_t row0, int32_t rows, int32_t req0, int32_t num_reqs,
+                           int32_t max_query_len, int32_t heads, int32_t kv_heads, int32_t dim,
+                           int32_t vdim, int32_t taps, float eps, void* workspace,
+                           int64_t workspace_bytes, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -142,20 +142,6 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
   }
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void conv_ring_update_kernel(const DeltaParams p) {
-  scalar_cache_acquire();
-  const int r = p.req0 + blockIdx.y;
-  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
-  const int ch = blockIdx.x * 256 + threadIdx.x;
-  if (L <= 1 || ch >= p.CH) return;
-  const int start = p.seq_lens[r] - L;
-  T* ring = reinterpret_cast<T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
-  const T* proj = reinterpret_cast<const T*>(p.proj);
-  for (int i = max(0, L - p.taps); i < L; ++i)
-    if (start + i >= 0) ring[(int64_t)((start + i) % p.taps) * p.CH + ch] = proj[(s0 + i) * p.ld + ch];
-}
-
 template <typename T, int VEC, int NT>
 int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
   const int groups = NT / (p.V / VEC);

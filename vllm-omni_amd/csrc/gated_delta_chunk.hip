@@ -1,0 +1,458 @@
+// Gated delta rule over prompt portions, in chunks of 64 tokens on the fp32 matrix cores.
+//
+// Within a chunk with entry state S0, G_i = sum of log decays up to i, u_i the corrected values:
+//   (I + A) U = diag(b) (V - diag(e^G) K S0),   A_ij = b_i e^(G_i - G_j) k_i . k_j  (j < i)
+//   O = diag(e^G) Q S0 + P U,                   P_ij = e^(G_i - G_j) q_i . k_j      (j <= i)
+//   S1 = e^(G_C) S0 + sum_j e^(G_C - G_j) k_j u_j^T
+// so everything but the S0 terms is independent between chunks:
+//   * prep (one workgroup per chunk and head): convolutions, silu, unit q / k, gates; A, its unit-triangular inverse T,
+//     P, and T diag(b) V, T diag(b e^G) K, diag(e^G) Q, (e^(G_C - G_j) k_j)^T to a workspace;
+//   * scan (one workgroup per request, head and 16 value columns): chunk after chunk, U, O and S with S in registers;
+//   * finish: o / rms(o) * norm * silu(gate).
+// All products run on v_mfma_f32_16x16x4_f32: q, k, decays and state are 32-bit quantities of the recurrence.  The k order
+// inside 16 consecutive k is permuted alike in both operands (step s takes k = 4 (lane / 16) + s), so an operand whose k is
+// contiguous is one 16-byte read for four steps, and an accumulator tile IS the B operand of a following product.
+#include "gated_delta.h"
+#include "mfma_attn_common.h"
+
+namespace mi {
+namespace {
+
+constexpr int kC = 64;             // tokens per chunk
+constexpr int kPrepThreads = 512;
+
+__device__ __forceinline__ f32x4_t mma4(const float (&a)[4], const float (&b)[4], f32x4_t c) {
+#pragma unroll
+  for (int s = 0; s < 4; ++s) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[s], b[s], c, 0, 0, 0);
+  return c;
+}
+__device__ __forceinline__ void frag_rows(const float* p, int ld, int lane, float (&f)[4]) {   // [row][k], k contiguous
+  const float4 v = *reinterpret_cast<const float4*>(p + (lane & 15) * ld + 4 * (lane >> 4));
+  f[0] = v.x, f[1] = v.y, f[2] = v.z, f[3] = v.w;
+}
+__device__ __forceinline__ void frag_cols(const float* p, int ld, int lane, float (&f)[4]) {   // [k][col]
+#pragma unroll
+  for (int s = 0; s < 4; ++s) f[s] = p[(4 * (lane >> 4) + s) * ld + (lane & 15)];
+}
+
+// workspace of one (chunk, head): W [C][Dp], Q [C][Dp], Kt [Dp][C], P [C][C], U [C][Vp], then e^(G_C)
+struct ChunkLayout {
+  int Dp, Vp;
+  __host__ __device__ int64_t w() const { return 0; }
+  __host__ __device__ int64_t q() const { return (int64_t)kC * Dp; }
+  __host__ __device__ int64_t kt() const { return 2 * (int64_t)kC * Dp; }
+  __host__ __device__ int64_t pm() const { return 3 * (int64_t)kC * Dp; }
+  __host__ __device__ int64_t u() const { return 3 * (int64_t)kC * Dp + kC * kC; }
+  __host__ __device__ int64_t g() const { return u() + (int64_t)kC * Vp; }
+  __host__ __device__ int64_t size() const { return g() + 16; }
+};
+
+__device__ __forceinline__ int64_t chunk_base(const DeltaParams& p, int r) {
+  return (p.qsl[r] - p.qsl[p.req0]) / kC + (r - p.req0);
+}
+
+// conv + silu of channels [ch0, ch0 + n) of the chunk's rows into buf [C][ld]; zeros in rows past len and columns past n
+template <typename T>
+__device__ __forceinline__ void conv_rows(const DeltaParams& p, float* buf, int ld, int np, int ch0, int n, int64_t row0, int i0,
+                                          int len, int start, const T* ring) {
+  const T* proj = reinterpret_cast<const T*>(p.proj);
+  const T* cw = reinterpret_cast<const T*>(p.convw);
+  const int segs = kPrepThreads / np > 0 ? kPrepThreads / np : 1;      // row segments worked on side by side
+  const int rows_per = (kC + segs - 1) / segs;
+  for (int item = threadIdx.x; item < segs * np; item += kPrepThreads) {
+    const int c = item % np, seg = item / np;
+    const int a = seg * rows_per, b = min(kC, a + rows_per);
+    if (c >= n) {
+      for (int i = a; i < b; ++i) buf[i * ld + c] = 0.f;
+      continue;
+    }
+    const int ch = ch0 + c;
+    // input of chunk row i (may be negative: rows of this portion in front of the chunk, then the ring, then zeros)
+    auto in = [&](int i) -> float {
+      if (i >= len) return 0.f;
+      if (i0 + i >= 0) return Io<T>::ld(proj + (row0 + i) * p.ld + ch);
+      const int pos = start + i0 + i;
+      return pos >= 0 ? Io<T>::ld(ring + (int64_t)(pos % p.taps) * p.CH + ch) : 0.f;
+    };
+    if (p.taps == 4) {
+      const float w0 = Io<T>::ld(cw + ch * 4), w1 = Io<T>::ld(cw + ch * 4 + 1), w2 = Io<T>::ld(cw + ch * 4 + 2),
+                  w3 = Io<T>::ld(cw + ch * 4 + 3);
+      float x0 = in(a - 3), x1 = in(a - 2), x2 = in(a - 1);
+      for (int i = a; i < b; ++i) {
+        float v = 0.f;
+        if (i < len) {
+          const float x3 = Io<T>::ld(proj + (row0 + i) * p.ld + ch);
+          v = silu_f(w0 * x0 + w1 * x1 + w2 * x2 + w3 * x3);
+          x0 = x1, x1 = x2, x2 = x3;
+        }
+        buf[i * ld + c] = v;
+      }
+    } else {
+      for (int i = a; i < b; ++i) {
+        float v = 0.f;
+        if (i < len) {
+          for (int t = 0; t < p.taps; ++t) v += Io<T>::ld(cw + (int64_t)ch * p.taps + t) * in(i - (p.taps - 1) + t);
+          v = silu_f(v);
+        }
+        buf[i * ld + c] = v;
+      }
+    }
+  }
+}
+
+// rows of buf made unit vectors (16 lanes a row), then times mul
+__device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul) {
+  const int sub = threadIdx.x & 15;
+  for (int i = threadIdx.x >> 4; i < kC; i += kPrepThreads / 16) {
+    float ss = 0.f;
+    for (int c = sub; c < np; c += 16) ss += buf[i * ld + c] * buf[i * ld + c];
+    ss = group_allreduce_sum<16>(ss);
+    const float f = mul / sqrtf(ss + 1e-6f);
+    for (int c = sub; c < np; c += 16) buf[i * ld + c] *= f;
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay) {
+  scalar_cache_acquire();
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int r = p.req0 + blockIdx.z, h = blockIdx.y, ck = blockIdx.x;
+  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
+  const int i0 = ck * kC;
+  if (i0 >= L) return;
+  const int len = min(kC, L - i0);
+  const int start = p.seq_lens[r] - L;
+  const int64_t row0 = s0 + i0;
+  const int Dp = lay.Dp, Vp = lay.Vp, ldk = Dp + 4, ldm = kC + 4;
+  const int ldv = Vp + 4, big = kC * max(ldk, ldv);
+  float* bufA = lds;                       // K, then V
+  float* bufB = bufA + big;                // Q, then T
+  float* mA = bufB + max(kC * ldk, kC * ldm);   // A
+  float* sG = mA + kC * ldm;               // G_i
+  float* sB = sG + kC;                     // b_i
+  float* sE = sB + kC;                     // b_i e^(G_i)
+  float* mT = bufB;
+  float* out = ws + ((chunk_base(p, r) + ck) * p.H + h) * lay.size();
+  const T* ring = reinterpret_cast<const T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int kh = h / (p.H / p.K);
+  conv_rows<T>(p, bufA, ldk, Dp, p.K * p.D + kh * p.D, p.D, row0, i0, len, start, ring);
+  conv_rows<T>(p, bufB, ldk, Dp, kh * p.D, p.D, row0, i0, len, start, ring);
+  if (wave == 0) {   // gates: cumulative log decay over the 64 tokens of the chunk
+    const T* pr = reinterpret_cast<const T*>(p.proj) + (row0 + lane) * p.ld;
+    float lg = 0.f, b = 0.f;
+    if (lane < len) {
+      lg = -expf(p.a_log[h]) * softplus_f(Io<T>::ld(pr + p.off_a + h) + p.dt_bias[h]);
+      b = sigmoid_f(Io<T>::ld(pr + p.off_b + h));
+    }
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float t = __shfl_up(lg, o, 64);
+      if (lane >= o) lg += t;
+    }
+    sG[lane] = lg;
+    sB[lane] = b;
+    sE[lane] = b * expf(lg);
+    if (lane == 63) out[lay.g()] = expf(lg);
+  }
+  __syncthreads();
+  unit_rows(bufA, ldk, Dp, 1.0f);
+  unit_rows(bufB, ldk, Dp, 1.0f / sqrtf((float)p.D));
+  __syncthreads();
+  // A and P: the 10 lower tiles of each
+  for (int t = wave; t < 32; t += kPrepThreads / 64) {
+    const bool isP = t >= 16;
+    const int ti = (t & 15) >> 2, tj = t & 3;
+    if (tj > ti) continue;   // above the diagonal: neither A nor P is read there
+    const float* a = (isP ? bufB : bufA) + ti * 16 * ldk;
+    const float* b = bufA + tj * 16 * ldk;
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < Dp; k += 16) {
+      float fa[4], fb[4];
+      frag_rows(a + k, ldk, lane, fa);
+      frag_rows(b + k, ldk, lane, fb);
+      acc = mma4(fa, fb, acc);
+    }
+    const int j = tj * 16 + (lane & 15);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const int i = ti * 16 + 4 * (lane >> 4) + s;
+      const float e = expf(fminf(sG[i] - sG[j], 0.f));
+      if (isP) out[lay.pm() + i * kC + j] = j <= i ? acc[s] * e : 0.f;
+      else mA[i * ldm + j] = j < i ? acc[s] * e * sB[i] : 0.f;
+    }
+  }
+  // diag(e^G) Q and the transposed, decayed keys
+  for (int n = tid; n < kC * Dp / 4; n += kPrepThreads) {
+    const int i = n / (Dp / 4), c = (n % (Dp / 4)) * 4;
+    const float e = expf(sG[i]);
+    const float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
+    *reinterpret_cast<float4*>(out + lay.q() + (int64_t)i * Dp + c) = make_float4(v.x * e, v.y * e, v.z * e, v.w * e);
+  }
+  for (int n = tid; n < kC * Dp; n += kPrepThreads) {
+    const int d = n / kC, j = n % kC;
+    out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * expf(sG[kC - 1] - sG[j]) : 0.f;
+  }
+  __syncthreads();   // Q is dead: T takes its place
+  // T = (I + A)^-1: diagonal 16 x 16 blocks by substitution, one column a lane
+  if (wave < 4 && lane < 16) {
+    const float* a = mA + wave * 16 * ldm + wave * 16;
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == lane ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) v -= a[i * ldm + j] * x[j];
+      x[i] = v;
+      mT[(wave * 16 + i) * ldm + wave * 16 + lane] = v;
+    }
+  }
+  __syncthreads();
+  for (int dist = 1; dist < 4; ++dist) {   // T_ij = -T_ii sum_k A_ik T_kj
+    if (wave < 4 - dist) {
+      const int tj = wave, ti = wave + dist;
+      f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+      float fa[4], fb[4];
+      for (int k = tj; k < ti; ++k) {
+        frag_rows(mA + ti * 16 * ldm + k * 16, ldm, lane, fa);
+        frag_cols(mT + k * 16 * ldm + tj * 16, ldm, lane, fb);
+        acc = mma4(fa, fb, acc);
+      }
+      frag_rows(mT + ti * 16 * ldm + ti * 16, ldm, lane, fa);
+      fb[0] = -acc[0], fb[1] = -acc[1], fb[2] = -acc[2], fb[3] = -acc[3];
+      f32x4_t z = {0.f, 0.f, 0.f, 0.f};
+      z = mma4(fa, fb, z);
+#pragma unroll
+      for (int s = 0; s < 4; ++s) mT[(ti * 16 + 4 * (lane >> 4) + s) * ldm + tj * 16 + (lane & 15)] = z[s];
+    }
+    __syncthreads();
+  }
+  // T diag(f) X, X [C][n] in bufA
+  auto times = [&](const float* f, int ld, int np, float* dst) {
+    const int nt = np / 16;
+    for (int t = wave; t < 4 * nt; t += kPrepThreads / 64) {
+      const int ti = t / nt, tn = t % nt;
+      f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k <= ti; ++k) {
+        float fa[4], fb[4];
+        frag_rows(mT + ti * 16 * ldm + k * 16, ldm, lane, fa);
+#pragma unroll
+        for (int s = 0; s < 4; ++s) fa[s] *= f[k * 16 + 4 * (lane >> 4) + s];
+        frag_cols(bufA + k * 16 * ld + tn * 16, ld, lane, fb);
+        acc = mma4(fa, fb, acc);
+      }
+#pragma unroll
+      for (int s = 0; s < 4; ++s) dst[(int64_t)(ti * 16 + 4 * (lane >> 4) + s) * np + tn * 16 + (lane & 15)] = acc[s];
+    }
+  };
+  times(sE, ldk, Dp, out + lay.w());
+  __syncthreads();
+  conv_rows<T>(p, bufA, ldv, Vp, 2 * p.K * p.D + h * p.V, p.V, row0, i0, len, start, ring);
+  __syncthreads();
+  times(sB, ldv, Vp, out + lay.u());
+}
+
+// LDS-only barrier: register loads in flight stay in flight
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+template <int DT>
+__global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, float* o,
+                                                               int nvt) {
+  scalar_cache_acquire();
+  constexpr int Dp = DT * 16, LS = Dp + 4, LU = kC + 4, MT = (DT + 3) / 4;
+  __shared__ __attribute__((aligned(16))) float sS[16 * LS];
+  __shared__ __attribute__((aligned(16))) float sU[16 * LU];
+  // the value tiles of a head on one XCD (workgroups go to the 8 XCDs in turn): they read the same workspace
+  const int bid = blockIdx.x;
+  const int h = (bid / (8 * nvt)) * 8 + bid % 8, vt = (bid / 8) % nvt;
+  const int r = p.req0 + blockIdx.y;
+  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
+  if (h >= p.H || L <= 0) return;
+  const int start = p.seq_lens[r] - L;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, lg = lane >> 4;
+  const int v = vt * 16 + lr;
+  float* S = p.state + (((int64_t)p.slots[r] * p.H + h) * p.D) * p.V;
+  f32x4_t st[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int mt = wave + 4 * m;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = mt * 16 + 4 * lg + i;
+      st[m][i] = start > 0 && d < p.D && v < p.V ? S[(int64_t)d * p.V + v] : 0.f;
+    }
+    if (mt < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + mt * 16 + 4 * lg) = st[m];
+  }
+  const int nck = (L + kC - 1) / kC;
+  const float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
+  const int64_t step = p.H * lay.size();
+  f32x4_t w[DT], q[DT];
+  f32x4_t u;
+  auto load_front = [&](const float* b) {
+    const int64_t ro = (int64_t)(16 * wave + lr) * Dp + 4 * lg;
+#pragma unroll
+    for (int k = 0; k < DT; ++k) {
+      w[k] = *reinterpret_cast<const f32x4_t*>(b + lay.w() + ro + 16 * k);
+      q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u[i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v];
+  };
+  load_front(base);
+  lds_barrier();
+  for (int c = 0; c < nck; ++c) {
+    const float* b = base + c * step;
+    // loads of the second half of this chunk, under the first half's products
+    f32x4_t pm[4], kt[MT][4];
+    for (int k = 0; k < 4; ++k) {
+      if (k <= wave) pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+        if (wave + 4 * m < DT)
+          kt[m][k] = *reinterpret_cast<const f32x4_t*>(b + lay.kt() + (int64_t)((wave + 4 * m) * 16 + lr) * kC + 16 * k + 4 * lg);
+    }
+    const float gc = b[lay.g()];
+    f32x4_t x = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < DT; ++k) {
+      const f32x4_t sv = *reinterpret_cast<const f32x4_t*>(sS + lr * LS + 16 * k + 4 * lg);
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        x = __builtin_amdgcn_mfma_f32_16x16x4f32(w[k][s], sv[s], x, 0, 0, 0);
+        ao = __builtin_amdgcn_mfma_f32_16x16x4f32(q[k][s], sv[s], ao, 0, 0, 0);
+      }
+    }
+    u -= x;
+    *reinterpret_cast<f32x4_t*>(sU + lr * LU + 16 * wave + 4 * lg) = u;
+    lds_barrier();
+    if (c + 1 < nck) load_front(b + step);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) st[m] *= gc;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const f32x4_t uv = *reinterpret_cast<const f32x4_t*>(sU + lr * LU + 16 * k + 4 * lg);
+      if (k <= wave)
+#pragma unroll
+        for (int s = 0; s < 4; ++s) ao = __builtin_amdgcn_mfma_f32_16x16x4f32(pm[k][s], uv[s], ao, 0, 0, 0);
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+        if (wave + 4 * m < DT)
+#pragma unroll
+          for (int s = 0; s < 4; ++s) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[m][k][s], uv[s], st[m], 0, 0, 0);
+    }
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+      if (wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + (wave + 4 * m) * 16 + 4 * lg) = st[m];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = c * kC + 16 * wave + 4 * lg + i;
+      if (t < L && v < p.V) o[((int64_t)(s0 + t) * p.H + h) * p.V + v] = ao[i];
+    }
+    lds_barrier();
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = (wave + 4 * m) * 16 + 4 * lg + i;
+      if (d < p.D && v < p.V) S[(int64_t)d * p.V + v] = st[m][i];
+    }
+}
+
+// out = o / rms(o) * norm * silu(gate), one wave per (row, head)
+template <typename T>
+__global__ __launch_bounds__(256) void gated_delta_finish_kernel(const DeltaParams p, const float* o, int row0, int rows) {
+  scalar_cache_acquire();
+  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63;
+  if (item >= (int64_t)rows * p.H) return;
+  const int64_t row = row0 + item / p.H;
+  const int h = (int)(item % p.H);
+  const float* x = o + (row * p.H + h) * (int64_t)p.V;
+  float ss = 0.f;
+  for (int v = lane; v < p.V; v += 64) ss += x[v] * x[v];
+  const float inv = inv_rms(wave_allreduce_sum(ss), p.V, p.eps);
+  const T* g = reinterpret_cast<const T*>(p.proj) + row * p.ld + p.off_g + h * p.V;
+  const T* nw = reinterpret_cast<const T*>(p.norm_w);
+  T* out = reinterpret_cast<T*>(p.out) + (row * p.H + h) * (int64_t)p.V;
+  for (int v = lane; v < p.V; v += 64) Io<T>::st(out + v, x[v] * inv * Io<T>::ld(nw + v) * silu_f(Io<T>::ld(g + v)));
+}
+
+inline int round_tiles(int n) {   // 16-column tiles of the built scans: 2, 4, 8, 16
+  const int t = (n + 15) / 16;
+  return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 16;
+}
+
+}  // namespace
+}  // namespace mi
+
+using namespace mi;
+
+static bool chunk_layout(int32_t dim, int32_t vdim, ChunkLayout* lay) {
+  if (dim <= 0 || vdim <= 0 || dim > 256 || vdim > 256) return false;
+  lay->Dp = 16 * round_tiles(dim);
+  lay->Vp = (vdim + 15) / 16 * 16;
+  return true;
+}
+
+extern "C" int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t dim, int32_t vdim) {
+  ChunkLayout lay;
+  if (rows < 0 || num_reqs < 0 || heads <= 0 || !chunk_layout(dim, vdim, &lay)) return 0;
+  const int64_t chunks = rows / kC + num_reqs;
+  return chunks * heads * lay.size() * 4;
+}
+
+extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w, const float* a_log,
+                                      const float* dt_bias, const void* norm_w, float* state, void* ring, const int32_t* slots,
+                                      const int32_t* query_start_loc, const int32_t* seq_lens, void* out, float* o_f32, int32_t row0,
+                                      int32_t rows, int32_t req0, int32_t num_reqs, int32_t max_query_len, int32_t heads,
+                                      int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps, float eps, void* workspace,
+                                      int64_t workspace_bytes, int dtype, void* stream) {
+  if (num_reqs == 0 || rows == 0) return MI_OK;
+  if (!proj || !conv_w || !a_log || !dt_bias || !norm_w || !state || !ring || !slots || !query_start_loc || !seq_lens || !out ||
+      !o_f32 || !workspace)
+    return MI_ERR_INVALID_ARG;
+  if (req0 < 0 || num_reqs < 0 || row0 < 0 || rows < 0 || max_query_len <= 0 || heads <= 0 || kv_heads <= 0 || taps <= 0 ||
+      heads % kv_heads)
+    return MI_ERR_INVALID_ARG;
+  ChunkLayout lay;
+  if (!chunk_layout(dim, vdim, &lay)) return MI_ERR_UNSUPPORTED;
+  if (workspace_bytes < mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, heads, dim, vdim)) return MI_ERR_WORKSPACE;
+  const int CH = 2 * kv_heads * dim + heads * vdim;
+  if (proj_stride < CH + heads * vdim + 2 * heads) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  const DeltaParams p{proj, conv_w, norm_w, ring, out, a_log, dt_bias, state, slots, query_start_loc, seq_lens, proj_stride, req0,
+                      heads, kv_heads, dim, vdim, taps, CH, CH, CH + heads * vdim, CH + heads * vdim + heads, eps};
+  hipStream_t s = (hipStream_t)stream;
+  float* ws = (float*)workspace;
+  const int ldk = lay.Dp + 4, ldv = lay.Vp + 4, ldm = kC + 4;
+  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > ldm ? ldk : ldm) + kC * ldm + 3 * kC) * 4;
+  const dim3 pg((max_query_len + kC - 1) / kC, heads, num_reqs);
+#define MI_PREP(T)                                                                                                        \
+  do {                                                                                                                    \
+    auto kern = gated_delta_prep_kernel<T>;                                                                               \
+    if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
+      return MI_ERR_LAUNCH;                                                                                               \
+    hipLaunchKernelGGL(kern, pg, dim3(kPrepThreads), lds, s, p, ws, lay);                                                 \
+  } while (0)
+  if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
+  else MI_PREP(float);
+#undef MI_PREP
+  const int nvt = lay.Vp / 16;
+  const dim3 sg((heads + 7) / 8 * 8 * nvt, num_reqs);
+  switch (lay.Dp / 16) {
+    case 2: hipLaunchKernelGGL((gated_delta_scan_kernel<2>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
+    case 4: hipLaunchKernelGGL((gated_delta_scan_kernel<4>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
+    case 8: hipLaunchKernelGGL((gated_delta_scan_kernel<8>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
+    default: hipLaunchKernelGGL((gated_delta_scan_kernel<16>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
+  }
+  const dim3 fg((unsigned)(((int64_t)rows * heads + 3) / 4)), rg((CH + 255) / 256, num_reqs);
+  if (dtype == MI_DTYPE_BF16) {
+    hipLaunchKernelGGL((gated_delta_finish_kernel<uint16_t>), fg, dim3(256), 0, s, p, o_f32, row0, rows);
+    hipLaunchKernelGGL((conv_ring_update_kernel<uint16_t>), rg, dim3(256), 0, s, p);
+  } else {
+    hipLaunchKernelGGL((gated_delta_finish_kernel<float>), fg, dim3(256), 0, s, p, o_f32, row0, rows);
+    hipLaunchKernelGGL((conv_ring_update_kernel<float>), rg, dim3(256), 0, s, p);
+  }
+  return launch_status();
+}

@@ -176,6 +176,10 @@ class DogulornForCausalLM:
                 src = layer.mixer.cfg.kv_from
                 layer.mixer.cache = caches[i if src is None else src]
 
+    def prefill_windows(self) -> list[int]:
+        """windows of the layers whose prompt attention runs on a gathered context"""
+        return sorted({layer.mixer.window for layer in self.layers if isinstance(layer.mixer, LatentAttention)})
+
     def state_specs(self) -> list[StateSpec]:
         specs = [StateSpec((), torch.int64)]          # the previous token
         for layer in self.layers:
@@ -240,6 +244,9 @@ class DogulornForCausalLM:
                 raise ValueError(f"{name}: checkpoint shape {tuple(w.shape)}, parameter {tuple(dst.shape)}")
             dst.copy_(w.to(dst.dtype))
             loaded.add(name)
+        for layer in self.layers:
+            if isinstance(layer.mixer, LatentAttention):
+                layer.mixer.weights_changed()
         return loaded
 
     def weight_bytes(self) -> int:

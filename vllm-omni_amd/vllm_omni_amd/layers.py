@@ -12,7 +12,7 @@ from __future__ import annotations
 import math
 import os
 from contextlib import contextmanager
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Optional, Sequence
 
 import torch
@@ -53,6 +53,10 @@ class AttentionMetadata:
     # models that take token ids and keep recurrent state (state_cache.py)
     state_rows: Optional[torch.Tensor] = None   # int32 [num_reqs], device: each request's state slot
     prev_ids: Optional[torch.Tensor] = None     # int64 [num_tokens], device: the token before each row (< 0: in the slot); None: all in the slots
+    # window -> (int32 [prefill requests + 1] device, rows): where each prompt portion's visible context starts in the dense
+    # matrix its attention runs on (64-row aligned)
+    prefill_ctx: dict = field(default_factory=dict)
+    step_cache: dict = field(default_factory=dict)   # what layers of one step share (gathered contexts)
     prev_slots: Optional[torch.Tensor] = None   # int32 [num_tokens], device: slot a row leaves its token in (a request's last row), else -1
 
 

@@ -8,6 +8,7 @@ from dataclasses import dataclass
 from typing import Iterable, Optional
 
 import torch
+import torch.nn.functional as F
 
 from . import ops
 from .kv_cache import LatentCacheSpec
@@ -69,6 +70,7 @@ class LatentAttention:
         self.dq_norm = torch.ones(cfg.q_rank, dtype=dtype, device=device)
         self.dkv_norm = torch.ones(cfg.kv_rank, dtype=dtype, device=device) if own else None
         self.cache: Optional[torch.Tensor] = None
+        self._uk_t: Optional[torch.Tensor] = None
 
     def kv_cache_spec(self, block_size: int) -> Optional[LatentCacheSpec]:
         return LatentCacheSpec(block_size, self.cfg.kv_rank, self.dtype) if self.cfg.kv_from is None else None
@@ -84,10 +86,53 @@ class LatentAttention:
         c = self.cfg
         cq = ops.latent_norm_cache(self.down(h), self.dq_norm, self.dkv_norm, self.cache, md.slot_mapping, self.eps)
         q = self.uq(cq)
-        qa = ops.head_gemm(q, self.uk.weight.view(c.heads, c.dim, c.kv_rank), transposed=True)
-        oa = ops.latent_attn_rows(qa, self.cache, md.block_table, md.seq_lens, md.query_start_loc, c.heads, self.window, c.scale)
-        o = ops.head_gemm(oa, self.uv.weight.view(c.heads, c.vdim, c.kv_rank))
+        nd, total = md.num_decodes, q.shape[0]
+        o = torch.empty(total, c.heads * c.vdim, dtype=q.dtype, device=q.device)
+        if nd:
+            self._decode(q[:nd], o[:nd], md)
+        if nd < total:
+            self._prefill(q, o, md)
         return self.o(o, defer_reduce)
+
+    def weights_changed(self) -> None:
+        self._uk_t = None
+
+    def _absorb_weight(self) -> torch.Tensor:
+        """W_uk per head transposed, [H, rank, dim]: the absorb product then reads rows"""
+        if self._uk_t is None:
+            c = self.cfg
+            self._uk_t = self.uk.weight.view(c.heads, c.dim, c.kv_rank).transpose(1, 2).contiguous()
+        return self._uk_t
+
+    def _rows(self, q: torch.Tensor, o: torch.Tensor, md: AttentionMetadata, row0: int) -> None:
+        """rows [row0, T) through the kernel that takes any sizes and types"""
+        c = self.cfg
+        qa = ops.head_gemm(q, self.uk.weight.view(c.heads, c.dim, c.kv_rank), transposed=True)
+        oa = ops.latent_attn_rows(qa, self.cache, md.block_table, md.seq_lens, md.query_start_loc, c.heads, self.window, c.scale,
+                                  row0=row0)
+        o[row0:] = ops.head_gemm(oa[row0:], self.uv.weight.view(c.heads, c.vdim, c.kv_rank))
+
+    def _decode(self, q: torch.Tensor, o: torch.Tensor, md: AttentionMetadata) -> None:
+        c = self.cfg
+        if not ops.latent_decode_supported(self.dtype, c.kv_rank, c.dim, c.vdim, self.cache.shape[1]):
+            return self._rows(q, o, md, 0)
+        qa = ops.head_gemm_nt(q, self._absorb_weight())
+        oa = ops.latent_decode(qa, self.cache, md.block_table, md.seq_lens, c.heads, self.window, md.max_seq_len, c.scale)
+        ops.head_gemm_nt(oa, self.uv.weight.view(c.heads, c.vdim, c.kv_rank), o)
+
+    def _prefill(self, q: torch.Tensor, o: torch.Tensor, md: AttentionMetadata) -> None:
+        c, nd = self.cfg, md.num_decodes
+        if not ops.latent_prefill_supported(self.dtype, c.kv_rank, c.dim, c.vdim):
+            return self._rows(q, o, md, nd)
+        start, rows = md.prefill_ctx[self.window]
+        table, lens, qsl = md.block_table[nd:], md.seq_lens[nd:], md.query_start_loc[nd:]
+        key = (self.cache.data_ptr(), self.window)      # layers that share a cache share its gathered rows
+        ctx = md.step_cache.get(key)
+        if ctx is None:
+            ctx = md.step_cache[key] = ops.latent_gather(self.cache, start, rows, table, lens, qsl, self.window)
+        # K by rows, V transposed: the attention kernel reads both along its k dimension
+        ops.latent_prefill(o, q, F.linear(ctx, self.uk.weight), F.linear(self.uv.weight, ctx), start, lens, qsl, md.max_query_len,
+                           c.heads, self.window, c.scale)
 
 
 @dataclass
@@ -146,7 +191,7 @@ class GatedDelta:
         if nd:
             ops.gated_delta_step(*args, 0, nd, update_ring=False)
         if nd < md.num_reqs:
-            ops.gated_delta_step(*args, nd, md.num_reqs - nd)
+            ops.gated_delta_chunked(*args, nd, md.num_reqs - nd, nd, md.max_query_len)
         return self.o(out, defer_reduce)
 
 

@@ -564,6 +564,12 @@ class GPUARModelRunner:
             self.model.bind_kv_caches(caches)
             self.state_cache = StateCache(self.max_num_reqs, self.device)
             self.model.bind_states(self.state_cache.allocate(self.model.state_specs()))
+            from .block_table import CpuGpuBuffer
+
+            # per window: where every prompt portion's context starts (written per step; not in the shared arena, whose size
+            # is fixed before the model is known)
+            self._ctx_starts = {w: CpuGpuBuffer(self.max_num_reqs + 1, dtype=torch.int32, device=self.device)
+                                for w in self.model.prefill_windows()}
             return
         self.kv_caches = allocate_kv_cache(self.config.num_hidden_layers, num_blocks, spec, self.device, self.kv_layout)
         for layer, kv in zip(self.model.language_model.model.layers, self.kv_caches):
@@ -848,7 +854,8 @@ class GPUARModelRunner:
         rows = self.state_rows.gpu[:n]
         if num_decodes == n == total:      # one row per request, the token before it is in its state slot
             return {"state_rows": rows, "prev_slots": rows}
-        return {"state_rows": rows, "prev_ids": self.prev_ids.gpu[:total], "prev_slots": self.prev_slots.gpu[:total]}
+        return {"state_rows": rows, "prev_ids": self.prev_ids.gpu[:total], "prev_slots": self.prev_slots.gpu[:total],
+                "prefill_ctx": {w: (b.gpu[:n - num_decodes + 1], int(b.np[n - num_decodes])) for w, b in self._ctx_starts.items()}}
 
     def _commit_state_rows(self, n: int, padded: int = 0) -> None:
         for i, rid in enumerate(self.input_batch.req_ids[:n]):
@@ -891,6 +898,12 @@ class GPUARModelRunner:
             t += k
         for b in (self.input_ids, self.prev_ids, self.prev_slots):
             b.copy_to_gpu(total)
+        computed, k = ib.num_computed_tokens_cpu[num_decodes:n], num_sched[num_decodes:n]
+        for w, b in self._ctx_starts.items():
+            seen = computed + k - np.maximum(computed - w + 1, 0)       # cache rows a portion can see
+            b.np[0] = 0
+            np.cumsum(-(-seen // 64) * 64, out=b.np[1:n - num_decodes + 1])
+            b.copy_to_gpu(n - num_decodes + 1)
         self._arena.flush()
 
     def _preprocess_embeds(self, n: int, total: int, num_sched: np.ndarray, num_decodes: int) -> None:

@@ -1221,17 +1221,127 @@ def latent_attn_rows(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Te
     return out
 
 
+def latent_decode_supported(dtype: torch.dtype, kv_rank: int, dim: int, vdim: int, block_size: int) -> bool:
+    return (dtype == torch.bfloat16 and kv_rank % 8 == 0 and kv_rank <= 512 and dim % 8 == 0 and vdim % 4 == 0
+            and block_size & (block_size - 1) == 0)
+
+
+def latent_prefill_supported(dtype: torch.dtype, kv_rank: int, dim: int, vdim: int) -> bool:
+    return dtype == torch.bfloat16 and kv_rank % 8 == 0 and dim % 8 == 0 and vdim % 8 == 0 and max(dim, vdim) <= 256
+
+
+def head_gemm_nt(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``head_gemm`` for w [H, N, K] on the matrix cores (bf16, K a multiple of 8, N of 4)."""
+    _gpu(x, w, out)
+    xs, cols = _rows(x)
+    hh, n, k = w.shape
+    if cols != hh * k or w.dtype != torch.bfloat16 or x.dtype != torch.bfloat16 or not w.is_contiguous():
+        raise ValueError("head_gemm_nt: bf16 x [T, heads * k] and contiguous w [heads, n, k]")
+    y = torch.empty(x.shape[0], hh * n, dtype=x.dtype, device=x.device) if out is None else out
+    check("mi_head_gemm_nt", lib.mi_head_gemm_nt(_p(y), _p(x), _p(w), x.shape[0], hh, n, k, y.stride(0), xs, n * k, _stream()))
+    return y
+
+
+def latent_decode(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, seq_lens: torch.Tensor, heads: int, window: int,
+                  max_seq_len: int, scale: float) -> torch.Tensor:
+    """Absorbed latent attention of one query per request, ``q`` [R, heads * rank] bf16."""
+    _gpu(q, cache, block_table, seq_lens)
+    _i32(seq_lens)
+    n, rank = q.shape[0], q.shape[1] // heads
+    bs, cb, ct = _latent_cache(cache, rank)
+    if not q.is_contiguous() or q.dtype != torch.bfloat16 or cache.dtype != torch.bfloat16 or block_table.dtype != torch.int32:
+        raise TypeError("latent_decode: contiguous bf16 q, bf16 cache, int32 block table")
+    if seq_lens.shape[0] < n or block_table.shape[0] < n or block_table.stride(1) != 1:
+        raise ValueError("latent_decode: one block-table row and length per query")
+    window = min(int(window), 2**31 - 1)
+    need = lib.mi_latent_decode_workspace_bytes(n, heads, rank, window, max_seq_len)
+    ws = torch.empty(need, dtype=torch.uint8, device=q.device) if need else None
+    out = torch.empty_like(q)
+    check("mi_latent_decode", lib.mi_latent_decode(
+        _p(out), _p(q), _p(cache), _p(block_table), _p(seq_lens), n, heads, rank, bs, window, max_seq_len, float(scale), cb, ct,
+        block_table.stride(0), _p(ws), need, _stream()))
+    return out
+
+
+def latent_gather(cache: torch.Tensor, ctx_start: torch.Tensor, ctx_rows: int, block_table: torch.Tensor, seq_lens: torch.Tensor,
+                  query_start_loc: torch.Tensor, window: int) -> torch.Tensor:
+    """[ctx_rows, rank]: per request the cache rows its portion can see, 64-row aligned, zero padded."""
+    _gpu(cache, ctx_start, block_table, seq_lens, query_start_loc)
+    _i32(ctx_start, seq_lens, query_start_loc)
+    rank, n = cache.shape[2], seq_lens.shape[0]
+    bs, cb, ct = _latent_cache(cache, rank)
+    if cache.dtype != torch.bfloat16 or ctx_start.shape[0] < n + 1 or query_start_loc.shape[0] < n + 1 or block_table.shape[0] < n:
+        raise ValueError("latent_gather: bf16 cache and one entry per request")
+    ctx = torch.empty(ctx_rows, rank, dtype=cache.dtype, device=cache.device)
+    check("mi_latent_gather", lib.mi_latent_gather(
+        _p(ctx), _p(cache), _p(ctx_start), _p(block_table), _p(seq_lens), _p(query_start_loc), n, ctx_rows, rank, bs,
+        min(int(window), 2**31 - 1), cb, ct, block_table.stride(0), _stream()))
+    return ctx
+
+
+def latent_prefill(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, vt: torch.Tensor, ctx_start: torch.Tensor,
+                   seq_lens: torch.Tensor, query_start_loc: torch.Tensor, max_query_len: int, heads: int, window: int,
+                   scale: float) -> torch.Tensor:
+    """Windowed attention of prompt portions: q [T, heads * dim], k [ctx, heads * dim], vt [heads * vdim, ctx] -> out rows."""
+    _gpu(out, q, k, vt, ctx_start, seq_lens, query_start_loc)
+    _i32(ctx_start, seq_lens, query_start_loc)
+    qs, qc = _rows(q)
+    ks, kc = _rows(k)
+    vs, vc = _rows(vt)
+    os_, oc = _rows(out)
+    n = seq_lens.shape[0]
+    if qc != kc or vt.shape[0] != oc or vc != k.shape[0] or qc % heads or oc % heads or out.shape[0] < q.shape[0]:
+        raise ValueError("latent_prefill: sizes do not fit")
+    if any(t.dtype != torch.bfloat16 for t in (out, q, k, vt)) or ctx_start.shape[0] < n + 1 or query_start_loc.shape[0] < n + 1:
+        raise TypeError("latent_prefill: bf16 operands and one entry per request")
+    check("mi_latent_prefill", lib.mi_latent_prefill(
+        _p(out), _p(q), _p(k), _p(vt), _p(ctx_start), _p(seq_lens), _p(query_start_loc), n, max_query_len, heads, qc // heads,
+        oc // heads, min(int(window), 2**31 - 1), float(scale), os_, qs, ks, vs, _stream()))
+    return out
+
+
 def gated_delta_step(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor,
                      state: torch.Tensor, ring: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
                      seq_lens: torch.Tensor, kv_heads: int, eps: float, out: torch.Tensor, req0: int, num_reqs: int,
                      update_ring: bool = True) -> torch.Tensor:
     """Gated delta rule of requests [req0, req0 + num_reqs), token by token.  ``state`` fp32 [slots, H, D, V], ``ring``
     [slots, taps, channels]; ``out`` [T, H * V] receives the requests' rows."""
+    ps, hh, d, v, taps = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
+                                     kv_heads, out, req0, num_reqs)
+    check("mi_gated_delta_step", lib.mi_gated_delta_step(
+        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
+        _p(seq_lens), _p(out), req0, num_reqs, hh, kv_heads, d, v, taps, float(eps), int(update_ring), _dt(proj.dtype), _stream()))
+    return out
+
+
+def gated_delta_chunked(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads: int,
+                        eps: float, out: torch.Tensor, req0: int, num_reqs: int, row0: int, max_query_len: int) -> torch.Tensor:
+    """The same for prompt portions (requests [req0, req0 + num_reqs) own the rows from ``row0`` to the end of ``proj``), 64
+    tokens at a time on the fp32 matrix cores; sizes outside its envelope (dim or vdim > 256) go token by token."""
+    ps, hh, d, v, taps = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
+                                     kv_heads, out, req0, num_reqs)
+    rows = proj.shape[0] - row0
+    need = lib.mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, hh, d, v)
+    if not need:
+        return gated_delta_step(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads,
+                                eps, out, req0, num_reqs)
+    ws = torch.empty(need, dtype=torch.uint8, device=proj.device)
+    o = torch.empty(proj.shape[0], hh * v, dtype=torch.float32, device=proj.device)
+    check("mi_gated_delta_chunked", lib.mi_gated_delta_chunked(
+        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
+        _p(seq_lens), _p(out), _p(o), row0, rows, req0, num_reqs, max_query_len, hh, kv_heads, d, v, taps, float(eps), _p(ws),
+        need, _dt(proj.dtype), _stream()))
+    return out
+
+
+def _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads, out, req0, num_reqs):
     _gpu(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, out)
     _i32(slots, query_start_loc, seq_lens)
-    ps, _ = _rows(proj)
+    ps, cols = _rows(proj)
     _, hh, d, v = state.shape
     taps, ch = ring.shape[1], ring.shape[2]
+    if cols < ch + hh * v + 2 * hh or out.shape[0] < proj.shape[0]:
+        raise ValueError("gated_delta: projection rows [q | k | v | gate | b | a], one output row each")
     if not (state.is_contiguous() and ring.is_contiguous() and conv_w.is_contiguous() and out.is_contiguous()):
         raise ValueError("gated_delta_step: contiguous state, ring, conv weights and output")
     if state.dtype != torch.float32 or a_log.dtype != torch.float32 or dt_bias.dtype != torch.float32:
@@ -1242,7 +1352,4 @@ def gated_delta_step(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tens
         raise TypeError("gated_delta_step: one activation dtype")
     if req0 + num_reqs > seq_lens.shape[0] or slots.shape[0] < req0 + num_reqs or query_start_loc.shape[0] < req0 + num_reqs + 1:
         raise ValueError("gated_delta_step: request range outside the metadata")
-    check("mi_gated_delta_step", lib.mi_gated_delta_step(
-        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
-        _p(seq_lens), _p(out), req0, num_reqs, hh, kv_heads, d, v, taps, float(eps), int(update_ring), _dt(proj.dtype), _stream()))
-    return out
+    return ps, hh, d, v, taps
