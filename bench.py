@@ -74,6 +74,12 @@ def parse_args():
                          "headline workload only), 'recorded' = the figure kept in profiles/, 'none' = null")
     ap.add_argument("--pmc-child", action="store_true", help=argparse.SUPPRESS)   # the profiled pass itself
     ap.add_argument("--cpu-baseline-batch", type=int, default=4)
+    ap.add_argument("--dogulorn", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the Dogulorn stack beside the "
+                         "talker stack of equal size (tools/bench_dogulorn.py; one JSON line per case)")
+    ap.add_argument("--dogulorn-size", default="2k,4k")
+    ap.add_argument("--dogulorn-mode", default="decode,prefill")
+    ap.add_argument("--dogulorn-models", default="dogulorn,talker")
     a = ap.parse_args()
     if a.pmc_child:   # a few steps of the same workload, nothing else: the parent reads the counters of the decode launches
         a.steps, a.warmup, a.no_cpu_baseline, a.roofline_steps, a.traffic = 2, 1, True, 0, "none"
@@ -575,6 +581,12 @@ def time_allreduce(dev, rows: int, cols: int, calls: int = 50) -> dict:
 
 def main():
     a = parse_args()
+    if a.dogulorn:
+        sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "tools"))
+        sys.modules.setdefault("bench", sys.modules[__name__])
+        import bench_dogulorn
+
+        return bench_dogulorn.run(a)
     launched = "WORLD_SIZE" in os.environ
     if a.gpus > 1 and not launched:
         # no launcher around us: become one.  Nothing has touched the GPU yet (device_count() does not).
