@@ -593,6 +593,10 @@ int mi_fused_add_rms_norm_splitk(void* out, const void* partials, int32_t split,
 int mi_linear_silu_mul(void* out, const void* x, const void* weight, int32_t m, int32_t inter,
                        int32_t k, int64_t x_row_stride, int64_t out_row_stride, int dtype,
                        void* stream);
+/* The same with the clamped gate of mi_clamped_glu as activation (alpha > 0). */
+int mi_linear_clamped_glu(void* out, const void* x, const void* weight, int32_t m, int32_t inter,
+                          int32_t k, int64_t x_row_stride, int64_t out_row_stride, float alpha,
+                          float limit, int dtype, void* stream);
 /* Tile plans measured for a deployment's shapes (tools/tune_linear_plans.py ->
  * vllm_omni_amd/tuned/linear_plans_gfx950.json), replacing the built-in heuristic of the
  * three entry points above for 16-bit operands — the counterpart of the TunableOp

@@ -17,12 +17,15 @@
 namespace mi {
 namespace {
 
-// LDS: q[D] k[D] v[V] red[2][groups * V]
-template <typename T, int VEC, int NT>
+typedef __attribute__((ext_vector_type(4))) float f32x4;
+
+// LDS: q[D] k[D] v[V] red[2][groups * V].  R: rows of the state a thread holds; TAPS: convolution taps, 0 = any (one load
+// after the other).  A decode step is one chain of memory latencies per workgroup, so everything a token needs is asked for
+// before the first use, the state with it.
+template <typename T, int VEC, int NT, int R, int TAPS>
 __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams p) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  constexpr int R = 64 / VEC;   // rows of the state a thread can hold
   const int h = blockIdx.x, r = p.req0 + blockIdx.y;
   const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
   if (L <= 0) return;
@@ -49,8 +52,8 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
     for (int j = 0; j < VEC; ++j) st[i][j] = 0.f;
     if (on && d < D && start > 0) {
       if constexpr (VEC == 4) {
-        const float4 a = *reinterpret_cast<const float4*>(S + (int64_t)d * V + c);
-        st[i][0] = a.x, st[i][1] = a.y, st[i][2] = a.z, st[i][3] = a.w;
+        const f32x4 a = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(S + (int64_t)d * V + c));
+        st[i][0] = a[0], st[i][1] = a[1], st[i][2] = a[2], st[i][3] = a[3];
       } else {
         st[i][0] = S[(int64_t)d * V + c];
       }
@@ -62,14 +65,36 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
     const int64_t row = s0 + i;
     const int pos = start + i;
     const T* pr = proj + row * p.ld;
+    const float raw_a = Io<T>::ld(pr + p.off_a + h), raw_b = Io<T>::ld(pr + p.off_b + h);
+    float gt[4], nw[4];                          // the first wave ends the token: its gate and norm weights (vdim <= 256)
+    if (tid < 64)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (tid + 64 * j < V) {
+          gt[j] = Io<T>::ld(pr + p.off_g + h * V + tid + 64 * j);
+          nw[j] = Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + tid + 64 * j);
+        }
     for (int n = tid; n < 2 * D + V; n += NT) {
       const int ch = n < D ? kh * D + n : n < 2 * D ? p.K * D + kh * D + (n - D) : 2 * p.K * D + h * V + (n - 2 * D);
       const float cur = Io<T>::ld(pr + ch);
-      float acc = cur * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1);
-      for (int b = 1; b < p.taps; ++b) {
-        if (pos - b < 0) break;
-        const float x = i >= b ? Io<T>::ld(pr - b * p.ld + ch) : Io<T>::ld(ring + (int64_t)((pos - b) % p.taps) * p.CH + ch);
-        acc += x * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1 - b);
+      auto tap = [&](int b, int taps) -> float {     // the input b tokens back
+        if (pos - b < 0) return 0.f;
+        return Io<T>::ld(i >= b ? pr - b * p.ld + ch : ring + (int64_t)((pos - b) % taps) * p.CH + ch);
+      };
+      float acc;
+      if constexpr (TAPS > 0) {
+        float x[TAPS], w[TAPS];
+        x[0] = cur;
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b) x[b] = tap(b, TAPS);
+#pragma unroll
+        for (int b = 0; b < TAPS; ++b) w[b] = Io<T>::ld(convw + (int64_t)ch * TAPS + TAPS - 1 - b);
+        acc = x[0] * w[0];
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b) acc += x[b] * w[b];
+      } else {
+        acc = cur * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1);
+        for (int b = 1; b < p.taps; ++b) acc += tap(b, p.taps) * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1 - b);
       }
       lds[n] = silu_f(acc);
       // one token: its row of the ring is nobody's to read this step (readers take the taps - 1 rows before it)
@@ -79,8 +104,8 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
     float qq = 0.f, kk = 0.f;
     for (int d = tid & 63; d < D; d += 64) qq += sq[d] * sq[d], kk += sk[d] * sk[d];
     const float qn = qs / sqrtf(wave_allreduce_sum(qq) + 1e-6f), kn = 1.0f / sqrtf(wave_allreduce_sum(kk) + 1e-6f);
-    const float decay = expf(neg_a * softplus_f(Io<T>::ld(pr + p.off_a + h) + dtb));
-    const float beta = sigmoid_f(Io<T>::ld(pr + p.off_b + h));
+    const float decay = expf(neg_a * softplus_f(raw_a + dtb));
+    const float beta = sigmoid_f(raw_b);
     float acc[VEC] = {};
 #pragma unroll
     for (int n = 0; n < R; ++n) {
@@ -127,26 +152,29 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
       }
       const float inv = inv_rms(wave_allreduce_sum(ss), V, p.eps);
       T* o = reinterpret_cast<T*>(p.out) + row * (int64_t)H * V + (int64_t)h * V;
-      for (int v = tid; v < V; v += 64)
-        Io<T>::st(o + v, red1[v] * inv * Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + v) *
-                             silu_f(Io<T>::ld(pr + p.off_g + h * V + v)));
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (tid + 64 * j < V) Io<T>::st(o + tid + 64 * j, red1[tid + 64 * j] * inv * nw[j] * silu_f(gt[j]));
     }
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) {
     const int d = g + i * groups;
     if (on && d < D) {
-      if constexpr (VEC == 4) *reinterpret_cast<float4*>(S + (int64_t)d * V + c) = make_float4(st[i][0], st[i][1], st[i][2], st[i][3]);
+      if constexpr (VEC == 4) {
+        const f32x4 a = {st[i][0], st[i][1], st[i][2], st[i][3]};
+        __builtin_nontemporal_store(a, reinterpret_cast<f32x4*>(S + (int64_t)d * V + c));
+      }
       else S[(int64_t)d * V + c] = st[i][0];
     }
   }
 }
 
-template <typename T, int VEC, int NT>
+template <typename T, int VEC, int NT, int R>
 int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
   const int groups = NT / (p.V / VEC);
   const size_t lds = (size_t)(2 * p.D + p.V + 2 * groups * p.V) * sizeof(float);
-  auto kern = gated_delta_step_kernel<T, VEC, NT>;
+  auto kern = p.taps == 4 ? gated_delta_step_kernel<T, VEC, NT, R, 4> : gated_delta_step_kernel<T, VEC, NT, R, 0>;
   if (lds > 65536) {
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
       return MI_ERR_LAUNCH;
@@ -157,16 +185,18 @@ int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
 
 template <typename T>
 int step_dispatch(const DeltaParams& p, int nreq, hipStream_t s) {
+  if (p.V > 256) return MI_ERR_UNSUPPORTED;
   const int vec = p.V % 4 == 0 ? 4 : 1;
   const int lv = p.V / vec;
-  // a thread holds at most 64 state elements: the smallest workgroup whose rows fit
-  auto fits = [&](int nt) { const int gr = nt / lv; return gr > 0 && (p.D + gr - 1) / gr <= 64 / vec; };
+  auto fits = [&](int nt, int r) { const int gr = nt / lv; return gr > 0 && (p.D + gr - 1) / gr <= r; };
   if (vec == 4) {
-    if (fits(256)) return launch_step<T, 4, 256>(p, nreq, s);
-    if (fits(1024)) return launch_step<T, 4, 1024>(p, nreq, s);
+    if (fits(256, 8)) return launch_step<T, 4, 256, 8>(p, nreq, s);
+    if (fits(512, 8)) return launch_step<T, 4, 512, 8>(p, nreq, s);
+    if (fits(512, 16)) return launch_step<T, 4, 512, 16>(p, nreq, s);
+    if (fits(1024, 16)) return launch_step<T, 4, 1024, 16>(p, nreq, s);
   } else {
-    if (fits(256)) return launch_step<T, 1, 256>(p, nreq, s);
-    if (fits(1024)) return launch_step<T, 1, 1024>(p, nreq, s);
+    if (fits(256, 32)) return launch_step<T, 1, 256, 32>(p, nreq, s);
+    if (fits(1024, 64)) return launch_step<T, 1, 1024, 64>(p, nreq, s);
   }
   return MI_ERR_UNSUPPORTED;
 }

@@ -100,6 +100,61 @@ __device__ __forceinline__ void conv_rows(const DeltaParams& p, float* buf, int 
   }
 }
 
+// the same, 8 channels a thread: every load of a thread is independent of the others.  Needs n, the channel offsets and the
+// row strides to be multiples of 8.
+template <typename T, int TAPS>
+__device__ __forceinline__ void conv_rows8(const DeltaParams& p, float* buf, int ld, int np, int ch0, int n, int64_t row0, int i0,
+                                           int len, int start, const T* ring) {
+  const T* proj = reinterpret_cast<const T*>(p.proj);
+  const T* cw = reinterpret_cast<const T*>(p.convw);
+  const int per = np / 8;
+  for (int item = threadIdx.x; item < kC * per; item += kPrepThreads) {
+    const int c = (item % per) * 8, i = item / per;
+    float acc[8] = {};
+    if (c < n && i < len) {
+      const int ch = ch0 + c;
+      float w[TAPS][8], x[TAPS][8];
+      float wf[8 * TAPS];
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t) Io<T>::template ldv<8>(cw + (int64_t)ch * TAPS + 8 * t, *reinterpret_cast<float(*)[8]>(wf + 8 * t));
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) w[t][j] = wf[j * TAPS + t];
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t) {
+        const int k = i - (TAPS - 1) + t;
+        const int pos = start + i0 + k;
+        if (i0 + k >= 0) {
+          Io<T>::template ldv<8>(proj + (row0 + k) * p.ld + ch, x[t]);
+        } else if (pos >= 0) {
+          Io<T>::template ldv<8>(ring + (int64_t)(pos % TAPS) * p.CH + ch, x[t]);
+        } else {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) x[t][j] = 0.f;
+        }
+      }
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[j] += w[t][j] * x[t][j];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] = silu_f(acc[j]);
+    }
+    *reinterpret_cast<float4*>(buf + i * ld + c) = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    *reinterpret_cast<float4*>(buf + i * ld + c + 4) = make_float4(acc[4], acc[5], acc[6], acc[7]);
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ void conv_tile(const DeltaParams& p, bool vec, float* buf, int ld, int np, int ch0, int n, int64_t row0,
+                                          int i0, int len, int start, const T* ring) {
+  if (vec && p.taps == 4) conv_rows8<T, 4>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
+  else if (vec && p.taps == 3) conv_rows8<T, 3>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
+  else if (vec && p.taps == 2) conv_rows8<T, 2>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
+  else conv_rows<T>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
+}
+
 // rows of buf made unit vectors (16 lanes a row), then times mul
 __device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul) {
   const int sub = threadIdx.x & 15;
@@ -113,7 +168,7 @@ __device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul)
 }
 
 template <typename T>
-__global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay) {
+__global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, bool vec) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = p.req0 + blockIdx.z, h = blockIdx.y, ck = blockIdx.x;
@@ -126,18 +181,20 @@ __global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const De
   const int Dp = lay.Dp, Vp = lay.Vp, ldk = Dp + 4, ldm = kC + 4;
   const int ldv = Vp + 4, big = kC * max(ldk, ldv);
   float* bufA = lds;                       // K, then V
-  float* bufB = bufA + big;                // Q, then T
-  float* mA = bufB + max(kC * ldk, kC * ldm);   // A
-  float* sG = mA + kC * ldm;               // G_i
+  float* bufB = bufA + big;                // Q, then A and T
+  float* mA = bufB;
+  float* mT = bufB + kC * ldm;
+  float* sG = bufB + max(kC * ldk, 2 * kC * ldm);   // G_i
   float* sB = sG + kC;                     // b_i
   float* sE = sB + kC;                     // b_i e^(G_i)
-  float* mT = bufB;
+  float* sQ = sE + kC;                     // e^(G_i)
+  float* sD = sQ + kC;                     // e^(G_C - G_i)
   float* out = ws + ((chunk_base(p, r) + ck) * p.H + h) * lay.size();
   const T* ring = reinterpret_cast<const T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int kh = h / (p.H / p.K);
-  conv_rows<T>(p, bufA, ldk, Dp, p.K * p.D + kh * p.D, p.D, row0, i0, len, start, ring);
-  conv_rows<T>(p, bufB, ldk, Dp, kh * p.D, p.D, row0, i0, len, start, ring);
+  conv_tile<T>(p, vec, bufA, ldk, Dp, p.K * p.D + kh * p.D, p.D, row0, i0, len, start, ring);
+  conv_tile<T>(p, vec, bufB, ldk, Dp, kh * p.D, p.D, row0, i0, len, start, ring);
   if (wave == 0) {   // gates: cumulative log decay over the 64 tokens of the chunk
     const T* pr = reinterpret_cast<const T*>(p.proj) + (row0 + lane) * p.ld;
     float lg = 0.f, b = 0.f;
@@ -152,18 +209,30 @@ __global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const De
     }
     sG[lane] = lg;
     sB[lane] = b;
-    sE[lane] = b * expf(lg);
-    if (lane == 63) out[lay.g()] = expf(lg);
+    const float e = expf(lg);
+    sE[lane] = b * e;
+    sQ[lane] = e;
+    sD[lane] = expf(__shfl(lg, 63, 64) - lg);
+    if (lane == 63) out[lay.g()] = e;
   }
   __syncthreads();
   unit_rows(bufA, ldk, Dp, 1.0f);
   unit_rows(bufB, ldk, Dp, 1.0f / sqrtf((float)p.D));
   __syncthreads();
-  // A and P: the 10 lower tiles of each
-  for (int t = wave; t < 32; t += kPrepThreads / 64) {
-    const bool isP = t >= 16;
+  // A and P, 16 tiles each, lower ones only: P goes out, A waits in registers until Q is dead
+  f32x4_t keep[2];
+#pragma unroll
+  for (int n = 0; n < 4; ++n) {
+    const int t = wave + n * (kPrepThreads / 64);
+    const bool isP = n >= 2;
     const int ti = (t & 15) >> 2, tj = t & 3;
-    if (tj > ti) continue;   // above the diagonal: neither A nor P is read there
+    if (!isP) keep[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (tj > ti) {
+      if (isP)      // the scan multiplies whole rows of P
+#pragma unroll
+        for (int s = 0; s < 4; ++s) out[lay.pm() + (ti * 16 + 4 * (lane >> 4) + s) * kC + tj * 16 + (lane & 15)] = 0.f;
+      continue;
+    }
     const float* a = (isP ? bufB : bufA) + ti * 16 * ldk;
     const float* b = bufA + tj * 16 * ldk;
     f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
@@ -179,21 +248,28 @@ __global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const De
       const int i = ti * 16 + 4 * (lane >> 4) + s;
       const float e = expf(fminf(sG[i] - sG[j], 0.f));
       if (isP) out[lay.pm() + i * kC + j] = j <= i ? acc[s] * e : 0.f;
-      else mA[i * ldm + j] = j < i ? acc[s] * e * sB[i] : 0.f;
+      else keep[n & 1][s] = j < i ? acc[s] * e * sB[i] : 0.f;
     }
   }
   // diag(e^G) Q and the transposed, decayed keys
   for (int n = tid; n < kC * Dp / 4; n += kPrepThreads) {
     const int i = n / (Dp / 4), c = (n % (Dp / 4)) * 4;
-    const float e = expf(sG[i]);
+    const float e = sQ[i];
     const float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
     *reinterpret_cast<float4*>(out + lay.q() + (int64_t)i * Dp + c) = make_float4(v.x * e, v.y * e, v.z * e, v.w * e);
   }
   for (int n = tid; n < kC * Dp; n += kPrepThreads) {
     const int d = n / kC, j = n % kC;
-    out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * expf(sG[kC - 1] - sG[j]) : 0.f;
+    out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * sD[j] : 0.f;
   }
-  __syncthreads();   // Q is dead: T takes its place
+  __syncthreads();   // Q is dead: A and T take its place
+#pragma unroll
+  for (int n = 0; n < 2; ++n) {
+    const int t = wave + n * (kPrepThreads / 64);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) mA[((t >> 2) * 16 + 4 * (lane >> 4) + s) * ldm + (t & 3) * 16 + (lane & 15)] = keep[n][s];
+  }
+  __syncthreads();
   // T = (I + A)^-1: diagonal 16 x 16 blocks by substitution, one column a lane
   if (wave < 4 && lane < 16) {
     const float* a = mA + wave * 16 * ldm + wave * 16;
@@ -247,7 +323,7 @@ __global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const De
   };
   times(sE, ldk, Dp, out + lay.w());
   __syncthreads();
-  conv_rows<T>(p, bufA, ldv, Vp, 2 * p.K * p.D + h * p.V, p.V, row0, i0, len, start, ring);
+  conv_tile<T>(p, vec, bufA, ldv, Vp, 2 * p.K * p.D + h * p.V, p.V, row0, i0, len, start, ring);
   __syncthreads();
   times(sB, ldv, Vp, out + lay.u());
 }
@@ -256,10 +332,11 @@ __global__ __launch_bounds__(kPrepThreads) void gated_delta_prep_kernel(const De
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 template <int DT>
-__global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, float* o,
+__global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, float* o,
                                                                int nvt) {
   scalar_cache_acquire();
   constexpr int Dp = DT * 16, LS = Dp + 4, LU = kC + 4, MT = (DT + 3) / 4;
+  constexpr bool whole = DT % 4 == 0;      // every wave owns MT tiles of the state
   __shared__ __attribute__((aligned(16))) float sS[16 * LS];
   __shared__ __attribute__((aligned(16))) float sU[16 * LU];
   // the value tiles of a head on one XCD (workgroups go to the 8 XCDs in turn): they read the same workspace
@@ -269,7 +346,7 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaParams
   const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
   if (h >= p.H || L <= 0) return;
   const int start = p.seq_lens[r] - L;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, lg = lane >> 4;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lg = lane >> 4;
   const int v = vt * 16 + lr;
   float* S = p.state + (((int64_t)p.slots[r] * p.H + h) * p.D) * p.V;
   f32x4_t st[MT];
@@ -286,69 +363,77 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaParams
   const int nck = (L + kC - 1) / kC;
   const float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
   const int64_t step = p.H * lay.size();
-  f32x4_t w[DT], q[DT];
-  f32x4_t u;
-  auto load_front = [&](const float* b) {
+  // one chunk's operands; the next chunk's are loaded a whole chunk ahead (the chain of chunks is the critical path, its
+  // loads must not be).  The loads are unconditional — past the last chunk they fetch what nobody uses — so that the number in
+  // flight is known at every wait.
+  struct Chunk {
+    f32x4_t w[DT], q[DT], pm[4], kt[MT][4], u;
+    float g;
+  };
+  auto load = [&](Chunk& x, int c) {
+    const float* b = base + c * step;
     const int64_t ro = (int64_t)(16 * wave + lr) * Dp + 4 * lg;
 #pragma unroll
     for (int k = 0; k < DT; ++k) {
-      w[k] = *reinterpret_cast<const f32x4_t*>(b + lay.w() + ro + 16 * k);
-      q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
+      x.w[k] = *reinterpret_cast<const f32x4_t*>(b + lay.w() + ro + 16 * k);
+      x.q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) u[i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v];
-  };
-  load_front(base);
-  lds_barrier();
-  for (int c = 0; c < nck; ++c) {
-    const float* b = base + c * step;
-    // loads of the second half of this chunk, under the first half's products
-    f32x4_t pm[4], kt[MT][4];
+    for (int i = 0; i < 4; ++i) x.u[i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v];
+#pragma unroll
     for (int k = 0; k < 4; ++k) {
-      if (k <= wave) pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
+      x.pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
 #pragma unroll
       for (int m = 0; m < MT; ++m)
-        if (wave + 4 * m < DT)
-          kt[m][k] = *reinterpret_cast<const f32x4_t*>(b + lay.kt() + (int64_t)((wave + 4 * m) * 16 + lr) * kC + 16 * k + 4 * lg);
+        x.kt[m][k] = *reinterpret_cast<const f32x4_t*>(b + lay.kt() + (int64_t)(min(wave + 4 * m, DT - 1) * 16 + lr) * kC + 16 * k + 4 * lg);
     }
-    const float gc = b[lay.g()];
-    f32x4_t x = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
+    x.g = b[lay.g()];
+  };
+  auto work = [&](Chunk& x, int c) {
+    f32x4_t d = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < DT; ++k) {
       const f32x4_t sv = *reinterpret_cast<const f32x4_t*>(sS + lr * LS + 16 * k + 4 * lg);
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
-        x = __builtin_amdgcn_mfma_f32_16x16x4f32(w[k][s], sv[s], x, 0, 0, 0);
-        ao = __builtin_amdgcn_mfma_f32_16x16x4f32(q[k][s], sv[s], ao, 0, 0, 0);
+        d = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w[k][s], sv[s], d, 0, 0, 0);
+        ao = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[k][s], sv[s], ao, 0, 0, 0);
       }
     }
-    u -= x;
-    *reinterpret_cast<f32x4_t*>(sU + lr * LU + 16 * wave + 4 * lg) = u;
+    *reinterpret_cast<f32x4_t*>(sU + lr * LU + 16 * wave + 4 * lg) = x.u - d;
     lds_barrier();
-    if (c + 1 < nck) load_front(b + step);
 #pragma unroll
-    for (int m = 0; m < MT; ++m) st[m] *= gc;
+    for (int m = 0; m < MT; ++m) st[m] *= x.g;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
       const f32x4_t uv = *reinterpret_cast<const f32x4_t*>(sU + lr * LU + 16 * k + 4 * lg);
-      if (k <= wave)
-#pragma unroll
-        for (int s = 0; s < 4; ++s) ao = __builtin_amdgcn_mfma_f32_16x16x4f32(pm[k][s], uv[s], ao, 0, 0, 0);
 #pragma unroll
       for (int m = 0; m < MT; ++m)
-        if (wave + 4 * m < DT)
+        if (whole || wave + 4 * m < DT)
 #pragma unroll
-          for (int s = 0; s < 4; ++s) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[m][k][s], uv[s], st[m], 0, 0, 0);
+          for (int s = 0; s < 4; ++s) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[m][k][s], uv[s], st[m], 0, 0, 0);
+#pragma unroll
+      for (int s = 0; s < 4; ++s) ao = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv[s], ao, 0, 0, 0);
     }
 #pragma unroll
     for (int m = 0; m < MT; ++m)
-      if (wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + (wave + 4 * m) * 16 + 4 * lg) = st[m];
+      if (whole || wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + (wave + 4 * m) * 16 + 4 * lg) = st[m];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = c * kC + 16 * wave + 4 * lg + i;
       if (t < L && v < p.V) o[((int64_t)(s0 + t) * p.H + h) * p.V + v] = ao[i];
     }
     lds_barrier();
+  };
+  Chunk a, b;
+  load(a, 0);
+  lds_barrier();
+  for (int c = 0; c < nck; c += 2) {
+    load(b, min(c + 1, nck - 1));
+    work(a, c);
+    if (c + 1 >= nck) break;
+    load(a, min(c + 2, nck - 1));
+    work(b, c + 1);
   }
 #pragma unroll
   for (int m = 0; m < MT; ++m)
@@ -359,7 +444,43 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaParams
     }
 }
 
-// out = o / rms(o) * norm * silu(gate), one wave per (row, head)
+// out = o / rms(o) * norm * silu(gate), 16 lanes per (row, head), 8 values a lane at a time; vdim a multiple of 8, <= 128 U
+template <typename T, int U>
+__global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaParams p, const float* o, int row0, int rows) {
+  scalar_cache_acquire();
+  const int64_t item = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const int sub = threadIdx.x & 15;
+  if (item >= (int64_t)rows * p.H) return;     // whole 16-lane groups leave
+  const int64_t row = row0 + item / p.H;
+  const int h = (int)(item % p.H);
+  const float* x = o + (row * p.H + h) * (int64_t)p.V;
+  const T* g = reinterpret_cast<const T*>(p.proj) + row * p.ld + p.off_g + h * p.V;
+  float v[U][8], gt[U][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int c = 8 * (sub + 16 * u);
+    if (c >= p.V) continue;
+    Io<float>::ldv<8>(x + c, v[u]);
+    Io<T>::template ldv<8>(g + c, gt[u]);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += v[u][j] * v[u][j];
+  }
+  const float inv = inv_rms(group_allreduce_sum<16>(ss), p.V, p.eps);
+  T* out = reinterpret_cast<T*>(p.out) + (row * p.H + h) * (int64_t)p.V;
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int c = 8 * (sub + 16 * u);
+    if (c >= p.V) continue;
+    float w[8];
+    Io<T>::template ldv<8>(reinterpret_cast<const T*>(p.norm_w) + c, w);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[u][j] *= inv * w[j] * silu_f(gt[u][j]);
+    Io<T>::template stv<8>(out + c, v[u]);
+  }
+}
+
+// the same for any vdim, one wave per (row, head)
 template <typename T>
 __global__ __launch_bounds__(256) void gated_delta_finish_kernel(const DeltaParams p, const float* o, int row0, int rows) {
   scalar_cache_acquire();
@@ -426,14 +547,17 @@ extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, con
   hipStream_t s = (hipStream_t)stream;
   float* ws = (float*)workspace;
   const int ldk = lay.Dp + 4, ldv = lay.Vp + 4, ldm = kC + 4;
-  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > ldm ? ldk : ldm) + kC * ldm + 3 * kC) * 4;
+  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC) * 4;
+  const int al = (dtype == MI_DTYPE_BF16 ? 8 : 4);
+  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && proj_stride % al == 0 && CH % al == 0 && aligned16(proj) && aligned16(conv_w) &&
+                   aligned16(ring);
   const dim3 pg((max_query_len + kC - 1) / kC, heads, num_reqs);
 #define MI_PREP(T)                                                                                                        \
   do {                                                                                                                    \
     auto kern = gated_delta_prep_kernel<T>;                                                                               \
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
       return MI_ERR_LAUNCH;                                                                                               \
-    hipLaunchKernelGGL(kern, pg, dim3(kPrepThreads), lds, s, p, ws, lay);                                                 \
+    hipLaunchKernelGGL(kern, pg, dim3(kPrepThreads), lds, s, p, ws, lay, vec);                                               \
   } while (0)
   if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
   else MI_PREP(float);
@@ -447,12 +571,21 @@ extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, con
     default: hipLaunchKernelGGL((gated_delta_scan_kernel<16>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
   }
   const dim3 fg((unsigned)(((int64_t)rows * heads + 3) / 4)), rg((CH + 255) / 256, num_reqs);
+  const dim3 f8((unsigned)(((int64_t)rows * heads + 15) / 16));
+  const bool vecf = vec && aligned16(out) && aligned16(norm_w) && aligned16(o_f32);
+#define MI_FINISH(T)                                                                                                              \
+  do {                                                                                                                            \
+    if (vecf && vdim <= 128) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 1>), f8, dim3(256), 0, s, p, o_f32, row0, rows);   \
+    else if (vecf) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 2>), f8, dim3(256), 0, s, p, o_f32, row0, rows);             \
+    else hipLaunchKernelGGL((gated_delta_finish_kernel<T>), fg, dim3(256), 0, s, p, o_f32, row0, rows);                           \
+  } while (0)
   if (dtype == MI_DTYPE_BF16) {
-    hipLaunchKernelGGL((gated_delta_finish_kernel<uint16_t>), fg, dim3(256), 0, s, p, o_f32, row0, rows);
+    MI_FINISH(uint16_t);
     hipLaunchKernelGGL((conv_ring_update_kernel<uint16_t>), rg, dim3(256), 0, s, p);
   } else {
-    hipLaunchKernelGGL((gated_delta_finish_kernel<float>), fg, dim3(256), 0, s, p, o_f32, row0, rows);
+    MI_FINISH(float);
     hipLaunchKernelGGL((conv_ring_update_kernel<float>), rg, dim3(256), 0, s, p);
   }
+#undef MI_FINISH
   return launch_status();
 }

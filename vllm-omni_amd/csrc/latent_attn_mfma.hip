@@ -30,6 +30,7 @@ __global__ __launch_bounds__(256) void head_gemm_nt_kernel(uint16_t* y, const ui
 #pragma unroll
   for (int i = 0; i < 4; ++i) xr[i] = x + (int64_t)min(t0 + 16 * i + lr, rows - 1) * x_row + (int64_t)h * Kd + 8 * lg;
   const int live = min(4, (rows - t0 + 15) / 16);
+#pragma unroll 4
   for (int k = 0; k < Kd; k += 32) {
     const bool in = k + 8 * lg < Kd;      // Kd is a multiple of 8
     const uint4 z = make_uint4(0, 0, 0, 0);
@@ -69,15 +70,33 @@ struct LatentDecodeParams {
   float scale;           // times log2(e)
 };
 
+constexpr int kBlockList = 256;
+
 __device__ __forceinline__ uint32_t lds_addr(const void* p) { return (uint32_t)(uintptr_t)(lds_void*)p; }
 
-// two transposed reads (4 key rows x 16 dims each) and their wait: the A operand of K = 32
+// transposed reads of the A operands (K = 32: two reads of 4 key rows x 16 dims) of one or four consecutive dim tiles, with
+// one wait
 template <int OFF>
 __device__ __forceinline__ uint4 tr_pair(uint32_t addr) {
   u32x2_t a, b;
   asm volatile("ds_read_b64_tr_b16 %0, %2\n\tds_read_b64_tr_b16 %1, %2 offset:%3\n\ts_waitcnt lgkmcnt(0)"
                : "=&v"(a), "=&v"(b) : "v"(addr), "i"(OFF) : "memory");
   return make_uint4(a[0], a[1], b[0], b[1]);
+}
+template <int OFF>
+__device__ __forceinline__ void tr_pair4(uint32_t addr, uint4 (&o)[4]) {
+  u32x2_t a[4], b[4];
+  asm volatile(
+      "ds_read_b64_tr_b16 %0, %8\n\tds_read_b64_tr_b16 %4, %8 offset:%9\n\t"
+      "ds_read_b64_tr_b16 %1, %8 offset:32\n\tds_read_b64_tr_b16 %5, %8 offset:%10\n\t"
+      "ds_read_b64_tr_b16 %2, %8 offset:64\n\tds_read_b64_tr_b16 %6, %8 offset:%11\n\t"
+      "ds_read_b64_tr_b16 %3, %8 offset:96\n\tds_read_b64_tr_b16 %7, %8 offset:%12\n\t"
+      "s_waitcnt lgkmcnt(0)"
+      : "=&v"(a[0]), "=&v"(a[1]), "=&v"(a[2]), "=&v"(a[3]), "=&v"(b[0]), "=&v"(b[1]), "=&v"(b[2]), "=&v"(b[3])
+      : "v"(addr), "i"(OFF), "i"(OFF + 32), "i"(OFF + 64), "i"(OFF + 96)
+      : "memory");
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o[i] = make_uint4(a[i][0], a[i][1], b[i][0], b[i][1]);
 }
 
 template <int RN, int NHT>
@@ -90,6 +109,7 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
   uint16_t* sC = reinterpret_cast<uint16_t*>(smem);           // [64][LD]
   uint16_t* sP = sC + 64 * LD;                                // [2 (hi, lo)][16 NHT][PL]
   float* sR = reinterpret_cast<float*>(sP + 2 * 16 * NHT * PL);   // [4][16 NHT]
+  int32_t* sB = reinterpret_cast<int32_t*>(sR + 4 * 16 * NHT);    // [kBlockList]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int kw = wave & 3, ht = wave >> 2;          // key group / dim group, head tile
   const int split = blockIdx.x, r = blockIdx.z;
@@ -109,8 +129,15 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
       const int c = 32 * k + 8 * lg;
       qf[k] = live && c < p.rank ? *reinterpret_cast<const uint4*>(qr + c) : make_uint4(0, 0, 0, 0);
     }
+    // the split's block ids in LDS (a load of the cache then waits for one memory access, not two); a split longer than the
+    // list reads the table itself
     const int32_t* tab = p.table + (int64_t)r * p.table_stride;
     const int bmask = (1 << p.bs_log2) - 1;
+    const int b0 = k0 >> p.bs_log2, nb = ((k1 - 1) >> p.bs_log2) - b0 + 1;
+    const bool listed = nb <= kBlockList;
+    if (listed)
+      for (int i = tid; i < nb; i += NT) sB[i] = tab[b0 + i];
+    __syncthreads();
     uint4 pre[CH];
     auto fetch = [&](int t0) {
 #pragma unroll
@@ -118,7 +145,7 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
         const int c = tid + i * NT, row = c / (Rp / 8), col = (c % (Rp / 8)) * 8, key = t0 + row;
         pre[i] = make_uint4(0, 0, 0, 0);
         if (key < k1 && col < p.rank)
-          pre[i] = *reinterpret_cast<const uint4*>(p.cache + (int64_t)tab[key >> p.bs_log2] * p.block_stride +
+          pre[i] = *reinterpret_cast<const uint4*>(p.cache + (int64_t)(listed ? sB[(key >> p.bs_log2) - b0] : tab[key >> p.bs_log2]) * p.block_stride +
                                                    (int64_t)(key & bmask) * p.token_stride + col);
       }
     };
@@ -133,12 +160,15 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
       }
       __syncthreads();
       if (t0 + 64 < k1) fetch(t0 + 64);
-      f32x4_t s = {};
+      f32x4_t s = {}, s2 = {};
 #pragma unroll
-      for (int k = 0; k < 2 * RN; ++k) {
+      for (int k = 0; k < 2 * RN; k += 2) {
         const uint4 a = *reinterpret_cast<const uint4*>(sC + (16 * kw + lr) * LD + 32 * k + 8 * lg);
+        const uint4 b = *reinterpret_cast<const uint4*>(sC + (16 * kw + lr) * LD + 32 * k + 32 + 8 * lg);
         s = mfma16<bf16_tag>(a, qf[k], s);
+        s2 = mfma16<bf16_tag>(b, qf[k + 1], s2);
       }
+      s += s2;
       float mx = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -171,11 +201,24 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
       for (int kb = 0; kb < 2; ++kb) {
         const uint4 bh = *reinterpret_cast<const uint4*>(sP + hl * PL + 32 * kb + 8 * lg);
         const uint4 bl = *reinterpret_cast<const uint4*>(sP + (16 * NHT + hl) * PL + 32 * kb + 8 * lg);
+        const uint32_t base = tr_base + (uint32_t)(32 * kb * LD * 2);
+        if constexpr (MT >= 4) {
 #pragma unroll
-        for (int i = 0; i < MT; ++i) {
-          const uint4 a = tr_pair<4 * LD * 2>(tr_base + (uint32_t)((32 * kb * LD + 16 * i) * 2));
-          acc[i] = mfma16<bf16_tag>(a, bh, acc[i]);
-          acc[i] = mfma16<bf16_tag>(a, bl, acc[i]);
+          for (int i = 0; i < MT; i += 4) {
+            uint4 a[4];
+            tr_pair4<4 * LD * 2>(base + 32 * i, a);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[i + j] = mfma16<bf16_tag>(a[j], bh, acc[i + j]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[i + j] = mfma16<bf16_tag>(a[j], bl, acc[i + j]);
+          }
+        } else {
+#pragma unroll
+          for (int i = 0; i < MT; ++i) {
+            const uint4 a = tr_pair<4 * LD * 2>(base + 32 * i);
+            acc[i] = mfma16<bf16_tag>(a, bh, acc[i]);
+            acc[i] = mfma16<bf16_tag>(a, bl, acc[i]);
+          }
         }
       }
     }
@@ -262,7 +305,7 @@ struct LatentPrefillParams {
 };
 
 template <int KT, int VN>   // dim padded to 16 KT, vdim to 32 VN
-__global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefillParams p) {
+__global__ __launch_bounds__(256, KT <= 8 && VN <= 4 ? 2 : 1) void latent_prefill_kernel(const LatentPrefillParams p) {
   scalar_cache_acquire();
   constexpr int Dp = 16 * KT, Vp = 32 * VN, LK = Dp + 8, LV = 64 + 4;
   constexpr int KCH = 64 * (Dp / 8) / 256, VCH = Vp * 8 / 256;
@@ -413,7 +456,7 @@ __global__ __launch_bounds__(256) void latent_prefill_kernel(const LatentPrefill
 template <int RN, int NHT>
 int launch_decode(const LatentDecodeParams& p, int reqs, hipStream_t s) {
   constexpr int LD = 64 * RN + 8, PL = 72;
-  constexpr int lds = (64 * LD + 2 * 16 * NHT * PL) * 2 + 4 * 16 * NHT * 4;
+  constexpr int lds = (64 * LD + 2 * 16 * NHT * PL) * 2 + 4 * 16 * NHT * 4 + kBlockList * 4;
   auto kern = latent_decode_kernel<RN, NHT>;
   if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess)
     return MI_ERR_LAUNCH;
@@ -434,8 +477,8 @@ int launch_prefill(const LatentPrefillParams& p, int reqs, int max_q, hipStream_
 inline int rank_tiles(int rank) { return rank <= 64 ? 1 : rank <= 128 ? 2 : rank <= 256 ? 4 : 8; }
 
 inline int decode_splits(int reqs, int head_groups, int span) {
-  // about two workgroups a CU, at least 128 cache rows each
-  const int want = (512 + reqs * head_groups - 1) / (reqs * head_groups);
+  // a workgroup for every CU, at least 128 cache rows each
+  const int want = (256 + reqs * head_groups - 1) / (reqs * head_groups);
   const int most = (span + 127) / 128;
   const int n = want < most ? want : most;
   return n < 1 ? 1 : n > 64 ? 64 : n;

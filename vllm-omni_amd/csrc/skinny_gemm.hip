@@ -173,7 +173,7 @@ struct V2 {
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const float gt = E::from_bits(E::to_bits(gq[r])), up = E::from_bits(E::to_bits(uq[r]));
-            v[r] = gt / (1.f + __expf(-gt)) * up;
+            v[r] = glu_value(p, gt, up);
           }
           uint2 o;
           o.x = E::pack(v[0], v[1]);
@@ -804,8 +804,8 @@ extern "C" int mi_linear_reduce(void* out, const void* partials, int32_t split, 
   return launch_status();
 }
 
-extern "C" int mi_linear_silu_mul(void* out, const void* x, const void* weight, int32_t m, int32_t inter, int32_t k,
-                                  int64_t x_row_stride, int64_t out_row_stride, int dtype, void* stream) {
+static int linear_glu(void* out, const void* x, const void* weight, int32_t m, int32_t inter, int32_t k, int64_t x_row_stride,
+                      int64_t out_row_stride, float alpha, float limit, int dtype, void* stream) {
   using namespace mi;
   if (m == 0 || inter == 0) return MI_OK;
   if (!out || !x || !weight || m < 0 || inter < 0 || k <= 0) return MI_ERR_INVALID_ARG;
@@ -825,7 +825,20 @@ extern "C" int mi_linear_silu_mul(void* out, const void* x, const void* weight, 
   p.dbg = linear_dbg();
   p.ldx = x_row_stride;
   p.ldo = out_row_stride;
+  p.glu_alpha = alpha;
+  p.glu_limit = limit;
   return launch_skinny(p, pl, true, dtype, reinterpret_cast<hipStream_t>(stream));
+}
+
+extern "C" int mi_linear_silu_mul(void* out, const void* x, const void* weight, int32_t m, int32_t inter, int32_t k,
+                                  int64_t x_row_stride, int64_t out_row_stride, int dtype, void* stream) {
+  return linear_glu(out, x, weight, m, inter, k, x_row_stride, out_row_stride, 0.f, 0.f, dtype, stream);
+}
+
+extern "C" int mi_linear_clamped_glu(void* out, const void* x, const void* weight, int32_t m, int32_t inter, int32_t k,
+                                     int64_t x_row_stride, int64_t out_row_stride, float alpha, float limit, int dtype, void* stream) {
+  if (!(alpha > 0.f)) return MI_ERR_INVALID_ARG;
+  return linear_glu(out, x, weight, m, inter, k, x_row_stride, out_row_stride, alpha, limit, dtype, stream);
 }
 
 // ------------------------------------------------------------------------------------------------ W8A8 entry points

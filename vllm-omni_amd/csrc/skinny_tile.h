@@ -55,6 +55,8 @@ struct SkinnyParams {
   // S > 1 with the reduce INSIDE the launch (mi_linear_fused_reduce): arrival counters [tiles x RB], zero before the
   // first launch and left at zero by every launch; the slice of a (tile, row block) that arrives last sums the slabs
   int32_t* cnt = nullptr;
+  // GATED: 0 = silu(gate) * up; > 0 = the clamped form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit)
+  float glu_alpha = 0.f, glu_limit = 0.f;
   // GROUPED (sparse-MoE expert GEMMs, fused_moe.hip): grid.y = one tile of `rpt` token rows that share one expert
   const int32_t* row_map;      // [max_rows] pair index per row or -1
   const int32_t* tile_expert;  // [max_tiles]
@@ -173,6 +175,12 @@ __device__ __forceinline__ void wait_steps_behind(int rem) {
 
 // NSLAB: 32-row weight slabs per tile (tile = 32 NSLAB rows); MT: 16-row m-tiles (x rows padded to 16 MT);
 // MH: consumer waves per slab, each with MT / MH m-tiles; NL: loader waves.
+__device__ __forceinline__ float glu_value(const SkinnyParams& p, float gt, float up) {
+  if (p.glu_alpha == 0.f) return gt / (1.f + __expf(-gt)) * up;
+  const float g = fminf(gt, p.glu_limit);
+  return g / (1.f + __expf(-p.glu_alpha * g)) * (fminf(fmaxf(up, -p.glu_limit), p.glu_limit) + 1.f);
+}
+
 // GATED: gate_up_proj with the SiluAndMul that follows it (qwen2_old.py:65-68: act_fn(gate_up_proj(x))) in the epilogue —
 // a slab is 16 gate rows and the 16 matching up rows, a tile covers 16 NSLAB output columns, and the [M, 2 I]
 // intermediate never goes to memory.
@@ -380,7 +388,7 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const float gt = E::from_bits(E::to_bits(gq[r])), up = E::from_bits(E::to_bits(uq[r]));
-        v[r] = gt / (1.f + __expf(-gt)) * up;
+        v[r] = glu_value(p, gt, up);
       }
       uint2 q;
       q.x = E::pack(v[0], v[1]);

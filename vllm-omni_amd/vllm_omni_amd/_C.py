@@ -99,6 +99,7 @@ SIGNATURES = {
     "mi_fused_add_rms_norm_splitk": (c_int, [_P, _P, c_int32, _P, _P, _P, c_float, c_int32, c_int32, c_int64, c_int64,
                                              c_int, _P]),
     "mi_linear_silu_mul": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_linear_clamped_glu": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_float, c_float, c_int, _P]),
     "mi_linear": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, _P, c_int64, c_int, _P]),
     "mi_linear_fused_reduce": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, _P, c_int64, _P, c_int64,
                                         c_int, _P]),

@@ -377,10 +377,11 @@ def _streaming_kernel_wins(m: int, n: int, k: int) -> bool:
     return m <= 256 and n <= 2048 and k <= 4096 and k > 2 * n and n * k >= (1 << 20)
 
 
-def fused_gate_up_silu(layer, x: torch.Tensor) -> Optional[torch.Tensor]:
+def fused_gate_up_silu(layer, x: torch.Tensor, clamped: Optional[tuple[float, float]] = None) -> Optional[torch.Tensor]:
     """``act_fn(gate_up_proj(x))`` in one launch (``ops.linear_silu_mul``) when the policy picks the streaming kernel
     for this shape, else None (the caller runs the GEMM and ``SiluAndMul`` apart).  Column-parallel, no bias, 16-bit
-    weights only; under TP a rank's weight is [gate shard; up shard], the layout the kernel expects."""
+    weights only; under TP a rank's weight is [gate shard; up shard], the layout the kernel expects.  ``clamped`` (alpha,
+    limit): the clamped gate (``ops.clamped_glu``) in SiLU's place."""
     if isinstance(x, ops.QuantizedActs):
         n2, k = layer.qweight.shape
         if layer.bias is None and n2 % 32 == 0 and ops.int8_linear_supported(min(x.xq.shape[0], ops.INT8_TILE_ROWS), n2 // 2, k):
@@ -404,10 +405,10 @@ def fused_gate_up_silu(layer, x: torch.Tensor) -> Optional[torch.Tensor]:
         return None
     e = _tuned(m, n // 2, k, gated=True)
     if e is not None and e.get("full"):
-        return ops.linear_silu_mul(x, w) if e["full"]["us"] < e["library_us"] else None
+        return ops.linear_silu_mul(x, w, clamped) if e["full"]["us"] < e["library_us"] else None
     if _LINEAR_MODE not in ("kernel", "mlp", "mlp+o") and not _fused_gate_up_wins(m, n // 2, k):
         return None
-    return ops.linear_silu_mul(x, w)
+    return ops.linear_silu_mul(x, w, clamped)
 
 
 def _deferred_kernel_wins(m: int, n: int, k: int) -> bool:

@@ -12,7 +12,7 @@ import torch.nn.functional as F
 
 from . import ops
 from .kv_cache import LatentCacheSpec
-from .layers import AttentionMetadata, _apply_linear, _init_weight
+from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu
 from .state_cache import StateSpec
 
 
@@ -208,7 +208,10 @@ class ClampedGluMLP:
         yield from self.down.named(p)
 
     def __call__(self, h: torch.Tensor, defer_reduce: bool = False):
-        return self.down(ops.clamped_glu(self.gate_up(h), self.alpha, self.limit), defer_reduce)
+        act = fused_gate_up_silu(self.gate_up, h, (self.alpha, self.limit))     # decode batches: one launch
+        if act is None:
+            act = ops.clamped_glu(self.gate_up(h), self.alpha, self.limit)
+        return self.down(act, defer_reduce)
 
 
 class TokenSideInput:

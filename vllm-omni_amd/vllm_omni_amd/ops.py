@@ -821,9 +821,10 @@ def rope_neox_and_cache_splitk(part: SplitKPartials, num_q_heads: int, num_kv_he
     return q_out
 
 
-def linear_silu_mul(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+def linear_silu_mul(x: torch.Tensor, weight: torch.Tensor, clamped: Optional[tuple[float, float]] = None) -> torch.Tensor:
     """silu(x Wg^T) * (x Wu^T) for a decode batch, weight = [gate rows; up rows] — ``gate_up_proj`` and the
-    ``SiluAndMul`` behind it (qwen2_old.py:65-68) in one launch; the [m, 2 I] intermediate never reaches memory."""
+    ``SiluAndMul`` behind it (qwen2_old.py:65-68) in one launch; the [m, 2 I] intermediate never reaches memory.
+    ``clamped`` (alpha, limit): the activation of ``clamped_glu`` instead."""
     _gpu(x, weight)
     x2 = x.reshape(-1, x.shape[-1])
     if x2.stride(-1) != 1:
@@ -833,6 +834,11 @@ def linear_silu_mul(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
         raise ValueError("weight must be a contiguous [2 * inter, k] tensor of x's dtype")
     inter = weight.shape[0] // 2
     out = torch.empty(m, inter, dtype=x.dtype, device=x.device)
+    if clamped is not None:
+        check("mi_linear_clamped_glu", lib.mi_linear_clamped_glu(
+            _p(out), _p(x2), _p(weight), m, inter, k, x2.stride(0), out.stride(0), float(clamped[0]), float(clamped[1]),
+            _dt(x.dtype), _stream()))
+        return out.view(*x.shape[:-1], inter)
     check("mi_linear_silu_mul", lib.mi_linear_silu_mul(_p(out), _p(x2), _p(weight), m, inter, k, x2.stride(0),
                                                        out.stride(0), _dt(x.dtype), _stream()))
     return out.view(*x.shape[:-1], inter)
