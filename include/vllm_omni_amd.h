@@ -817,14 +817,14 @@ int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_
                         float eps, int32_t update_ring, int dtype, void* stream);
 /* The same for prompt portions, 64 tokens at a time on the fp32 matrix cores
  * (dim, vdim <= 256): requests [req0, req0 + num_reqs) own rows [row0, row0 +
- * rows); o_f32 [total rows][heads vdim] and the workspace are scratch. */
+ * rows); the workspace is scratch. */
 int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads,
                                                int32_t dim, int32_t vdim);
 int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w,
                            const float* a_log, const float* dt_bias, const void* norm_w,
                            float* state, void* ring, const int32_t* slots,
                            const int32_t* query_start_loc, const int32_t* seq_lens, void* out,
-                           float* o_f32, int32_t row0, int32_t rows, int32_t req0, int32_t num_reqs,
+                           int32_t row0, int32_t rows, int32_t req0, int32_t num_reqs,
                            int32_t max_query_len, int32_t heads, int32_t kv_heads, int32_t dim,
                            int32_t vdim, int32_t taps, float eps, void* workspace,
                            int64_t workspace_bytes, int dtype, void* stream);

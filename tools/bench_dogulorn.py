@@ -131,7 +131,8 @@ def run(a):
         for mode in a.dogulorn_mode.split(","):
             for name in a.dogulorn_models.split(","):
                 cfg = (dogulorn_config if name == "dogulorn" else talker_config)(s)
-                cases = [(32, 4096), (256, 4096)] if mode == "decode" else [[8192], [2048] * 4]
+                cases = ([(int(b), 4096) for b in a.dogulorn_batches.split(",")] if mode == "decode" else
+                         [[int(n) for n in c.split(",")] for c in a.dogulorn_prompts.split(";")])
                 for case in cases:
                     with torch.inference_mode():
                         if mode == "decode":

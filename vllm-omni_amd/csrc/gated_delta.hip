@@ -20,17 +20,18 @@ namespace {
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 // LDS: q[D] k[D] v[V] red[2][groups * V].  R: rows of the state a thread holds; TAPS: convolution taps, 0 = any (one load
-// after the other).  A decode step is one chain of memory latencies per workgroup, so everything a token needs is asked for
-// before the first use, the state with it.
-template <typename T, int VEC, int NT, int R, int TAPS>
-__global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams p) {
+// after the other); FULL: the threads' tiles cover the state exactly.  A decode step is one chain of memory latencies per
+// workgroup, so everything a token needs is asked for before the first use, the state with it; loads are unconditional on
+// clamped addresses and their values selected afterwards (a load behind a branch is waited for on its own).
+template <typename T, int VEC, int NT, int R, int TAPS, bool FULL>
+__global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(const DeltaParams p) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int h = blockIdx.x, r = p.req0 + blockIdx.y;
-  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
-  if (L <= 0) return;
-  const int start = p.seq_lens[r] - L;     // < 0: a padded row of a graph replay (scratch slot)
+  const int s0 = p.qsl[r], s1 = p.qsl[r + 1], seq = p.seq_lens[r];
   const int64_t slot = p.slots[r];
+  const int L = s1 - s0, start = seq - L;      // start < 0: a padded row of a graph replay (scratch slot)
+  if (L <= 0) return;
   const int D = p.D, V = p.V, H = p.H, per = H / p.K, kh = h / per;
   float* sq = lds;
   float* sk = sq + D;
@@ -39,52 +40,51 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
   float* red0 = sv + V;
   float* red1 = red0 + groups * V;
   const int tid = threadIdx.x, g = tid / lv, c = (tid % lv) * VEC;
-  const bool on = g < groups;
+  const bool on = FULL || g < groups;
   float* S = p.state + ((slot * H + h) * D) * (int64_t)V;
   const T* proj = reinterpret_cast<const T*>(p.proj);
   const T* convw = reinterpret_cast<const T*>(p.convw);
   T* ring = reinterpret_cast<T*>(p.ring) + slot * p.taps * (int64_t)p.CH;
+  auto has = [&](int n) { return FULL || (on && g + n * groups < D); };      // row n of the thread's tile exists
   float st[R][VEC];
 #pragma unroll
   for (int i = 0; i < R; ++i) {
-    const int d = g + i * groups;
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) st[i][j] = 0.f;
-    if (on && d < D && start > 0) {
-      if constexpr (VEC == 4) {
-        const f32x4 a = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(S + (int64_t)d * V + c));
-        st[i][0] = a[0], st[i][1] = a[1], st[i][2] = a[2], st[i][3] = a[3];
-      } else {
-        st[i][0] = S[(int64_t)d * V + c];
-      }
+    const int d = FULL ? g + i * groups : min(g + i * groups, D - 1);
+    if constexpr (VEC == 4) {
+      const f32x4 a = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(S + (int64_t)d * V + c));
+      st[i][0] = a[0], st[i][1] = a[1], st[i][2] = a[2], st[i][3] = a[3];
+    } else {
+      st[i][0] = S[(int64_t)d * V + c];
     }
   }
   const float neg_a = -expf(p.a_log[h]), dtb = p.dt_bias[h];
   const float qs = 1.0f / sqrtf((float)D);
+  const int nch = 2 * D + V;
   for (int i = 0; i < L; ++i) {
     const int64_t row = s0 + i;
     const int pos = start + i;
     const T* pr = proj + row * p.ld;
     const float raw_a = Io<T>::ld(pr + p.off_a + h), raw_b = Io<T>::ld(pr + p.off_b + h);
-    float gt[4], nw[4];                          // the first wave ends the token: its gate and norm weights (vdim <= 256)
-    if (tid < 64)
+    float gt[4], nw[4];                          // what the first wave ends the token with: gate and norm weights (vdim <= 256)
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (tid + 64 * j < V) {
-          gt[j] = Io<T>::ld(pr + p.off_g + h * V + tid + 64 * j);
-          nw[j] = Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + tid + 64 * j);
-        }
-    for (int n = tid; n < 2 * D + V; n += NT) {
+    for (int j = 0; j < 4; ++j) {
+      const int v = min((tid & 63) + 64 * j, V - 1);
+      gt[j] = Io<T>::ld(pr + p.off_g + h * V + v);
+      nw[j] = Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + v);
+    }
+    for (int n0 = 0; n0 < nch; n0 += NT) {
+      const int n = min(n0 + tid, nch - 1);
       const int ch = n < D ? kh * D + n : n < 2 * D ? p.K * D + kh * D + (n - D) : 2 * p.K * D + h * V + (n - 2 * D);
-      const float cur = Io<T>::ld(pr + ch);
       auto tap = [&](int b, int taps) -> float {     // the input b tokens back
-        if (pos - b < 0) return 0.f;
-        return Io<T>::ld(i >= b ? pr - b * p.ld + ch : ring + (int64_t)((pos - b) % taps) * p.CH + ch);
+        const T* src = i >= b ? pr - b * p.ld : ring + (int64_t)((pos - b) % taps) * p.CH;
+        const float x = Io<T>::ld((pos >= b ? src : pr) + ch);
+        return pos >= b ? x : 0.f;
       };
+      const T cur = pr[ch];
       float acc;
       if constexpr (TAPS > 0) {
         float x[TAPS], w[TAPS];
-        x[0] = cur;
+        x[0] = Io<T>::ld(&cur);
 #pragma unroll
         for (int b = 1; b < TAPS; ++b) x[b] = tap(b, TAPS);
 #pragma unroll
@@ -93,12 +93,18 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
 #pragma unroll
         for (int b = 1; b < TAPS; ++b) acc += x[b] * w[b];
       } else {
-        acc = cur * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1);
+        acc = Io<T>::ld(&cur) * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1);
         for (int b = 1; b < p.taps; ++b) acc += tap(b, p.taps) * Io<T>::ld(convw + (int64_t)ch * p.taps + p.taps - 1 - b);
       }
-      lds[n] = silu_f(acc);
+      if (n0 + tid < nch) lds[n] = silu_f(acc);
       // one token: its row of the ring is nobody's to read this step (readers take the taps - 1 rows before it)
-      if (L == 1 && pos >= 0 && (n >= 2 * D || h % per == 0)) ring[(int64_t)(pos % p.taps) * p.CH + ch] = pr[ch];
+      if (L == 1 && pos >= 0 && n0 + tid < nch && (n >= 2 * D || h % per == 0)) ring[(int64_t)(pos % p.taps) * p.CH + ch] = cur;
+    }
+    if (i == 0) {
+#pragma unroll
+      for (int n = 0; n < R; ++n)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) st[n][j] = start > 0 && has(n) ? st[n][j] : 0.f;
     }
     __syncthreads();
     float qq = 0.f, kk = 0.f;
@@ -109,12 +115,9 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
     float acc[VEC] = {};
 #pragma unroll
     for (int n = 0; n < R; ++n) {
-      const int d = g + n * groups;
-      if (on && d < D) {
-        const float k = sk[d] * kn;
+      const float k = has(n) ? sk[g + n * groups] * kn : 0.f;
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) st[n][j] *= decay, acc[j] += st[n][j] * k;
-      }
+      for (int j = 0; j < VEC; ++j) st[n][j] *= decay, acc[j] += st[n][j] * k;
     }
     if (on)
 #pragma unroll
@@ -131,12 +134,9 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
     }
 #pragma unroll
     for (int n = 0; n < R; ++n) {
-      const int d = g + n * groups;
-      if (on && d < D) {
-        const float k = sk[d] * kn, q = sq[d] * qn;
+      const float k = has(n) ? sk[g + n * groups] * kn : 0.f, q = has(n) ? sq[g + n * groups] * qn : 0.f;
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) st[n][j] += k * u[j], acc[j] += st[n][j] * q;
-      }
+      for (int j = 0; j < VEC; ++j) st[n][j] += k * u[j], acc[j] += st[n][j] * q;
     }
     if (on)
 #pragma unroll
@@ -159,13 +159,13 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaParams 
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) {
+    if (!has(i)) continue;
     const int d = g + i * groups;
-    if (on && d < D) {
-      if constexpr (VEC == 4) {
-        const f32x4 a = {st[i][0], st[i][1], st[i][2], st[i][3]};
-        __builtin_nontemporal_store(a, reinterpret_cast<f32x4*>(S + (int64_t)d * V + c));
-      }
-      else S[(int64_t)d * V + c] = st[i][0];
+    if constexpr (VEC == 4) {
+      const f32x4 a = {st[i][0], st[i][1], st[i][2], st[i][3]};
+      __builtin_nontemporal_store(a, reinterpret_cast<f32x4*>(S + (int64_t)d * V + c));
+    } else {
+      S[(int64_t)d * V + c] = st[i][0];
     }
   }
 }
@@ -174,7 +174,10 @@ template <typename T, int VEC, int NT, int R>
 int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
   const int groups = NT / (p.V / VEC);
   const size_t lds = (size_t)(2 * p.D + p.V + 2 * groups * p.V) * sizeof(float);
-  auto kern = p.taps == 4 ? gated_delta_step_kernel<T, VEC, NT, R, 4> : gated_delta_step_kernel<T, VEC, NT, R, 0>;
+  const bool full = VEC == 4 && NT % (p.V / VEC) == 0 && p.D == R * groups;
+  auto kern = p.taps != 4 ? gated_delta_step_kernel<T, VEC, NT, R, 0, false>
+              : full      ? gated_delta_step_kernel<T, VEC, NT, R, 4, true>
+                          : gated_delta_step_kernel<T, VEC, NT, R, 4, false>;
   if (lds > 65536) {
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
       return MI_ERR_LAUNCH;

@@ -331,43 +331,47 @@ __global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const
 // LDS-only barrier: register loads in flight stay in flight
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
-template <int DT>
-__global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, float* o,
-                                                               int nvt) {
+// NV 16-column value tiles a workgroup: its four waves read every operand of a chunk once for all of them (the bound is the
+// L2 traffic of those operands, each head's tiles reading the same ones)
+template <int DT, int NV>
+__global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, int nvg) {
   scalar_cache_acquire();
   constexpr int Dp = DT * 16, LS = Dp + 4, LU = kC + 4, MT = (DT + 3) / 4;
   constexpr bool whole = DT % 4 == 0;      // every wave owns MT tiles of the state
-  __shared__ __attribute__((aligned(16))) float sS[16 * LS];
-  __shared__ __attribute__((aligned(16))) float sU[16 * LU];
-  // the value tiles of a head on one XCD (workgroups go to the 8 XCDs in turn): they read the same workspace
+  __shared__ __attribute__((aligned(16))) float sS[NV * 16 * LS];
+  __shared__ __attribute__((aligned(16))) float sU[NV * 16 * LU];
+  // the workgroups of a head on one XCD (workgroups go to the 8 XCDs in turn)
   const int bid = blockIdx.x;
-  const int h = (bid / (8 * nvt)) * 8 + bid % 8, vt = (bid / 8) % nvt;
+  const int h = (bid / (8 * nvg)) * 8 + bid % 8, vg = (bid / 8) % nvg;
   const int r = p.req0 + blockIdx.y;
   const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
   if (h >= p.H || L <= 0) return;
   const int start = p.seq_lens[r] - L;
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lg = lane >> 4;
-  const int v = vt * 16 + lr;
+  const int v0 = vg * 16 * NV + lr;        // + 16 n: this lane's value columns
   float* S = p.state + (((int64_t)p.slots[r] * p.H + h) * p.D) * p.V;
-  f32x4_t st[MT];
+  f32x4_t st[NV][MT];
 #pragma unroll
-  for (int m = 0; m < MT; ++m) {
-    const int mt = wave + 4 * m;
+  for (int n = 0; n < NV; ++n)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = mt * 16 + 4 * lg + i;
-      st[m][i] = start > 0 && d < p.D && v < p.V ? S[(int64_t)d * p.V + v] : 0.f;
+    for (int m = 0; m < MT; ++m) {
+      const int mt = wave + 4 * m, v = v0 + 16 * n;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = mt * 16 + 4 * lg + i;
+        st[n][m][i] = start > 0 && d < p.D && v < p.V ? S[(int64_t)d * p.V + v] : 0.f;
+      }
+      if (mt < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + mt * 16 + 4 * lg) = st[n][m];
     }
-    if (mt < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + mt * 16 + 4 * lg) = st[m];
-  }
   const int nck = (L + kC - 1) / kC;
-  const float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
+  float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
   const int64_t step = p.H * lay.size();
   // one chunk's operands; the next chunk's are loaded a whole chunk ahead (the chain of chunks is the critical path, its
-  // loads must not be).  The loads are unconditional — past the last chunk they fetch what nobody uses — so that the number in
-  // flight is known at every wait.
+  // loads must not be).  Loads and stores are unconditional — past the last chunk the loads fetch what nobody uses, read-outs
+  // replace U in the workspace — so that the number in flight is known at every wait: memory operations retire in order, and a
+  // store that may or may not be there makes the wait for the loads behind it wait for its acknowledgement as well.
   struct Chunk {
-    f32x4_t w[DT], q[DT], pm[4], kt[MT][4], u;
+    f32x4_t w[DT], q[DT], pm[4], kt[MT][4], u[NV];
     float g;
   };
   auto load = [&](Chunk& x, int c) {
@@ -379,7 +383,10 @@ __global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaPar
       x.q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) x.u[i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v];
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        x.u[n][i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n];
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
       x.pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
@@ -390,38 +397,57 @@ __global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaPar
     x.g = b[lay.g()];
   };
   auto work = [&](Chunk& x, int c) {
-    f32x4_t d = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
+    f32x4_t d[NV] = {}, ao[NV] = {};
+    f32x4_t sv[2][NV];       // the next k block's reads under this one's products
+    auto get = [&](f32x4_t (&f)[NV], const float* b, int ld, int k) {
+#pragma unroll
+      for (int n = 0; n < NV; ++n) f[n] = *reinterpret_cast<const f32x4_t*>(b + (16 * n + lr) * ld + 16 * k + 4 * lg);
+    };
+    get(sv[0], sS, LS, 0);
 #pragma unroll
     for (int k = 0; k < DT; ++k) {
-      const f32x4_t sv = *reinterpret_cast<const f32x4_t*>(sS + lr * LS + 16 * k + 4 * lg);
+      if (k + 1 < DT) get(sv[(k + 1) & 1], sS, LS, k + 1);
 #pragma unroll
-      for (int s = 0; s < 4; ++s) {
-        d = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w[k][s], sv[s], d, 0, 0, 0);
-        ao = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[k][s], sv[s], ao, 0, 0, 0);
-      }
+      for (int n = 0; n < NV; ++n)
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          d[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w[k][s], sv[k & 1][n][s], d[n], 0, 0, 0);
+          ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[k][s], sv[k & 1][n][s], ao[n], 0, 0, 0);
+        }
+      __builtin_amdgcn_sched_barrier(0);
     }
-    *reinterpret_cast<f32x4_t*>(sU + lr * LU + 16 * wave + 4 * lg) = x.u - d;
+#pragma unroll
+    for (int n = 0; n < NV; ++n) *reinterpret_cast<f32x4_t*>(sU + (16 * n + lr) * LU + 16 * wave + 4 * lg) = x.u[n] - d[n];
     lds_barrier();
 #pragma unroll
-    for (int m = 0; m < MT; ++m) st[m] *= x.g;
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int m = 0; m < MT; ++m) st[n][m] *= x.g;
+    get(sv[0], sU, LU, 0);
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      const f32x4_t uv = *reinterpret_cast<const f32x4_t*>(sU + lr * LU + 16 * k + 4 * lg);
+      if (k < 3) get(sv[(k + 1) & 1], sU, LU, k + 1);
 #pragma unroll
-      for (int m = 0; m < MT; ++m)
-        if (whole || wave + 4 * m < DT)
+      for (int n = 0; n < NV; ++n)
 #pragma unroll
-          for (int s = 0; s < 4; ++s) st[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[m][k][s], uv[s], st[m], 0, 0, 0);
+        for (int s = 0; s < 4; ++s) {
+          const float uv = sv[k & 1][n][s];
 #pragma unroll
-      for (int s = 0; s < 4; ++s) ao = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv[s], ao, 0, 0, 0);
+          for (int m = 0; m < MT; ++m)
+            if (whole || wave + 4 * m < DT) st[n][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[m][k][s], uv, st[n][m], 0, 0, 0);
+          ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv, ao[n], 0, 0, 0);
+        }
+      __builtin_amdgcn_sched_barrier(0);
     }
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
-      if (whole || wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + lr * LS + (wave + 4 * m) * 16 + 4 * lg) = st[m];
+    for (int n = 0; n < NV; ++n) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = c * kC + 16 * wave + 4 * lg + i;
-      if (t < L && v < p.V) o[((int64_t)(s0 + t) * p.H + h) * p.V + v] = ao[i];
+      for (int m = 0; m < MT; ++m)
+        if (whole || wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + (wave + 4 * m) * 16 + 4 * lg) = st[n][m];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        base[c * step + lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n] = ao[n][i];
+      }
     }
     lds_barrier();
   };
@@ -436,24 +462,33 @@ __global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaPar
     work(b, c + 1);
   }
 #pragma unroll
-  for (int m = 0; m < MT; ++m)
+  for (int n = 0; n < NV; ++n)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = (wave + 4 * m) * 16 + 4 * lg + i;
-      if (d < p.D && v < p.V) S[(int64_t)d * p.V + v] = st[m][i];
-    }
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = (wave + 4 * m) * 16 + 4 * lg + i, v = v0 + 16 * n;
+        if (d < p.D && v < p.V) S[(int64_t)d * p.V + v] = st[n][m][i];
+      }
+}
+
+// the read-out of (row, head), where the scan left it
+__device__ __forceinline__ const float* readout(const DeltaParams& p, const float* ws, const ChunkLayout& lay, int nreq, int row, int h) {
+  const int r = p.req0 + row_request(p.qsl + p.req0, nreq, row);
+  const int i = row - p.qsl[r];
+  return ws + ((chunk_base(p, r) + i / kC) * p.H + h) * lay.size() + lay.u() + (int64_t)(i % kC) * lay.Vp;
 }
 
 // out = o / rms(o) * norm * silu(gate), 16 lanes per (row, head), 8 values a lane at a time; vdim a multiple of 8, <= 128 U
 template <typename T, int U>
-__global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaParams p, const float* o, int row0, int rows) {
+__global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, int nreq, int row0, int rows) {
   scalar_cache_acquire();
   const int64_t item = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
   const int sub = threadIdx.x & 15;
   if (item >= (int64_t)rows * p.H) return;     // whole 16-lane groups leave
   const int64_t row = row0 + item / p.H;
   const int h = (int)(item % p.H);
-  const float* x = o + (row * p.H + h) * (int64_t)p.V;
+  const float* x = readout(p, ws, lay, nreq, (int)row, h);
   const T* g = reinterpret_cast<const T*>(p.proj) + row * p.ld + p.off_g + h * p.V;
   float v[U][8], gt[U][8];
   float ss = 0.f;
@@ -482,14 +517,14 @@ __global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaPar
 
 // the same for any vdim, one wave per (row, head)
 template <typename T>
-__global__ __launch_bounds__(256) void gated_delta_finish_kernel(const DeltaParams p, const float* o, int row0, int rows) {
+__global__ __launch_bounds__(256) void gated_delta_finish_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, int nreq, int row0, int rows) {
   scalar_cache_acquire();
   const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (item >= (int64_t)rows * p.H) return;
   const int64_t row = row0 + item / p.H;
   const int h = (int)(item % p.H);
-  const float* x = o + (row * p.H + h) * (int64_t)p.V;
+  const float* x = readout(p, ws, lay, nreq, (int)row, h);
   float ss = 0.f;
   for (int v = lane; v < p.V; v += 64) ss += x[v] * x[v];
   const float inv = inv_rms(wave_allreduce_sum(ss), p.V, p.eps);
@@ -525,13 +560,13 @@ extern "C" int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t 
 
 extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w, const float* a_log,
                                       const float* dt_bias, const void* norm_w, float* state, void* ring, const int32_t* slots,
-                                      const int32_t* query_start_loc, const int32_t* seq_lens, void* out, float* o_f32, int32_t row0,
+                                      const int32_t* query_start_loc, const int32_t* seq_lens, void* out, int32_t row0,
                                       int32_t rows, int32_t req0, int32_t num_reqs, int32_t max_query_len, int32_t heads,
                                       int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps, float eps, void* workspace,
                                       int64_t workspace_bytes, int dtype, void* stream) {
   if (num_reqs == 0 || rows == 0) return MI_OK;
   if (!proj || !conv_w || !a_log || !dt_bias || !norm_w || !state || !ring || !slots || !query_start_loc || !seq_lens || !out ||
-      !o_f32 || !workspace)
+      !workspace)
     return MI_ERR_INVALID_ARG;
   if (req0 < 0 || num_reqs < 0 || row0 < 0 || rows < 0 || max_query_len <= 0 || heads <= 0 || kv_heads <= 0 || taps <= 0 ||
       heads % kv_heads)
@@ -562,22 +597,29 @@ extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, con
   if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
   else MI_PREP(float);
 #undef MI_PREP
-  const int nvt = lay.Vp / 16;
-  const dim3 sg((heads + 7) / 8 * 8 * nvt, num_reqs);
+  // two value tiles a workgroup where that still leaves one for every CU
+  const int nvt = lay.Vp / 16, nv = nvt % 2 == 0 && (int64_t)num_reqs * heads * (nvt / 2) >= 256 ? 2 : 1, nvg = nvt / nv;
+  const dim3 sg((heads + 7) / 8 * 8 * nvg, num_reqs);
+#define MI_SCAN(DT)                                                                                                            \
+  do {                                                                                                                         \
+    if (nv == 2) hipLaunchKernelGGL((gated_delta_scan_kernel<DT, 2>), sg, dim3(256), 0, s, p, ws, lay, nvg);                   \
+    else hipLaunchKernelGGL((gated_delta_scan_kernel<DT, 1>), sg, dim3(256), 0, s, p, ws, lay, nvg);                           \
+  } while (0)
   switch (lay.Dp / 16) {
-    case 2: hipLaunchKernelGGL((gated_delta_scan_kernel<2>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
-    case 4: hipLaunchKernelGGL((gated_delta_scan_kernel<4>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
-    case 8: hipLaunchKernelGGL((gated_delta_scan_kernel<8>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
-    default: hipLaunchKernelGGL((gated_delta_scan_kernel<16>), sg, dim3(256), 0, s, p, ws, lay, o_f32, nvt); break;
+    case 2: MI_SCAN(2); break;
+    case 4: MI_SCAN(4); break;
+    case 8: MI_SCAN(8); break;
+    default: MI_SCAN(16); break;
   }
+#undef MI_SCAN
   const dim3 fg((unsigned)(((int64_t)rows * heads + 3) / 4)), rg((CH + 255) / 256, num_reqs);
   const dim3 f8((unsigned)(((int64_t)rows * heads + 15) / 16));
-  const bool vecf = vec && aligned16(out) && aligned16(norm_w) && aligned16(o_f32);
+  const bool vecf = vec && aligned16(out) && aligned16(norm_w);
 #define MI_FINISH(T)                                                                                                              \
   do {                                                                                                                            \
-    if (vecf && vdim <= 128) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 1>), f8, dim3(256), 0, s, p, o_f32, row0, rows);   \
-    else if (vecf) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 2>), f8, dim3(256), 0, s, p, o_f32, row0, rows);             \
-    else hipLaunchKernelGGL((gated_delta_finish_kernel<T>), fg, dim3(256), 0, s, p, o_f32, row0, rows);                           \
+    if (vecf && vdim <= 128) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 1>), f8, dim3(256), 0, s, p, ws, lay, num_reqs, row0, rows);   \
+    else if (vecf) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 2>), f8, dim3(256), 0, s, p, ws, lay, num_reqs, row0, rows);             \
+    else hipLaunchKernelGGL((gated_delta_finish_kernel<T>), fg, dim3(256), 0, s, p, ws, lay, num_reqs, row0, rows);                           \
   } while (0)
   if (dtype == MI_DTYPE_BF16) {
     MI_FINISH(uint16_t);

@@ -16,44 +16,40 @@ namespace {
 using E16 = Elem<bf16_tag>;
 
 // ------------------------------------------------------------------------------------------------ per-head GEMM
-// y[t][h][n] = sum_k x[t][h][k] w[h][n][k]; wave = 16 n x 64 t, operands straight from global memory
+// y[t][h][n] = sum_k x[t][h][k] w[h][n][k]; wave = 16 n x 16 TT t, operands straight from global memory, 128 k of them in
+// flight.  Loads are unconditional on clamped addresses; FULL: Kd is a multiple of 32, nothing to blank out.
+template <int TT, bool FULL>
 __global__ __launch_bounds__(256) void head_gemm_nt_kernel(uint16_t* y, const uint16_t* x, const uint16_t* w, int rows, int N, int Kd,
                                                            int64_t y_row, int64_t x_row, int64_t w_head) {
   scalar_cache_acquire();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
-  const int h = blockIdx.y, n0 = blockIdx.x * 64 + wave * 16, t0 = blockIdx.z * 64;
+  const int h = blockIdx.y, n0 = blockIdx.x * 64 + wave * 16, t0 = blockIdx.z * 16 * TT;
   if (n0 >= N) return;
-  const int n = n0 + lr;
-  const uint16_t* wr = w + h * w_head + (int64_t)min(n, N - 1) * Kd + 8 * lg;
-  f32x4_t acc[4] = {};
-  const uint16_t* xr[4];
+  const uint16_t* wr = w + h * w_head + (int64_t)min(n0 + lr, N - 1) * Kd;
+  const uint16_t* xh = x + (int64_t)h * Kd;
+  f32x4_t acc[TT] = {};
+  for (int k0 = 0; k0 < Kd; k0 += 128) {
+    u32x4_t a[4], b[4][TT];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) xr[i] = x + (int64_t)min(t0 + 16 * i + lr, rows - 1) * x_row + (int64_t)h * Kd + 8 * lg;
-  const int live = min(4, (rows - t0 + 15) / 16);
-#pragma unroll 4
-  for (int k = 0; k < Kd; k += 32) {
-    const bool in = k + 8 * lg < Kd;      // Kd is a multiple of 8
-    const uint4 z = make_uint4(0, 0, 0, 0);
-    const uint4 a = in ? *reinterpret_cast<const uint4*>(wr + k) : z;
+    for (int u = 0; u < 4; ++u) {
+      const int k = min(k0 + 32 * u + 8 * lg, Kd - 8);      // Kd is a multiple of 8
+      a[u] = *reinterpret_cast<const u32x4_t*>(wr + k);
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i < live) {
-        const uint4 b = in ? *reinterpret_cast<const uint4*>(xr[i] + k) : z;
-        acc[i] = mfma16<bf16_tag>(a, b, acc[i]);
-      }
+      for (int i = 0; i < TT; ++i) b[u][i] = *reinterpret_cast<const u32x4_t*>(xh + (int64_t)min(t0 + 16 * i + lr, rows - 1) * x_row + k);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (FULL && k0 + 32 * u >= Kd) break;
+      if (!FULL && k0 + 32 * u + 8 * lg >= Kd) a[u] = u32x4_t{0, 0, 0, 0};
+#pragma unroll
+      for (int i = 0; i < TT; ++i) acc[i] = mfma16<bf16_tag>(__builtin_bit_cast(uint4, a[u]), __builtin_bit_cast(uint4, b[u][i]), acc[i]);
+    }
   }
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int t = t0 + 16 * i + lr;
-    if (t >= rows) continue;
-    uint16_t* o = y + t * y_row + (int64_t)h * N + n0 + 4 * lg;
-    if (n0 + 16 <= N && (N & 3) == 0) {
-      *reinterpret_cast<uint2*>(o) = make_uint2(E16::pack(acc[i][0], acc[i][1]), E16::pack(acc[i][2], acc[i][3]));
-    } else {
-#pragma unroll
-      for (int s = 0; s < 4; ++s)
-        if (n0 + 4 * lg + s < N) o[s] = E16::to_bits(acc[i][s]);
-    }
+  for (int i = 0; i < TT; ++i) {
+    const int t = t0 + 16 * i + lr, n = n0 + 4 * lg;
+    if (t < rows && n < N)      // N is a multiple of 4
+      *reinterpret_cast<uint2*>(y + t * y_row + (int64_t)h * N + n) = make_uint2(E16::pack(acc[i][0], acc[i][1]), E16::pack(acc[i][2], acc[i][3]));
   }
 }
 
@@ -69,8 +65,6 @@ struct LatentDecodeParams {
   int H, rank, bs_log2, window, nsplit;
   float scale;           // times log2(e)
 };
-
-constexpr int kBlockList = 256;
 
 __device__ __forceinline__ uint32_t lds_addr(const void* p) { return (uint32_t)(uintptr_t)(lds_void*)p; }
 
@@ -109,7 +103,6 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
   uint16_t* sC = reinterpret_cast<uint16_t*>(smem);           // [64][LD]
   uint16_t* sP = sC + 64 * LD;                                // [2 (hi, lo)][16 NHT][PL]
   float* sR = reinterpret_cast<float*>(sP + 2 * 16 * NHT * PL);   // [4][16 NHT]
-  int32_t* sB = reinterpret_cast<int32_t*>(sR + 4 * 16 * NHT);    // [kBlockList]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int kw = wave & 3, ht = wave >> 2;          // key group / dim group, head tile
   const int split = blockIdx.x, r = blockIdx.z;
@@ -129,37 +122,38 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
       const int c = 32 * k + 8 * lg;
       qf[k] = live && c < p.rank ? *reinterpret_cast<const uint4*>(qr + c) : make_uint4(0, 0, 0, 0);
     }
-    // the split's block ids in LDS (a load of the cache then waits for one memory access, not two); a split longer than the
-    // list reads the table itself
+    // a tile's block ids are loaded a tile ahead of its rows, its rows a tile ahead of their use.  Loads are unconditional on
+    // clamped addresses (rows past the split get weight 0, columns past the rank meet zeros of q and are not stored): the
+    // number in flight is known at every wait.
     const int32_t* tab = p.table + (int64_t)r * p.table_stride;
     const int bmask = (1 << p.bs_log2) - 1;
-    const int b0 = k0 >> p.bs_log2, nb = ((k1 - 1) >> p.bs_log2) - b0 + 1;
-    const bool listed = nb <= kBlockList;
-    if (listed)
-      for (int i = tid; i < nb; i += NT) sB[i] = tab[b0 + i];
-    __syncthreads();
-    uint4 pre[CH];
+    u32x4_t pre[CH];
+    int32_t blk[CH];
+    auto ids = [&](int t0) {
+#pragma unroll
+      for (int i = 0; i < CH; ++i) blk[i] = tab[min(t0 + (tid + i * NT) / (Rp / 8), k1 - 1) >> p.bs_log2];
+    };
     auto fetch = [&](int t0) {
 #pragma unroll
       for (int i = 0; i < CH; ++i) {
-        const int c = tid + i * NT, row = c / (Rp / 8), col = (c % (Rp / 8)) * 8, key = t0 + row;
-        pre[i] = make_uint4(0, 0, 0, 0);
-        if (key < k1 && col < p.rank)
-          pre[i] = *reinterpret_cast<const uint4*>(p.cache + (int64_t)(listed ? sB[(key >> p.bs_log2) - b0] : tab[key >> p.bs_log2]) * p.block_stride +
-                                                   (int64_t)(key & bmask) * p.token_stride + col);
+        const int c = tid + i * NT, key = min(t0 + c / (Rp / 8), k1 - 1), col = min((c % (Rp / 8)) * 8, p.rank - 8);
+        pre[i] = *reinterpret_cast<const u32x4_t*>(p.cache + (int64_t)blk[i] * p.block_stride + (int64_t)(key & bmask) * p.token_stride + col);
       }
     };
+    ids(k0);
     fetch(k0);
+    ids(k0 + 64);
     const uint32_t tr_base = lds_addr(sC) + (uint32_t)(((8 * lg + (lr >> 2)) * LD + kw * (Rp / 4) + 4 * (lr & 3)) * 2);
     for (int t0 = k0; t0 < k1; t0 += 64) {
       __syncthreads();        // the previous tile's readers are done
 #pragma unroll
       for (int i = 0; i < CH; ++i) {
         const int c = tid + i * NT, row = c / (Rp / 8), col = (c % (Rp / 8)) * 8;
-        *reinterpret_cast<uint4*>(sC + row * LD + col) = pre[i];
+        *reinterpret_cast<u32x4_t*>(sC + row * LD + col) = pre[i];
       }
       __syncthreads();
-      if (t0 + 64 < k1) fetch(t0 + 64);
+      fetch(t0 + 64);      // (past the end: the last row again)
+      ids(t0 + 128);
       f32x4_t s = {}, s2 = {};
 #pragma unroll
       for (int k = 0; k < 2 * RN; k += 2) {
@@ -456,7 +450,7 @@ __global__ __launch_bounds__(256, KT <= 8 && VN <= 4 ? 2 : 1) void latent_prefil
 template <int RN, int NHT>
 int launch_decode(const LatentDecodeParams& p, int reqs, hipStream_t s) {
   constexpr int LD = 64 * RN + 8, PL = 72;
-  constexpr int lds = (64 * LD + 2 * 16 * NHT * PL) * 2 + 4 * 16 * NHT * 4 + kBlockList * 4;
+  constexpr int lds = (64 * LD + 2 * 16 * NHT * PL) * 2 + 4 * 16 * NHT * 4;
   auto kern = latent_decode_kernel<RN, NHT>;
   if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess)
     return MI_ERR_LAUNCH;
@@ -496,8 +490,18 @@ extern "C" int mi_head_gemm_nt(void* y, const void* x, const void* w, int32_t ro
   if (y_row_stride < (int64_t)heads * n || x_row_stride < (int64_t)heads * k || w_head_stride < (int64_t)n * k) return MI_ERR_INVALID_ARG;
   if (k % 8 || n % 4 || x_row_stride % 8 || y_row_stride % 4 || w_head_stride % 8 || !aligned16(x) || !aligned16(w) || ((uintptr_t)y & 7))
     return MI_ERR_UNSUPPORTED;
-  hipLaunchKernelGGL(head_gemm_nt_kernel, dim3((n + 63) / 64, heads, (rows + 63) / 64), dim3(256), 0, (hipStream_t)stream, (uint16_t*)y,
-                     (const uint16_t*)x, (const uint16_t*)w, rows, n, k, y_row_stride, x_row_stride, w_head_stride);
+#define MI_HG(TT, FULL)                                                                                                           \
+  hipLaunchKernelGGL((head_gemm_nt_kernel<TT, FULL>), dim3((n + 63) / 64, heads, (rows + 16 * TT - 1) / (16 * TT)), dim3(256), 0, \
+                     (hipStream_t)stream, (uint16_t*)y, (const uint16_t*)x, (const uint16_t*)w, rows, n, k, y_row_stride, x_row_stride, w_head_stride)
+  if (k % 32 == 0) {
+    if (rows <= 16) MI_HG(1, true);
+    else if (rows <= 32) MI_HG(2, true);
+    else MI_HG(4, true);
+  } else {
+    if (rows <= 16) MI_HG(1, false);
+    else MI_HG(4, false);
+  }
+#undef MI_HG
   return launch_status();
 }
 

@@ -1332,10 +1332,9 @@ def gated_delta_chunked(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots
         return gated_delta_step(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads,
                                 eps, out, req0, num_reqs)
     ws = torch.empty(need, dtype=torch.uint8, device=proj.device)
-    o = torch.empty(proj.shape[0], hh * v, dtype=torch.float32, device=proj.device)
     check("mi_gated_delta_chunked", lib.mi_gated_delta_chunked(
         _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
-        _p(seq_lens), _p(out), _p(o), row0, rows, req0, num_reqs, max_query_len, hh, kv_heads, d, v, taps, float(eps), _p(ws),
+        _p(seq_lens), _p(out), row0, rows, req0, num_reqs, max_query_len, hh, kv_heads, d, v, taps, float(eps), _p(ws),
         need, _dt(proj.dtype), _stream()))
     return out
 
