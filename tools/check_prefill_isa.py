@@ -15,7 +15,8 @@ import tempfile
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 SRC = os.path.join(ROOT, "vllm-omni_amd", "csrc", "paged_attn_prefill.hip")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
-FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950", "-Wno-pass-failed", "-fno-slp-vectorize", "--cuda-device-only", "-S"]
+FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950", "-Wno-pass-failed", "-fno-slp-vectorize", "-Xclang", "-target-feature",
+         "-Xclang", "-packed-fp32-ops", "--cuda-device-only", "-S"]
 
 
 def regs(tok: str):

@@ -1,5 +1,5 @@
 """Per-phase timing of the code predictor's one-launch stack from inside the kernel (debug build):
-    cd vllm-omni_amd/csrc && hipcc -O3 -std=c++17 -fPIC --offload-arch=gfx950 -DMI_CP_TIMING -DMI_CP_TIMING_WG=0 -shared cp_stack.hip \
+    cd vllm-omni_amd/csrc && hipcc -O3 -std=c++17 -fPIC -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 -DMI_CP_TIMING -DMI_CP_TIMING_WG=0 -shared cp_stack.hip \
         -o ../build/libcp_stack_timing.so
     python tools/debug_cp_stack_timing.py [rows]
 Loads the debug library for mi_cp_stack_decode only; prints work / barrier microseconds of every phase of the first layers."""

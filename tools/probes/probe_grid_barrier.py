@@ -1,5 +1,5 @@
 """Cost of a grid-wide barrier inside one persistent launch, and of streaming a phase's weights between two of them.
-    hipcc --offload-arch=gfx950 -O3 -shared -fPIC tools/probes/grid_barrier.hip -o tools/probes/grid_barrier.so
+    hipcc --offload-arch=gfx950 -O3 -Xclang -target-feature -Xclang -packed-fp32-ops -shared -fPIC tools/probes/grid_barrier.hip -o tools/probes/grid_barrier.so
     python tools/probes/probe_grid_barrier.py
 """
 import ctypes

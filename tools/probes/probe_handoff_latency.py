@@ -1,5 +1,5 @@
 """Producer -> consumer hand-off of freshly written rows between two workgroups of one launch (device scope).
-    hipcc --offload-arch=gfx950 -O3 -shared -fPIC tools/probes/handoff_latency.hip -o tools/probes/handoff_latency.so
+    hipcc --offload-arch=gfx950 -O3 -Xclang -target-feature -Xclang -packed-fp32-ops -shared -fPIC tools/probes/handoff_latency.hip -o tools/probes/handoff_latency.so
     python tools/probes/probe_handoff_latency.py
 """
 import ctypes

@@ -1,5 +1,5 @@
 """Round-trip latency of dependent loads / acknowledged stores of ONE wave at the scopes the one-launch stack uses.
-    hipcc --offload-arch=gfx950 -O3 -shared -fPIC tools/probes/scope_latency.hip -o tools/probes/scope_latency.so
+    hipcc --offload-arch=gfx950 -O3 -Xclang -target-feature -Xclang -packed-fp32-ops -shared -fPIC tools/probes/scope_latency.hip -o tools/probes/scope_latency.so
     python tools/probes/probe_scope_latency.py
 """
 import ctypes

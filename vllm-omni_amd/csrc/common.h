@@ -53,11 +53,17 @@ struct Elem<f16_tag> {
   static __device__ __forceinline__ float from_bits(uint16_t b) {
     return (float)__builtin_bit_cast(_Float16, b);
   }
+  // The value is an fp32 value first: without the (empty) asm hipcc folds the operation in front and the conversion into one
+  // `v_fma_mixlo_f16` — a single rounding — in some kernels and not in others, and kernels that must agree bit for bit do not.
+  static __device__ __forceinline__ float as_f32(float f) {
+    asm("" : "+v"(f));
+    return f;
+  }
   static __device__ __forceinline__ uint16_t to_bits(float f) {
-    return __builtin_bit_cast(uint16_t, (_Float16)f);
+    return __builtin_bit_cast(uint16_t, (_Float16)as_f32(f));
   }
   static __device__ __forceinline__ uint32_t pack(float a, float b) {
-    f16x2_t v = {(_Float16)a, (_Float16)b};
+    f16x2_t v = {(_Float16)as_f32(a), (_Float16)as_f32(b)};
     return __builtin_bit_cast(uint32_t, v);
   }
   static __device__ __forceinline__ float dot2(uint32_t a, uint32_t b, float acc) {
