@@ -303,6 +303,26 @@ class AsyncOmniModelRunnerOutput:
         return self._out
 
 
+_KEPT_GRAPHS: dict = {}      # device index -> the capture of `keep_generator_tensors_normal`, alive with the process
+
+
+def keep_generator_tensors_normal() -> None:
+    """torch's default generator owns seed / offset tensors while any captured graph is alive; they are created by the first
+    capture.  Created under inference mode (the runner's step) they are inference tensors: every capture OUTSIDE inference mode
+    then fails on their in-place update and leaves the generator marked as capturing.  One capture of a single small kernel in
+    normal mode, kept for the life of the process, makes them ordinary tensors, which both modes may update."""
+    dev = torch.cuda.current_device()
+    if dev in _KEPT_GRAPHS:
+        return
+    with torch.inference_mode(False):
+        x = torch.zeros(1, device=f"cuda:{dev}")
+        g = torch.cuda.CUDAGraph()
+        torch.cuda.synchronize()
+        with torch.cuda.graph(g):
+            x.add_(1)
+        _KEPT_GRAPHS[dev] = (g, x)
+
+
 class no_gc_during_capture:
     """The cyclic garbage collector must not run while a stream is capturing: collecting a dead tensor / graph / event
     there issues HIP calls that are illegal during capture and the process aborts (seen: "Fatal Python error: Aborted
@@ -315,6 +335,7 @@ class no_gc_during_capture:
         self._was_enabled = gc.isenabled()
         gc.collect()
         gc.disable()
+        keep_generator_tensors_normal()
         return self
 
     def __exit__(self, *exc):
