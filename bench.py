@@ -81,6 +81,7 @@ def parse_args():
     ap.add_argument("--dogulorn-mode", default="decode,prefill")
     ap.add_argument("--dogulorn-models", default="dogulorn,talker")
     ap.add_argument("--dogulorn-batches", default="32,256", help="decode batch sizes")
+    ap.add_argument("--dogulorn-ctx", type=int, default=4096, help="context of the decode cases")
     ap.add_argument("--dogulorn-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
     a = ap.parse_args()
     if a.pmc_child:   # a few steps of the same workload, nothing else: the parent reads the counters of the decode launches

@@ -131,7 +131,7 @@ def run(a):
         for mode in a.dogulorn_mode.split(","):
             for name in a.dogulorn_models.split(","):
                 cfg = (dogulorn_config if name == "dogulorn" else talker_config)(s)
-                cases = ([(int(b), 4096) for b in a.dogulorn_batches.split(",")] if mode == "decode" else
+                cases = ([(int(b), a.dogulorn_ctx) for b in a.dogulorn_batches.split(",")] if mode == "decode" else
                          [[int(n) for n in c.split(",")] for c in a.dogulorn_prompts.split(";")])
                 for case in cases:
                     with torch.inference_mode():

@@ -115,13 +115,10 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
   f32x4_t acc[MT] = {};
   float m = -INFINITY, l = 0.f;
   if (k0 < k1) {
-    uint4 qf[2 * RN];
+    u32x4_t qv[2 * RN];
     const uint16_t* qr = p.q + ((int64_t)r * p.H + (live ? head : 0)) * p.rank;
 #pragma unroll
-    for (int k = 0; k < 2 * RN; ++k) {
-      const int c = 32 * k + 8 * lg;
-      qf[k] = live && c < p.rank ? *reinterpret_cast<const uint4*>(qr + c) : make_uint4(0, 0, 0, 0);
-    }
+    for (int k = 0; k < 2 * RN; ++k) qv[k] = *reinterpret_cast<const u32x4_t*>(qr + min(32 * k + 8 * lg, p.rank - 8));
     // a tile's block ids are loaded a tile ahead of its rows, its rows a tile ahead of their use.  Loads are unconditional on
     // clamped addresses (rows past the split get weight 0, columns past the rank meet zeros of q and are not stored): the
     // number in flight is known at every wait.
@@ -143,6 +140,12 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
     ids(k0);
     fetch(k0);
     ids(k0 + 64);
+    uint4 qf[2 * RN];
+#pragma unroll
+    for (int k = 0; k < 2 * RN; ++k) {
+      const bool in = 32 * k + 8 * lg < p.rank;
+      qf[k] = make_uint4(in ? qv[k][0] : 0, in ? qv[k][1] : 0, in ? qv[k][2] : 0, in ? qv[k][3] : 0);
+    }
     const uint32_t tr_base = lds_addr(sC) + (uint32_t)(((8 * lg + (lr >> 2)) * LD + kw * (Rp / 4) + 4 * (lr & 3)) * 2);
     for (int t0 = k0; t0 < k1; t0 += 64) {
       __syncthreads();        // the previous tile's readers are done
@@ -247,21 +250,32 @@ __global__ __launch_bounds__(256 * NHT) void latent_decode_kernel(const LatentDe
 
 __global__ __launch_bounds__(128) void latent_decode_merge_kernel(uint16_t* out, const float* part, int H, int rank, int nsplit) {
   scalar_cache_acquire();
-  const int h = blockIdx.x, r = blockIdx.y;
+  const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x & 63;
   const int64_t st = (int64_t)H * (rank + 4);
   const float* b = part + ((int64_t)r * nsplit * H + h) * (rank + 4);
-  float m = -INFINITY;
-  for (int s = 0; s < nsplit; ++s) m = fmaxf(m, b[s * st + rank]);
-  float l = 0.f;
-  for (int s = 0; s < nsplit; ++s) l += b[s * st + rank + 1] * (b[s * st + rank + 1] > 0.f ? fast_exp2(b[s * st + rank] - m) : 0.f);
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
-  for (int d = threadIdx.x * 4; d < rank; d += 512) {
-    f32x4_t a = {};
-    for (int s = 0; s < nsplit; ++s)
-      if (b[s * st + rank + 1] > 0.f) a += *reinterpret_cast<const f32x4_t*>(b + s * st + d) * fast_exp2(b[s * st + rank] - m);
-    a *= inv;
-    *reinterpret_cast<uint2*>(out + ((int64_t)r * H + h) * rank + d) = make_uint2(E16::pack(a[0], a[1]), E16::pack(a[2], a[3]));
+  const int d = threadIdx.x * 4;
+  const float* bd = b + min(d, rank - 4);
+  // lane s holds split s's maximum and sum (at most 64 splits); eight splits' values are in flight at a time
+  f32x4_t v[8];
+  auto fetch = [&](int s0) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = *reinterpret_cast<const f32x4_t*>(bd + min(s0 + j, nsplit - 1) * st);
+  };
+  const float* bs = b + min(lane, nsplit - 1) * st + rank;
+  const float ms = bs[0], ls = lane < nsplit ? bs[1] : 0.f;
+  fetch(0);
+  const float m = wave_allreduce_max(ls > 0.f ? ms : -INFINITY);
+  const float w = ls > 0.f ? fast_exp2(ms - m) : 0.f;      // a split without tokens: 0
+  const float l = wave_allreduce_sum(ls * w);
+  f32x4_t a = {};
+  for (int s0 = 0; s0 < nsplit; s0 += 8) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) a += v[j] * __shfl(w, s0 + j, 64);
+    fetch(s0 + 8);
   }
+  a *= l > 0.f ? 1.0f / l : 0.f;
+  if (d < rank)
+    *reinterpret_cast<uint2*>(out + ((int64_t)r * H + h) * rank + d) = make_uint2(E16::pack(a[0], a[1]), E16::pack(a[2], a[3]));
 }
 
 // ------------------------------------------------------------------------------------------------ prefill
