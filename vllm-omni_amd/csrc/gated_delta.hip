@@ -2,9 +2,9 @@
 //
 // Per v-head h (its q/k head is h / (heads / kv_heads)) and token:
 //   q, k, v   = silu(causal conv over time of the projections);  q, k made unit vectors, q times dim^-1/2
-//   S        <- g S,  u = beta (v - S^T k),  S <- S + k u^T,  o = S^T q        g = exp(-exp(A_log) softplus(a + dt_bias))
-//   out       = o / rms(o) * norm * silu(gate)
-// The projections of a row arrive as one row [q | k | v | gate | b | a].  Per request slot the state is S [dim][vdim]
+//   M_t = g M_(t-1) + k (x) e   with  e = b (v - g k M_(t-1)),   y = q M_t        ln g = -exp(A_log) softplus(a + dt_bias)
+//   out       = y / rms(y) * norm * silu(gate)
+// The projections of a row arrive as one row [q | k | v | gate | b | a].  Per request slot the state is M [dim][vdim]
 // fp32 per head and a ring of the last `taps` projection rows (row p % taps holds position p); a request whose first
 // token is position 0 starts from zeros whatever the slot holds, so slots need no clearing.
 //

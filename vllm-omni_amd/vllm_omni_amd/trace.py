@@ -1,12 +1,12 @@
-"""``trace_run``: replay given token ids through a model, step by step, and write logits.
+"""``trace_run``: drive a model with tokens chosen by the caller instead of sampled ones, and write the logits it gives.
 
-Steps arrive on standard input, one JSON object a line::
+The input has a line of JSON per step, for instance::
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17], "want": [0, 1]}], "end": []}
+    {"step": 3, "entries": [{"id": "req7", "tokens": [40, 8, 2], "want": [2]}], "end": ["req5"]}
 
-All entries of a step run as one batch.  For a step that wants something ``OUT/<step>.f32`` gets the logits (little-endian
-fp32, [wanted, vocab], in the order of the entries); ``done <step>`` is printed after every step.  Ids in ``end`` give back
-their cache blocks and state slot.
+The entries form one batch: each appends its tokens to its request (a new id starts one).  ``want`` lists places among the
+entry's own tokens; their logits go to ``OUT/<step>.f32`` as little-endian fp32 rows, entry after entry.  ``end`` finishes
+requests, whose blocks and state slots become free.  ``done <step>`` follows on standard output.
 """
 from __future__ import annotations
 
