@@ -23,7 +23,7 @@
 extern "C" {
 #endif
 
-#define MI_ABI_VERSION 3
+#define MI_ABI_VERSION 4
 
 /* dtype enum shared by every entry point */
 enum {
@@ -802,32 +802,137 @@ int mi_latent_prefill(void* out, const void* q, const void* k, const void* vt,
                       int32_t heads, int32_t dim, int32_t vdim, int32_t window, float scale,
                       int64_t out_stride, int64_t q_stride, int64_t k_stride, int64_t vt_stride,
                       void* stream);
-/* Gated delta rule over requests [req0, req0 + num_reqs), token by token:
- * proj rows [q | k | v | gate | b | a] (heads / kv_heads q-k sharing), short
- * causal convolutions (conv_w [2 kv_heads dim + heads vdim][taps]) + silu, unit
- * q / k, decayed state update and read-out, gated norm; out [rows][heads vdim].
- * state [slots][heads][dim][vdim] fp32, ring [slots][taps][conv channels].
- * update_ring: also leave multi-token portions' last rows in the ring (a
- * one-token portion's row is always left there). */
-int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_w,
-                        const float* a_log, const float* dt_bias, const void* norm_w, float* state,
-                        void* ring, const int32_t* slots, const int32_t* query_start_loc,
-                        const int32_t* seq_lens, void* out, int32_t req0, int32_t num_reqs,
-                        int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps,
-                        float eps, int32_t update_ring, int dtype, void* stream);
+/* Gated delta rule over requests [req0, req0 + num_reqs): short causal
+ * convolutions (conv_w [2 kv_heads dim + heads vdim][taps]) of the q | k | v
+ * projections + silu, unit q / k, decayed state update and read-out, gated norm;
+ * out[row] = heads x vdim values.  decay: the projection softplus takes, one per
+ * head (a_log [heads], dt_bias [heads]) or, channel_decay, one per head and key
+ * channel (dt_bias [heads dim]).  The output gate is silu(gate), or
+ * sigmoid(gate).  state [slots][heads][dim][vdim] fp32, ring [slots][taps][conv
+ * channels]. */
+typedef struct {
+  const void *qkv, *gate, *beta, *decay; /* rows of the model's dtype */
+  const void *conv_w, *norm_w;
+  const float *a_log, *dt_bias;
+  float* state;
+  void* ring;
+  const int32_t *slots, *query_start_loc, *seq_lens;
+  void* out;
+  int64_t qkv_stride, gate_stride, beta_stride, decay_stride, out_stride;
+  int32_t req0, num_reqs, heads, kv_heads, dim, vdim, taps;
+  int32_t channel_decay, sigmoid_gate;
+  float eps;
+} mi_gated_delta_args;
+/* token by token.  update_ring: also leave multi-token portions' last rows in
+ * the ring (a one-token portion's row is always left there). */
+int mi_gated_delta_step(const mi_gated_delta_args* args, int32_t update_ring, int dtype, void* stream);
 /* The same for prompt portions, 64 tokens at a time on the fp32 matrix cores
- * (dim, vdim <= 256): requests [req0, req0 + num_reqs) own rows [row0, row0 +
- * rows); the workspace is scratch. */
+ * (dim, vdim <= 256; channel_decay: dim <= 128): the requests own rows [row0,
+ * row0 + rows); the workspace is scratch, 0 bytes = sizes not built. */
 int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads,
-                                               int32_t dim, int32_t vdim);
-int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w,
-                           const float* a_log, const float* dt_bias, const void* norm_w,
-                           float* state, void* ring, const int32_t* slots,
-                           const int32_t* query_start_loc, const int32_t* seq_lens, void* out,
-                           int32_t row0, int32_t rows, int32_t req0, int32_t num_reqs,
-                           int32_t max_query_len, int32_t heads, int32_t kv_heads, int32_t dim,
-                           int32_t vdim, int32_t taps, float eps, void* workspace,
-                           int64_t workspace_bytes, int dtype, void* stream);
+                                               int32_t dim, int32_t vdim, int32_t channel_decay);
+int mi_gated_delta_chunked(const mi_gated_delta_args* args, int32_t row0, int32_t rows,
+                           int32_t max_query_len, void* workspace, int64_t workspace_bytes,
+                           int dtype, void* stream);
+
+/* ------------------------------------------------------------------------
+ * Decoders whose layers run mixer and feed-forward side by side (Pupopel):
+ * bf16 or fp32 as above.
+ * ---------------------------------------------------------------------- */
+enum { MI_ACT_SILU = 0, MI_ACT_GELU_TANH = 1 };
+/* x[row] += y[row] + sum_j weights[row][j] part[row_of_pair[row][j]] (start: x
+ * is not read);  h[row] = x / rms(x) * (w_pre + w_shift), or the cast of x when
+ * w_pre == NULL.  y: rows of dtype (split == 0) or fp32 slabs [split][rows]
+ * [y_stride].  part == NULL: no routed experts; row_of_pair == NULL: pair
+ * row * top + j is its own row. */
+int mi_residual_add_norm(void* x, const void* y, int32_t split, const void* part,
+                         const int32_t* row_of_pair, const float* weights, int32_t top,
+                         const void* w_pre, float w_shift, void* h, int32_t start, float eps,
+                         int32_t rows, int32_t width, int64_t x_stride, int64_t y_stride,
+                         int64_t h_stride, int64_t part_stride, int dtype, void* stream);
+/* x = table[id] (fp32; zeros for ids outside the table), copy = the same in
+ * dtype (NULL: none);  h as above. */
+int mi_embed_norm(void* x, void* h, void* copy, const void* table, const void* w_pre, float w_shift,
+                  const int64_t* ids, float eps, int32_t rows, int32_t width, int32_t vocab,
+                  int64_t x_stride, int64_t h_stride, int64_t copy_stride, int dtype, void* stream);
+/* out = act(gate) * up */
+int mi_glu(void* out, const void* gate, const void* up, int32_t rows, int32_t ff, int64_t gu_stride,
+           int64_t out_stride, int32_t act, int dtype, void* stream);
+/* Rows q (heads x dim) | k (kv x dim) | v (kv x vdim): q and k RMS-normed per
+ * head (NULL weight: not), q times 1 + coef ln(floor((position + 1) / every) +
+ * 1); q to q_out, k and v to their cache rows, heads head_dim apart and padded
+ * with zeros up to it. */
+int mi_head_norm_cache(const void* x, int64_t x_stride, const void* q_weight, const void* k_weight,
+                       void* q_out, int64_t q_stride, void* k_cache, void* v_cache,
+                       const int64_t* slot_mapping, const int64_t* positions, int32_t rows,
+                       int32_t num_q_heads, int32_t num_kv_heads, int32_t dim, int32_t vdim,
+                       int32_t head_dim, int32_t block_size, int64_t cache_block_stride,
+                       int64_t cache_token_stride, int64_t cache_head_stride, float temp_coef,
+                       int64_t temp_every, float eps, int dtype, void* stream);
+/* Causal attention of rows [row0, row0 + rows) with a distance bias (slopes
+ * [num_q_heads] or NULL: score -= slope (position - key position)) and a sink
+ * (sinks [num_q_heads] or NULL: exp(sink) in the denominator), the output times
+ * out_scale: any sizes, bf16 or fp32. */
+int mi_attn_rows(void* out, const void* q, const void* k_cache, const void* v_cache,
+                 const int32_t* block_table, const int32_t* seq_lens, const int32_t* query_start_loc,
+                 const float* slopes, const float* sinks, float out_scale, int32_t row0, int32_t rows,
+                 int32_t num_reqs, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                 int32_t block_size, float scale, int64_t q_stride, int64_t out_stride,
+                 int64_t cache_block_stride, int64_t cache_token_stride, int64_t cache_head_stride,
+                 int64_t table_stride, int dtype, void* stream);
+/* mi_paged_attn_decode / mi_paged_attn_prefill_split with the same bias and
+ * sink: bf16, head_dim 64 or 128, block_size >= 16, scale > 0. */
+int mi_paged_attn_decode_biased(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                const int32_t* block_table, const int32_t* seq_lens,
+                                const float* slopes, const float* sinks, float out_scale,
+                                int32_t num_seqs, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                                int32_t block_size, int32_t block_table_stride, int32_t max_seq_len,
+                                float scale, int64_t q_token_stride, int64_t out_token_stride,
+                                int64_t cache_block_stride, int64_t cache_token_stride,
+                                int64_t cache_head_stride, int32_t partition_size, void* workspace,
+                                int64_t workspace_bytes, int dtype, void* stream);
+int mi_paged_attn_prefill_biased(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                 const int32_t* block_table, const int32_t* seq_lens,
+                                 const int32_t* query_start_loc, const float* slopes,
+                                 const float* sinks, float out_scale, int32_t num_seqs,
+                                 int32_t num_tokens, int32_t max_query_len, int32_t num_q_heads, int32_t num_kv_heads,
+                                 int32_t head_dim, int32_t block_size, int32_t block_table_stride,
+                                 float scale, int64_t q_token_stride, int64_t out_token_stride,
+                                 int64_t cache_block_stride, int64_t cache_token_stride,
+                                 int64_t cache_head_stride, int dtype, int32_t max_seq_len,
+                                 int32_t force_segments, void* workspace, int64_t workspace_bytes,
+                                 void* stream);
+/* Decayed linear attention over requests [req0, req0 + num_reqs): q, k, v =
+ * silu of rows q (heads x dim) | k (heads x dim) | v (heads x vdim); S = decay S
+ * + k v^T, o = S^T q; out[row] = o / rms(o over all heads) * norm_w *
+ * sigmoid(gate) * mul.  state [slots][heads][dim][vdim] fp32. */
+typedef struct {
+  const void *qkv, *gate, *norm_w;
+  const float *decay, *log2_decay; /* [heads] */
+  float* state;
+  const int32_t *slots, *query_start_loc, *seq_lens;
+  void* out;
+  int64_t qkv_stride, gate_stride, out_stride;
+  int32_t req0, num_reqs, heads, dim, vdim;
+  float eps, mul;
+} mi_lightning_args;
+/* The requests own rows [row0, row0 + rows).  chunked: 64 tokens at a time on
+ * the fp32 matrix cores (dim, vdim <= 256), else token by token.  The workspace
+ * is scratch; 0 bytes = sizes not built. */
+int64_t mi_lightning_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t dim,
+                                     int32_t vdim, int32_t chunked);
+int mi_lightning_attn(const mi_lightning_args* args, int32_t row0, int32_t rows,
+                      int32_t max_query_len, int32_t chunked, void* workspace,
+                      int64_t workspace_bytes, int dtype, void* stream);
+/* fp32 router logits of bf16 rows: out[t][e] = h[t] . weight[e] + bias[e] */
+int mi_moe_router_logits(float* out, const void* h, const void* weight, const float* bias,
+                         int32_t rows, int32_t num_experts, int32_t k, int64_t h_stride, void* stream);
+/* mi_moe_expert_gemm for any sizes and for fp32, pairs ungrouped: row p of out
+ * (and of a_rows, gated == 0) belongs to pair p = token * top_k + j. */
+int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const int32_t* topk_ids,
+                     int32_t num_pairs, int32_t num_experts, int32_t gated, int32_t n_out, int32_t k,
+                     int32_t top_k, int64_t a_row_stride, int64_t out_row_stride,
+                     int64_t weight_expert_stride, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -38,6 +38,11 @@ struct DecodeParams {
   const void* q_norm_w = nullptr;
   const void* k_norm_w = nullptr;
   float norm_eps = 0.f;
+  // distance bias and sink (matrix-core kernel, bf16): score -= slopes[head] * (position - key position), the softmax's
+  // denominator also holds exp(sinks[head]).  fp32 [num_q_heads] each, nullptr = none
+  const float* slopes = nullptr;
+  const float* sinks = nullptr;
+  float out_scale = 1.f;   // the output times this (matrix-core kernel and the merge)
 };
 
 // paged_attn_decode_mfma.hip

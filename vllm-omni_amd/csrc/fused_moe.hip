@@ -19,6 +19,7 @@
 #include "common.h"
 #include "skinny_grouped.h"
 #include "mfma_attn_common.h"
+#include "row_io.h"
 
 namespace mi {
 namespace {
@@ -43,8 +44,8 @@ __device__ __forceinline__ float wave_max_valu(float v) {
   return rows_allreduce_max(v);
 }
 
-template <int DT, int EPL>  // EPL = experts per lane = E / 64
-__global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict__ logits, int64_t row_stride,
+template <int DT, int EPL>  // EPL = experts per lane = E / 64, rounded up
+__global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict__ logits, int64_t row_stride, int num_experts,
                                                          int32_t* __restrict__ ids, float* __restrict__ weights,
                                                          int32_t* __restrict__ counts, int T, int top_k, int norm,
                                                          int round_dt) {
@@ -61,7 +62,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
     float mx = -INFINITY;
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
-      const int e = lane + 64 * i;
+      const int e = min(lane + 64 * i, num_experts - 1);
       if constexpr (DT == MI_DTYPE_F32) p[i] = reinterpret_cast<const float*>(logits)[t * row_stride + e];
       else if constexpr (DT == MI_DTYPE_BF16)
         p[i] = Elem<bf16_tag>::from_bits(reinterpret_cast<const uint16_t*>(logits)[t * row_stride + e]);
@@ -73,7 +74,8 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
       p[i] = __expf(p[i] - mx);
-      s += p[i];
+      if (lane + 64 * i >= num_experts) p[i] = -1.f;   // not an expert
+      else s += p[i];
     }
     s = wave_allreduce_sum(s);
     const float inv = 1.f / s;
@@ -117,7 +119,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
   __syncthreads();
   for (int e = threadIdx.x; e < 64 * EPL; e += 1024) {
     const int c = hist[e];
-    if (c) atomicAdd(&counts[e], c);
+    if (c) atomicAdd(&counts[e], c);   // (only experts that exist are ever chosen)
   }
 }
 
@@ -236,7 +238,8 @@ struct MoeGemmParams {
 
 // GATED: gemm 1 — a wave owns 16 gate rows and the 16 matching up rows; WG = 4 waves = 64 outputs.
 // !GATED: gemm 2 — a wave owns 32 weight rows; WG = 4 waves = 128 outputs.
-template <typename Tag, bool GATED, int MT>  // MT = 16-row token tiles per workgroup tile (2 or 4)
+// GUARD: any n_out that is a multiple of 4 and any K that is a multiple of 8 (weight rows and k past the end are blanked out)
+template <typename Tag, bool GATED, int MT, bool GUARD = false>  // MT = 16-row token tiles per workgroup tile (2 or 4)
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
   constexpr int kMoeRows = 16 * MT;
   scalar_cache_acquire();
@@ -269,8 +272,10 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
   const int n_base = GATED ? blockIdx.y * 64 + 16 * wid : blockIdx.y * 128 + 32 * wid;
   const uint16_t* wexp = p.w + (int64_t)e * p.w_expert_stride;
   const uint16_t* arow[2];
-  arow[0] = wexp + (int64_t)(n_base + r16) * p.K + 16 * kg;                                  // gate / rows 0-15
-  arow[1] = wexp + (int64_t)(GATED ? p.N_out + n_base + r16 : n_base + 16 + r16) * p.K + 16 * kg;  // up / rows 16-31
+  const int wr0 = GUARD ? min(n_base + r16, p.N_out - 1) : n_base + r16;
+  const int wr1 = GATED ? wr0 : GUARD ? min(n_base + 16 + r16, p.N_out - 1) : n_base + 16 + r16;
+  arow[0] = wexp + (int64_t)wr0 * p.K + 16 * kg;                                  // gate / rows 0-15
+  arow[1] = wexp + (int64_t)(GATED ? p.N_out + wr1 : wr1) * p.K + 16 * kg;        // up / rows 16-31
   f32x4_t acc[2][MT];
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -288,8 +293,9 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
       // elements 16 kg .. 16 kg + 7 for the even k-step and 16 kg + 8 .. + 15 for the odd one, so the four lanes of
       // a row cover one whole 128-byte line per instruction pair instead of two half lines
       const int k = k0 + 64 * (u >> 1);
-      const bool ok = k < p.K;   // K is a multiple of 64, not necessarily of 32 * UNR
-      const int kk = (ok ? k : 0) + 8 * (u & 1);
+      // K is a multiple of 64, not necessarily of 32 * UNR; GUARD: of 8, and the lane's own eight are in or out
+      const bool ok = GUARD ? k + 16 * kg + 8 * (u & 1) < p.K : k < p.K;
+      const int kk = GUARD ? (ok ? k + 8 * (u & 1) : -16 * kg) : (ok ? k : 0) + 8 * (u & 1);
 #pragma unroll
       for (int i = 0; i < 2; ++i) fa[buf][u][i] = *reinterpret_cast<const uint4*>(arow[i] + kk);
 #pragma unroll
@@ -332,16 +338,85 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
       uint2 q;
       q.x = E::pack(v[0], v[1]);
       q.y = E::pack(v[2], v[3]);
-      *reinterpret_cast<uint2*>(o + n_base + 4 * kg) = q;
+      if (!GUARD || n_base + 4 * kg < p.N_out) *reinterpret_cast<uint2*>(o + n_base + 4 * kg) = q;
     } else {
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
         uint2 q;
         q.x = E::pack(acc[i][mt][0], acc[i][mt][1]);
         q.y = E::pack(acc[i][mt][2], acc[i][mt][3]);
-        *reinterpret_cast<uint2*>(o + n_base + 16 * i + 4 * kg) = q;
+        if (!GUARD || n_base + 16 * i + 4 * kg < p.N_out) *reinterpret_cast<uint2*>(o + n_base + 16 * i + 4 * kg) = q;
       }
     }
+  }
+}
+
+// ---------------------------------------------------------------- any sizes and types
+// One workgroup per (pair, 16 outputs), a wave per four of them, pairs in their own order (no grouping): 32-bit models and
+// sizes the matrix-core kernels do not take.  GATED: out[pair] = silu(x[tok] Wg^T) * (x[tok] Wu^T), else out[pair] = a[pair] W^T.
+template <typename T, bool GATED>
+__global__ __launch_bounds__(256) void moe_pair_gemm_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ w,
+                                                            const int32_t* __restrict__ ids, int n_out, int K, int top_k, int E,
+                                                            int64_t a_stride, int64_t out_stride, int64_t w_stride) {
+  scalar_cache_acquire();
+  const int64_t pair = blockIdx.x;
+  const int lane = threadIdx.x & 63, n0 = blockIdx.y * 16 + (threadIdx.x >> 6) * 4;
+  const int e = ids[pair];
+  const bool known = e >= 0 && e < E;
+  const T* x = a + (GATED ? pair / top_k : pair) * a_stride;
+  const T* we = w + (known ? e : 0) * w_stride;
+  for (int n = n0; n < min(n0 + 4, n_out); ++n) {
+    float g = 0.f, u = 0.f;
+    for (int k = lane; k < K; k += 64) {
+      const float xv = Io<T>::ld(x + k);
+      g += xv * Io<T>::ld(we + (int64_t)n * K + k);
+      if constexpr (GATED) u += xv * Io<T>::ld(we + (int64_t)(n_out + n) * K + k);
+    }
+    g = wave_allreduce_sum(g);
+    if constexpr (GATED) g = silu_f(g) * wave_allreduce_sum(u);
+    if (lane == 0) Io<T>::st(out + pair * out_stride + n, known ? g : 0.f);
+  }
+}
+
+// ---------------------------------------------------------------- router
+// fp32 logits[t][e] = h[t] . w[e] + bias[e] of 16-bit rows.  A wave takes a quarter of K for 16 experts x 16 tokens, operands
+// straight from global memory; the four quarters meet in LDS.  Loads are unconditional on clamped addresses.
+__global__ __launch_bounds__(256) void moe_router_kernel(float* __restrict__ out, const uint16_t* __restrict__ h,
+                                                         const uint16_t* __restrict__ w, const float* __restrict__ bias, int rows, int E,
+                                                         int K, int64_t h_stride) {
+  scalar_cache_acquire();
+  __shared__ f32x4_t red[4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
+  const int t0 = blockIdx.x * 16, e0 = blockIdx.y * 16;
+  const int steps = (K + 31) / 32, per = (steps + 3) / 4;
+  const int s0 = wave * per, s1 = min(steps, s0 + per);
+  const uint16_t* wr = w + (int64_t)min(e0 + lr, E - 1) * K;
+  const uint16_t* hr = h + (int64_t)min(t0 + lr, rows - 1) * h_stride;
+  f32x4_t acc = {};
+  for (int s = s0; s < s1; s += 4) {
+    uint4 a[4], b[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int k = min(32 * (s + u) + 8 * lg, K - 8);      // K is a multiple of 8
+      a[u] = *reinterpret_cast<const uint4*>(wr + k);
+      b[u] = *reinterpret_cast<const uint4*>(hr + k);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (s + u >= s1 || 32 * (s + u) + 8 * lg >= K) a[u] = make_uint4(0, 0, 0, 0);
+      acc = mfma16<bf16_tag>(a[u], b[u], acc);
+    }
+  }
+  red[wave][lane] = acc;
+  __syncthreads();
+  if (wave) return;
+  acc = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]);
+  const int t = t0 + lr;
+  if (t >= rows) return;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int e = e0 + 4 * lg + i;
+    if (e < E) out[(int64_t)t * E + e] = acc[i] + (bias ? bias[e] : 0.f);
   }
 }
 
@@ -426,7 +501,7 @@ extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* exp
   using namespace mi;
   if (num_tokens == 0) return MI_OK;
   if (!topk_ids || !topk_weights || !router_logits || num_tokens < 0) return MI_ERR_INVALID_ARG;
-  if (num_experts != 64 && num_experts != 128 && num_experts != 256) return MI_ERR_UNSUPPORTED;
+  if (num_experts <= 0 || num_experts > 256) return MI_ERR_UNSUPPORTED;
   if (top_k <= 0 || top_k > 16 || top_k > num_experts) return MI_ERR_INVALID_ARG;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   // expert_counts == NULL: no counting (and no launch to zero the counters) — mi_moe_align counts the ids itself.
@@ -437,12 +512,12 @@ extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* exp
   const int tpw = num_tokens >= 8192 ? 4 : num_tokens >= 1024 ? 2 : 1;
   const dim3 grid((num_tokens + 16 * tpw - 1) / (16 * tpw)), block(1024);
 #define MI_ROUTE(DT, EPL)                                                                                        \
-  hipLaunchKernelGGL((moe_route_kernel<DT, EPL>), grid, block, 0, s, router_logits, logits_row_stride, topk_ids, \
+  hipLaunchKernelGGL((moe_route_kernel<DT, EPL>), grid, block, 0, s, router_logits, logits_row_stride, num_experts, topk_ids, \
                      topk_weights, expert_counts, num_tokens, top_k, norm_topk_prob, weight_round_dtype)
 #define MI_ROUTE_E(DT)                                  \
   do {                                                  \
-    if (num_experts == 64) MI_ROUTE(DT, 1);             \
-    else if (num_experts == 128) MI_ROUTE(DT, 2);       \
+    if (num_experts <= 64) MI_ROUTE(DT, 1);             \
+    else if (num_experts <= 128) MI_ROUTE(DT, 2);       \
     else MI_ROUTE(DT, 4);                               \
   } while (0)
   switch (logits_dtype) {
@@ -483,12 +558,14 @@ extern "C" int mi_moe_expert_gemm(void* out, const void* a_rows, const void* wei
   if (max_tiles == 0) return MI_OK;
   if (!out || !a_rows || !weights || !sorted_pairs || !tile_expert || !num_tiles || max_tiles < 0)
     return MI_ERR_INVALID_ARG;
-  if (k <= 0 || k % 64 || n_out <= 0 || n_out % (gated ? 64 : 128)) return MI_ERR_UNSUPPORTED;
+  if (k <= 0 || k % 8 || n_out <= 0 || n_out % 4) return MI_ERR_UNSUPPORTED;
+  const bool guard = k % 64 || n_out % (gated ? 64 : 128);      // outside the tiles of the ring kernel
+  if (guard && (dtype != MI_DTYPE_BF16 || rows_per_tile > 64)) return MI_ERR_UNSUPPORTED;
   if (!moe_rows_per_tile_ok(rows_per_tile)) return MI_ERR_INVALID_ARG;
   if (a_row_stride % 8 || out_row_stride % 4 || weight_expert_stride % 8) return MI_ERR_INVALID_ARG;
   if (((uintptr_t)a_rows | (uintptr_t)weights) & 15 || ((uintptr_t)out & 7)) return MI_ERR_INVALID_ARG;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  {
+  if (!guard) {
     // default: the decode-batch linear kernel's grouped form (skinny_gemm.hip: row-contiguous LDS-DMA weight images,
     // `ds_read_b128` fragments, loader / consumer waves); MI_MOE_GEMM=direct keeps the fragments-from-global kernel
     // below (A/B runs, and shapes outside the ring kernel's envelope)
@@ -519,7 +596,16 @@ extern "C" int mi_moe_expert_gemm(void* out, const void* a_rows, const void* wei
   p.a_stride = a_row_stride;
   p.out_stride = out_row_stride;
   p.w_expert_stride = weight_expert_stride;
-  const dim3 grid((max_tiles + 7) / 8 * 8, gated ? n_out / 64 : n_out / 128), block(256);
+  const dim3 grid((max_tiles + 7) / 8 * 8, gated ? (n_out + 63) / 64 : (n_out + 127) / 128), block(256);
+  if (guard) {
+#define MI_MOE_GUARD(G, M) hipLaunchKernelGGL((moe_gemm_kernel<bf16_tag, G, M, true>), grid, block, 0, s, p)
+    if (gated && rows_per_tile == 32) MI_MOE_GUARD(true, 2);
+    else if (gated) MI_MOE_GUARD(true, 4);
+    else if (rows_per_tile == 32) MI_MOE_GUARD(false, 2);
+    else MI_MOE_GUARD(false, 4);
+#undef MI_MOE_GUARD
+    return launch_status();
+  }
 #define MI_MOE_GEMM(TAG, G, M) hipLaunchKernelGGL((moe_gemm_kernel<TAG, G, M>), grid, block, 0, s, p)
 #define MI_MOE_GEMM_T(TAG)                                \
   do {                                                    \
@@ -559,5 +645,40 @@ extern "C" int mi_moe_combine(void* out, const void* partial, const int32_t* row
     hipLaunchKernelGGL((moe_combine_kernel<f16_tag>), dim3(num_tokens), dim3(256), 0, s, o, pp, row_of_pair, topk_weights, sh, xx, gw, hidden, top_k, partial_row_stride, out_row_stride, x_row_stride, shared_row_stride);
   else
     return MI_ERR_UNSUPPORTED;
+  return launch_status();
+}
+
+extern "C" int mi_moe_router_logits(float* out, const void* h, const void* weight, const float* bias, int32_t rows,
+                                    int32_t num_experts, int32_t k, int64_t h_stride, void* stream) {
+  using namespace mi;
+  if (rows == 0) return MI_OK;
+  if (!out || !h || !weight || rows < 0 || num_experts <= 0 || k <= 0 || h_stride < k) return MI_ERR_INVALID_ARG;
+  if (k % 8 || h_stride % 8 || !aligned16(h) || !aligned16(weight)) return MI_ERR_UNSUPPORTED;
+  hipLaunchKernelGGL(moe_router_kernel, dim3((rows + 15) / 16, (num_experts + 15) / 16), dim3(256), 0, reinterpret_cast<hipStream_t>(stream),
+                     out, (const uint16_t*)h, (const uint16_t*)weight, bias, rows, num_experts, k, h_stride);
+  return launch_status();
+}
+
+extern "C" int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const int32_t* topk_ids, int32_t num_pairs,
+                                int32_t num_experts, int32_t gated, int32_t n_out, int32_t k, int32_t top_k, int64_t a_row_stride,
+                                int64_t out_row_stride, int64_t weight_expert_stride, int dtype, void* stream) {
+  using namespace mi;
+  if (num_pairs == 0) return MI_OK;
+  if (!out || !a_rows || !weights || !topk_ids || num_pairs < 0 || num_experts <= 0 || n_out <= 0 || k <= 0 || top_k <= 0 ||
+      a_row_stride < k || out_row_stride < n_out || weight_expert_stride < (int64_t)(gated ? 2 : 1) * n_out * k)
+    return MI_ERR_INVALID_ARG;
+  const dim3 grid(num_pairs, (n_out + 15) / 16), block(256);
+  hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+#define MI_PAIR(T)                                                                                                                  \
+  do {                                                                                                                              \
+    if (gated) hipLaunchKernelGGL((moe_pair_gemm_kernel<T, true>), grid, block, 0, s, (T*)out, (const T*)a_rows, (const T*)weights, \
+                                  topk_ids, n_out, k, top_k, num_experts, a_row_stride, out_row_stride, weight_expert_stride);      \
+    else hipLaunchKernelGGL((moe_pair_gemm_kernel<T, false>), grid, block, 0, s, (T*)out, (const T*)a_rows, (const T*)weights,      \
+                            topk_ids, n_out, k, top_k, num_experts, a_row_stride, out_row_stride, weight_expert_stride);            \
+  } while (0)
+  if (dtype == MI_DTYPE_BF16) MI_PAIR(uint16_t);
+  else if (dtype == MI_DTYPE_F32) MI_PAIR(float);
+  else return MI_ERR_UNSUPPORTED;
+#undef MI_PAIR
   return launch_status();
 }

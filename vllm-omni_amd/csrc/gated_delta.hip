@@ -3,8 +3,9 @@
 // Per v-head h (its q/k head is h / (heads / kv_heads)) and token:
 //   q, k, v   = silu(causal conv over time of the projections);  q, k made unit vectors, q times dim^-1/2
 //   M_t = g M_(t-1) + k (x) e   with  e = b (v - g k M_(t-1)),   y = q M_t        ln g = -exp(A_log) softplus(a + dt_bias)
-//   out       = y / rms(y) * norm * silu(gate)
-// The projections of a row arrive as one row [q | k | v | gate | b | a].  Per request slot the state is M [dim][vdim]
+//   out       = y / rms(y) * norm * silu(gate), or sigmoid(gate)
+// g is one number per head, or one per head and key channel (a diagonal in front of the rows of M).  A row's q, k, v
+// projections arrive side by side, gate, b and a wherever the caller has them.  Per request slot the state is M [dim][vdim]
 // fp32 per head and a ring of the last `taps` projection rows (row p % taps holds position p); a request whose first
 // token is position 0 starts from zeros whatever the slot holds, so slots need no clearing.
 //
@@ -12,6 +13,8 @@
 //   * gated_delta_step: one workgroup per (head, request), the state in registers, tokens one after the other: decode
 //     (HBM bound: the state is read and written once), and any shape the chunked pair does not build.
 //   * conv_ring_update: leaves a multi-token portion's last rows in the ring (after every reader of the old rows).
+#include <type_traits>
+
 #include "gated_delta.h"
 
 namespace mi {
@@ -19,11 +22,11 @@ namespace {
 
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
-// LDS: q[D] k[D] v[V] red[2][groups * V].  R: rows of the state a thread holds; TAPS: convolution taps, 0 = any (one load
+// LDS: q[D] k[D] v[V] red[2][groups * V] decay[D].  R: rows of the state a thread holds; TAPS: convolution taps, 0 = any (one load
 // after the other); FULL: the threads' tiles cover the state exactly.  A decode step is one chain of memory latencies per
 // workgroup, so everything a token needs is asked for before the first use, the state with it; loads are unconditional on
 // clamped addresses and their values selected afterwards (a load behind a branch is waited for on its own).
-template <typename T, int VEC, int NT, int R, int TAPS, bool FULL>
+template <typename T, int VEC, int NT, int R, int TAPS, bool FULL, bool CHN>
 __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(const DeltaParams p) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -39,6 +42,7 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
   const int lv = V / VEC, groups = NT / lv;
   float* red0 = sv + V;
   float* red1 = red0 + groups * V;
+  float* sdec = red1 + groups * V;       // CHN: decays of the key channels
   const int tid = threadIdx.x, g = tid / lv, c = (tid % lv) * VEC;
   const bool on = FULL || g < groups;
   float* S = p.state + ((slot * H + h) * D) * (int64_t)V;
@@ -57,19 +61,21 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
       st[i][0] = S[(int64_t)d * V + c];
     }
   }
-  const float neg_a = -expf(p.a_log[h]), dtb = p.dt_bias[h];
+  const float neg_a = -expf(p.a_log[h]), dtb = CHN ? 0.f : p.dt_bias[h];
   const float qs = 1.0f / sqrtf((float)D);
   const int nch = 2 * D + V;
   for (int i = 0; i < L; ++i) {
     const int64_t row = s0 + i;
     const int pos = start + i;
     const T* pr = proj + row * p.ld;
-    const float raw_a = Io<T>::ld(pr + p.off_a + h), raw_b = Io<T>::ld(pr + p.off_b + h);
+    const T* ar = reinterpret_cast<const T*>(p.a) + row * p.ld_a + (int64_t)h * (CHN ? D : 1);
+    const float raw_a = Io<T>::ld(ar + (CHN ? min(tid, D - 1) : 0));
+    const float raw_b = Io<T>::ld(reinterpret_cast<const T*>(p.b) + row * p.ld_b + h);
     float gt[4], nw[4];                          // what the first wave ends the token with: gate and norm weights (vdim <= 256)
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int v = min((tid & 63) + 64 * j, V - 1);
-      gt[j] = Io<T>::ld(pr + p.off_g + h * V + v);
+      gt[j] = Io<T>::ld(reinterpret_cast<const T*>(p.gate) + row * p.ld_gate + h * V + v);
       nw[j] = Io<T>::ld(reinterpret_cast<const T*>(p.norm_w) + v);
     }
     for (int n0 = 0; n0 < nch; n0 += NT) {
@@ -100,6 +106,10 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
       // one token: its row of the ring is nobody's to read this step (readers take the taps - 1 rows before it)
       if (L == 1 && pos >= 0 && n0 + tid < nch && (n >= 2 * D || h % per == 0)) ring[(int64_t)(pos % p.taps) * p.CH + ch] = cur;
     }
+    if constexpr (CHN) {
+      for (int d = tid; d < D; d += NT)
+        sdec[d] = expf(neg_a * softplus_f((d < NT ? raw_a : Io<T>::ld(ar + d)) + p.dt_bias[h * D + d]));
+    }
     if (i == 0) {
 #pragma unroll
       for (int n = 0; n < R; ++n)
@@ -110,14 +120,15 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
     float qq = 0.f, kk = 0.f;
     for (int d = tid & 63; d < D; d += 64) qq += sq[d] * sq[d], kk += sk[d] * sk[d];
     const float qn = qs / sqrtf(wave_allreduce_sum(qq) + 1e-6f), kn = 1.0f / sqrtf(wave_allreduce_sum(kk) + 1e-6f);
-    const float decay = expf(neg_a * softplus_f(raw_a + dtb));
+    const float decay = CHN ? 1.f : expf(neg_a * softplus_f(raw_a + dtb));
     const float beta = sigmoid_f(raw_b);
     float acc[VEC] = {};
 #pragma unroll
     for (int n = 0; n < R; ++n) {
       const float k = has(n) ? sk[g + n * groups] * kn : 0.f;
+      const float f = CHN ? (has(n) ? sdec[g + n * groups] : 0.f) : decay;
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) st[n][j] *= decay, acc[j] += st[n][j] * k;
+      for (int j = 0; j < VEC; ++j) st[n][j] *= f, acc[j] += st[n][j] * k;
     }
     if (on)
 #pragma unroll
@@ -151,10 +162,10 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
         ss += t * t;
       }
       const float inv = inv_rms(wave_allreduce_sum(ss), V, p.eps);
-      T* o = reinterpret_cast<T*>(p.out) + row * (int64_t)H * V + (int64_t)h * V;
+      T* o = reinterpret_cast<T*>(p.out) + row * p.ld_out + (int64_t)h * V;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        if (tid + 64 * j < V) Io<T>::st(o + tid + 64 * j, red1[tid + 64 * j] * inv * nw[j] * silu_f(gt[j]));
+        if (tid + 64 * j < V) Io<T>::st(o + tid + 64 * j, red1[tid + 64 * j] * inv * nw[j] * out_gate(p, gt[j]));
     }
   }
 #pragma unroll
@@ -173,11 +184,15 @@ __global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void gated_delta_step_kernel(co
 template <typename T, int VEC, int NT, int R>
 int launch_step(const DeltaParams& p, int nreq, hipStream_t s) {
   const int groups = NT / (p.V / VEC);
-  const size_t lds = (size_t)(2 * p.D + p.V + 2 * groups * p.V) * sizeof(float);
+  const size_t lds = (size_t)(2 * p.D + p.V + 2 * groups * p.V + (p.channel ? p.D : 0)) * sizeof(float);
   const bool full = VEC == 4 && NT % (p.V / VEC) == 0 && p.D == R * groups;
-  auto kern = p.taps != 4 ? gated_delta_step_kernel<T, VEC, NT, R, 0, false>
-              : full      ? gated_delta_step_kernel<T, VEC, NT, R, 4, true>
-                          : gated_delta_step_kernel<T, VEC, NT, R, 4, false>;
+  auto pick = [&](auto chn) {
+    constexpr bool C = decltype(chn)::value;
+    return p.taps != 4 ? gated_delta_step_kernel<T, VEC, NT, R, 0, false, C>
+           : full      ? gated_delta_step_kernel<T, VEC, NT, R, 4, true, C>
+                       : gated_delta_step_kernel<T, VEC, NT, R, 4, false, C>;
+  };
+  auto kern = p.channel ? pick(std::true_type{}) : pick(std::false_type{});
   if (lds > 65536) {
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
       return MI_ERR_LAUNCH;
@@ -209,30 +224,12 @@ int step_dispatch(const DeltaParams& p, int nreq, hipStream_t s) {
 
 using namespace mi;
 
-static int delta_fill(DeltaParams& p, const void* proj, int64_t ld, const void* convw, const float* a_log, const float* dt_bias,
-                      const void* norm_w, float* state, void* ring, const int32_t* slots, const int32_t* qsl,
-                      const int32_t* seq_lens, void* out, int32_t req0, int32_t nreq, int32_t H, int32_t K, int32_t D, int32_t V,
-                      int32_t taps, float eps) {
-  if (!proj || !convw || !a_log || !dt_bias || !norm_w || !state || !ring || !slots || !qsl || !seq_lens || !out)
-    return MI_ERR_INVALID_ARG;
-  if (req0 < 0 || nreq < 0 || H <= 0 || K <= 0 || D <= 0 || V <= 0 || taps <= 0 || H % K) return MI_ERR_INVALID_ARG;
-  const int CH = 2 * K * D + H * V;
-  if (ld < CH + H * V + 2 * H) return MI_ERR_INVALID_ARG;
-  p = DeltaParams{proj, convw, norm_w, ring, out, a_log, dt_bias, state, slots, qsl, seq_lens, ld, req0, H, K, D, V, taps, CH,
-                  CH, CH + H * V, CH + H * V + H, eps};
-  return MI_OK;
-}
-
-extern "C" int mi_gated_delta_step(const void* proj, int64_t proj_stride, const void* conv_w, const float* a_log,
-                                   const float* dt_bias, const void* norm_w, float* state, void* ring, const int32_t* slots,
-                                   const int32_t* query_start_loc, const int32_t* seq_lens, void* out, int32_t req0,
-                                   int32_t num_reqs, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps,
-                                   float eps, int32_t update_ring, int dtype, void* stream) {
-  if (num_reqs == 0) return MI_OK;
+extern "C" int mi_gated_delta_step(const mi_gated_delta_args* args, int32_t update_ring, int dtype, void* stream) {
+  if (args && args->num_reqs == 0) return MI_OK;
   DeltaParams p;
-  const int rc = delta_fill(p, proj, proj_stride, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
-                            out, req0, num_reqs, heads, kv_heads, dim, vdim, taps, eps);
+  const int rc = delta_fill(p, args);
   if (rc != MI_OK) return rc;
+  const int num_reqs = args->num_reqs;
   hipStream_t s = (hipStream_t)stream;
   int st;
   if (dtype == MI_DTYPE_BF16) st = step_dispatch<uint16_t>(p, num_reqs, s);

@@ -8,48 +8,19 @@
 //   * prep (one workgroup per chunk and head): convolutions, silu, unit q / k, gates; A, its unit-triangular inverse T,
 //     P, and T diag(b) V, T diag(b e^G) K, diag(e^G) Q, (e^(G_C - G_j) k_j)^T to a workspace;
 //   * scan (one workgroup per request, head and 16 value columns): chunk after chunk, U, O and S with S in registers;
-//   * finish: o / rms(o) * norm * silu(gate).
+//   * finish: o / rms(o) * norm * gate.
+// With one decay per key channel G_i is a vector: e^(G_i) and e^(G_C - G_i) scale the columns of K and Q, and A and P take
+// sum_d k_id e^(G_id - G_jd) k_jd, whose exponential is split at a row between j and i so that no factor exceeds one.
 // All products run on v_mfma_f32_16x16x4_f32: q, k, decays and state are 32-bit quantities of the recurrence.  The k order
 // inside 16 consecutive k is permuted alike in both operands (step s takes k = 4 (lane / 16) + s), so an operand whose k is
 // contiguous is one 16-byte read for four steps, and an accumulator tile IS the B operand of a following product.
+#include "chunk_scan.h"
 #include "gated_delta.h"
-#include "mfma_attn_common.h"
 
 namespace mi {
 namespace {
 
-constexpr int kC = 64;             // tokens per chunk
 constexpr int kPrepThreads = 512;
-
-__device__ __forceinline__ f32x4_t mma4(const float (&a)[4], const float (&b)[4], f32x4_t c) {
-#pragma unroll
-  for (int s = 0; s < 4; ++s) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[s], b[s], c, 0, 0, 0);
-  return c;
-}
-__device__ __forceinline__ void frag_rows(const float* p, int ld, int lane, float (&f)[4]) {   // [row][k], k contiguous
-  const float4 v = *reinterpret_cast<const float4*>(p + (lane & 15) * ld + 4 * (lane >> 4));
-  f[0] = v.x, f[1] = v.y, f[2] = v.z, f[3] = v.w;
-}
-__device__ __forceinline__ void frag_cols(const float* p, int ld, int lane, float (&f)[4]) {   // [k][col]
-#pragma unroll
-  for (int s = 0; s < 4; ++s) f[s] = p[(4 * (lane >> 4) + s) * ld + (lane & 15)];
-}
-
-// workspace of one (chunk, head): W [C][Dp], Q [C][Dp], Kt [Dp][C], P [C][C], U [C][Vp], then e^(G_C)
-struct ChunkLayout {
-  int Dp, Vp;
-  __host__ __device__ int64_t w() const { return 0; }
-  __host__ __device__ int64_t q() const { return (int64_t)kC * Dp; }
-  __host__ __device__ int64_t kt() const { return 2 * (int64_t)kC * Dp; }
-  __host__ __device__ int64_t pm() const { return 3 * (int64_t)kC * Dp; }
-  __host__ __device__ int64_t u() const { return 3 * (int64_t)kC * Dp + kC * kC; }
-  __host__ __device__ int64_t g() const { return u() + (int64_t)kC * Vp; }
-  __host__ __device__ int64_t size() const { return g() + 16; }
-};
-
-__device__ __forceinline__ int64_t chunk_base(const DeltaParams& p, int r) {
-  return (p.qsl[r] - p.qsl[p.req0]) / kC + (r - p.req0);
-}
 
 // conv + silu of channels [ch0, ch0 + n) of the chunk's rows into buf [C][ld]; zeros in rows past len and columns past n
 template <typename T>
@@ -167,8 +138,70 @@ __device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul)
   }
 }
 
-template <typename T>
-__global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, bool vec) {
+// A and P of one 16 x 16 tile (rows ti, columns tj < ti) with a decay per key channel.  e^(G_i - G_j) is split at the tile's
+// first row r: e^(G_i - G_r) on the row's side, e^(G_r - G_j) on the column's; both exponents are <= 0 (G falls with time).
+// gk, gq, gG: [C][ld] keys, queries, G in log2.
+__device__ __forceinline__ void channel_tile(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti, int tj, int lane,
+                                             f32x4_t& aA, f32x4_t& aP) {
+  for (int k = 0; k < Dp; k += 16) {
+    float kf[4], qf[4], gf[4], cf[4], hf[4], rf[4];
+    frag_rows(kb + ti * 16 * ld + k, ld, lane, kf);
+    frag_rows(qb + ti * 16 * ld + k, ld, lane, qf);
+    frag_rows(gb + ti * 16 * ld + k, ld, lane, gf);
+    frag_rows(kb + tj * 16 * ld + k, ld, lane, cf);
+    frag_rows(gb + tj * 16 * ld + k, ld, lane, hf);
+    frag_rows(gb + ti * 16 * ld + k, 0, lane, rf);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const float e = fast_exp2(gf[s] - rf[s]);
+      kf[s] *= e, qf[s] *= e;
+      cf[s] *= fast_exp2(rf[s] - hf[s]);
+    }
+    aA = mma4(kf, cf, aA);
+    aP = mma4(qf, cf, aP);
+  }
+}
+
+// the same on the diagonal (ti == tj), in four levels of halving: pairs (i, j) whose highest differing bit is `half` are split
+// at the first row of the upper half of their block of 2 half rows.  A lane's token is in a row's role (upper half) or a
+// column's (lower half) on each level, so one exponential per level serves both.  dg: q_i . k_i of the lane's token.
+__device__ __forceinline__ void channel_diag(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti, int lane,
+                                             f32x4_t (&aA)[4], f32x4_t (&aP)[4], float& dg) {
+  const int t = lane & 15;
+  const float* g0 = gb + ti * 16 * ld;
+  dg = 0.f;
+  for (int k = 0; k < Dp; k += 16) {
+    float kf[4], qf[4], gf[4];
+    frag_rows(kb + ti * 16 * ld + k, ld, lane, kf);
+    frag_rows(qb + ti * 16 * ld + k, ld, lane, qf);
+    frag_rows(g0 + k, ld, lane, gf);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) dg += qf[s] * kf[s];
+#pragma unroll
+    for (int lv = 0; lv < 4; ++lv) {
+      const int half = 1 << lv, ref = (t & ~(2 * half - 1)) + half;
+      const bool up = t & half;
+      const float4 rv = *reinterpret_cast<const float4*>(g0 + ref * ld + k + 4 * (lane >> 4));
+      const float rf[4] = {rv.x, rv.y, rv.z, rv.w};
+      float rk[4], rq[4], ck[4];
+#pragma unroll
+      for (int s = 0; s < 4; ++s) {
+        const float d = gf[s] - rf[s], e = fast_exp2(up ? d : -d);
+        rk[s] = up ? kf[s] * e : 0.f;
+        rq[s] = up ? qf[s] * e : 0.f;
+        ck[s] = up ? 0.f : kf[s] * e;
+      }
+      aA[lv] = mma4(rk, ck, aA[lv]);
+      aP[lv] = mma4(rq, ck, aP[lv]);
+    }
+  }
+  dg += __shfl_xor(dg, 16, 64);
+  dg += __shfl_xor(dg, 32, 64);
+}
+
+// CHN: one decay per head and key channel
+template <typename T, bool CHN>
+__global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, bool vec) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = p.req0 + blockIdx.z, h = blockIdx.y, ck = blockIdx.x;
@@ -189,18 +222,18 @@ __global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const
   float* sE = sB + kC;                     // b_i e^(G_i)
   float* sQ = sE + kC;                     // e^(G_i)
   float* sD = sQ + kC;                     // e^(G_C - G_i)
+  float* bufG = sD + kC;                   // CHN: G_i per channel, in log2
   float* out = ws + ((chunk_base(p, r) + ck) * p.H + h) * lay.size();
   const T* ring = reinterpret_cast<const T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int kh = h / (p.H / p.K);
   conv_tile<T>(p, vec, bufA, ldk, Dp, p.K * p.D + kh * p.D, p.D, row0, i0, len, start, ring);
   conv_tile<T>(p, vec, bufB, ldk, Dp, kh * p.D, p.D, row0, i0, len, start, ring);
-  if (wave == 0) {   // gates: cumulative log decay over the 64 tokens of the chunk
-    const T* pr = reinterpret_cast<const T*>(p.proj) + (row0 + lane) * p.ld;
+  if (!CHN && wave == 0) {   // gates: cumulative log decay over the 64 tokens of the chunk
     float lg = 0.f, b = 0.f;
     if (lane < len) {
-      lg = -expf(p.a_log[h]) * softplus_f(Io<T>::ld(pr + p.off_a + h) + p.dt_bias[h]);
-      b = sigmoid_f(Io<T>::ld(pr + p.off_b + h));
+      lg = -expf(p.a_log[h]) * softplus_f(Io<T>::ld(reinterpret_cast<const T*>(p.a) + (row0 + lane) * p.ld_a + h) + p.dt_bias[h]);
+      b = sigmoid_f(Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + lane) * p.ld_b + h));
     }
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -213,16 +246,71 @@ __global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const
     sE[lane] = b * e;
     sQ[lane] = e;
     sD[lane] = expf(__shfl(lg, 63, 64) - lg);
-    if (lane == 63) out[lay.g()] = e;
+    const float last = __shfl(e, 63, 64);
+    for (int d = lane; d < Dp; d += 64) out[lay.g() + d] = last;
+  }
+  if constexpr (CHN) {
+    const float neg_a = -expf(p.a_log[h]) * kLog2e;
+    const T* ar = reinterpret_cast<const T*>(p.a) + row0 * p.ld_a + (int64_t)h * p.D;
+    for (int n = tid; n < kC * Dp; n += kPrepThreads) {
+      const int i = n / Dp, c = n % Dp;
+      const bool in = i < len && c < p.D;
+      const float v = Io<T>::ld(ar + (int64_t)min(i, len - 1) * p.ld_a + min(c, p.D - 1)) + p.dt_bias[h * p.D + min(c, p.D - 1)];
+      bufG[i * ldk + c] = in ? neg_a * softplus_f(v) : 0.f;
+    }
+    if (wave == 0) sB[lane] = lane < len ? sigmoid_f(Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + min(lane, len - 1)) * p.ld_b + h)) : 0.f;
+    __syncthreads();
+    // running sums over the chunk, a segment of rows a thread, then what the segments in front add up to
+    const int segs = kPrepThreads / Dp, c = tid % Dp, sg = tid / Dp, per = kC / segs;
+    float acc = 0.f;
+    for (int i = sg * per; i < (sg + 1) * per; ++i) acc += bufG[i * ldk + c], bufG[i * ldk + c] = acc;
+    __syncthreads();
+    float before = 0.f;
+    for (int n = 0; n < sg; ++n) before += bufG[(n * per + per - 1) * ldk + c];
+    __syncthreads();
+    for (int i = sg * per; i < (sg + 1) * per; ++i) bufG[i * ldk + c] += before;
+    if (sg == segs - 1) out[lay.g() + c] = fast_exp2(acc + before);
   }
   __syncthreads();
   unit_rows(bufA, ldk, Dp, 1.0f);
   unit_rows(bufB, ldk, Dp, 1.0f / sqrtf((float)p.D));
   __syncthreads();
   // A and P, 16 tiles each, lower ones only: P goes out, A waits in registers until Q is dead
-  f32x4_t keep[2];
+  f32x4_t keep[2] = {};
+  if constexpr (CHN) {
+    auto store = [&](int ti, int tj, int s, float a, float pv, f32x4_t& kp) {
+      const int i = ti * 16 + 4 * (lane >> 4) + s, j = tj * 16 + (lane & 15);
+      out[lay.pm() + i * kC + j] = pv;
+      kp[s] = a * sB[i];
+    };
+    if (wave < 4) {          // a diagonal tile each, as much work as two others
+      f32x4_t aA[4] = {}, aP[4] = {};
+      float dg;
+      channel_diag(bufA, bufB, bufG, ldk, Dp, wave, lane, aA, aP, dg);
 #pragma unroll
-  for (int n = 0; n < 4; ++n) {
+      for (int s = 0; s < 4; ++s) {
+        const int i = 4 * (lane >> 4) + s, j = lane & 15, x = i ^ j;
+        const float a = x >= 8 ? aA[3][s] : x >= 4 ? aA[2][s] : x >= 2 ? aA[1][s] : aA[0][s];
+        const float q = x >= 8 ? aP[3][s] : x >= 4 ? aP[2][s] : x >= 2 ? aP[1][s] : aP[0][s];
+        store(wave, wave, s, i > j ? a : 0.f, i > j ? q : i == j ? dg : 0.f, keep[0]);
+      }
+    } else {
+#pragma unroll
+      for (int n = 0; n < 2; ++n) {
+        const int t = wave - 4 + 4 * n, ti = t < 1 ? 1 : t < 3 ? 2 : 3, tj = t - ti * (ti - 1) / 2;
+        if (t >= 6) continue;
+        f32x4_t aA = {}, aP = {};
+        channel_tile(bufA, bufB, bufG, ldk, Dp, ti, tj, lane, aA, aP);
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          store(ti, tj, s, aA[s], aP[s], keep[n]);
+          out[lay.pm() + (tj * 16 + 4 * (lane >> 4) + s) * kC + ti * 16 + (lane & 15)] = 0.f;   // its mirror: whole rows of P are multiplied
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int n = 0; n < (CHN ? 0 : 4); ++n) {
     const int t = wave + n * (kPrepThreads / 64);
     const bool isP = n >= 2;
     const int ti = (t & 15) >> 2, tj = t & 3;
@@ -254,17 +342,37 @@ __global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const
   // diag(e^G) Q and the transposed, decayed keys
   for (int n = tid; n < kC * Dp / 4; n += kPrepThreads) {
     const int i = n / (Dp / 4), c = (n % (Dp / 4)) * 4;
-    const float e = sQ[i];
-    const float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
-    *reinterpret_cast<float4*>(out + lay.q() + (int64_t)i * Dp + c) = make_float4(v.x * e, v.y * e, v.z * e, v.w * e);
+    float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
+    if constexpr (CHN) {
+      const float4 g = *reinterpret_cast<const float4*>(bufG + i * ldk + c);
+      v = make_float4(v.x * fast_exp2(g.x), v.y * fast_exp2(g.y), v.z * fast_exp2(g.z), v.w * fast_exp2(g.w));
+    } else {
+      const float e = sQ[i];
+      v = make_float4(v.x * e, v.y * e, v.z * e, v.w * e);
+    }
+    *reinterpret_cast<float4*>(out + lay.q() + (int64_t)i * Dp + c) = v;
   }
   for (int n = tid; n < kC * Dp; n += kPrepThreads) {
     const int d = n / kC, j = n % kC;
-    out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * sD[j] : 0.f;
+    const float e = CHN ? fast_exp2(bufG[(kC - 1) * ldk + d] - bufG[j * ldk + d]) : sD[j];
+    out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * e : 0.f;
   }
   __syncthreads();   // Q is dead: A and T take its place
+  if constexpr (CHN) {   // and nobody needs the plain keys again
+    for (int n = tid; n < kC * Dp; n += kPrepThreads) {
+      const int i = n / Dp, c = n % Dp;
+      bufA[i * ldk + c] *= fast_exp2(bufG[i * ldk + c]);
+    }
 #pragma unroll
-  for (int n = 0; n < 2; ++n) {
+    for (int n = 0; n < 2; ++n) {
+      const int t = wave - 4 + 4 * n, ti = wave < 4 ? wave : t < 1 ? 1 : t < 3 ? 2 : 3, tj = wave < 4 ? wave : t - ti * (ti - 1) / 2;
+      if (wave < 4 ? n > 0 : t >= 6) continue;
+#pragma unroll
+      for (int s = 0; s < 4; ++s) mA[(ti * 16 + 4 * (lane >> 4) + s) * ldm + tj * 16 + (lane & 15)] = keep[n][s];
+    }
+  }
+#pragma unroll
+  for (int n = 0; n < (CHN ? 0 : 2); ++n) {
     const int t = wave + n * (kPrepThreads / 64);
 #pragma unroll
     for (int s = 0; s < 4; ++s) mA[((t >> 2) * 16 + 4 * (lane >> 4) + s) * ldm + (t & 3) * 16 + (lane & 15)] = keep[n][s];
@@ -321,155 +429,11 @@ __global__ __launch_bounds__(kPrepThreads, 4) void gated_delta_prep_kernel(const
       for (int s = 0; s < 4; ++s) dst[(int64_t)(ti * 16 + 4 * (lane >> 4) + s) * np + tn * 16 + (lane & 15)] = acc[s];
     }
   };
-  times(sE, ldk, Dp, out + lay.w());
+  times(CHN ? sB : sE, ldk, Dp, out + lay.w());
   __syncthreads();
   conv_tile<T>(p, vec, bufA, ldv, Vp, 2 * p.K * p.D + h * p.V, p.V, row0, i0, len, start, ring);
   __syncthreads();
   times(sB, ldv, Vp, out + lay.u());
-}
-
-// LDS-only barrier: register loads in flight stay in flight
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-
-// NV 16-column value tiles a workgroup: its four waves read every operand of a chunk once for all of them (the bound is the
-// L2 traffic of those operands, each head's tiles reading the same ones)
-template <int DT, int NV>
-__global__ __launch_bounds__(256, 1) void gated_delta_scan_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, int nvg) {
-  scalar_cache_acquire();
-  constexpr int Dp = DT * 16, LS = Dp + 4, LU = kC + 4, MT = (DT + 3) / 4;
-  constexpr bool whole = DT % 4 == 0;      // every wave owns MT tiles of the state
-  __shared__ __attribute__((aligned(16))) float sS[NV * 16 * LS];
-  __shared__ __attribute__((aligned(16))) float sU[NV * 16 * LU];
-  // the workgroups of a head on one XCD (workgroups go to the 8 XCDs in turn)
-  const int bid = blockIdx.x;
-  const int h = (bid / (8 * nvg)) * 8 + bid % 8, vg = (bid / 8) % nvg;
-  const int r = p.req0 + blockIdx.y;
-  const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
-  if (h >= p.H || L <= 0) return;
-  const int start = p.seq_lens[r] - L;
-  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lg = lane >> 4;
-  const int v0 = vg * 16 * NV + lr;        // + 16 n: this lane's value columns
-  float* S = p.state + (((int64_t)p.slots[r] * p.H + h) * p.D) * p.V;
-  f32x4_t st[NV][MT];
-#pragma unroll
-  for (int n = 0; n < NV; ++n)
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      const int mt = wave + 4 * m, v = v0 + 16 * n;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = mt * 16 + 4 * lg + i;
-        st[n][m][i] = start > 0 && d < p.D && v < p.V ? S[(int64_t)d * p.V + v] : 0.f;
-      }
-      if (mt < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + mt * 16 + 4 * lg) = st[n][m];
-    }
-  const int nck = (L + kC - 1) / kC;
-  float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
-  const int64_t step = p.H * lay.size();
-  // one chunk's operands; the next chunk's are loaded a whole chunk ahead (the chain of chunks is the critical path, its
-  // loads must not be).  Loads and stores are unconditional — past the last chunk the loads fetch what nobody uses, read-outs
-  // replace U in the workspace — so that the number in flight is known at every wait: memory operations retire in order, and a
-  // store that may or may not be there makes the wait for the loads behind it wait for its acknowledgement as well.
-  struct Chunk {
-    f32x4_t w[DT], q[DT], pm[4], kt[MT][4], u[NV];
-    float g;
-  };
-  auto load = [&](Chunk& x, int c) {
-    const float* b = base + c * step;
-    const int64_t ro = (int64_t)(16 * wave + lr) * Dp + 4 * lg;
-#pragma unroll
-    for (int k = 0; k < DT; ++k) {
-      x.w[k] = *reinterpret_cast<const f32x4_t*>(b + lay.w() + ro + 16 * k);
-      x.q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
-    }
-#pragma unroll
-    for (int n = 0; n < NV; ++n)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        x.u[n][i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n];
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      x.pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
-#pragma unroll
-      for (int m = 0; m < MT; ++m)
-        x.kt[m][k] = *reinterpret_cast<const f32x4_t*>(b + lay.kt() + (int64_t)(min(wave + 4 * m, DT - 1) * 16 + lr) * kC + 16 * k + 4 * lg);
-    }
-    x.g = b[lay.g()];
-  };
-  auto work = [&](Chunk& x, int c) {
-    f32x4_t d[NV] = {}, ao[NV] = {};
-    f32x4_t sv[2][NV];       // the next k block's reads under this one's products
-    auto get = [&](f32x4_t (&f)[NV], const float* b, int ld, int k) {
-#pragma unroll
-      for (int n = 0; n < NV; ++n) f[n] = *reinterpret_cast<const f32x4_t*>(b + (16 * n + lr) * ld + 16 * k + 4 * lg);
-    };
-    get(sv[0], sS, LS, 0);
-#pragma unroll
-    for (int k = 0; k < DT; ++k) {
-      if (k + 1 < DT) get(sv[(k + 1) & 1], sS, LS, k + 1);
-#pragma unroll
-      for (int n = 0; n < NV; ++n)
-#pragma unroll
-        for (int s = 0; s < 4; ++s) {
-          d[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w[k][s], sv[k & 1][n][s], d[n], 0, 0, 0);
-          ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[k][s], sv[k & 1][n][s], ao[n], 0, 0, 0);
-        }
-      __builtin_amdgcn_sched_barrier(0);
-    }
-#pragma unroll
-    for (int n = 0; n < NV; ++n) *reinterpret_cast<f32x4_t*>(sU + (16 * n + lr) * LU + 16 * wave + 4 * lg) = x.u[n] - d[n];
-    lds_barrier();
-#pragma unroll
-    for (int n = 0; n < NV; ++n)
-#pragma unroll
-      for (int m = 0; m < MT; ++m) st[n][m] *= x.g;
-    get(sv[0], sU, LU, 0);
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      if (k < 3) get(sv[(k + 1) & 1], sU, LU, k + 1);
-#pragma unroll
-      for (int n = 0; n < NV; ++n)
-#pragma unroll
-        for (int s = 0; s < 4; ++s) {
-          const float uv = sv[k & 1][n][s];
-#pragma unroll
-          for (int m = 0; m < MT; ++m)
-            if (whole || wave + 4 * m < DT) st[n][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[m][k][s], uv, st[n][m], 0, 0, 0);
-          ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv, ao[n], 0, 0, 0);
-        }
-      __builtin_amdgcn_sched_barrier(0);
-    }
-#pragma unroll
-    for (int n = 0; n < NV; ++n) {
-#pragma unroll
-      for (int m = 0; m < MT; ++m)
-        if (whole || wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + (wave + 4 * m) * 16 + 4 * lg) = st[n][m];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        base[c * step + lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n] = ao[n][i];
-      }
-    }
-    lds_barrier();
-  };
-  Chunk a, b;
-  load(a, 0);
-  lds_barrier();
-  for (int c = 0; c < nck; c += 2) {
-    load(b, min(c + 1, nck - 1));
-    work(a, c);
-    if (c + 1 >= nck) break;
-    load(a, min(c + 2, nck - 1));
-    work(b, c + 1);
-  }
-#pragma unroll
-  for (int n = 0; n < NV; ++n)
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = (wave + 4 * m) * 16 + 4 * lg + i, v = v0 + 16 * n;
-        if (d < p.D && v < p.V) S[(int64_t)d * p.V + v] = st[n][m][i];
-      }
 }
 
 // the read-out of (row, head), where the scan left it
@@ -479,7 +443,7 @@ __device__ __forceinline__ const float* readout(const DeltaParams& p, const floa
   return ws + ((chunk_base(p, r) + i / kC) * p.H + h) * lay.size() + lay.u() + (int64_t)(i % kC) * lay.Vp;
 }
 
-// out = o / rms(o) * norm * silu(gate), 16 lanes per (row, head), 8 values a lane at a time; vdim a multiple of 8, <= 128 U
+// out = o / rms(o) * norm * gate, 16 lanes per (row, head), 8 values a lane at a time; vdim a multiple of 8, <= 128 U
 template <typename T, int U>
 __global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaParams p, const float* ws, const ChunkLayout lay, int nreq, int row0, int rows) {
   scalar_cache_acquire();
@@ -489,7 +453,7 @@ __global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaPar
   const int64_t row = row0 + item / p.H;
   const int h = (int)(item % p.H);
   const float* x = readout(p, ws, lay, nreq, (int)row, h);
-  const T* g = reinterpret_cast<const T*>(p.proj) + row * p.ld + p.off_g + h * p.V;
+  const T* g = reinterpret_cast<const T*>(p.gate) + row * p.ld_gate + h * p.V;
   float v[U][8], gt[U][8];
   float ss = 0.f;
 #pragma unroll
@@ -502,7 +466,7 @@ __global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaPar
     for (int j = 0; j < 8; ++j) ss += v[u][j] * v[u][j];
   }
   const float inv = inv_rms(group_allreduce_sum<16>(ss), p.V, p.eps);
-  T* out = reinterpret_cast<T*>(p.out) + (row * p.H + h) * (int64_t)p.V;
+  T* out = reinterpret_cast<T*>(p.out) + row * p.ld_out + (int64_t)h * p.V;
 #pragma unroll
   for (int u = 0; u < U; ++u) {
     const int c = 8 * (sub + 16 * u);
@@ -510,7 +474,7 @@ __global__ __launch_bounds__(256) void gated_delta_finish8_kernel(const DeltaPar
     float w[8];
     Io<T>::template ldv<8>(reinterpret_cast<const T*>(p.norm_w) + c, w);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[u][j] *= inv * w[j] * silu_f(gt[u][j]);
+    for (int j = 0; j < 8; ++j) v[u][j] *= inv * w[j] * out_gate(p, gt[u][j]);
     Io<T>::template stv<8>(out + c, v[u]);
   }
 }
@@ -528,15 +492,10 @@ __global__ __launch_bounds__(256) void gated_delta_finish_kernel(const DeltaPara
   float ss = 0.f;
   for (int v = lane; v < p.V; v += 64) ss += x[v] * x[v];
   const float inv = inv_rms(wave_allreduce_sum(ss), p.V, p.eps);
-  const T* g = reinterpret_cast<const T*>(p.proj) + row * p.ld + p.off_g + h * p.V;
+  const T* g = reinterpret_cast<const T*>(p.gate) + row * p.ld_gate + h * p.V;
   const T* nw = reinterpret_cast<const T*>(p.norm_w);
-  T* out = reinterpret_cast<T*>(p.out) + (row * p.H + h) * (int64_t)p.V;
-  for (int v = lane; v < p.V; v += 64) Io<T>::st(out + v, x[v] * inv * Io<T>::ld(nw + v) * silu_f(Io<T>::ld(g + v)));
-}
-
-inline int round_tiles(int n) {   // 16-column tiles of the built scans: 2, 4, 8, 16
-  const int t = (n + 15) / 16;
-  return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 16;
+  T* out = reinterpret_cast<T*>(p.out) + row * p.ld_out + (int64_t)h * p.V;
+  for (int v = lane; v < p.V; v += 64) Io<T>::st(out + v, x[v] * inv * Io<T>::ld(nw + v) * out_gate(p, Io<T>::ld(g + v)));
 }
 
 }  // namespace
@@ -544,52 +503,37 @@ inline int round_tiles(int n) {   // 16-column tiles of the built scans: 2, 4, 8
 
 using namespace mi;
 
-static bool chunk_layout(int32_t dim, int32_t vdim, ChunkLayout* lay) {
-  if (dim <= 0 || vdim <= 0 || dim > 256 || vdim > 256) return false;
-  lay->Dp = 16 * round_tiles(dim);
-  lay->Vp = (vdim + 15) / 16 * 16;
-  return true;
-}
-
-extern "C" int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t dim, int32_t vdim) {
+extern "C" int64_t mi_gated_delta_chunked_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t dim, int32_t vdim,
+                                                          int32_t channel_decay) {
   ChunkLayout lay;
   if (rows < 0 || num_reqs < 0 || heads <= 0 || !chunk_layout(dim, vdim, &lay)) return 0;
+  if (channel_decay && dim > 128) return 0;      // K, Q and the cumulative decays of a chunk must fit the LDS together
   const int64_t chunks = rows / kC + num_reqs;
   return chunks * heads * lay.size() * 4;
 }
 
-extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, const void* conv_w, const float* a_log,
-                                      const float* dt_bias, const void* norm_w, float* state, void* ring, const int32_t* slots,
-                                      const int32_t* query_start_loc, const int32_t* seq_lens, void* out, int32_t row0,
-                                      int32_t rows, int32_t req0, int32_t num_reqs, int32_t max_query_len, int32_t heads,
-                                      int32_t kv_heads, int32_t dim, int32_t vdim, int32_t taps, float eps, void* workspace,
-                                      int64_t workspace_bytes, int dtype, void* stream) {
-  if (num_reqs == 0 || rows == 0) return MI_OK;
-  if (!proj || !conv_w || !a_log || !dt_bias || !norm_w || !state || !ring || !slots || !query_start_loc || !seq_lens || !out ||
-      !workspace)
-    return MI_ERR_INVALID_ARG;
-  if (req0 < 0 || num_reqs < 0 || row0 < 0 || rows < 0 || max_query_len <= 0 || heads <= 0 || kv_heads <= 0 || taps <= 0 ||
-      heads % kv_heads)
-    return MI_ERR_INVALID_ARG;
+extern "C" int mi_gated_delta_chunked(const mi_gated_delta_args* args, int32_t row0, int32_t rows, int32_t max_query_len,
+                                      void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
+  if (args && (args->num_reqs == 0 || rows == 0)) return MI_OK;
+  DeltaParams p;
+  const int rc = delta_fill(p, args);
+  if (rc != MI_OK) return rc;
+  if (!workspace || row0 < 0 || rows < 0 || max_query_len <= 0) return MI_ERR_INVALID_ARG;
+  const int heads = p.H, dim = p.D, vdim = p.V, num_reqs = args->num_reqs, CH = p.CH;
   ChunkLayout lay;
-  if (!chunk_layout(dim, vdim, &lay)) return MI_ERR_UNSUPPORTED;
-  if (workspace_bytes < mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, heads, dim, vdim)) return MI_ERR_WORKSPACE;
-  const int CH = 2 * kv_heads * dim + heads * vdim;
-  if (proj_stride < CH + heads * vdim + 2 * heads) return MI_ERR_INVALID_ARG;
+  if (!chunk_layout(dim, vdim, &lay) || (p.channel && dim > 128)) return MI_ERR_UNSUPPORTED;
+  if (workspace_bytes < mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, heads, dim, vdim, p.channel)) return MI_ERR_WORKSPACE;
   if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
-  const DeltaParams p{proj, conv_w, norm_w, ring, out, a_log, dt_bias, state, slots, query_start_loc, seq_lens, proj_stride, req0,
-                      heads, kv_heads, dim, vdim, taps, CH, CH, CH + heads * vdim, CH + heads * vdim + heads, eps};
   hipStream_t s = (hipStream_t)stream;
   float* ws = (float*)workspace;
   const int ldk = lay.Dp + 4, ldv = lay.Vp + 4, ldm = kC + 4;
-  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC) * 4;
+  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC + (p.channel ? kC * ldk : 0)) * 4;
   const int al = (dtype == MI_DTYPE_BF16 ? 8 : 4);
-  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && proj_stride % al == 0 && CH % al == 0 && aligned16(proj) && aligned16(conv_w) &&
-                   aligned16(ring);
+  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && p.ld % al == 0 && CH % al == 0 && aligned16(p.proj) && aligned16(p.convw) && aligned16(p.ring);
   const dim3 pg((max_query_len + kC - 1) / kC, heads, num_reqs);
 #define MI_PREP(T)                                                                                                        \
   do {                                                                                                                    \
-    auto kern = gated_delta_prep_kernel<T>;                                                                               \
+    auto kern = p.channel ? gated_delta_prep_kernel<T, true> : gated_delta_prep_kernel<T, false>;                                                                               \
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
       return MI_ERR_LAUNCH;                                                                                               \
     hipLaunchKernelGGL(kern, pg, dim3(kPrepThreads), lds, s, p, ws, lay, vec);                                               \
@@ -597,24 +541,11 @@ extern "C" int mi_gated_delta_chunked(const void* proj, int64_t proj_stride, con
   if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
   else MI_PREP(float);
 #undef MI_PREP
-  // two value tiles a workgroup where that still leaves one for every CU
-  const int nvt = lay.Vp / 16, nv = nvt % 2 == 0 && (int64_t)num_reqs * heads * (nvt / 2) >= 256 ? 2 : 1, nvg = nvt / nv;
-  const dim3 sg((heads + 7) / 8 * 8 * nvg, num_reqs);
-#define MI_SCAN(DT)                                                                                                            \
-  do {                                                                                                                         \
-    if (nv == 2) hipLaunchKernelGGL((gated_delta_scan_kernel<DT, 2>), sg, dim3(256), 0, s, p, ws, lay, nvg);                   \
-    else hipLaunchKernelGGL((gated_delta_scan_kernel<DT, 1>), sg, dim3(256), 0, s, p, ws, lay, nvg);                           \
-  } while (0)
-  switch (lay.Dp / 16) {
-    case 2: MI_SCAN(2); break;
-    case 4: MI_SCAN(4); break;
-    case 8: MI_SCAN(8); break;
-    default: MI_SCAN(16); break;
-  }
-#undef MI_SCAN
+  const int sc = launch_scan<true>(ScanParams{p.state, p.slots, p.qsl, p.seq_lens, p.req0, heads, dim, vdim}, ws, lay, num_reqs, s);
+  if (sc != MI_OK) return sc;
   const dim3 fg((unsigned)(((int64_t)rows * heads + 3) / 4)), rg((CH + 255) / 256, num_reqs);
   const dim3 f8((unsigned)(((int64_t)rows * heads + 15) / 16));
-  const bool vecf = vec && aligned16(out) && aligned16(norm_w);
+  const bool vecf = vec && p.ld_gate % al == 0 && p.ld_out % al == 0 && aligned16(p.gate) && aligned16(p.out) && aligned16(p.norm_w);
 #define MI_FINISH(T)                                                                                                              \
   do {                                                                                                                            \
     if (vecf && vdim <= 128) hipLaunchKernelGGL((gated_delta_finish8_kernel<T, 1>), f8, dim3(256), 0, s, p, ws, lay, num_reqs, row0, rows);   \

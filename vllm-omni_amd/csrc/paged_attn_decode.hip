@@ -382,7 +382,7 @@ __global__ __launch_bounds__(64) void decode_reduce_kernel(const DecodeParams p)
         for (int d = 0; d < DPL; ++d) a1[d] += w * po[j][d];
       }
     }
-    const float inv1 = np > 0 ? 1.f / L1 : 0.f;
+    const float inv1 = np > 0 ? p.out_scale / L1 : 0.f;
     const int64_t o1 = (int64_t)seq * p.out_stride + (int64_t)qh * HD + lane * DPL;
 #pragma unroll
     for (int d = 0; d < DPL; ++d) {
@@ -424,7 +424,7 @@ __global__ __launch_bounds__(64) void decode_reduce_kernel(const DecodeParams p)
       }
     }
   }
-  const float inv = np > 0 ? 1.f / L : 0.f;
+  const float inv = np > 0 ? p.out_scale / L : 0.f;
   const int64_t o = (int64_t)seq * p.out_stride + (int64_t)qh * HD + lane * DPL;
 #pragma unroll
   for (int d = 0; d < DPL; ++d) {
@@ -551,7 +551,8 @@ int decode_call(void* out, const void* q, const void* k_cache, const void* v_cac
                 int32_t block_size, int32_t block_table_stride, int32_t max_seq_len, float scale, int64_t q_token_stride,
                 int64_t out_token_stride, int64_t cache_block_stride, int64_t cache_token_stride,
                 int64_t cache_head_stride, int32_t partition_size, void* workspace, int64_t workspace_bytes, int dtype,
-                int out_dtype, int32_t flags, void* stream, const RopeFusion* rope) {
+                int out_dtype, int32_t flags, void* stream, const RopeFusion* rope, const float* slopes = nullptr,
+                const float* sinks = nullptr, float out_scale = 1.f) {
   using namespace mi;
   if (num_seqs == 0) return MI_OK;
   if (!out || !q || !k_cache || !v_cache || !block_table || !seq_lens) return MI_ERR_INVALID_ARG;
@@ -625,6 +626,10 @@ int decode_call(void* out, const void* q, const void* k_cache, const void* v_cac
   // fp32-P VALU kernel, so every production launch is inside the rtol 1e-3 / atol 1e-4 bound.
   const bool packed = (flags & MI_DECODE_PACKED_PV) && (flags & MI_DECODE_FORCE_VALU);
   int rc;
+  p.slopes = slopes;
+  p.sinks = sinks;
+  p.out_scale = out_scale;
+  if ((slopes || sinks) && (rope || !use_mfma)) return MI_ERR_UNSUPPORTED;
   if (rope) {
     // built for the production form only: matrix-core kernel, nt streams, P as a hi + lo pair
     if (!use_mfma || !(flags & MI_DECODE_NONTEMPORAL) || (flags & MI_DECODE_ROUNDED_P)) return MI_ERR_UNSUPPORTED;
@@ -668,6 +673,21 @@ extern "C" int mi_paged_attn_decode(void* out, const void* q, const void* k_cach
                      block_size, block_table_stride, max_seq_len, scale, q_token_stride, out_token_stride,
                      cache_block_stride, cache_token_stride, cache_head_stride, partition_size, workspace,
                      workspace_bytes, dtype, out_dtype, flags, stream, nullptr);
+}
+
+extern "C" int mi_paged_attn_decode_biased(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                           const int32_t* block_table, const int32_t* seq_lens, const float* slopes,
+                                           const float* sinks, float out_scale, int32_t num_seqs, int32_t num_q_heads, int32_t num_kv_heads,
+                                           int32_t head_dim, int32_t block_size, int32_t block_table_stride,
+                                           int32_t max_seq_len, float scale, int64_t q_token_stride,
+                                           int64_t out_token_stride, int64_t cache_block_stride,
+                                           int64_t cache_token_stride, int64_t cache_head_stride, int32_t partition_size,
+                                           void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
+  return decode_call(out, q, k_cache, v_cache, block_table, seq_lens, num_seqs, num_q_heads, num_kv_heads, head_dim,
+                     block_size, block_table_stride, max_seq_len, scale, q_token_stride, out_token_stride,
+                     cache_block_stride, cache_token_stride, cache_head_stride, partition_size, workspace,
+                     workspace_bytes, dtype, dtype, MI_DECODE_PACKED_PV | MI_DECODE_NONTEMPORAL, stream, nullptr, slopes,
+                     sinks, out_scale);
 }
 
 extern "C" int mi_rope_cache_paged_attn_decode(void* out, const void* q, const void* k, const void* v,

@@ -127,7 +127,9 @@ __device__ __forceinline__ float item_sumsq(const uint4& xr, const uint4& yr) {
   return ss;
 }
 
-template <typename Tag, int HD, int AUX, bool SPLIT, int NS, bool ROPE = false, bool NORM = false>
+// BIAS: a distance bias and a sink.  The bias is the MFMA's C operand — S^T = K . Q^T + slope / scale * (key - position) — so
+// the softmax does not know of it; the sink is what partition 0 starts its running maximum and sum from.
+template <typename Tag, int HD, int AUX, bool SPLIT, int NS, bool ROPE = false, bool NORM = false, bool BIAS = false>
 __global__ __launch_bounds__(64, 2) void decode_mfma_kernel(const DecodeParams p, const int gh) {
   scalar_cache_acquire();
   using E = Elem<Tag>;
@@ -366,6 +368,14 @@ __global__ __launch_bounds__(64, 2) void decode_mfma_kernel(const DecodeParams p
   };
 
   float m = -3.0e38f, l = 0.f;
+  float slope = 0.f;      // in units of the raw scores
+  if constexpr (BIAS) {
+    if (p.slopes && head_ok) slope = p.slopes[qh0 + h] * kLog2e / p.scale_log2e;
+    if (p.sinks && head_ok && part == 0) {
+      m = p.sinks[qh0 + h] * kLog2e;
+      l = g == 0 ? 1.f : 0.f;      // summed over the four lanes of the head at the end
+    }
+  }
   f32x4_t acc[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n) acc[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -385,6 +395,14 @@ __global__ __launch_bounds__(64, 2) void decode_mfma_kernel(const DecodeParams p
     else lds_read_rows4<SB, SB + 16 * ROWB>(k_rd, k0, k1);
     if (refill) issue_k(t + NS, ST);  // K image of this stage is free again: refill it now
     f32x4_t s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+    if constexpr (BIAS) {
+      const float b = slope * (float)(t * kStep + 4 * g - (seq_len - 1));
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s0[r] = __builtin_fmaf(slope, (float)r, b);
+        s1[r] = __builtin_fmaf(slope, (float)(16 + r), b);
+      }
+    }
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
       s0 = mfma16<Tag>(__builtin_bit_cast(uint4, k0[s]), qf[s], s0);
@@ -534,7 +552,7 @@ __global__ __launch_bounds__(64, 2) void decode_mfma_kernel(const DecodeParams p
   l = rows_allreduce_sum(l);
   if (direct) {
     if (!head_ok) return;
-    const float inv = 1.f / l;
+    const float inv = p.out_scale / l;
     const int64_t o = (int64_t)seq * p.out_stride + (int64_t)(qh0 + h) * HD + 4 * g;
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
@@ -604,7 +622,7 @@ __global__ __launch_bounds__(64, 2) void decode_mfma_kernel(const DecodeParams p
 #pragma unroll
       for (int d = 0; d < DPL; ++d) a[d] += w * __hip_atomic_load(po + d, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     }
-    const float inv = 1.f / L;
+    const float inv = p.out_scale / L;
     const int64_t o = (int64_t)seq * p.out_stride + (int64_t)qh * HD + lane * DPL;
 #pragma unroll
     for (int d = 0; d < DPL; ++d) {
@@ -624,6 +642,12 @@ int launch_decode_mfma(const DecodeParams& p, int gh, int head_dim, int dtype, b
   const int64_t waves = (int64_t)p.num_seqs * (p.num_q_heads / gh) * p.num_parts;
   if (waves > INT32_MAX) return MI_ERR_UNSUPPORTED;
   const dim3 grid((unsigned)waves), block(64);
+  if (p.slopes || p.sinks) {
+    if (dtype != MI_DTYPE_BF16 || !split_p) return MI_ERR_UNSUPPORTED;
+    if (head_dim == 128) hipLaunchKernelGGL((decode_mfma_kernel<bf16_tag, 128, 2, true, 2, false, false, true>), grid, block, 0, stream, p, gh);
+    else hipLaunchKernelGGL((decode_mfma_kernel<bf16_tag, 64, 2, true, MI_DECODE_NS64, false, false, true>), grid, block, 0, stream, p, gh);
+    return launch_status();
+  }
 #define MI_LAUNCH_NS(TAG, HDIM, NS_)                                                                        \
   do {                                                                                                      \
     if (split_p) {                                                                                          \

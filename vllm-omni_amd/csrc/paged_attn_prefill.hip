@@ -32,6 +32,7 @@
 // FLOPs per layer: 2 * S^2 * d * n_q (causal).  MFMA-bound by design; K/V bytes are read once per
 // (16*NC query tokens x G heads) and served from L2/MALL for any but the first tile of a sequence.
 #include <cstdlib>
+#include <type_traits>
 
 #include "common.h"
 #include "mfma_attn_common.h"
@@ -56,7 +57,31 @@ struct PrefillParams {
   float* ws;    // [token][q head][nseg][head_dim + 1]
   float scale_log2e;
   int64_t q_stride, out_stride, blk_stride, tok_stride, head_stride;
+  // BIAS kernels: score -= slopes[head] * (position - key position); the denominator also holds exp(sinks[head]).
+  // fp32 [num_q_heads] each, nullptr = none
+  const float* slopes;
+  const float* sinks;
+  float out_scale;      // the output times this
 };
+
+// A distance bias is the C operand of the score MFMAs: S^T = K . Q^T + slope / scale * (key - position), so the softmax does
+// not know of it.  It climbs by 32 slopes a step, hence a larger headroom before the reference maximum is raised.
+// A sink is one more term of the denominator: the segment that holds key 0 takes it in its epilogue.
+constexpr float kThrPlain = 6.0f, kThrBias = 40.0f;
+// acc / l with reference mu (log2) -> factor of acc and log2 of the denominator
+template <bool BIAS>
+__device__ __forceinline__ float close_row(const PrefillParams& p, int head, int seg, float mu_l2, float l, float& lse) {
+  if constexpr (BIAS) {
+    if (p.sinks && seg == 0) {
+      const float sk = p.sinks[head] * kLog2e, m = fmaxf(mu_l2, sk), f = fast_exp2(mu_l2 - m);
+      const float den = l * f + fast_exp2(sk - m);
+      lse = m + __builtin_amdgcn_logf(den);
+      return f / den;
+    }
+  }
+  lse = l > 0.f ? mu_l2 + __builtin_amdgcn_logf(l) : -INFINITY;
+  return l > 0.f ? 1.f / l : 0.f;      // l == 0: a column that saw no key of this segment
+}
 
 constexpr int kColTile = 16;  // query tokens per MFMA column tile
 #ifndef MI_PREFILL_ABLATE
@@ -123,7 +148,7 @@ namespace {
 // waves per workgroup = query heads per KV head handled together; NI = waves that issue DMA;
 // NC = column tiles (of 16 query tokens) per wave.
 // SPLIT: see prefill_mfma32_kernel — P as a hi + lo pair of cache-dtype values, one extra MFMA per d-tile.
-template <typename Tag, int HD, int NI, int NC, bool SPLIT>
+template <typename Tag, int HD, int NI, int NC, bool SPLIT, bool BIAS = false>
 __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p) {
   scalar_cache_acquire();
   using E = Elem<Tag>;
@@ -293,7 +318,8 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
   // slow path BEFORE its exponentials: row maximum across the four lane rows, mu raised, acc and l (which hold exactly
   // the steps before this one) rescaled by exp2(-growth).  The first step of a tile has no reference yet and always
   // takes that path.
-  constexpr float kThr = 6.0f;
+  constexpr float kThr = BIAS ? kThrBias : kThrPlain;
+  const float slope = BIAS && p.slopes ? p.slopes[head] * kLog2e / p.scale_log2e : 0.f;   // in units of the raw scores
   const float thr_raw = kThr / p.scale_log2e;   // the threshold in unscaled score units
   float mu[NC], nms[NC], mu_thr[NC], l[NC];     // reference, -mu * scale (the exponent's addend), mu + threshold
   f32x4_t acc[NC][NT];
@@ -340,11 +366,19 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
     } else if constexpr (KS == 4) lds_read_rows8<SB, SB + 16 * ROWB>(k_rd, k0, k1);
     else lds_read_rows4<SB, SB + 16 * ROWB>(k_rd, k0, k1);
   };
-  auto qk_mfma = [&](const u32x4_t (&k0)[KS], const u32x4_t (&k1)[KS], f32x4_t (&s0)[NC], f32x4_t (&s1)[NC]) {
+  auto qk_mfma = [&](int t, const u32x4_t (&k0)[KS], const u32x4_t (&k1)[KS], f32x4_t (&s0)[NC], f32x4_t (&s1)[NC]) {
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       s0[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
       s1[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if constexpr (BIAS) {
+        const float b = slope * (float)(t * kStep + 4 * g - (qpos0 + kColTile * c));
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s0[c][r] = __builtin_fmaf(slope, (float)r, b);
+          s1[c][r] = __builtin_fmaf(slope, (float)(16 + r), b);
+        }
+      }
     }
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
@@ -520,7 +554,7 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
       u32x4_t k0[KS], k1[KS];
       kread(NEXT{}, k0, k1);
       MI_TICK(4);
-      qk_mfma(k0, k1, sc0[(ST + 1) & 1], sc1[(ST + 1) & 1]);
+      qk_mfma(t + 1, k0, k1, sc0[(ST + 1) & 1], sc1[(ST + 1) & 1]);
       expo(sc0[ST & 1], sc1[ST & 1]);
       if constexpr (MI_PREFILL_SCHED) {
 #pragma unroll
@@ -549,7 +583,7 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
   if (active) {
     u32x4_t k0[KS], k1[KS];
     kread(S0{}, k0, k1);
-    qk_mfma(k0, k1, sc0[0], sc1[0]);
+    qk_mfma(t_begin, k0, k1, sc0[0], sc1[0]);
   }
   // interior steps [0, t_int): t + 3 < t_end, (t + 1) * 32 <= first diagonal key of the tile; whole groups of four
   const int t_int = max(t_begin, min(t_end - 3, (ctx_off + tile0 + 1) / kStep)) & ~3;
@@ -582,7 +616,8 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
     float lc = l[c];
     lc = rows_allreduce_sum(lc);
     if (active && kColTile * c + col < rows) {
-      const float inv = lc > 0.f ? 1.f / lc : 0.f;   // lc == 0: a column that saw no key of this segment
+      float lse;
+      const float inv = close_row<BIAS>(p, head, seg, mu[c] * p.scale_log2e, lc, lse);
       if (split) {
         // normalised fp32 partial + log2-sum-exp of the segment; merged by prefill_merge_kernel
         float* w = p.ws + (((int64_t)(q0 + tile0 + kColTile * c + col) * p.num_q_heads + head) * p.nseg + seg) * (HD + 1);
@@ -590,15 +625,16 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
         for (int n = 0; n < NT; ++n)
           *reinterpret_cast<f32x4_t*>(w + 16 * n + 4 * g) =
               f32x4_t{acc[c][n][0] * inv, acc[c][n][1] * inv, acc[c][n][2] * inv, acc[c][n][3] * inv};
-        if (g == 0) w[HD] = lc > 0.f ? mu[c] * p.scale_log2e + __builtin_amdgcn_logf(lc) : -INFINITY;
+        if (g == 0) w[HD] = lse;
       } else {
         uint16_t* o = reinterpret_cast<uint16_t*>(p.out) + (int64_t)(q0 + tile0 + kColTile * c + col) * p.out_stride +
                       (int64_t)head * HD + 4 * g;
+        const float mul = BIAS ? inv * p.out_scale : inv;
 #pragma unroll
         for (int n = 0; n < NT; ++n) {
           uint2 r;
-          r.x = E::pack(acc[c][n][0] * inv, acc[c][n][1] * inv);
-          r.y = E::pack(acc[c][n][2] * inv, acc[c][n][3] * inv);
+          r.x = E::pack(acc[c][n][0] * mul, acc[c][n][1] * mul);
+          r.y = E::pack(acc[c][n][2] * mul, acc[c][n][3] * mul);
           *reinterpret_cast<uint2*>(o + 16 * n) = r;
         }
       }
@@ -629,7 +665,7 @@ __global__ __launch_bounds__(512) void prefill_mfma_kernel(const PrefillParams p
 // significant bits instead of 8 / 11), one extra MFMA per (d-block, key half) against the same V operand — what brings the
 // kernel inside rtol 1e-3 / atol 1e-4 of the fp32 oracle, as the decode kernel's split does.  SPLIT = false is the
 // single-rounding P of flash kernels (`dot(P.to(V.dtype), V)`), kept for A/B (MI_PREFILL_ROUNDED_P=1).
-template <typename Tag, int HD, int NI, int NC, bool SPLIT>
+template <typename Tag, int HD, int NI, int NC, bool SPLIT, bool BIAS = false>
 __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(const PrefillParams p) {
   scalar_cache_acquire();
   using E = Elem<Tag>;
@@ -784,10 +820,13 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
   };
 
   // ---- online softmax state (deferred reference maximum: see the 16x16x32 kernel)
-  constexpr float kThr = 6.0f;
+  constexpr float kThr = BIAS ? kThrBias : kThrPlain;
   const float thr_raw = kThr / p.scale_log2e;
   float mu[NC], nms[NC], mu_thr[NC], l[NC];
   f32x16_t acc[NC][NB];
+  float slope[NC];      // in units of the raw scores
+#pragma unroll
+  for (int c = 0; c < NC; ++c) slope[c] = BIAS && p.slopes ? p.slopes[head[c]] * kLog2e / p.scale_log2e : 0.f;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
     mu[c] = nms[c] = mu_thr[c] = l[c] = 0.f;
@@ -815,11 +854,13 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
   // vector instructions the scheduler places behind each MFMA (the same totals per step whatever the head size)
   constexpr int kExpPerMfma = 16 / KS, kPackPerMfma = 8 / KS;
   constexpr int kLoPerMfma = 40 / (2 * NB), kSumPerMfma = (30 + 2 * NB - 1) / (2 * NB);
-  auto qk_mfma = [&](const u32x4_t (&k)[KS], f32x16_t (&s)[NC]) {
+  auto qk_mfma = [&](int t, const u32x4_t (&k)[KS], f32x16_t (&s)[NC]) {
 #pragma unroll
-    for (int c = 0; c < NC; ++c)
+    for (int c = 0; c < NC; ++c) {
+      const float b = BIAS ? slope[c] * (float)(t * kStep + 4 * h - qpos[c]) : 0.f;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) s[c][i] = 0.f;
+      for (int i = 0; i < 16; ++i) s[c][i] = BIAS ? __builtin_fmaf(slope[c], (float)(8 * (i >> 2) + (i & 3)), b) : 0.f;
+    }
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
@@ -971,7 +1012,7 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
       v_issue(std::integral_constant<int, SB>{}, o);
       __builtin_amdgcn_sched_barrier(0);
       MI_TICK(4);
-      qk_mfma(k, sc[(ST + 1) & 1]);
+      qk_mfma(t + 1, k, sc[(ST + 1) & 1]);
       float v[NC][16];
       expo(sc[ST & 1], v);
       if constexpr (MI_PREFILL_SCHED) {
@@ -1085,7 +1126,7 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
       pre(t, sc[ST & 1], interior);
       v_issue(std::integral_constant<int, SB>{}, o_keep);   // V(t): under the S^T MFMAs
       __builtin_amdgcn_sched_barrier(0);
-      qk_mfma(k, sc[(ST + 1) & 1]);
+      qk_mfma(t + 1, k, sc[(ST + 1) & 1]);
       expo(sc[ST & 1], v_keep);
       if constexpr (MI_PREFILL_SCHED) {
 #pragma unroll
@@ -1112,7 +1153,7 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
   if (active) {
     u32x4_t k[KS];
     kread(S0{}, k);
-    qk_mfma(k, sc[0]);
+    qk_mfma(t_begin, k, sc[0]);
 #pragma unroll
     for (int c = 0; c < NC; ++c) mx_pre[c] = row_max(sc[0][c]);
   }
@@ -1169,7 +1210,8 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
     permlane32_swap(la, lb);
     const float lsum = la + lb;
     if (valid[c]) {
-      const float inv = lsum > 0.f ? 1.f / lsum : 0.f;   // lsum == 0: a column that saw no key of this segment
+      float lse;
+      const float inv = close_row<BIAS>(p, head[c], seg, mu[c] * p.scale_log2e, lsum, lse);
       if (split) {
         float* w = p.ws + (((int64_t)(q0 + tile0 + qi[c]) * p.num_q_heads + head[c]) * p.nseg + seg) * (HD + 1);
 #pragma unroll
@@ -1178,16 +1220,17 @@ __global__ __launch_bounds__(NC == 2 ? 256 : 512) void prefill_mfma32_kernel(con
           for (int q4 = 0; q4 < 4; ++q4)
             *reinterpret_cast<f32x4_t*>(w + 32 * n + 8 * q4 + 4 * h) =
                 f32x4_t{acc[c][n][4 * q4] * inv, acc[c][n][4 * q4 + 1] * inv, acc[c][n][4 * q4 + 2] * inv, acc[c][n][4 * q4 + 3] * inv};
-        if (h == 0) w[HD] = lsum > 0.f ? mu[c] * p.scale_log2e + __builtin_amdgcn_logf(lsum) : -INFINITY;
+        if (h == 0) w[HD] = lse;
       } else {
         uint16_t* o = reinterpret_cast<uint16_t*>(p.out) + (int64_t)(q0 + tile0 + qi[c]) * p.out_stride + (int64_t)head[c] * HD + 4 * h;
+        const float mul = BIAS ? inv * p.out_scale : inv;
 #pragma unroll
         for (int n = 0; n < NB; ++n)
 #pragma unroll
           for (int q4 = 0; q4 < 4; ++q4) {
             uint2 r;
-            r.x = E::pack(acc[c][n][4 * q4] * inv, acc[c][n][4 * q4 + 1] * inv);
-            r.y = E::pack(acc[c][n][4 * q4 + 2] * inv, acc[c][n][4 * q4 + 3] * inv);
+            r.x = E::pack(acc[c][n][4 * q4] * mul, acc[c][n][4 * q4 + 1] * mul);
+            r.y = E::pack(acc[c][n][4 * q4 + 2] * mul, acc[c][n][4 * q4 + 3] * mul);
             *reinterpret_cast<uint2*>(o + 32 * n + 8 * q4) = r;
           }
       }
@@ -1226,7 +1269,7 @@ __global__ __launch_bounds__(256) void prefill_merge_kernel(const PrefillParams 
       den += wt;
       a += *reinterpret_cast<const f32x4_t*>(w + sidx * (HD + 1) + 4 * d4) * wt;
     }
-    const float inv = 1.f / den;
+    const float inv = p.out_scale / den;
     uint2 o;
     o.x = E::pack(a[0] * inv, a[1] * inv);
     o.y = E::pack(a[2] * inv, a[3] * inv);
@@ -1356,6 +1399,25 @@ int launch_prefill(PrefillParams p, const PrefillPlan& pl, int num_kv_heads, int
     const char* e = getenv("MI_PREFILL_ROUNDED_P");
     return e && atoi(e) != 0;
   }();
+  if (p.slopes || p.sinks) {
+    if constexpr (std::is_same_v<Tag, bf16_tag>) {
+      if (pl.w4) return MI_ERR_UNSUPPORTED;
+#define MI_LAUNCH_BIAS(KERN, NC_)                                                                                     \
+  do {                                                                                                                \
+    if (pl.waves >= 4) hipLaunchKernelGGL((KERN<Tag, HD, 4, NC_, true, true>), grid, block, 0, s, p);                 \
+    else if (pl.waves >= 2) hipLaunchKernelGGL((KERN<Tag, HD, 2, NC_, true, true>), grid, block, 0, s, p);            \
+    else hipLaunchKernelGGL((KERN<Tag, HD, 1, NC_, true, true>), grid, block, 0, s, p);                               \
+  } while (0)
+      if (pl.kernel32) MI_LAUNCH_BIAS(prefill_mfma32_kernel, 1);
+      else if (pl.nc >= 2) MI_LAUNCH_BIAS(prefill_mfma_kernel, 2);
+      else MI_LAUNCH_BIAS(prefill_mfma_kernel, 1);
+#undef MI_LAUNCH_BIAS
+      const int rc = launch_status();
+      return rc != MI_OK ? rc : launch_prefill_merge<Tag, HD>(p, max_query_len, s);
+    } else {
+      return MI_ERR_UNSUPPORTED;
+    }
+  }
 #define MI_LAUNCH32(NI_, NC_)                                                                              \
   do {                                                                                                     \
     if (rounded_p) hipLaunchKernelGGL((prefill_mfma32_kernel<Tag, HD, NI_, NC_, false>), grid, block, 0, s, p); \
@@ -1409,7 +1471,7 @@ extern "C" int64_t mi_paged_attn_prefill_workspace_bytes(int32_t num_tokens, int
   return pl.nseg > 1 ? (int64_t)num_tokens * num_q_heads * pl.nseg * (head_dim + 1) * (int64_t)sizeof(float) : 0;
 }
 
-extern "C" int mi_paged_attn_prefill_split(void* out, const void* q, const void* k_cache, const void* v_cache,
+static int prefill_call(void* out, const void* q, const void* k_cache, const void* v_cache,
                                            const int32_t* block_table, const int32_t* seq_lens,
                                            const int32_t* query_start_loc, int32_t num_seqs, int32_t num_tokens,
                                            int32_t max_query_len, int32_t num_q_heads, int32_t num_kv_heads,
@@ -1418,7 +1480,7 @@ extern "C" int mi_paged_attn_prefill_split(void* out, const void* q, const void*
                                            int64_t cache_block_stride, int64_t cache_token_stride,
                                            int64_t cache_head_stride, int dtype, int32_t max_seq_len,
                                            int32_t force_segments, void* workspace, int64_t workspace_bytes,
-                                           void* stream) {
+                                           const float* slopes, const float* sinks, float out_scale, void* stream) {
   using namespace mi;
   if (num_seqs == 0 || num_tokens == 0) return MI_OK;
   if (!out || !q || !k_cache || !v_cache || !block_table || !seq_lens || !query_start_loc)
@@ -1465,12 +1527,47 @@ extern "C" int mi_paged_attn_prefill_split(void* out, const void* q, const void*
   p.nseg = pl.nseg;
   p.seg_steps = pl.seg_steps;
   p.ws = reinterpret_cast<float*>(workspace);
+  p.slopes = slopes;
+  p.sinks = sinks;
+  p.out_scale = out_scale;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   if (dtype == MI_DTYPE_BF16)
     return head_dim == 128 ? launch_prefill<bf16_tag, 128>(p, pl, num_kv_heads, max_query_len, s)
                            : launch_prefill<bf16_tag, 64>(p, pl, num_kv_heads, max_query_len, s);
   return head_dim == 128 ? launch_prefill<f16_tag, 128>(p, pl, num_kv_heads, max_query_len, s)
                          : launch_prefill<f16_tag, 64>(p, pl, num_kv_heads, max_query_len, s);
+}
+
+extern "C" int mi_paged_attn_prefill_split(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                           const int32_t* block_table, const int32_t* seq_lens,
+                                           const int32_t* query_start_loc, int32_t num_seqs, int32_t num_tokens,
+                                           int32_t max_query_len, int32_t num_q_heads, int32_t num_kv_heads,
+                                           int32_t head_dim, int32_t block_size, int32_t block_table_stride,
+                                           float scale, int64_t q_token_stride, int64_t out_token_stride,
+                                           int64_t cache_block_stride, int64_t cache_token_stride,
+                                           int64_t cache_head_stride, int dtype, int32_t max_seq_len,
+                                           int32_t force_segments, void* workspace, int64_t workspace_bytes,
+                                           void* stream) {
+  return prefill_call(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, num_seqs, num_tokens, max_query_len,
+                      num_q_heads, num_kv_heads, head_dim, block_size, block_table_stride, scale, q_token_stride,
+                      out_token_stride, cache_block_stride, cache_token_stride, cache_head_stride, dtype, max_seq_len,
+                      force_segments, workspace, workspace_bytes, nullptr, nullptr, 1.f, stream);
+}
+
+extern "C" int mi_paged_attn_prefill_biased(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                            const int32_t* block_table, const int32_t* seq_lens,
+                                            const int32_t* query_start_loc, const float* slopes, const float* sinks,
+                                            float out_scale, int32_t num_seqs, int32_t num_tokens, int32_t max_query_len,
+                                            int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                                            int32_t block_size, int32_t block_table_stride, float scale,
+                                            int64_t q_token_stride, int64_t out_token_stride, int64_t cache_block_stride,
+                                            int64_t cache_token_stride, int64_t cache_head_stride, int dtype,
+                                            int32_t max_seq_len, int32_t force_segments, void* workspace,
+                                            int64_t workspace_bytes, void* stream) {
+  return prefill_call(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, num_seqs, num_tokens, max_query_len,
+                      num_q_heads, num_kv_heads, head_dim, block_size, block_table_stride, scale, q_token_stride,
+                      out_token_stride, cache_block_stride, cache_token_stride, cache_head_stride, dtype, max_seq_len,
+                      force_segments, workspace, workspace_bytes, slopes, sinks, out_scale, stream);
 }
 
 extern "C" int mi_paged_attn_prefill(void* out, const void* q, const void* k_cache, const void* v_cache,

@@ -1,9 +1,13 @@
-// Row kernels of decoders whose residual stream is 32-bit and whose sublayers are normed on both sides
-// (x <- x + norm_b(f(norm_a(x)))), and the small gates of such decoders:
+// Row kernels of decoders whose residual stream is 32-bit, and the small gates of such decoders:
 //   * residual_norm:   post-norm of a sublayer's output + residual add + pre-norm (or plain cast) for the next one
+//     (sublayers normed on both sides: x <- x + norm_b(f(norm_a(x))))
+//   * residual_add_norm: residual add of a layer's output (and of its routed experts' rows, weighted) + pre-norm or cast
+//     for what follows; also starts a stream from a projection (no add)
+//   * embed_norm:      token embedding + the first pre-norm or cast
 //   * pair_embed_norm: scaled token embedding + the row of the (previous, current) token pair + the first pre-norm
 //   * gelu_lookup_mul: gelu_tanh(z) * (a slice of a per-token table row)
 //   * clamped_glu:     g sigmoid(alpha g) (u + 1) on clamped g, u
+//   * glu:             act(g) * u, act silu or the tanh form of gelu
 // One workgroup per row, the row stays in registers; fp32 arithmetic, one rounding to the output type.  All of them
 // stream: the bound is HBM (or launch latency at decode sizes).
 #include "row_io.h"
@@ -81,6 +85,128 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualNormPa
     }
     Io<T>::template stv<VEC>(hr + c, x[k]);
   }
+}
+
+// h = norm(x) w, norm(x) (1 + w) or x itself, of a row whose sum of squares over the thread's values is ss
+template <typename T, int VEC, int MAXC>
+__device__ __forceinline__ void store_normed(float (&x)[MAXC][VEC], float ss, const void* w_pre, float w_shift, void* h, int width,
+                                             float eps, float* smem) {
+  const bool pre = w_pre != nullptr;
+  const float inv = pre ? inv_rms(wg_sum(ss, smem), width, eps) : 1.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= width) continue;
+    if (pre) {
+      float w[VEC];
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(w_pre) + c, w);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] *= inv * (w[j] + w_shift);
+    }
+    Io<T>::template stv<VEC>(reinterpret_cast<T*>(h) + c, x[k]);
+  }
+}
+
+struct ResidualAddParams {
+  float* x;
+  const void* y;                // T rows, fp32 rows, or fp32 split-K partials [split][rows][width]
+  const void* part;             // routed experts' output rows, T; nullptr: none
+  const int32_t* row_of_pair;   // [rows][top] -> row of `part`; nullptr: pair t * top + j is its row t * top + j
+  const float* weights;         // [rows][top]
+  const void* w_pre;            // nullptr: h = x cast
+  void* h;
+  int64_t x_stride, y_stride, h_stride, part_stride;
+  int rows, width, split, top, start;      // start: x is not read, the sum starts the stream
+  float w_shift, eps;
+};
+
+template <typename T, int VEC, int MAXC>
+__global__ __launch_bounds__(256) void residual_add_norm_kernel(const ResidualAddParams p) {
+  scalar_cache_acquire();
+  __shared__ float smem[16];
+  const int64_t row = blockIdx.x;
+  float* xr = p.x + row * p.x_stride;
+  float x[MAXC][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float t[VEC];
+    if (p.start) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] = 0.f;
+    } else {
+      Io<float>::ldv<VEC>(xr + c, x[k]);
+    }
+    if (p.split) {
+      const float* yp = reinterpret_cast<const float*>(p.y) + row * p.y_stride + c;
+      for (int s = 0; s < p.split; ++s) {
+        Io<float>::ldv<VEC>(yp + (int64_t)s * p.rows * p.y_stride, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) x[k][j] += t[j];
+      }
+    } else {
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.y) + row * p.y_stride + c, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] += t[j];
+    }
+    if (p.part) {
+      float e[VEC] = {};
+      for (int j0 = 0; j0 < p.top; ++j0) {
+        const int64_t pair = row * p.top + j0;
+        const int64_t pr = p.row_of_pair ? p.row_of_pair[pair] : pair;
+        const float w = p.weights[pair];
+        Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.part) + pr * p.part_stride + c, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) e[j] += w * t[j];
+      }
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] += e[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss += x[k][j] * x[k][j];
+    Io<float>::stv<VEC>(xr + c, x[k]);
+  }
+  store_normed<T, VEC, MAXC>(x, ss, p.w_pre, p.w_shift, reinterpret_cast<T*>(p.h) + row * p.h_stride, p.width, p.eps, smem);
+}
+
+struct EmbedNormParams {
+  float* x;
+  void* h;
+  void* copy;              // nullptr: none; the row in the table's type (a loop's second input)
+  const void* table;
+  const void* w_pre;       // nullptr: h = x cast
+  const int64_t* ids;
+  int64_t x_stride, h_stride, copy_stride;
+  int width, vocab;
+  float w_shift, eps;
+};
+
+template <typename T, int VEC, int MAXC>
+__global__ __launch_bounds__(256) void embed_norm_kernel(const EmbedNormParams p) {
+  scalar_cache_acquire();
+  __shared__ float smem[16];
+  const int64_t row = blockIdx.x;
+  const int64_t id = p.ids[row];
+  const bool known = id >= 0 && id < p.vocab;   // an id outside the table reads as a zero row
+  const T* er = reinterpret_cast<const T*>(p.table) + (known ? id : 0) * p.width;
+  float x[MAXC][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    Io<T>::template ldv<VEC>(er + c, x[k]);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      x[k][j] = known ? x[k][j] : 0.f;
+      ss += x[k][j] * x[k][j];
+    }
+    Io<float>::stv<VEC>(p.x + row * p.x_stride + c, x[k]);
+    if (p.copy) Io<T>::template stv<VEC>(reinterpret_cast<T*>(p.copy) + row * p.copy_stride + c, x[k]);
+  }
+  store_normed<T, VEC, MAXC>(x, ss, p.w_pre, p.w_shift, reinterpret_cast<T*>(p.h) + row * p.h_stride, p.width, p.eps, smem);
 }
 
 struct PairEmbedParams {
@@ -194,6 +320,24 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(T* out, const T* gu, i
   }
 }
 
+template <typename T, int VEC, int ACT>
+__global__ __launch_bounds__(256) void glu_kernel(T* out, const T* gate, const T* up, int rows, int ff, int64_t gu_stride,
+                                                  int64_t out_stride) {
+  scalar_cache_acquire();
+  const int per = ff / VEC;
+  const int64_t n = (int64_t)rows * per;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+    const int64_t row = i / per;
+    const int c = (int)(i % per) * VEC;
+    float g[VEC], u[VEC];
+    Io<T>::template ldv<VEC>(gate + row * gu_stride + c, g);
+    Io<T>::template ldv<VEC>(up + row * gu_stride + c, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) g[j] = (ACT == MI_ACT_SILU ? silu_f(g[j]) : gelu_tanh_f(g[j])) * u[j];
+    Io<T>::template stv<VEC>(out + row * out_stride + c, g);
+  }
+}
+
 #define MI_ROW_DISPATCH(KERN, T, width, vec_ok, ...)                                         \
   do {                                                                                       \
     if (vec_ok) {                                                                            \
@@ -283,5 +427,65 @@ extern "C" int mi_clamped_glu(void* out, const void* gate_up, int32_t rows, int3
   else if (dtype == MI_DTYPE_F32) { if (vec) MI_CG(float, 8); else MI_CG(float, 1); }
   else return MI_ERR_UNSUPPORTED;
 #undef MI_CG
+  return launch_status();
+}
+
+extern "C" int mi_residual_add_norm(void* x, const void* y, int32_t split, const void* part, const int32_t* row_of_pair,
+                                    const float* weights, int32_t top, const void* w_pre, float w_shift, void* h, int32_t start,
+                                    float eps, int32_t rows, int32_t width, int64_t x_stride, int64_t y_stride, int64_t h_stride,
+                                    int64_t part_stride, int dtype, void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!x || !y || !h || rows < 0 || width <= 0 || split < 0 || y_stride < width || h_stride < width || x_stride < width)
+    return MI_ERR_INVALID_ARG;
+  if (part && (!weights || top <= 0 || part_stride < width)) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  const ResidualAddParams p{(float*)x, y, part, row_of_pair, weights, w_pre, h, x_stride, y_stride, h_stride, part_stride,
+                            rows, width, split, part ? top : 0, start, w_shift, eps};
+  const bool vec = width % 8 == 0 && x_stride % 8 == 0 && y_stride % 8 == 0 && h_stride % 8 == 0 && (!part || part_stride % 8 == 0) &&
+                   aligned16(x) && aligned16(y) && aligned16(w_pre) && aligned16(h) && aligned16(part);
+  const dim3 grid(rows), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(residual_add_norm_kernel, uint16_t, width, vec, p);
+  else MI_ROW_DISPATCH(residual_add_norm_kernel, float, width, vec, p);
+  return launch_status();
+}
+
+extern "C" int mi_embed_norm(void* x, void* h, void* copy, const void* table, const void* w_pre, float w_shift, const int64_t* ids,
+                             float eps, int32_t rows, int32_t width, int32_t vocab, int64_t x_stride, int64_t h_stride,
+                             int64_t copy_stride, int dtype, void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!x || !h || !table || !ids || rows < 0 || width <= 0 || vocab <= 0 || x_stride < width || h_stride < width)
+    return MI_ERR_INVALID_ARG;
+  if (copy && copy_stride < width) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  const EmbedNormParams p{(float*)x, h, copy, table, w_pre, ids, x_stride, h_stride, copy_stride, width, vocab, w_shift, eps};
+  const bool vec = width % 8 == 0 && x_stride % 8 == 0 && h_stride % 8 == 0 && (!copy || copy_stride % 8 == 0) && aligned16(x) &&
+                   aligned16(h) && aligned16(copy) && aligned16(table) && aligned16(w_pre);
+  const dim3 grid(rows), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(embed_norm_kernel, uint16_t, width, vec, p);
+  else MI_ROW_DISPATCH(embed_norm_kernel, float, width, vec, p);
+  return launch_status();
+}
+
+extern "C" int mi_glu(void* out, const void* gate, const void* up, int32_t rows, int32_t ff, int64_t gu_stride, int64_t out_stride,
+                      int32_t act, int dtype, void* stream) {
+  if (rows == 0 || ff == 0) return MI_OK;
+  if (!out || !gate || !up || rows < 0 || ff < 0 || gu_stride < ff || out_stride < ff) return MI_ERR_INVALID_ARG;
+  if (act != MI_ACT_SILU && act != MI_ACT_GELU_TANH) return MI_ERR_INVALID_ARG;
+  const bool vec = ff % 8 == 0 && gu_stride % 8 == 0 && out_stride % 8 == 0 && aligned16(out) && aligned16(gate) && aligned16(up);
+  const int64_t n = (int64_t)rows * (vec ? ff / 8 : ff);
+  const int64_t want = (n + 255) / 256;
+  const dim3 grid((unsigned)(want < 65536 ? want : 65536)), block(256);
+  hipStream_t s = (hipStream_t)stream;
+#define MI_GLU(T, V, A) \
+  hipLaunchKernelGGL((glu_kernel<T, V, A>), grid, block, 0, s, (T*)out, (const T*)gate, (const T*)up, rows, ff, gu_stride, out_stride)
+#define MI_GLU_A(T, V) \
+  do { if (act == MI_ACT_SILU) MI_GLU(T, V, MI_ACT_SILU); else MI_GLU(T, V, MI_ACT_GELU_TANH); } while (0)
+  if (dtype == MI_DTYPE_BF16) { if (vec) MI_GLU_A(uint16_t, 8); else MI_GLU_A(uint16_t, 1); }
+  else if (dtype == MI_DTYPE_F32) { if (vec) MI_GLU_A(float, 8); else MI_GLU_A(float, 1); }
+  else return MI_ERR_UNSUPPORTED;
+#undef MI_GLU_A
+#undef MI_GLU
   return launch_status();
 }

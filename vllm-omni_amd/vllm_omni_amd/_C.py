@@ -19,7 +19,7 @@ MI_DTYPE_F16, MI_DTYPE_BF16, MI_DTYPE_F32 = 0, 1, 2
 MI_OK = 0
 MI_ERR_INVALID_ARG, MI_ERR_UNSUPPORTED, MI_ERR_WORKSPACE = -1, -2, -3
 MI_ERR_LAUNCH, MI_ERR_EXHAUSTED, MI_ERR_STATE = -4, -5, -6
-ABI_VERSION = 3
+ABI_VERSION = 4
 MI_LINEAR_PLAN_FULL, MI_LINEAR_PLAN_PARTIALS, MI_LINEAR_PLAN_GATED = 0, 1, 2
 MI_LINEAR_COUNTER_BYTES = 16 << 10
 MI_DECODE_PACKED_PV = 1
@@ -30,6 +30,28 @@ MI_DECODE_FUSED_MERGE = 16
 MI_DECODE_SKIP_MERGE = 32
 MI_DECODE_COUNTER_BYTES = 1 << 20
 MI_ALLREDUCE_MAX_RANKS, MI_ALLREDUCE_HANDLE_BYTES = 8, 64
+
+MI_ACT_SILU, MI_ACT_GELU_TANH = 0, 1
+
+
+class GatedDeltaArgs(ctypes.Structure):
+    """mi_gated_delta_args"""
+
+    _fields_ = [(n, c_void_p) for n in ("qkv", "gate", "beta", "decay", "conv_w", "norm_w", "a_log", "dt_bias", "state", "ring",
+                                        "slots", "query_start_loc", "seq_lens", "out")] \
+        + [(n, c_int64) for n in ("qkv_stride", "gate_stride", "beta_stride", "decay_stride", "out_stride")] \
+        + [(n, c_int32) for n in ("req0", "num_reqs", "heads", "kv_heads", "dim", "vdim", "taps", "channel_decay", "sigmoid_gate")] \
+        + [("eps", c_float)]
+
+
+class LightningArgs(ctypes.Structure):
+    """mi_lightning_args"""
+
+    _fields_ = [(n, c_void_p) for n in ("qkv", "gate", "norm_w", "decay", "log2_decay", "state", "slots", "query_start_loc",
+                                        "seq_lens", "out")] \
+        + [(n, c_int64) for n in ("qkv_stride", "gate_stride", "out_stride")] \
+        + [(n, c_int32) for n in ("req0", "num_reqs", "heads", "dim", "vdim")] + [("eps", c_float), ("mul", c_float)]
+
 
 # name -> (restype, argtypes); mirrors include/vllm_omni_amd.h declaration by declaration
 _P = c_void_p
@@ -138,11 +160,28 @@ SIGNATURES = {
     "mi_head_gemm": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, c_int64, c_int64, c_int, _P]),
     "mi_latent_attn_rows": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float,
                                     c_int64, c_int64, c_int64, c_int, _P]),
-    "mi_gated_delta_step": (c_int, [_P, c_int64, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32,
-                                    c_int32, c_int32, c_float, c_int32, c_int, _P]),
-    "mi_gated_delta_chunked_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32]),
-    "mi_gated_delta_chunked": (c_int, [_P, c_int64, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32,
-                                       c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float, _P, c_int64, c_int, _P]),
+    "mi_gated_delta_step": (c_int, [POINTER(GatedDeltaArgs), c_int32, c_int, _P]),
+    "mi_gated_delta_chunked_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32]),
+    "mi_gated_delta_chunked": (c_int, [POINTER(GatedDeltaArgs), c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
+    "mi_residual_add_norm": (c_int, [_P, _P, c_int32, _P, _P, _P, c_int32, _P, c_float, _P, c_int32, c_float, c_int32, c_int32, c_int64,
+                                     c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_embed_norm": (c_int, [_P, _P, _P, _P, _P, c_float, _P, c_float, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, c_int,
+                              _P]),
+    "mi_glu": (c_int, [_P, _P, _P, c_int32, c_int32, c_int64, c_int64, c_int32, c_int, _P]),
+    "mi_head_norm_cache": (c_int, [_P, c_int64, _P, _P, _P, c_int64, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32,
+                                   c_int32, c_int32, c_int64, c_int64, c_int64, c_float, c_int64, c_float, c_int, _P]),
+    "mi_attn_rows": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, _P, c_float, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float,
+                             c_int64, c_int64, c_int64, c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_paged_attn_decode_biased": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, c_float, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32,
+                                            c_float, c_int64, c_int64, c_int64, c_int64, c_int64, c_int32, _P, c_int64, c_int, _P]),
+    "mi_paged_attn_prefill_biased": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, _P, c_float, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32,
+                                             c_int32, c_int32, c_float, c_int64, c_int64, c_int64, c_int64, c_int64, c_int, c_int32,
+                                             c_int32, _P, c_int64, _P]),
+    "mi_lightning_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32]),
+    "mi_lightning_attn": (c_int, [POINTER(LightningArgs), c_int32, c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
+    "mi_moe_router_logits": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int64, _P]),
+    "mi_moe_pair_gemm": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64,
+                                 c_int, _P]),
     "mi_head_gemm_nt": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, _P]),
     "mi_latent_decode_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32]),
     "mi_latent_decode": (c_int, [_P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float, c_int64, c_int64,

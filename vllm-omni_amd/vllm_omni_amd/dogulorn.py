@@ -16,9 +16,10 @@ import torch
 
 from . import ops
 from .kv_cache import LatentCacheSpec
-from .layers import _init_weight, get_forward_context, tuned_linear
+from .layers import _init_weight, get_forward_context
 from .mixers import (ClampedGluMLP, GatedDelta, GatedDeltaConfig, LatentAttention, LatentAttentionConfig, TokenSideInput)
 from .state_cache import StateSpec
+from .text_model import TokenDecoder
 
 GLU_ALPHA = 1.702       # slope of the gate's sigmoid, fixed by the design
 
@@ -130,27 +131,12 @@ class DogulornDecoderLayer:
         return ops.residual_norm(x, self.side(h, side_table, ids, True), self.side.norm, next_norm, self.eps)
 
 
-class DogulornForCausalLM:
+class DogulornForCausalLM(TokenDecoder):
     """Takes token ids (and each request's state slot) from the step's metadata; returns final-normed hidden rows."""
 
-    consumes_token_ids = True
-    extra_dtypes = (torch.float32,)      # runs in true 32-bit as well
-    has_preprocess = False
-    has_postprocess = False
-    prefer_model_sampler = False
-
     def __init__(self, cfg: DogulornConfig, dtype=torch.bfloat16, device=None, seed: Optional[int] = 0):
-        from .distributed import get_tensor_model_parallel_world_size
-
-        if get_tensor_model_parallel_world_size() > 1:
-            raise NotImplementedError("this model runs data-parallel only (tp_size 1)")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError(f"this model runs in bfloat16 or float32, not {dtype}")
-        self.config, self.dtype, self.device = cfg, dtype, device
-        gen = None
-        if seed is not None:
-            gen = torch.Generator(device=device)
-            gen.manual_seed(seed)
+        super().__init__(cfg, dtype, device)
+        gen = self.generator(seed)
         w, v = cfg.hidden_size, cfg.vocab_size
         self.embed = _init_weight(v, w, dtype, device, gen, std=1.0)
         self.bigram = _init_weight(cfg.bigram_buckets + 1, w, dtype, device, gen, std=1.0)
@@ -159,7 +145,6 @@ class DogulornForCausalLM:
         self.final_norm = torch.ones(w, dtype=dtype, device=device)
         self.head = _init_weight(v, w, dtype, device, gen, std=w ** -0.5)
         self.last_token: Optional[torch.Tensor] = None
-        self.residual_tap: Optional[list] = None      # a list collects the stream after every layer (inspection)
 
     # ---- caches -------------------------------------------------------------------
     def kv_cache_specs(self, block_size: int) -> dict[int, LatentCacheSpec]:
@@ -215,13 +200,6 @@ class DogulornForCausalLM:
 
     __call__ = forward
 
-    def compute_logits(self, hidden_states: torch.Tensor) -> torch.Tensor:
-        return tuned_linear(hidden_states, self.head)
-
-    def compute_logits_and_greedy(self, hidden_states: torch.Tensor, ids: Optional[torch.Tensor] = None):
-        logits = self.compute_logits(hidden_states)
-        return logits, ops.mask_logits_argmax(logits, ids=ids)
-
     # ---- weights ----------------------------------------------------------------------
     def named_weights(self) -> Iterable[tuple[str, torch.Tensor]]:
         """checkpoint name -> parameter (a row block of a fused one where the checkpoint stores the pieces apart)"""
@@ -233,24 +211,7 @@ class DogulornForCausalLM:
         yield "final.norm", self.final_norm
         yield "head", self.head
 
-    def load_weights(self, weights) -> set[str]:
-        params = dict(self.named_weights())
-        loaded: set[str] = set()
-        for name, w in (weights.items() if isinstance(weights, dict) else weights):
-            dst = params.get(name)
-            if dst is None:
-                raise KeyError(f"checkpoint tensor maps to no parameter: {name!r}")
-            if tuple(dst.shape) != tuple(w.shape):
-                raise ValueError(f"{name}: checkpoint shape {tuple(w.shape)}, parameter {tuple(dst.shape)}")
-            dst.copy_(w.to(dst.dtype))
-            loaded.add(name)
+    def weights_changed(self) -> None:
         for layer in self.layers:
             if isinstance(layer.mixer, LatentAttention):
                 layer.mixer.weights_changed()
-        return loaded
-
-    def weight_bytes(self) -> int:
-        return sum(w.numel() * w.element_size() for _, w in self.named_weights())
-
-    def quantize_int8(self) -> None:
-        raise ValueError("int8 quantization is not built for this model")

@@ -728,6 +728,13 @@ def allocate_latent_cache(num_blocks: int, spec: LatentCacheSpec, device) -> tor
     return torch.zeros(num_blocks, spec.block_size, spec.rank, dtype=spec.dtype, device=device)
 
 
+def allocate_layer_cache(num_blocks: int, spec, device, layout: str):
+    """One layer's cache by its spec: a latent cache, or a K/V pair in ``layout``."""
+    if isinstance(spec, LatentCacheSpec):
+        return allocate_latent_cache(num_blocks, spec, device)
+    return allocate_kv_cache(1, num_blocks, spec, device, layout)[0]
+
+
 def normalize_layer_kv(layer_kv):
     """(key_blocks, value_blocks) views of any accepted layout, else ``None``.
 

@@ -1,17 +1,24 @@
 """Sequence mixers and small blocks of decoders with a 32-bit residual stream: latent attention without positions
-(its cache row shared by all heads, optionally by several layers) and the gated delta rule.  Constants that a design
-fixes are parameters here; the layers know nothing of the model they are in.
+(its cache row shared by all heads, optionally by several layers), the gated delta rule with a decay per head or per key
+channel, attention with a distance bias and a sink, decayed linear attention, and several mixers side by side.  Constants
+that a design fixes are parameters here; the layers know nothing of the model they are in.
+
+Two kinds: mixers that own their projections (``LatentAttention``, ``GatedDelta``: rows in, rows out), and mixers for layers
+whose sublayers all read one normed row and add up (``ChannelDelta``, ``SinkAttention``, ``LightningAttention``,
+``ParallelMixers``, ``DenseGlu``): such a layer has ONE input product and ONE output product (``SharedProjections``), and a
+sublayer names its blocks of both, turning columns of the first into columns the second reads.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Iterable, Optional
+import math
+from dataclasses import dataclass, field
+from typing import Iterable, Optional, Sequence
 
 import torch
 import torch.nn.functional as F
 
 from . import ops
-from .kv_cache import LatentCacheSpec
+from .kv_cache import KVCacheSpec, LatentCacheSpec, normalize_layer_kv
 from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu
 from .state_cache import StateSpec
 
@@ -230,3 +237,329 @@ class TokenSideInput:
 
     def __call__(self, x: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, defer_reduce: bool = False):
         return self.proj(ops.gelu_lookup_mul(self.gate(x), table, ids, self.offset), defer_reduce)
+
+
+# ------------------------------------------------------------------------------------------ sublayers side by side
+@dataclass
+class InBlock:
+    """Neighbouring rows of the shared input product, stored apart in the checkpoint: name -> rows"""
+
+    parts: dict[str, int]
+
+    @property
+    def size(self) -> int:
+        return sum(self.parts.values())
+
+
+@dataclass
+class OutBlock:
+    """Columns of the shared output product: ``groups`` groups of ``width`` columns, laid out ``pitch`` apart"""
+
+    name: str
+    groups: int
+    width: int
+    pitch: int
+
+    @property
+    def size(self) -> int:
+        return self.groups * self.pitch
+
+
+class SharedProjections:
+    """The input and output product of a layer whose sublayers read the same row and whose outputs add up.  Blocks start on
+    multiples of eight (16-byte rows for the kernels that read and write them); what lies between them is zero."""
+
+    ALIGN = 8
+
+    def __init__(self, width: int, ins: Sequence[InBlock], outs: Sequence[OutBlock], dtype, device, generator=None):
+        self.ins, self.outs = list(ins), list(outs)
+        self.in_at, n = self._place([b.size for b in self.ins])
+        self.out_at, k = self._place([b.size for b in self.outs])
+        self.gaps = k != sum(b.groups * b.width for b in self.outs)
+        self.inp = ReplicatedLinear(width, {"in": n}, dtype, device, generator, pad=True)
+        real = sum(b.groups * b.width for b in self.outs)
+        self.out = ReplicatedLinear(k, {"out": width}, dtype, device, generator)
+        self.out.weight.mul_((k / real) ** 0.5)
+        keep = torch.zeros(k, dtype=torch.bool, device=device)
+        for b, a in zip(self.outs, self.out_at):
+            keep[a:a + b.size].view(b.groups, b.pitch)[:, :b.width] = True
+        self.out.weight[:, ~keep] = 0
+        used = torch.zeros(self.inp.weight.shape[0], dtype=torch.bool, device=device)
+        for b, a in zip(self.ins, self.in_at):
+            used[a:a + b.size] = True
+        self.inp.weight[~used] = 0
+
+    def _place(self, sizes: Sequence[int]) -> tuple[list[int], int]:
+        at, n = [], 0
+        for s in sizes:
+            at.append(n)
+            n += -(-s // self.ALIGN) * self.ALIGN
+        return at, n
+
+    def named_weights(self) -> Iterable[tuple[str, torch.Tensor]]:
+        for b, a in zip(self.ins, self.in_at):
+            for name, n in b.parts.items():
+                yield name, self.inp.weight[a:a + n]
+                a += n
+        for b, a in zip(self.outs, self.out_at):
+            w = self.out.weight[:, a:a + b.size].view(-1, b.groups, b.pitch)[:, :, :b.width]
+            yield b.name, w if b.pitch != b.width else self.out.weight[:, a:a + b.size]
+
+    def project(self, h: torch.Tensor) -> list[torch.Tensor]:
+        """a view per input block"""
+        y = self.inp(h)
+        return [y[:, a:a + b.size] for b, a in zip(self.ins, self.in_at)]
+
+    def buffers(self, rows: int) -> tuple[torch.Tensor, list[torch.Tensor]]:
+        """the output product's operand and a view per block (sublayers fill whole blocks; gaps between blocks stay zero)"""
+        w = self.out.weight
+        exact = sum(b.size for b in self.outs) == w.shape[1]
+        buf = (torch.empty if exact else torch.zeros)(rows, w.shape[1], dtype=w.dtype, device=w.device)
+        return buf, [buf[:, a:a + b.size] for b, a in zip(self.outs, self.out_at)]
+
+
+@dataclass
+class StepInfo:
+    """what a sublayer needs of the step besides its own rows"""
+
+    md: AttentionMetadata
+    positions: torch.Tensor
+
+
+class Sublayer:
+    """``ins`` / ``outs``: its blocks of the shared products (names below the layer's prefix).  ``run`` fills its output views
+    from its input views; ``memory`` holds its cache and state tensors of this layer run."""
+
+    ins: list[InBlock]
+    outs: list[OutBlock]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        """parameters outside the shared products"""
+        return ()
+
+    def kv_cache_spec(self, block_size: int) -> Optional[KVCacheSpec]:
+        return None
+
+    def state_specs(self) -> list[StateSpec]:
+        return []
+
+    def run(self, x: list[torch.Tensor], y: list[torch.Tensor], step: StepInfo, memory: "LayerMemory") -> None:
+        raise NotImplementedError
+
+
+@dataclass
+class LayerMemory:
+    """one layer run's cache and state tensors (a layer that runs several times has one of these per run)"""
+
+    kv: Optional[tuple[torch.Tensor, torch.Tensor]] = None
+    states: list[torch.Tensor] = field(default_factory=list)
+
+    def bind_kv(self, layer_kv) -> None:
+        self.kv = normalize_layer_kv(layer_kv)
+
+
+def _vec(n: int, dtype, device, value: float = 1.0) -> torch.Tensor:
+    return torch.full((n,), value, dtype=dtype, device=device)
+
+
+@dataclass
+class ChannelDeltaConfig(GatedDeltaConfig):
+    """decay (one per head and key channel) and output gate come through products of low rank"""
+
+    decay_rank: int = 0
+    gate_rank: int = 0
+
+
+class ChannelDelta(Sublayer):
+    """Gated delta rule with one decay per head and key channel (``csrc/gated_delta.hip``)."""
+
+    def __init__(self, cfg: ChannelDeltaConfig, width: int, eps: float, dtype, device, generator=None, prefix: str = ""):
+        if cfg.heads % cfg.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.cfg, self.eps, self.dtype = cfg, eps, dtype
+        kd, hd, hv = cfg.kv_heads * cfg.dim, cfg.heads * cfg.dim, cfg.heads * cfg.vdim
+        p = prefix
+        self.ins = [InBlock({p + "q": kd, p + "k": kd, p + "v": hv}), InBlock({p + "a1": cfg.decay_rank, p + "g1": cfg.gate_rank}),
+                    InBlock({p + "b": cfg.heads})]
+        self.outs = [OutBlock(p + "o", 1, hv, hv)]
+        self.channels = 2 * kd + hv
+        self.conv_w = _init_weight(self.channels, cfg.conv, dtype, device, generator, std=0.5)
+        # both second factors in one product, block-diagonal: [a1 h; g1 h] -> [decay; gate]
+        self.gate_at = -(-hd // 8) * 8
+        self.low = torch.zeros(self.gate_at + hv, cfg.decay_rank + cfg.gate_rank, dtype=dtype, device=device)
+        self._low_blocks = {"a2": self.low[:hd, :cfg.decay_rank], "g2": self.low[self.gate_at:, cfg.decay_rank:]}
+        for w in self._low_blocks.values():
+            w.copy_(_init_weight(*w.shape, dtype, device, generator, std=w.shape[1] ** -0.5))
+        self.a_log = _vec(cfg.heads, torch.float32, device, 0.0)
+        self.dt_bias = _vec(hd, torch.float32, device, 0.0)
+        self.norm = _vec(cfg.vdim, dtype, device)
+
+    def state_specs(self) -> list[StateSpec]:
+        c = self.cfg
+        return [StateSpec((c.heads, c.dim, c.vdim), torch.float32), StateSpec((c.conv, self.channels), self.dtype)]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        kd = self.cfg.kv_heads * self.cfg.dim
+        for name, lo, hi in (("q", 0, kd), ("k", kd, 2 * kd), ("v", 2 * kd, self.channels)):
+            yield p + name + ".conv", self.conv_w[lo:hi]
+        for name, w in self._low_blocks.items():
+            yield p + name, w
+        yield p + "A_log", self.a_log
+        yield p + "dt_bias", self.dt_bias
+        yield p + "norm", self.norm
+
+    def run(self, x, y, step, memory) -> None:
+        c, md = self.cfg, step.md
+        qkv, low, beta = x
+        both = F.linear(low, self.low)
+        hd = c.heads * c.dim
+        args = (qkv, self.conv_w, self.a_log, self.dt_bias, self.norm, *memory.states, md.state_rows, md.query_start_loc, md.seq_lens,
+                c.kv_heads, self.eps, y[0])
+        kw = dict(gate=both[:, self.gate_at:], beta=beta, decay=both[:, :hd], sigmoid_gate=True)
+        nd = md.num_decodes
+        if nd:
+            ops.gated_delta_step(*args, 0, nd, update_ring=False, **kw)
+        if nd < md.num_reqs:
+            ops.gated_delta_chunked(*args, nd, md.num_reqs - nd, nd, md.max_query_len, **kw)
+
+
+@dataclass
+class SinkAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    slopes: Optional[list[float]] = None      # per head, taken off per token of distance; None: no distance bias
+    temp_coef: float = 0.0                    # q times 1 + coef ln(floor((p + 1) / every) + 1)
+    temp_every: int = 1
+
+
+class SinkAttention(Sublayer):
+    """Grouped-query attention with normed heads, a query temperature, a distance bias and a sink (``csrc/biased_attn.hip`` and
+    the paged-attention kernels)."""
+
+    def __init__(self, cfg: SinkAttentionConfig, width: int, eps: float, dtype, device, generator=None, prefix: str = "",
+                 out_scale: float = 1.0):
+        if cfg.heads % cfg.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if cfg.scale <= 0:
+            raise ValueError("the score scale must be positive")
+        self.cfg, self.eps, self.dtype, self.out_scale = cfg, eps, dtype, out_scale
+        big = max(cfg.dim, cfg.vdim)
+        # heads are laid out to the sizes the matrix-core kernels are built for
+        self.head_dim = -(-big // 8) * 8 if dtype != torch.bfloat16 or big > 128 else 64 if big <= 64 else 128
+        p = prefix
+        self.ins = [InBlock({p + "q": cfg.heads * cfg.dim, p + "k": cfg.kv_heads * cfg.dim, p + "v": cfg.kv_heads * cfg.vdim})]
+        self.outs = [OutBlock(p + "o", cfg.heads, cfg.vdim, self.head_dim)]
+        self.q_norm, self.k_norm = _vec(cfg.dim, dtype, device), _vec(cfg.dim, dtype, device)
+        self.sink = _vec(cfg.heads, torch.float32, device, 0.0)
+        self.slopes = None if cfg.slopes is None else torch.tensor(cfg.slopes, dtype=torch.float32, device=device)
+
+    def kv_cache_spec(self, block_size: int) -> KVCacheSpec:
+        return KVCacheSpec(block_size, self.cfg.kv_heads, self.head_dim, self.dtype)
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield p + "q.norm", self.q_norm
+        yield p + "k.norm", self.k_norm
+        yield p + "sink", self.sink
+
+    def run(self, x, y, step, memory) -> None:
+        c, md = self.cfg, step.md
+        kc, vc = memory.kv
+        q = ops.head_norm_cache(x[0], self.q_norm, self.k_norm, kc, vc, md.slot_mapping, step.positions, c.heads, c.dim, c.vdim, self.eps,
+                                c.temp_coef, c.temp_every)
+        out, nd = y[0], md.num_decodes
+        bias = dict(slopes=self.slopes, sinks=self.sink, out_scale=self.out_scale)
+        if not ops.paged_attn_bias_supported(self.dtype, self.head_dim, kc.shape[1]):
+            ops.attn_rows(out, q, kc, vc, md.block_table, md.seq_lens, md.query_start_loc, c.scale, **bias)
+            return
+        if nd:
+            ops.paged_attn_decode(out[:nd], q[:nd], kc, vc, md.block_table[:nd], md.seq_lens[:nd], md.max_seq_len, c.scale,
+                                  workspace=md.decode_workspace, **bias)
+        if nd < md.num_reqs:      # the portions' row offsets count from the step's first row, so q and out go whole
+            ops.paged_attn_prefill(out, q, kc, vc, md.block_table[nd:md.num_reqs], md.seq_lens[nd:md.num_reqs],
+                                   md.query_start_loc[nd:md.num_reqs + 1], md.max_query_len, c.scale, max_seq_len=md.max_seq_len, **bias)
+
+
+@dataclass
+class LightningConfig:
+    heads: int
+    dim: int
+    vdim: int
+    decay: list[float]
+
+
+class LightningAttention(Sublayer):
+    """Decayed linear attention, its heads normed together and gated (``csrc/lightning_attn.hip``)."""
+
+    def __init__(self, cfg: LightningConfig, width: int, eps: float, dtype, device, generator=None, prefix: str = "",
+                 out_scale: float = 1.0):
+        if len(cfg.decay) != cfg.heads or any(d <= 0 for d in cfg.decay):
+            raise ValueError(f"one positive decay per head ({cfg.heads}), got {cfg.decay}")
+        self.cfg, self.eps, self.dtype, self.out_scale = cfg, eps, dtype, out_scale
+        hd, hv = cfg.heads * cfg.dim, cfg.heads * cfg.vdim
+        p = prefix
+        self.ins = [InBlock({p + "q": hd, p + "k": hd, p + "v": hv}), InBlock({p + "g": hv})]
+        self.outs = [OutBlock(p + "o", 1, hv, hv)]
+        self.norm = _vec(hv, dtype, device)
+        self.decay = torch.tensor(cfg.decay, dtype=torch.float32, device=device)
+        self.log2_decay = torch.tensor([math.log2(d) for d in cfg.decay], dtype=torch.float32, device=device)
+
+    def state_specs(self) -> list[StateSpec]:
+        c = self.cfg
+        return [StateSpec((c.heads, c.dim, c.vdim), torch.float32)]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield p + "norm", self.norm
+
+    def run(self, x, y, step, memory) -> None:
+        md, nd = step.md, step.md.num_decodes
+        args = (x[0], x[1], self.norm, self.decay, self.log2_decay, memory.states[0], md.state_rows, md.query_start_loc, md.seq_lens,
+                self.eps, y[0])
+        if nd:
+            ops.lightning_attn(*args, 0, nd, 0, nd, 1, self.out_scale, chunked=False)
+        if nd < md.num_reqs:
+            ops.lightning_attn(*args, nd, md.num_reqs - nd, nd, x[0].shape[0] - nd, md.max_query_len, self.out_scale)
+
+
+class ParallelMixers(Sublayer):
+    """Mixers that read the same row and whose outputs (each scaled by its own ``out_scale``) add up; name -> mixer"""
+
+    def __init__(self, mixers: dict[str, Sublayer]):
+        self.mixers = mixers
+        self.ins = [b for m in mixers.values() for b in m.ins]
+        self.outs = [b for m in mixers.values() for b in m.outs]
+
+    def kv_cache_spec(self, block_size: int) -> Optional[KVCacheSpec]:
+        specs = [s for s in (m.kv_cache_spec(block_size) for m in self.mixers.values()) if s is not None]
+        if len(specs) > 1:
+            raise NotImplementedError("one of the mixers side by side may keep a KV cache")
+        return specs[0] if specs else None
+
+    def state_specs(self) -> list[StateSpec]:
+        return [s for m in self.mixers.values() for s in m.state_specs()]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        for name, m in self.mixers.items():
+            yield from m.named_weights(f"{p}{name}.")
+
+    def run(self, x, y, step, memory) -> None:
+        i = o = s = 0
+        for m in self.mixers.values():
+            ni, no, ns = len(m.ins), len(m.outs), len(m.state_specs())
+            m.run(x[i:i + ni], y[o:o + no], step, LayerMemory(memory.kv, memory.states[s:s + ns]))
+            i, o, s = i + ni, o + no, s + ns
+
+
+class DenseGlu(Sublayer):
+    """down(act(gate) * up)"""
+
+    def __init__(self, ff: int, act: str, prefix: str = ""):
+        self.ff, self.act = ff, act
+        # gate and up on 16-byte rows of their own: two blocks
+        self.ins = [InBlock({prefix + "gate": ff}), InBlock({prefix + "up": ff})]
+        self.outs = [OutBlock(prefix + "down", 1, ff, ff)]
+
+    def run(self, x, y, step, memory) -> None:
+        ops.glu(y[0], x[0], x[1], self.act)

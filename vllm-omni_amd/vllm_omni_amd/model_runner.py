@@ -30,7 +30,7 @@ import torch.nn.functional as F
 
 from . import ops
 from .block_table import MultiGroupBlockTable
-from .kv_cache import KVCacheSpec, allocate_kv_cache, allocate_latent_cache, extract_request_kv
+from .kv_cache import KVCacheSpec, allocate_kv_cache, allocate_layer_cache, extract_request_kv
 from .layers import AttentionMetadata, set_forward_context
 from .sched_output import (EMPTY_MODEL_RUNNER_OUTPUT, CachedRequestData, NewRequestData, OmniModelRunnerOutput,
                            SamplingMetadata, SamplingParams, SchedulerOutput)
@@ -580,7 +580,7 @@ class GPUARModelRunner:
         if self._token_ids:
             if self.enable_prefix_caching and self.model.is_recurrent:
                 raise ValueError("prefix caching re-uses KV blocks only: a model with recurrent layers cannot start behind them")
-            caches = {i: allocate_latent_cache(num_blocks, s, self.device) for i, s in spec.items()}
+            caches = {i: allocate_layer_cache(num_blocks, s, self.device, self.kv_layout) for i, s in spec.items()}
             self.kv_caches = list(caches.values())
             self.model.bind_kv_caches(caches)
             self.state_cache = StateCache(self.max_num_reqs, self.device)
@@ -620,7 +620,7 @@ class GPUARModelRunner:
         idx = torch.as_tensor(block_ids, dtype=torch.int64, device=self.device)
         for kv in self.kv_caches:
             from .kv_cache import normalize_layer_kv
-            if self._token_ids:
+            if isinstance(kv, torch.Tensor) and kv.dim() == 3:      # a latent cache
                 kv.index_fill_(0, idx, 0)
                 continue
             kb, vb = normalize_layer_kv(kv)

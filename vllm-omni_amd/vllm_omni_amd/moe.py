@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass
-from typing import Optional
+from typing import Iterable, Optional
 
 import torch
 import torch.nn.functional as F
@@ -100,3 +100,35 @@ class Qwen3OmniMoeSparseMoeBlock:
                 dst.copy_(w[name].to(self.dtype))
                 loaded.add(name)
         return loaded
+
+
+class RoutedExperts:
+    """Routed gated experts whose output rows the caller sums (``ops.residual_add_norm``): the ``top`` largest of the router's
+    32-bit logits (+ bias), weighted by the softmax over these alone.  Weight names: ``router``, ``router.b``, ``e<i>.gate`` /
+    ``.up`` / ``.down``."""
+
+    def __init__(self, width: int, experts: int, top: int, ff: int, dtype, device=None, generator=None):
+        if not 0 < top <= min(experts, 16) or experts > 256:
+            raise ValueError(f"{top} of {experts} experts: at most 16 of at most 256")
+        self.top, self.ff = top, ff
+        step = 64 if width % 128 == 0 else 8           # columns of zeros bring a small expert to a tile of the grouped products
+        pad = -(-ff // step) * step
+        self.router = _init_weight(experts, width, dtype, device, generator, std=width ** -0.5)
+        self.router_b = torch.zeros(experts, dtype=torch.float32, device=device)
+        self.gate_up = _init_weight(experts * 2 * pad, width, dtype, device, generator, std=width ** -0.5).view(experts, 2, pad, width)
+        self.down = _init_weight(experts * width, pad, dtype, device, generator, std=ff ** -0.5).view(experts, width, pad)
+        self.gate_up[:, :, ff:].zero_()
+        self.down[:, :, ff:].zero_()
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield p + "router", self.router
+        yield p + "router.b", self.router_b
+        for i in range(self.router.shape[0]):
+            yield f"{p}e{i}.gate", self.gate_up[i, 0, :self.ff]
+            yield f"{p}e{i}.up", self.gate_up[i, 1, :self.ff]
+            yield f"{p}e{i}.down", self.down[i, :, :self.ff]
+
+    def __call__(self, h: torch.Tensor) -> ops.ExpertRows:
+        logits = ops.moe_router_logits(h, self.router, self.router_b)
+        ids, weights, _ = ops.moe_route(logits, self.top, True, want_counts=False)
+        return ops.moe_expert_rows(h, ids, weights, self.gate_up.flatten(1, 2), self.down)

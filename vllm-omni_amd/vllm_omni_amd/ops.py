@@ -343,12 +343,19 @@ DECODE_FUSED_MERGE = os.environ.get("VLLM_OMNI_AMD_DECODE_FUSED_MERGE", "0") == 
 ROPE_DECODE_FUSION = os.environ.get("VLLM_OMNI_AMD_ROPE_DECODE_FUSION", "1") != "0"
 
 
+def _head_vectors(nq: int, *ts: Optional[torch.Tensor]) -> None:
+    for t in ts:
+        if t is not None and (t.dtype != torch.float32 or t.numel() != nq or not t.is_contiguous()):
+            raise ValueError(f"expected {nq} contiguous fp32 values, one per query head")
+
+
 def paged_attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                       block_table: torch.Tensor, seq_lens: torch.Tensor, max_seq_len: int, scale: float,
                       partition_size: int = 0, workspace: Optional[torch.Tensor] = None,
                       packed_pv: Optional[bool] = None, force_valu: bool = False,
                       nontemporal: Optional[bool] = None, rounded_p: bool = False,
-                      fused_merge: Optional[bool] = None, _skip_merge: bool = False) -> torch.Tensor:
+                      fused_merge: Optional[bool] = None, _skip_merge: bool = False, slopes: Optional[torch.Tensor] = None,
+                      sinks: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
     """out[s, h] = softmax(q[s,h] . K^T * scale) . V over the paged cache (one query per sequence).
 
     q, out: [S, nq*d] (or [S, nq, d]); block_table int32 [S, max_blocks]; seq_lens int32 [S].
@@ -360,8 +367,10 @@ def paged_attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
     P of flash kernels (A/B measurements only).  ``fused_merge`` (None = on for workspaces made by
     ``new_decode_workspace``): the context partitions are merged inside the attention launch by the last-arriving
     wave of each (sequence, head group) instead of a second kernel — same bits.  Returns ``out``.
+    ``slopes`` / ``sinks`` (fp32 [nq]): a distance bias (score - slope * (position - key position)) and one more term
+    exp(sink) of the softmax's denominator, and the output times ``out_scale``; bf16 and the default mode only.
     """
-    _gpu(out, q, k_cache, v_cache, block_table, seq_lens, workspace)
+    _gpu(out, q, k_cache, v_cache, block_table, seq_lens, workspace, slopes, sinks)
     nb, bs, hkv, d = k_cache.shape
     s = q.shape[0]
     nq = q.numel() // (s * d) if s else 0
@@ -381,6 +390,17 @@ def paged_attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         fused_merge = DECODE_FUSED_MERGE and ready
     elif fused_merge and not ready:
         raise ValueError("fused_merge needs a workspace from ops.new_decode_workspace (zeroed arrival counters)")
+    if slopes is None and sinks is None and out_scale != 1.0:
+        raise ValueError("out_scale goes with a distance bias or a sink")
+    if slopes is not None or sinks is not None:
+        _head_vectors(nq, slopes, sinks)
+        if force_valu or rounded_p or packed_pv is False or out.dtype != q.dtype:
+            raise ValueError("a distance bias or a sink runs in the default mode only")
+        check("mi_paged_attn_decode_biased", lib.mi_paged_attn_decode_biased(
+            _p(out), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(seq_lens), _p(slopes), _p(sinks), float(out_scale), s, nq, hkv, d, bs,
+            block_table.stride(0), int(max_seq_len), float(scale), q.stride(0), out.stride(0), cb, ct, ch, int(partition_size),
+            _p(workspace), workspace.numel() * workspace.element_size() if workspace is not None else 0, _dt(q.dtype), _stream()))
+        return out
     check("mi_paged_attn_decode", lib.mi_paged_attn_decode(
         _p(out), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(seq_lens), s, nq, hkv, d, bs,
         block_table.stride(0), int(max_seq_len), float(scale), q.stride(0), out.stride(0), cb, ct, ch,
@@ -458,14 +478,16 @@ _PREFILL_WS: dict = {}   # device -> grow-only fp32 workspace of the split-conte
 def paged_attn_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                        block_table: torch.Tensor, seq_lens: torch.Tensor, query_start_loc: torch.Tensor,
                        max_query_len: int, scale: float, max_seq_len: Optional[int] = None,
-                       segments: int = 0) -> torch.Tensor:
+                       segments: int = 0, slopes: Optional[torch.Tensor] = None,
+                       sinks: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
     """Varlen causal attention of query chunks against the paged cache (chunked prefill).
 
     ``max_seq_len`` (host upper bound of ``seq_lens``) lets a launch that would leave most CUs idle — the ragged last
     chunk of a long prompt, a TP shard with one KV head — split every tile's context into segments run by separate
     workgroups and merged afterwards (``mi_paged_attn_prefill_split``).  Without it nothing is split.
-    ``segments``: 0 automatic, 1 never, n > 1 force n (tests)."""
-    _gpu(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc)
+    ``segments``: 0 automatic, 1 never, n > 1 force n (tests).  ``slopes`` / ``sinks`` /
+    ``out_scale``: as in ``paged_attn_decode``."""
+    _gpu(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, slopes, sinks)
     nb, bs, hkv, d = k_cache.shape
     t = q.shape[0]
     nq = q.numel() // (t * d) if t else 0
@@ -481,11 +503,16 @@ def paged_attn_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor
             ws = _PREFILL_WS.get(q.device)
             if ws is None or ws.numel() * 4 < ws_bytes:
                 ws = _PREFILL_WS[q.device] = torch.empty((ws_bytes + 3) // 4, dtype=torch.float32, device=q.device)
-    check("mi_paged_attn_prefill_split", lib.mi_paged_attn_prefill_split(
-        _p(out), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(seq_lens), _p(query_start_loc),
-        s, t, int(max_query_len), nq, hkv, d, bs, block_table.stride(0), float(scale),
-        q.stride(0), out.stride(0), cb, ct, ch, _dt(q.dtype), msl, int(segments) if ws is not None else 1,
-        _p(ws) if ws is not None else None, ws.numel() * 4 if ws is not None else 0, _stream()))
+    tail = (s, t, int(max_query_len), nq, hkv, d, bs, block_table.stride(0), float(scale), q.stride(0), out.stride(0), cb, ct, ch,
+            _dt(q.dtype), msl, int(segments) if ws is not None else 1, _p(ws), ws.numel() * 4 if ws is not None else 0, _stream())
+    head = (_p(out), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(seq_lens), _p(query_start_loc))
+    if slopes is not None or sinks is not None:
+        _head_vectors(nq, slopes, sinks)
+        check("mi_paged_attn_prefill_biased", lib.mi_paged_attn_prefill_biased(*head, _p(slopes), _p(sinks), float(out_scale), *tail))
+    else:
+        if out_scale != 1.0:
+            raise ValueError("out_scale goes with a distance bias or a sink")
+        check("mi_paged_attn_prefill_split", lib.mi_paged_attn_prefill_split(*head, *tail))
     return out
 
 
@@ -1023,6 +1050,15 @@ def moe_route(router_logits: torch.Tensor, top_k: int, norm_topk_prob: bool, rou
     return ids, w, counts
 
 
+def _moe_align(ids: torch.Tensor, num_experts: int, max_rows: int, rows_per_tile: int):
+    """(token, choice) pairs grouped by expert in tiles: -> sorted_pairs, row_of_pair, tile_expert, num_tiles"""
+    i32 = dict(dtype=torch.int32, device=ids.device)
+    out = (torch.empty(max_rows, **i32), torch.empty(ids.numel(), **i32), torch.empty(max_rows // rows_per_tile, **i32),
+           torch.empty(1, **i32))
+    check("mi_moe_align", lib.mi_moe_align(*map(_p, out), _p(ids), None, ids.numel(), num_experts, max_rows, rows_per_tile, _stream()))
+    return out
+
+
 def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, top_k: int,
               norm_topk_prob: bool = False, shared_out: Optional[torch.Tensor] = None,
               shared_gate_weight: Optional[torch.Tensor] = None, routing=None,
@@ -1039,17 +1075,9 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gate_up: torch.Ten
         ids, w, _ = moe_route(router_logits, top_k, norm_topk_prob, round_to=x.dtype, want_counts=False)
     else:
         ids, w = routing
-    counts = None     # mi_moe_align derives the per-expert counts from the ids
-    pairs = t * top_k
     rpt = rows_per_tile or int(lib.mi_moe_rows_per_tile(t, top_k, e))
     max_rows = int(lib.mi_moe_max_rows(t, top_k, e, rpt))
-    i32 = dict(dtype=torch.int32, device=dev)
-    sorted_pairs = torch.empty(max_rows, **i32)
-    row_of_pair = torch.empty(pairs, **i32)
-    tile_expert = torch.empty(max_rows // rpt, **i32)
-    num_tiles = torch.empty(1, **i32)
-    check("mi_moe_align", lib.mi_moe_align(_p(sorted_pairs), _p(row_of_pair), _p(tile_expert), _p(num_tiles), _p(ids),
-                                           _p(counts), pairs, e, max_rows, rpt, _stream()))
+    sorted_pairs, row_of_pair, tile_expert, num_tiles = _moe_align(ids, e, max_rows, rpt)   # counts the ids itself
     act = torch.empty(max_rows, i, dtype=x.dtype, device=dev)
     part = torch.empty(max_rows, h, dtype=x.dtype, device=dev)
     dt = _dt(x.dtype)
@@ -1309,52 +1337,289 @@ def latent_prefill(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, vt: torc
 def gated_delta_step(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor,
                      state: torch.Tensor, ring: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
                      seq_lens: torch.Tensor, kv_heads: int, eps: float, out: torch.Tensor, req0: int, num_reqs: int,
-                     update_ring: bool = True) -> torch.Tensor:
+                     update_ring: bool = True, gate: Optional[torch.Tensor] = None, beta: Optional[torch.Tensor] = None,
+                     decay: Optional[torch.Tensor] = None, sigmoid_gate: bool = False) -> torch.Tensor:
     """Gated delta rule of requests [req0, req0 + num_reqs), token by token.  ``state`` fp32 [slots, H, D, V], ``ring``
-    [slots, taps, channels]; ``out`` [T, H * V] receives the requests' rows."""
-    ps, hh, d, v, taps = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
-                                     kv_heads, out, req0, num_reqs)
-    check("mi_gated_delta_step", lib.mi_gated_delta_step(
-        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
-        _p(seq_lens), _p(out), req0, num_reqs, hh, kv_heads, d, v, taps, float(eps), int(update_ring), _dt(proj.dtype), _stream()))
+    [slots, taps, channels]; ``out`` [T, H * V] receives the requests' rows.  ``proj`` holds rows q | k | v, and behind them
+    gate | b | a where these do not come as tensors of their own; ``decay`` [T, H] or, one per key channel, [T, H * D]
+    (``dt_bias`` has as many)."""
+    a = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads, eps, out, req0,
+                    num_reqs, gate, beta, decay, sigmoid_gate)
+    check("mi_gated_delta_step", lib.mi_gated_delta_step(ctypes.byref(a), int(update_ring), _dt(proj.dtype), _stream()))
     return out
 
 
 def gated_delta_chunked(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads: int,
-                        eps: float, out: torch.Tensor, req0: int, num_reqs: int, row0: int, max_query_len: int) -> torch.Tensor:
+                        eps: float, out: torch.Tensor, req0: int, num_reqs: int, row0: int, max_query_len: int, gate=None, beta=None,
+                        decay=None, sigmoid_gate: bool = False) -> torch.Tensor:
     """The same for prompt portions (requests [req0, req0 + num_reqs) own the rows from ``row0`` to the end of ``proj``), 64
     tokens at a time on the fp32 matrix cores; sizes outside its envelope (dim or vdim > 256) go token by token."""
-    ps, hh, d, v, taps = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens,
-                                     kv_heads, out, req0, num_reqs)
+    a = _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads, eps, out, req0,
+                    num_reqs, gate, beta, decay, sigmoid_gate)
     rows = proj.shape[0] - row0
-    need = lib.mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, hh, d, v)
+    need = lib.mi_gated_delta_chunked_workspace_bytes(rows, num_reqs, a.heads, a.dim, a.vdim, a.channel_decay)
     if not need:
-        return gated_delta_step(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads,
-                                eps, out, req0, num_reqs)
+        check("mi_gated_delta_step", lib.mi_gated_delta_step(ctypes.byref(a), 1, _dt(proj.dtype), _stream()))
+        return out
     ws = torch.empty(need, dtype=torch.uint8, device=proj.device)
-    check("mi_gated_delta_chunked", lib.mi_gated_delta_chunked(
-        _p(proj), ps, _p(conv_w), _p(a_log), _p(dt_bias), _p(norm_w), _p(state), _p(ring), _p(slots), _p(query_start_loc),
-        _p(seq_lens), _p(out), row0, rows, req0, num_reqs, max_query_len, hh, kv_heads, d, v, taps, float(eps), _p(ws),
-        need, _dt(proj.dtype), _stream()))
+    check("mi_gated_delta_chunked", lib.mi_gated_delta_chunked(ctypes.byref(a), row0, rows, max_query_len, _p(ws), need,
+                                                               _dt(proj.dtype), _stream()))
     return out
 
 
-def _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads, out, req0, num_reqs):
-    _gpu(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, out)
+def _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, kv_heads, eps, out, req0, num_reqs,
+                gate, beta, decay, sigmoid_gate) -> "_C.GatedDeltaArgs":
+    _gpu(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_start_loc, seq_lens, out, gate, beta, decay)
     _i32(slots, query_start_loc, seq_lens)
     ps, cols = _rows(proj)
+    os_, oc = _rows(out)
     _, hh, d, v = state.shape
     taps, ch = ring.shape[1], ring.shape[2]
-    if cols < ch + hh * v + 2 * hh or out.shape[0] < proj.shape[0]:
+    at = ch                       # what is not given apart follows q | k | v in the rows of ``proj``
+    views = []
+    for t, n in ((gate, hh * v), (beta, hh), (decay, hh)):
+        if t is None:
+            t = proj[:, at:at + n]
+            at += n
+        views.append(t)
+    gate, beta, decay = views
+    channel = d > 1 and decay.shape[1] == hh * d      # one key channel: the same thing
+    if cols < at or out.shape[0] < proj.shape[0]:
         raise ValueError("gated_delta: projection rows [q | k | v | gate | b | a], one output row each")
-    if not (state.is_contiguous() and ring.is_contiguous() and conv_w.is_contiguous() and out.is_contiguous()):
-        raise ValueError("gated_delta_step: contiguous state, ring, conv weights and output")
+    if not (state.is_contiguous() and ring.is_contiguous() and conv_w.is_contiguous()):
+        raise ValueError("gated_delta: contiguous state, ring and conv weights")
     if state.dtype != torch.float32 or a_log.dtype != torch.float32 or dt_bias.dtype != torch.float32:
         raise TypeError("recurrent state, A_log and dt_bias are fp32")
-    if ch != 2 * kv_heads * d + hh * v or tuple(conv_w.shape) != (ch, taps) or out.shape[1] != hh * v or norm_w.numel() != v:
-        raise ValueError("gated_delta_step: sizes do not fit")
-    if any(t.dtype != proj.dtype for t in (conv_w, norm_w, ring, out)):
-        raise TypeError("gated_delta_step: one activation dtype")
+    if (ch != 2 * kv_heads * d + hh * v or tuple(conv_w.shape) != (ch, taps) or oc != hh * v or norm_w.numel() != v
+            or a_log.numel() != hh or dt_bias.numel() != (hh * d if channel else hh)):
+        raise ValueError("gated_delta: sizes do not fit")
+    if any(t.shape[0] < proj.shape[0] or t.stride(1) != 1 or t.shape[1] != n
+           for t, n in ((gate, hh * v), (beta, hh), (decay, hh * d if channel else hh))):
+        raise ValueError("gated_delta: gate, b and decay rows do not fit")
+    if any(t.dtype != proj.dtype for t in (conv_w, norm_w, ring, out, gate, beta, decay)):
+        raise TypeError("gated_delta: one activation dtype")
     if req0 + num_reqs > seq_lens.shape[0] or slots.shape[0] < req0 + num_reqs or query_start_loc.shape[0] < req0 + num_reqs + 1:
-        raise ValueError("gated_delta_step: request range outside the metadata")
-    return ps, hh, d, v, taps
+        raise ValueError("gated_delta: request range outside the metadata")
+    return _C.GatedDeltaArgs(_p(proj), _p(gate), _p(beta), _p(decay), _p(conv_w), _p(norm_w), _p(a_log), _p(dt_bias), _p(state), _p(ring),
+                             _p(slots), _p(query_start_loc), _p(seq_lens), _p(out), ps, gate.stride(0), beta.stride(0), decay.stride(0),
+                             os_, req0, num_reqs, hh, kv_heads, d, v, taps, int(channel), int(sigmoid_gate), float(eps))
+
+
+# ------------------------------------------------- layers with mixer and feed-forward side by side
+class ExpertRows:
+    """Output rows of routed experts, one per (token, choice), and how they sum up: ``residual_add_norm`` does it."""
+
+    def __init__(self, part: torch.Tensor, weights: torch.Tensor, row_of_pair: Optional[torch.Tensor]):
+        self.part, self.weights, self.row_of_pair = part, weights, row_of_pair
+
+
+def residual_add_norm(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials"], w_pre: Optional[torch.Tensor], eps: float,
+                      h: torch.Tensor, experts: Optional[ExpertRows] = None, w_shift: float = 0.0, start: bool = False) -> torch.Tensor:
+    """``x += y (+ the experts' rows)`` in place (x fp32 [T, W]; ``start``: x = y instead), then ``h`` = x / rms(x) * (w_pre +
+    w_shift), or x cast when ``w_pre`` is None.  ``y``: rows of h's dtype, fp32 rows, or split-K partials."""
+    part = isinstance(y, SplitKPartials)
+    if part:
+        y._live()
+        if y.bias is not None:
+            raise ValueError("residual_add_norm takes partials of a linear without bias")
+    src = y.part if part else y
+    _gpu(x, src, w_pre, h)
+    xs, width = _rows(x)
+    hs, hw = _rows(h)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or hw != width or h.shape[0] < rows or (w_pre is not None and (w_pre.numel() != width or w_pre.dtype != h.dtype)):
+        raise ValueError("residual_add_norm: fp32 stream, h and weights of its width")
+    if part:
+        if (y.m, y.n) != (rows, width):
+            raise ValueError("partials of another shape")
+        split, ys = y.split, width
+    else:
+        ys, yw = _rows(y)
+        if y.shape[0] != rows or yw != width or y.dtype not in (h.dtype, torch.float32):
+            raise ValueError("layer output of another shape or dtype")
+        split = 1 if y.dtype == torch.float32 and h.dtype != torch.float32 else 0
+    top, rp, ww, ps, prt = 0, None, None, 0, None
+    if experts is not None:
+        prt, rp, ww = experts.part, experts.row_of_pair, experts.weights
+        _gpu(prt, rp, ww)
+        ps, pw = _rows(prt)
+        top = ww.shape[1]
+        if pw != width or prt.dtype != h.dtype or ww.shape[0] != rows or ww.dtype != torch.float32 or not ww.is_contiguous():
+            raise ValueError("expert rows of another shape or dtype")
+        if rp is None and prt.shape[0] < rows * top:
+            raise ValueError("one row per pair expected")
+        _i32(rp)
+    check("mi_residual_add_norm", lib.mi_residual_add_norm(
+        _p(x), _p(src), split, _p(prt), _p(rp), _p(ww), top, _p(w_pre), float(w_shift), _p(h), int(start), float(eps), rows, width, xs,
+        ys, hs, ps, _dt(h.dtype), _stream()))
+    return h
+
+
+def embed_norm(table: torch.Tensor, ids: torch.Tensor, x: torch.Tensor, w_pre: Optional[torch.Tensor], eps: float, h: torch.Tensor,
+               copy: Optional[torch.Tensor] = None, w_shift: float = 0.0) -> None:
+    """x = table[ids] (fp32), ``copy`` = the same in the table's dtype, ``h`` as in ``residual_add_norm``"""
+    _gpu(table, ids, x, w_pre, h, copy)
+    _i64(ids)
+    xs, width = _rows(x)
+    hs, hw = _rows(h)
+    cs, cw = _rows(copy) if copy is not None else (0, width)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or not table.is_contiguous() or (table.shape[1], hw, cw) != (width,) * 3 or ids.numel() != rows:
+        raise ValueError("embed_norm: sizes do not fit")
+    if h.shape[0] < rows or (copy is not None and copy.shape[0] < rows) or (w_pre is not None and w_pre.numel() != width):
+        raise ValueError("embed_norm: sizes do not fit")
+    if any(t is not None and t.dtype != table.dtype for t in (h, copy, w_pre)):
+        raise TypeError("embed_norm: one dtype")
+    check("mi_embed_norm", lib.mi_embed_norm(_p(x), _p(h), _p(copy), _p(table), _p(w_pre), float(w_shift), _p(ids), float(eps), rows, width,
+                                             table.shape[0], xs, hs, cs, _dt(table.dtype), _stream()))
+
+
+def glu(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, act: str) -> torch.Tensor:
+    """``out = act(gate) * up``; act "silu" or "gelu_tanh".  gate and up are column blocks of one matrix."""
+    _gpu(out, gate, up)
+    gs, ff = _rows(gate)
+    us, uf = _rows(up)
+    os_, of = _rows(out)
+    if gs != us or not ff == uf == of or not gate.shape[0] == up.shape[0] == out.shape[0] or not gate.dtype == up.dtype == out.dtype:
+        raise ValueError("glu: gate, up and out of one shape, gate and up of one row stride")
+    check("mi_glu", lib.mi_glu(_p(out), _p(gate), _p(up), gate.shape[0], ff, gs, os_,
+                               {"silu": _C.MI_ACT_SILU, "gelu_tanh": _C.MI_ACT_GELU_TANH}[act], _dt(gate.dtype), _stream()))
+    return out
+
+
+def head_norm_cache(x: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], k_cache: torch.Tensor,
+                    v_cache: torch.Tensor, slot_mapping: torch.Tensor, positions: torch.Tensor, num_q_heads: int, dim: int, vdim: int,
+                    eps: float, temp_coef: float = 0.0, temp_every: int = 1) -> torch.Tensor:
+    """Rows q | k | v: per-head norms, the query temperature, K / V cache write; returns q, heads laid out as in the cache."""
+    _gpu(x, q_weight, k_weight, k_cache, v_cache, slot_mapping, positions)
+    _i64(slot_mapping, positions)
+    xs, cols = _rows(x)
+    rows = x.shape[0]
+    _, bs, g, hd = k_cache.shape
+    cb, ct, ch = _cache_strides(k_cache, v_cache)
+    if cols != (num_q_heads + g) * dim + g * vdim or slot_mapping.numel() < rows or positions.numel() < rows:
+        raise ValueError("head_norm_cache: sizes do not fit")
+    for w in (q_weight, k_weight):
+        if w is not None and (w.numel() != dim or w.dtype != x.dtype):
+            raise ValueError("head_norm_cache: norm weights of one head's size")
+    if x.dtype != k_cache.dtype:
+        raise TypeError("cache and activations share a dtype")
+    q = torch.empty(rows, num_q_heads * hd, dtype=x.dtype, device=x.device)
+    check("mi_head_norm_cache", lib.mi_head_norm_cache(
+        _p(x), xs, _p(q_weight), _p(k_weight), _p(q), q.stride(0), _p(k_cache), _p(v_cache), _p(slot_mapping), _p(positions), rows,
+        num_q_heads, g, dim, vdim, hd, bs, cb, ct, ch, float(temp_coef), int(temp_every), float(eps), _dt(x.dtype), _stream()))
+    return q
+
+
+def attn_rows(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+              seq_lens: torch.Tensor, query_start_loc: torch.Tensor, scale: float, slopes: Optional[torch.Tensor] = None,
+              sinks: Optional[torch.Tensor] = None, row0: int = 0, out_scale: float = 1.0) -> torch.Tensor:
+    """Causal attention of rows [row0, T), any sizes and types; ``slopes`` / ``sinks`` as in ``paged_attn_decode``."""
+    _gpu(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, slopes, sinks)
+    _i32(seq_lens, query_start_loc)
+    _, bs, g, hd = k_cache.shape
+    cb, ct, ch = _cache_strides(k_cache, v_cache)
+    qs, qc = _rows(q)
+    os_, oc = _rows(out)
+    nq = qc // hd
+    if qc != nq * hd or oc != qc or out.shape[0] < q.shape[0] or block_table.dtype != torch.int32 or block_table.stride(1) != 1:
+        raise ValueError("attn_rows: sizes do not fit")
+    if not q.dtype == out.dtype == k_cache.dtype:
+        raise TypeError("attn_rows: one dtype")
+    _head_vectors(nq, slopes, sinks)
+    check("mi_attn_rows", lib.mi_attn_rows(
+        _p(out), _p(q), _p(k_cache), _p(v_cache), _p(block_table), _p(seq_lens), _p(query_start_loc), _p(slopes), _p(sinks), float(out_scale), row0,
+        q.shape[0] - row0, seq_lens.shape[0], nq, g, hd, bs, float(scale), qs, os_, cb, ct, ch, block_table.stride(0), _dt(q.dtype),
+        _stream()))
+    return out
+
+
+def paged_attn_bias_supported(dtype: torch.dtype, head_dim: int, block_size: int) -> bool:
+    """whether the matrix-core paged-attention kernels take a distance bias and a sink at these sizes"""
+    return dtype == torch.bfloat16 and head_dim in (64, 128) and block_size >= 16 and block_size & (block_size - 1) == 0
+
+
+def lightning_attn(qkv: torch.Tensor, gate: torch.Tensor, norm_w: torch.Tensor, decay: torch.Tensor, log2_decay: torch.Tensor,
+                   state: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor, seq_lens: torch.Tensor, eps: float,
+                   out: torch.Tensor, req0: int, num_reqs: int, row0: int, rows: int, max_query_len: int, mul: float = 1.0,
+                   chunked: bool = True) -> torch.Tensor:
+    """Decayed linear attention of requests [req0, req0 + num_reqs), which own rows [row0, row0 + rows).  ``state`` fp32 [slots,
+    H, D, V]; ``chunked``: 64 tokens at a time (sizes outside that form go token by token)."""
+    _gpu(qkv, gate, norm_w, decay, log2_decay, state, slots, query_start_loc, seq_lens, out)
+    _i32(slots, query_start_loc, seq_lens)
+    ps, cols = _rows(qkv)
+    gs, gc = _rows(gate)
+    os_, oc = _rows(out)
+    _, hh, d, v = state.shape
+    if cols != hh * (2 * d + v) or gc != hh * v or oc != hh * v or norm_w.numel() != hh * v or decay.numel() != hh or log2_decay.numel() != hh:
+        raise ValueError("lightning_attn: sizes do not fit")
+    if any(t.dtype != torch.float32 for t in (state, decay, log2_decay)) or not state.is_contiguous():
+        raise TypeError("lightning_attn: contiguous fp32 state and decays")
+    if any(t.dtype != qkv.dtype for t in (gate, norm_w, out)):
+        raise TypeError("lightning_attn: one activation dtype")
+    if min(qkv.shape[0], gate.shape[0], out.shape[0]) < row0 + rows:
+        raise ValueError("lightning_attn: rows outside the tensors")
+    if req0 + num_reqs > seq_lens.shape[0] or slots.shape[0] < req0 + num_reqs or query_start_loc.shape[0] < req0 + num_reqs + 1:
+        raise ValueError("lightning_attn: request range outside the metadata")
+    need = lib.mi_lightning_workspace_bytes(rows, num_reqs, hh, d, v, 1) if chunked else 0
+    chunked = need > 0
+    if not chunked:
+        need = lib.mi_lightning_workspace_bytes(rows, num_reqs, hh, d, v, 0)
+    ws = torch.empty(max(need, 1), dtype=torch.uint8, device=qkv.device)
+    a = _C.LightningArgs(_p(qkv), _p(gate), _p(norm_w), _p(decay), _p(log2_decay), _p(state), _p(slots), _p(query_start_loc), _p(seq_lens),
+                         _p(out), ps, gs, os_, req0, num_reqs, hh, d, v, float(eps), float(mul))
+    check("mi_lightning_attn", lib.mi_lightning_attn(ctypes.byref(a), row0, rows, max_query_len, int(chunked), _p(ws), need,
+                                                     _dt(qkv.dtype), _stream()))
+    return out
+
+
+def moe_router_logits(h: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor]) -> torch.Tensor:
+    """fp32 logits h weight^T + bias of bf16 rows (fp32 sums; fp32 rows take the library product)"""
+    _gpu(h, weight, bias)
+    hs, k = _rows(h)
+    if h.dtype == torch.float32 or k % 8 or hs % 8:
+        y = torch.nn.functional.linear(h.float(), weight.float())
+        return y if bias is None else y + bias
+    if weight.dtype != h.dtype or h.dtype != torch.bfloat16 or not weight.is_contiguous() or weight.shape[1] != k:
+        raise ValueError("moe_router_logits: contiguous bf16 weight of the rows' width")
+    if bias is not None:
+        _head_vectors(weight.shape[0], bias)
+    out = torch.empty(h.shape[0], weight.shape[0], dtype=torch.float32, device=h.device)
+    check("mi_moe_router_logits", lib.mi_moe_router_logits(_p(out), _p(h), _p(weight), _p(bias), h.shape[0], weight.shape[0], k, hs,
+                                                           _stream()))
+    return out
+
+
+def moe_expert_rows(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor,
+                    w_down: torch.Tensor) -> ExpertRows:
+    """Gated (silu) experts on the rows routed to them, not yet summed: grouped matrix-core products where the sizes allow,
+    the any-size kernel (fp32, odd sizes) elsewhere."""
+    _gpu(x, ids, weights, w_gate_up, w_down)
+    _i32(ids)
+    t, h = x.shape
+    top = ids.shape[1]
+    e, two_i, k = w_gate_up.shape
+    i = two_i // 2
+    xs = _rows(x)[0]
+    if k != h or tuple(w_down.shape) != (e, h, i) or not w_gate_up.is_contiguous() or not w_down.is_contiguous() or w_gate_up.dtype != x.dtype:
+        raise ValueError("moe_expert_rows: expert weights do not fit")
+    dt, dev = _dt(x.dtype), x.device
+    if x.dtype == torch.bfloat16 and h % 8 == 0 and i % 8 == 0 and xs % 8 == 0:
+        guard = h % 128 or i % 64
+        rpt = int(lib.mi_moe_rows_per_tile(t, top, e))
+        rpt = min(rpt, 64) if guard else rpt
+        max_rows = int(lib.mi_moe_max_rows(t, top, e, rpt))
+        sorted_pairs, row_of_pair, tile_expert, num_tiles = _moe_align(ids, e, max_rows, rpt)
+        act = torch.empty(max_rows, i, dtype=x.dtype, device=dev)
+        part = torch.empty(max_rows, h, dtype=x.dtype, device=dev)
+        for out, a, w, gated, n, kk in ((act, x, w_gate_up, 1, i, h), (part, act, w_down, 0, h, i)):
+            check("mi_moe_expert_gemm", lib.mi_moe_expert_gemm(
+                _p(out), _p(a), _p(w), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, gated, n, kk, top, a.stride(0),
+                out.stride(0), w.stride(0), rpt, dt, _stream()))
+        return ExpertRows(part, weights, row_of_pair)
+    act = torch.empty(t * top, i, dtype=x.dtype, device=dev)
+    part = torch.empty(t * top, h, dtype=x.dtype, device=dev)
+    for out, a, w, gated, n, kk in ((act, x, w_gate_up, 1, i, h), (part, act, w_down, 0, h, i)):
+        check("mi_moe_pair_gemm", lib.mi_moe_pair_gemm(_p(out), _p(a), _p(w), _p(ids), t * top, e, gated, n, kk, top, a.stride(0),
+                                                       out.stride(0), w.stride(0), dt, _stream()))
+    return ExpertRows(part, weights, None)

@@ -17,6 +17,7 @@ from .compat import _get
 ARCHITECTURES = {
     "Qwen2_5OmniTalkerForConditionalGeneration": ("talker", "TalkerConfig", "Qwen2_5OmniTalkerForConditionalGeneration"),
     "Dogulorn": ("dogulorn", "DogulornConfig", "DogulornForCausalLM"),
+    "Pupopel": ("pupopel", "PupopelConfig", "PupopelForCausalLM"),
 }
 DEFAULT_ARCHITECTURE = "Qwen2_5OmniTalkerForConditionalGeneration"
 
@@ -51,9 +52,26 @@ def config_from_hf(hf: Any):
     return _load(arch, 1).from_dict(hf if isinstance(hf, dict) else hf.to_dict())
 
 
+def checkpoint_shapes(path: str) -> dict[str, tuple[int, ...]]:
+    """name -> shape of every tensor in a folder's ``*.safetensors`` files (headers only)"""
+    from safetensors import safe_open
+
+    out = {}
+    for name in sorted(f for f in os.listdir(path) if f.endswith(".safetensors")):
+        with safe_open(os.path.join(path, name), framework="pt") as f:
+            out.update((key, tuple(f.get_slice(key).get_shape())) for key in f.keys())
+    return out
+
+
 def config_from_dir(path: str):
+    """Configuration of a checkpoint folder.  A class with ``from_checkpoint`` also sees the tensors' shapes: its
+    ``config.json`` does not give every size."""
     with open(os.path.join(path, "config.json")) as f:
-        return config_from_hf(json.load(f))
+        d = json.load(f)
+    cls = _load(architecture_of(d), 1)
+    if hasattr(cls, "from_checkpoint"):
+        return cls.from_checkpoint(d, checkpoint_shapes(path))
+    return config_from_hf(d)
 
 
 def model_class_for(config: Any):
