@@ -242,12 +242,19 @@ def test_argument_validation_without_gpu():
     assert lib.mi_latent_decode(p, p, p, p, p, 1, 4, 64, 16, 4096, 4096, 1.0, 1024, 64, 4, p, need - 1, None) == _C.MI_ERR_WORKSPACE
     assert lib.mi_latent_prefill(p, p, p, p, p, p, p, 1, 8, 2, 12, 16, 8, 1.0, 32, 24, 24, 64, None) == _C.MI_ERR_UNSUPPORTED
     # heads that do not divide, a projection row too short, a workspace too small
-    assert lib.mi_gated_delta_step(p, 400, p, p, p, p, p, p, p, p, p, p, 0, 1, 3, 2, 16, 16, 4, 1e-6, 1, 1, None) == bad
-    assert lib.mi_gated_delta_step(p, 100, p, p, p, p, p, p, p, p, p, p, 0, 1, 4, 2, 16, 16, 4, 1e-6, 1, 1, None) == bad
-    assert lib.mi_gated_delta_chunked_workspace_bytes(64, 1, 4, 300, 64) == 0
-    ws = lib.mi_gated_delta_chunked_workspace_bytes(64, 1, 4, 64, 64)
-    assert lib.mi_gated_delta_chunked(p, 400, p, p, p, p, p, p, p, p, p, p, 0, 64, 0, 1, 64, 4, 2, 64, 64, 4, 1e-6, p, ws - 1, 1,
-                                      None) == _C.MI_ERR_WORKSPACE
+    def delta(**kw):
+        n = [f for f, t in _C.GatedDeltaArgs._fields_ if t is ctypes.c_void_p]
+        a = _C.GatedDeltaArgs(**{**dict.fromkeys(n, p), **dict(qkv_stride=400, gate_stride=400, beta_stride=400, decay_stride=400,
+                              out_stride=400, num_reqs=1, heads=4, kv_heads=2, dim=16, vdim=16, taps=4, eps=1e-6), **kw})
+        return ctypes.byref(a)
+
+    assert lib.mi_gated_delta_step(delta(kv_heads=3), 1, 1, None) == bad
+    assert lib.mi_gated_delta_step(delta(qkv_stride=100), 1, 1, None) == bad
+    assert lib.mi_gated_delta_step(delta(channel_decay=1, decay_stride=32), 1, 1, None) == bad
+    assert lib.mi_gated_delta_chunked_workspace_bytes(64, 1, 4, 300, 64, 0) == 0
+    assert lib.mi_gated_delta_chunked_workspace_bytes(64, 1, 4, 136, 64, 1) == 0
+    ws = lib.mi_gated_delta_chunked_workspace_bytes(64, 1, 4, 64, 64, 0)
+    assert lib.mi_gated_delta_chunked(delta(dim=64, vdim=64, qkv_stride=600), 0, 64, 64, p, ws - 1, 1, None) == _C.MI_ERR_WORKSPACE
     assert lib.mi_linear_clamped_glu(p, p, p, 1, 16, 64, 64, 16, 0.0, 1.0, 1, None) == bad
 
 

@@ -10,7 +10,7 @@
 //   * scan (one workgroup per request, head and 16 value columns): chunk after chunk, U, O and S with S in registers;
 //   * finish: o / rms(o) * norm * gate.
 // With one decay per key channel G_i is a vector: e^(G_i) and e^(G_C - G_i) scale the columns of K and Q, and A and P take
-// sum_d k_id e^(G_id - G_jd) k_jd, whose exponential is split at a row between j and i so that no factor exceeds one.
+// sum_d k_id e^(G_id - G_jd) k_jd, whose exponential is split between j and i so that no factor exceeds one.
 // All products run on v_mfma_f32_16x16x4_f32: q, k, decays and state are 32-bit quantities of the recurrence.  The k order
 // inside 16 consecutive k is permuted alike in both operands (step s takes k = 4 (lane / 16) + s), so an operand whose k is
 // contiguous is one 16-byte read for four steps, and an accumulator tile IS the B operand of a following product.
@@ -139,23 +139,31 @@ __device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul)
 }
 
 // A and P of one 16 x 16 tile (rows ti, columns tj < ti) with a decay per key channel.  e^(G_i - G_j) is split at the tile's
-// first row r: e^(G_i - G_r) on the row's side, e^(G_r - G_j) on the column's; both exponents are <= 0 (G falls with time).
-// gk, gq, gG: [C][ld] keys, queries, G in log2.
-__device__ __forceinline__ void channel_tile(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti, int tj, int lane,
-                                             f32x4_t& aA, f32x4_t& aP) {
+// entry: e^(sum of the row's tile up to i) on the row's side, what is left of tile tj behind j and the tiles between on the
+// column's; all of these are sums of log decays, <= 0.  kb, qb, gb: [C][ld] keys, queries, log2 decays summed from the
+// start of each 16-row tile (sums over a whole chunk would leave differences of large numbers).
+__device__ __forceinline__ void channel_tile(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti,
+                                             int tj, int lane, f32x4_t& aA, f32x4_t& aP) {
   for (int k = 0; k < Dp; k += 16) {
-    float kf[4], qf[4], gf[4], cf[4], hf[4], rf[4];
+    float kf[4], qf[4], gf[4], cf[4], hf[4], lf[4], bf[4];
     frag_rows(kb + ti * 16 * ld + k, ld, lane, kf);
     frag_rows(qb + ti * 16 * ld + k, ld, lane, qf);
     frag_rows(gb + ti * 16 * ld + k, ld, lane, gf);
     frag_rows(kb + tj * 16 * ld + k, ld, lane, cf);
     frag_rows(gb + tj * 16 * ld + k, ld, lane, hf);
-    frag_rows(gb + ti * 16 * ld + k, 0, lane, rf);
+    frag_rows(gb + (tj * 16 + 15) * ld + k, 0, lane, lf);
+    for (int s = 0; s < 4; ++s) bf[s] = 0.f;
+    for (int t = tj + 1; t < ti; ++t) {
+      float mf[4];
+      frag_rows(gb + (t * 16 + 15) * ld + k, 0, lane, mf);
+#pragma unroll
+      for (int s = 0; s < 4; ++s) bf[s] += mf[s];
+    }
 #pragma unroll
     for (int s = 0; s < 4; ++s) {
-      const float e = fast_exp2(gf[s] - rf[s]);
+      const float e = fast_exp2(gf[s]);
       kf[s] *= e, qf[s] *= e;
-      cf[s] *= fast_exp2(rf[s] - hf[s]);
+      cf[s] *= fast_exp2((lf[s] - hf[s]) + bf[s]);
     }
     aA = mma4(kf, cf, aA);
     aP = mma4(qf, cf, aP);
@@ -222,7 +230,9 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   float* sE = sB + kC;                     // b_i e^(G_i)
   float* sQ = sE + kC;                     // e^(G_i)
   float* sD = sQ + kC;                     // e^(G_C - G_i)
-  float* bufG = sD + kC;                   // CHN: G_i per channel, in log2
+  float* bufG = sD + kC;                   // CHN: log2 decays per channel, summed from the start of each 16-row tile
+  float* sPre = bufG + kC * ldk;           // CHN: [4][Dp] sums of the tiles in front of a tile, and of those behind it
+  float* sSuf = sPre + 4 * Dp;
   float* out = ws + ((chunk_base(p, r) + ck) * p.H + h) * lay.size();
   const T* ring = reinterpret_cast<const T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -256,20 +266,31 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
       const int i = n / Dp, c = n % Dp;
       const bool in = i < len && c < p.D;
       const float v = Io<T>::ld(ar + (int64_t)min(i, len - 1) * p.ld_a + min(c, p.D - 1)) + p.dt_bias[h * p.D + min(c, p.D - 1)];
-      bufG[i * ldk + c] = in ? neg_a * softplus_f(v) : 0.f;
+      // (a decay below 2^-64 forgets as completely in 32 bits, and keeps the sums short)
+      bufG[i * ldk + c] = in ? fmaxf(neg_a * softplus_f(v), -64.f) : 0.f;
     }
     if (wave == 0) sB[lane] = lane < len ? sigmoid_f(Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + min(lane, len - 1)) * p.ld_b + h)) : 0.f;
     __syncthreads();
-    // running sums over the chunk, a segment of rows a thread, then what the segments in front add up to
-    const int segs = kPrepThreads / Dp, c = tid % Dp, sg = tid / Dp, per = kC / segs;
+    // running sums over each 16-row tile, a segment of a tile's rows a thread, then the tile's segments in front
+    const int segs = kPrepThreads / Dp, c = tid % Dp, sg = tid / Dp, per = kC / segs;     // per <= 16: Dp <= 128
     float acc = 0.f;
     for (int i = sg * per; i < (sg + 1) * per; ++i) acc += bufG[i * ldk + c], bufG[i * ldk + c] = acc;
     __syncthreads();
     float before = 0.f;
-    for (int n = 0; n < sg; ++n) before += bufG[(n * per + per - 1) * ldk + c];
+    for (int n = sg * per / 16 * 16 / per; n < sg; ++n) before += bufG[(n * per + per - 1) * ldk + c];
     __syncthreads();
     for (int i = sg * per; i < (sg + 1) * per; ++i) bufG[i * ldk + c] += before;
-    if (sg == segs - 1) out[lay.g() + c] = fast_exp2(acc + before);
+    __syncthreads();
+    if (tid < Dp) {
+      float e[4], a = 0.f, b = 0.f;
+#pragma unroll
+      for (int t = 0; t < 4; ++t) e[t] = bufG[(16 * t + 15) * ldk + tid];
+#pragma unroll
+      for (int t = 0; t < 4; ++t) sPre[t * Dp + tid] = a, a += e[t];
+#pragma unroll
+      for (int t = 3; t >= 0; --t) sSuf[t * Dp + tid] = b, b += e[t];
+      out[lay.g() + tid] = fast_exp2(a);
+    }
   }
   __syncthreads();
   unit_rows(bufA, ldk, Dp, 1.0f);
@@ -344,8 +365,8 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
     const int i = n / (Dp / 4), c = (n % (Dp / 4)) * 4;
     float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
     if constexpr (CHN) {
-      const float4 g = *reinterpret_cast<const float4*>(bufG + i * ldk + c);
-      v = make_float4(v.x * fast_exp2(g.x), v.y * fast_exp2(g.y), v.z * fast_exp2(g.z), v.w * fast_exp2(g.w));
+      const float4 g = *reinterpret_cast<const float4*>(bufG + i * ldk + c), b = *reinterpret_cast<const float4*>(sPre + (i >> 4) * Dp + c);
+      v = make_float4(v.x * fast_exp2(g.x + b.x), v.y * fast_exp2(g.y + b.y), v.z * fast_exp2(g.z + b.z), v.w * fast_exp2(g.w + b.w));
     } else {
       const float e = sQ[i];
       v = make_float4(v.x * e, v.y * e, v.z * e, v.w * e);
@@ -354,14 +375,14 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   }
   for (int n = tid; n < kC * Dp; n += kPrepThreads) {
     const int d = n / kC, j = n % kC;
-    const float e = CHN ? fast_exp2(bufG[(kC - 1) * ldk + d] - bufG[j * ldk + d]) : sD[j];
+    const float e = CHN ? fast_exp2((bufG[(j | 15) * ldk + d] - bufG[j * ldk + d]) + sSuf[(j >> 4) * Dp + d]) : sD[j];
     out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * e : 0.f;
   }
   __syncthreads();   // Q is dead: A and T take its place
   if constexpr (CHN) {   // and nobody needs the plain keys again
     for (int n = tid; n < kC * Dp; n += kPrepThreads) {
       const int i = n / Dp, c = n % Dp;
-      bufA[i * ldk + c] *= fast_exp2(bufG[i * ldk + c]);
+      bufA[i * ldk + c] *= fast_exp2(bufG[i * ldk + c] + sPre[(i >> 4) * Dp + c]);
     }
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
@@ -527,7 +548,7 @@ extern "C" int mi_gated_delta_chunked(const mi_gated_delta_args* args, int32_t r
   hipStream_t s = (hipStream_t)stream;
   float* ws = (float*)workspace;
   const int ldk = lay.Dp + 4, ldv = lay.Vp + 4, ldm = kC + 4;
-  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC + (p.channel ? kC * ldk : 0)) * 4;
+  const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC + (p.channel ? kC * ldk + 8 * lay.Dp : 0)) * 4;
   const int al = (dtype == MI_DTYPE_BF16 ? 8 : 4);
   const bool vec = dim % 8 == 0 && vdim % 8 == 0 && p.ld % al == 0 && CH % al == 0 && aligned16(p.proj) && aligned16(p.convw) && aligned16(p.ring);
   const dim3 pg((max_query_len + kC - 1) / kC, heads, num_reqs);
