@@ -27,6 +27,7 @@ Rank 0 prints ONE JSON line.
 from __future__ import annotations
 
 import argparse
+import importlib
 import json
 import os
 import sys
@@ -83,6 +84,15 @@ def parse_args():
     ap.add_argument("--dogulorn-batches", default="32,256", help="decode batch sizes")
     ap.add_argument("--dogulorn-ctx", type=int, default=4096, help="context of the decode cases")
     ap.add_argument("--dogulorn-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
+    ap.add_argument("--pupopel", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the Pupopel stack beside the Dogulorn "
+                         "and talker stacks of equal size (tools/bench_pupopel.py; one JSON line per case)")
+    ap.add_argument("--pupopel-size", default="2k,4k")
+    ap.add_argument("--pupopel-mode", default="decode,prefill")
+    ap.add_argument("--pupopel-models", default="pupopel,dogulorn,talker")
+    ap.add_argument("--pupopel-batches", default="32,256", help="decode batch sizes")
+    ap.add_argument("--pupopel-ctx", type=int, default=4096, help="context of the decode cases")
+    ap.add_argument("--pupopel-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
     a = ap.parse_args()
     if a.pmc_child:   # a few steps of the same workload, nothing else: the parent reads the counters of the decode launches
         a.steps, a.warmup, a.no_cpu_baseline, a.roofline_steps, a.traffic = 2, 1, True, 0, "none"
@@ -584,12 +594,10 @@ def time_allreduce(dev, rows: int, cols: int, calls: int = 50) -> dict:
 
 def main():
     a = parse_args()
-    if a.dogulorn:
+    if a.dogulorn or a.pupopel:
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "tools"))
         sys.modules.setdefault("bench", sys.modules[__name__])
-        import bench_dogulorn
-
-        return bench_dogulorn.run(a)
+        return importlib.import_module("bench_pupopel" if a.pupopel else "bench_dogulorn").run(a)
     launched = "WORLD_SIZE" in os.environ
     if a.gpus > 1 and not launched:
         # no launcher around us: become one.  Nothing has touched the GPU yet (device_count() does not).

@@ -378,14 +378,15 @@ int mi_mask_logits_argmax(void* logits, int64_t* ids, int32_t num_tokens, int32_
  *                  gated == 0: out[row, :n_out] = a[row] . W_e^T, weights
  *                  [E, n_out, k], a = the gated output.  max_tiles bounds the
  *                  grid; tiles >= num_tiles[0] exit.  k % 64 == 0; n_out % 64
- *                  (gated) / % 128 == 0.
+ *                  (gated) / % 128 == 0; bf16 and at most 64 rows per tile also
+ *                  k % 8 == 0, n_out % 4 == 0.
  *   mi_moe_combine out[t] = sum_j w[t, j] * partial[row_of_pair[t*k + j]]
  *                  (+ g * shared_out[t], g = sigmoid(x[t] . shared_gate_weight) or 1).
  * ---------------------------------------------------------------------- */
 int32_t mi_moe_rows_per_tile(int32_t num_tokens, int32_t top_k, int32_t num_experts); /* 32, 64 or (prefill chunks) 256 */
 int64_t mi_moe_max_rows(int32_t num_tokens, int32_t top_k, int32_t num_experts, int32_t rows_per_tile);
 int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* expert_counts, const void* router_logits,
-                 int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
+                 const float* bias /* [num_experts], added to the logits, or NULL */, int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
                  int32_t norm_topk_prob, int logits_dtype, int weight_round_dtype, void* stream);
 int mi_moe_align(int32_t* sorted_pairs, int32_t* row_of_pair, int32_t* tile_expert, int32_t* num_tiles,
                  const int32_t* topk_ids, const int32_t* expert_counts, int32_t num_pairs,
@@ -924,9 +925,6 @@ int64_t mi_lightning_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t hea
 int mi_lightning_attn(const mi_lightning_args* args, int32_t row0, int32_t rows,
                       int32_t max_query_len, int32_t chunked, void* workspace,
                       int64_t workspace_bytes, int dtype, void* stream);
-/* fp32 router logits of bf16 rows: out[t][e] = h[t] . weight[e] + bias[e] */
-int mi_moe_router_logits(float* out, const void* h, const void* weight, const float* bias,
-                         int32_t rows, int32_t num_experts, int32_t k, int64_t h_stride, void* stream);
 /* mi_moe_expert_gemm for any sizes and for fp32, pairs ungrouped: row p of out
  * (and of a_rows, gated == 0) belongs to pair p = token * top_k + j. */
 int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const int32_t* topk_ids,

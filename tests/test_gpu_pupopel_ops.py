@@ -389,10 +389,26 @@ def test_lightning_attention(dev, dtype, sizes):
             close(outs[1], wants[1][16 * n:16 * n + 16], **t)
 
 
+@pytest.mark.parametrize("sizes", [(2, 64, 64), (3, 24, 40), (1, 128, 128)], ids=lambda s: "x".join(map(str, s)))
+def test_lightning_attention_in_segments(dev, sizes):
+    """long portions: chunks run in segments side by side; requests of unequal length, then a second portion from the states"""
+    c = LightningCase(*sizes, torch.float32, dev)
+    c.decay = [1.0, 0.999, 0.9997][:sizes[0]]
+    lens = [2100, 70, 1030, 512]
+    ps = [c.rows(n, 30 + i) for i, n in enumerate(lens)]
+    wants = [c.want(p) for p in ps]
+    cut = [1500, 60, 1000, 1]
+    for got, w, n in zip(c.run([(i, [x[:n] for x in p], 0) for i, (p, n) in enumerate(zip(ps, cut))], True), wants, cut):
+        close(got, w[:n], rtol=2e-4, atol=2e-4)
+    for got, w, n in zip(c.run([(i, [x[n:] for x in p], n) for i, (p, n) in enumerate(zip(ps, cut))], True), wants, cut):
+        close(got, w[n:], rtol=2e-4, atol=2e-4)
+
+
 # ------------------------------------------------------------------------------------------------ routed experts
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("t,width,experts,top,ff", [(7, 96, 6, 2, 40), (70, 128, 8, 3, 64), (33, 100, 5, 1, 21), (300, 320, 9, 4, 96),
-                                                    (90, 256, 40, 4, 64), (20, 128, 130, 16, 16), (3, 200, 4, 4, 24)])
+                                                    (90, 256, 40, 4, 64), (20, 128, 130, 16, 16), (3, 200, 4, 4, 24),
+                                                    (1500, 72, 20, 2, 16)])
 def test_routed_experts(dev, dtype, t, width, experts, top, ff):
     from vllm_omni_amd import ops
     from vllm_omni_amd.moe import RoutedExperts
@@ -410,9 +426,9 @@ def test_routed_experts(dev, dtype, t, width, experts, top, ff):
     hg.copy_(h)
     wd = {k: v.double() for k, v in w.items()}
     idx, p = ref.route(h.double(), wd["router"], wd["router.b"], top)
-    logits = ops.moe_router_logits(hg, m.router, m.router_b)
-    close(logits, h.double() @ wd["router"].T + wd["router.b"], rtol=1e-5, atol=2e-5)      # 32-bit whatever the rows are
-    ids, wt, _ = ops.moe_route(logits, top, True, want_counts=False)
+    logits = ops.moe_router_logits(hg, m.router)
+    close(logits, h.double() @ wd["router"].T, rtol=1e-5, atol=2e-5)      # 32-bit whatever the rows are
+    ids, wt, _ = ops.moe_route(logits, top, True, want_counts=False, bias=m.router_b)
     assert torch.equal(ids.cpu().long().sort(-1).values, idx.sort(-1).values)
     got = torch.zeros(t, experts, dtype=torch.float64).scatter_(1, ids.cpu().long(), wt.cpu().double())
     close(got, torch.zeros(t, experts, dtype=torch.float64).scatter_(1, idx, p), rtol=1e-5, atol=1e-6)

@@ -44,7 +44,13 @@ struct ScanParams {
   const int32_t* qsl;
   const int32_t* seq_lens;
   int req0, H, D, V;
+  // segments (recurrences without a delta term and one decay per head): a request's chunks in runs of seg_chunks
+  const float* log2_decay = nullptr;   // [H]
+  float* seg_state = nullptr;          // [requests][nseg][H][D][V]: end state of each run but the last, from zeros except the
+                                       // first; the last place holds what the request started from
+  int nseg = 1, seg_chunks = 1 << 28;
 };
+constexpr int kMaxSegments = 8;
 
 template <typename P>
 __device__ __forceinline__ int64_t chunk_base(const P& p, int r) {
@@ -55,8 +61,8 @@ __device__ __forceinline__ int64_t chunk_base(const P& p, int r) {
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 // NV 16-column value tiles a workgroup: its four waves read every operand of a chunk once for all of them (the bound is the
-// L2 traffic of those operands, each head's tiles reading the same ones)
-template <int DT, int NV, bool DELTA>
+// L2 traffic of those operands, each head's tiles reading the same ones).  ENDS: only the end state of a segment.
+template <int DT, int NV, bool DELTA, bool ENDS = false>
 __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, float* ws, const ChunkLayout lay, int nvg) {
   scalar_cache_acquire();
   constexpr int Dp = DT * 16, LS = Dp + 4, LU = kC + 4, MT = (DT + 3) / 4;
@@ -70,31 +76,66 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
   const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
   if (h >= p.H || L <= 0) return;
   const int start = p.seq_lens[r] - L;
+  const int all = (L + kC - 1) / kC;                                   // the request's chunks
+  const int seg = DELTA ? 0 : blockIdx.z, segs = DELTA ? 1 : (all + p.seg_chunks - 1) / p.seg_chunks;
+  if (!DELTA && (ENDS ? seg >= segs - 1 : seg >= segs)) return;
+  const int first = DELTA ? 0 : seg * p.seg_chunks;
+  const int nck = DELTA ? all : min(p.seg_chunks, all - first);
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lg = lane >> 4;
   const int v0 = vg * 16 * NV + lr;        // + 16 n: this lane's value columns
   float* S = p.state + (((int64_t)p.slots[r] * p.H + h) * p.D) * p.V;
-  f32x4_t st[NV][MT];
+  auto seg_at = [&](int k) { return p.seg_state + ((((int64_t)(r - p.req0) * p.nseg + k) * p.H + h) * p.D) * p.V; };
+  f32x4_t st[NV][MT] = {};
+  auto add_state = [&](const float* src, float keep) {      // st <- keep st + src
+#pragma unroll
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int d = (wave + 4 * m) * 16 + 4 * lg + i, v = v0 + 16 * n;
+          const bool in = d < p.D && v < p.V;
+          const float x = src[in ? (int64_t)d * p.V + v : 0];
+          st[n][m][i] = st[n][m][i] * keep + (in ? x : 0.f);
+        }
+  };
+  auto put_state = [&](float* dst) {
+#pragma unroll
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int d = (wave + 4 * m) * 16 + 4 * lg + i, v = v0 + 16 * n;
+          if (d < p.D && v < p.V) dst[(int64_t)d * p.V + v] = st[n][m][i];
+        }
+  };
+  if (DELTA || segs == 1) {
+    if (start > 0) add_state(S, 0.f);
+  } else if constexpr (ENDS) {
+    // the first segment starts from the request's state and leaves a copy of it: the pass behind this one overwrites it
+    if (seg == 0) {
+      if (start > 0) add_state(S, 0.f);
+      put_state(seg_at(p.nseg - 1));
+    }
+  } else {
+    if (seg == 0) add_state(seg_at(p.nseg - 1), 0.f);
+    const float keep = seg > 1 ? fast_exp2(p.log2_decay[h] * (float)(p.seg_chunks * kC)) : 0.f;
+    for (int k = 0; k < seg; ++k) add_state(seg_at(k), keep);
+  }
 #pragma unroll
   for (int n = 0; n < NV; ++n)
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      const int mt = wave + 4 * m, v = v0 + 16 * n;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = mt * 16 + 4 * lg + i;
-        st[n][m][i] = start > 0 && d < p.D && v < p.V ? S[(int64_t)d * p.V + v] : 0.f;
-      }
-      if (mt < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + mt * 16 + 4 * lg) = st[n][m];
-    }
-  const int nck = (L + kC - 1) / kC;
-  float* base = ws + (chunk_base(p, r) * p.H + h) * lay.size();
+    for (int m = 0; m < MT; ++m)
+      if (wave + 4 * m < DT) *reinterpret_cast<f32x4_t*>(sS + (16 * n + lr) * LS + (wave + 4 * m) * 16 + 4 * lg) = st[n][m];
+  float* base = ws + ((chunk_base(p, r) + first) * p.H + h) * lay.size();
   const int64_t step = p.H * lay.size();
   // one chunk's operands; the next chunk's are loaded a whole chunk ahead (the chain of chunks is the critical path, its
   // loads must not be).  Loads and stores are unconditional — past the last chunk the loads fetch what nobody uses, read-outs
   // replace U in the workspace — so that the number in flight is known at every wait: memory operations retire in order, and a
   // store that may or may not be there makes the wait for the loads behind it wait for its acknowledgement as well.
   struct Chunk {
-    f32x4_t w[DELTA ? DT : 1], q[DT], pm[4], kt[MT][4], u[NV], g[MT];
+    f32x4_t w[DELTA ? DT : 1], q[ENDS ? 1 : DT], pm[ENDS ? 1 : 4], kt[MT][4], u[NV], g[MT];
   };
   auto load = [&](Chunk& x, int c) {
     const float* b = base + c * step;
@@ -102,7 +143,7 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
 #pragma unroll
     for (int k = 0; k < DT; ++k) {
       if constexpr (DELTA) x.w[k] = *reinterpret_cast<const f32x4_t*>(b + lay.w() + ro + 16 * k);
-      x.q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
+      if constexpr (!ENDS) x.q[k] = *reinterpret_cast<const f32x4_t*>(b + lay.q() + ro + 16 * k);
     }
 #pragma unroll
     for (int n = 0; n < NV; ++n)
@@ -111,7 +152,7 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
         x.u[n][i] = b[lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n];
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      x.pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
+      if constexpr (!ENDS) x.pm[k] = *reinterpret_cast<const f32x4_t*>(b + lay.pm() + (16 * wave + lr) * kC + 16 * k + 4 * lg);
 #pragma unroll
       for (int m = 0; m < MT; ++m)
         x.kt[m][k] = *reinterpret_cast<const f32x4_t*>(b + lay.kt() + (int64_t)(min(wave + 4 * m, DT - 1) * 16 + lr) * kC + 16 * k + 4 * lg);
@@ -126,6 +167,7 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
 #pragma unroll
       for (int n = 0; n < NV; ++n) f[n] = *reinterpret_cast<const f32x4_t*>(b + (16 * n + lr) * ld + 16 * k + 4 * lg);
     };
+    if constexpr (!ENDS) {
     get(sv[0], sS, LS, 0);
 #pragma unroll
     for (int k = 0; k < DT; ++k) {
@@ -138,6 +180,7 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
           ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[k][s], sv[k & 1][n][s], ao[n], 0, 0, 0);
         }
       __builtin_amdgcn_sched_barrier(0);
+    }
     }
 #pragma unroll
     for (int n = 0; n < NV; ++n) *reinterpret_cast<f32x4_t*>(sU + (16 * n + lr) * LU + 16 * wave + 4 * lg) = x.u[n] - d[n];
@@ -158,10 +201,11 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
 #pragma unroll
           for (int m = 0; m < MT; ++m)
             if (whole || wave + 4 * m < DT) st[n][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[m][k][s], uv, st[n][m], 0, 0, 0);
-          ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv, ao[n], 0, 0, 0);
+          if constexpr (!ENDS) ao[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.pm[k][s], uv, ao[n], 0, 0, 0);
         }
       __builtin_amdgcn_sched_barrier(0);
     }
+    if constexpr (!ENDS) {
 #pragma unroll
     for (int n = 0; n < NV; ++n) {
 #pragma unroll
@@ -171,6 +215,7 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
       for (int i = 0; i < 4; ++i) {
         base[c * step + lay.u() + (int64_t)(16 * wave + 4 * lg + i) * lay.Vp + v0 + 16 * n] = ao[n][i];
       }
+    }
     }
     lds_barrier();
   };
@@ -184,15 +229,8 @@ __global__ __launch_bounds__(256, 1) void chunk_scan_kernel(const ScanParams p, 
     load(a, min(c + 2, nck - 1));
     work(b, c + 1);
   }
-#pragma unroll
-  for (int n = 0; n < NV; ++n)
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = (wave + 4 * m) * 16 + 4 * lg + i, v = v0 + 16 * n;
-        if (d < p.D && v < p.V) S[(int64_t)d * p.V + v] = st[n][m][i];
-      }
+  if constexpr (ENDS) put_state(seg_at(seg));
+  else if (seg == segs - 1) put_state(S);
 }
 
 inline int round_tiles(int n) {   // 16-column tiles of the built scans: 2, 4, 8, 16
@@ -200,15 +238,15 @@ inline int round_tiles(int n) {   // 16-column tiles of the built scans: 2, 4, 8
   return t <= 2 ? 2 : t <= 4 ? 4 : t <= 8 ? 8 : 16;
 }
 
-template <bool DELTA>
+template <bool DELTA, bool ENDS>
 int launch_scan(const ScanParams& p, float* ws, const ChunkLayout& lay, int num_reqs, hipStream_t s) {
   // two value tiles a workgroup where that still leaves one for every CU
-  const int nvt = lay.Vp / 16, nv = nvt % 2 == 0 && (int64_t)num_reqs * p.H * (nvt / 2) >= 256 ? 2 : 1, nvg = nvt / nv;
-  const dim3 sg((p.H + 7) / 8 * 8 * nvg, num_reqs);
+  const int nvt = lay.Vp / 16, nv = nvt % 2 == 0 && (int64_t)num_reqs * p.H * p.nseg * (nvt / 2) >= 256 ? 2 : 1, nvg = nvt / nv;
+  const dim3 sg((p.H + 7) / 8 * 8 * nvg, num_reqs, ENDS ? p.nseg - 1 : p.nseg);
 #define MI_SCAN(DT)                                                                                                            \
   do {                                                                                                                         \
-    if (nv == 2) hipLaunchKernelGGL((chunk_scan_kernel<DT, 2, DELTA>), sg, dim3(256), 0, s, p, ws, lay, nvg);                  \
-    else hipLaunchKernelGGL((chunk_scan_kernel<DT, 1, DELTA>), sg, dim3(256), 0, s, p, ws, lay, nvg);                          \
+    if (nv == 2) hipLaunchKernelGGL((chunk_scan_kernel<DT, 2, DELTA, ENDS>), sg, dim3(256), 0, s, p, ws, lay, nvg);            \
+    else hipLaunchKernelGGL((chunk_scan_kernel<DT, 1, DELTA, ENDS>), sg, dim3(256), 0, s, p, ws, lay, nvg);                    \
   } while (0)
   switch (lay.Dp / 16) {
     case 2: MI_SCAN(2); break;
@@ -218,6 +256,24 @@ int launch_scan(const ScanParams& p, float* ws, const ChunkLayout& lay, int num_
   }
 #undef MI_SCAN
   return launch_status();
+}
+
+// recurrences without a delta term: where heads and requests leave CUs idle, a request's chunks run in segments side by side —
+// one pass for the segments' end states, one for the read-outs
+inline int launch_linear_scan(ScanParams p, float* ws, const ChunkLayout& lay, int num_reqs, int max_chunks, hipStream_t s) {
+  const int64_t tiles = (int64_t)num_reqs * p.H * (lay.Vp / 16);
+  int n = (int)(1024 / tiles);
+  if (n > max_chunks / 8) n = max_chunks / 8;
+  if (n > kMaxSegments) n = kMaxSegments;
+  if (n > 1) {
+    p.seg_chunks = (max_chunks + n - 1) / n;
+    p.nseg = (max_chunks + p.seg_chunks - 1) / p.seg_chunks;
+  }
+  if (p.nseg > 1) {
+    const int rc = launch_scan<false, true>(p, ws, lay, num_reqs, s);
+    if (rc != MI_OK) return rc;
+  }
+  return launch_scan<false, false>(p, ws, lay, num_reqs, s);
 }
 
 inline bool chunk_layout(int32_t dim, int32_t vdim, ChunkLayout* lay) {

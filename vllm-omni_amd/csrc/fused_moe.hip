@@ -45,7 +45,8 @@ __device__ __forceinline__ float wave_max_valu(float v) {
 }
 
 template <int DT, int EPL>  // EPL = experts per lane = E / 64, rounded up
-__global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict__ logits, int64_t row_stride, int num_experts,
+__global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict__ logits, const float* __restrict__ bias,
+                                                         int64_t row_stride, int num_experts,
                                                          int32_t* __restrict__ ids, float* __restrict__ weights,
                                                          int32_t* __restrict__ counts, int T, int top_k, int norm,
                                                          int round_dt) {
@@ -67,6 +68,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
       else if constexpr (DT == MI_DTYPE_BF16)
         p[i] = Elem<bf16_tag>::from_bits(reinterpret_cast<const uint16_t*>(logits)[t * row_stride + e]);
       else p[i] = Elem<f16_tag>::from_bits(reinterpret_cast<const uint16_t*>(logits)[t * row_stride + e]);
+      if (bias) p[i] += bias[e];
       mx = fmaxf(mx, p[i]);
     }
     mx = wave_max_valu(mx);
@@ -378,48 +380,6 @@ __global__ __launch_bounds__(256) void moe_pair_gemm_kernel(T* __restrict__ out,
   }
 }
 
-// ---------------------------------------------------------------- router
-// fp32 logits[t][e] = h[t] . w[e] + bias[e] of 16-bit rows.  A wave takes a quarter of K for 16 experts x 16 tokens, operands
-// straight from global memory; the four quarters meet in LDS.  Loads are unconditional on clamped addresses.
-__global__ __launch_bounds__(256) void moe_router_kernel(float* __restrict__ out, const uint16_t* __restrict__ h,
-                                                         const uint16_t* __restrict__ w, const float* __restrict__ bias, int rows, int E,
-                                                         int K, int64_t h_stride) {
-  scalar_cache_acquire();
-  __shared__ f32x4_t red[4][64];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
-  const int t0 = blockIdx.x * 16, e0 = blockIdx.y * 16;
-  const int steps = (K + 31) / 32, per = (steps + 3) / 4;
-  const int s0 = wave * per, s1 = min(steps, s0 + per);
-  const uint16_t* wr = w + (int64_t)min(e0 + lr, E - 1) * K;
-  const uint16_t* hr = h + (int64_t)min(t0 + lr, rows - 1) * h_stride;
-  f32x4_t acc = {};
-  for (int s = s0; s < s1; s += 4) {
-    uint4 a[4], b[4];
-#pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int k = min(32 * (s + u) + 8 * lg, K - 8);      // K is a multiple of 8
-      a[u] = *reinterpret_cast<const uint4*>(wr + k);
-      b[u] = *reinterpret_cast<const uint4*>(hr + k);
-    }
-#pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      if (s + u >= s1 || 32 * (s + u) + 8 * lg >= K) a[u] = make_uint4(0, 0, 0, 0);
-      acc = mfma16<bf16_tag>(a[u], b[u], acc);
-    }
-  }
-  red[wave][lane] = acc;
-  __syncthreads();
-  if (wave) return;
-  acc = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]);
-  const int t = t0 + lr;
-  if (t >= rows) return;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int e = e0 + 4 * lg + i;
-    if (e < E) out[(int64_t)t * E + e] = acc[i] + (bias ? bias[e] : 0.f);
-  }
-}
-
 // ---------------------------------------------------------------- combine
 template <typename Tag>
 __global__ __launch_bounds__(256) void moe_combine_kernel(uint16_t* __restrict__ out, const uint16_t* __restrict__ part,
@@ -496,7 +456,7 @@ extern "C" int64_t mi_moe_max_rows(int32_t num_tokens, int32_t top_k, int32_t nu
 }
 
 extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* expert_counts, const void* router_logits,
-                            int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
+                            const float* bias, int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
                             int32_t norm_topk_prob, int logits_dtype, int weight_round_dtype, void* stream) {
   using namespace mi;
   if (num_tokens == 0) return MI_OK;
@@ -512,7 +472,7 @@ extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* exp
   const int tpw = num_tokens >= 8192 ? 4 : num_tokens >= 1024 ? 2 : 1;
   const dim3 grid((num_tokens + 16 * tpw - 1) / (16 * tpw)), block(1024);
 #define MI_ROUTE(DT, EPL)                                                                                        \
-  hipLaunchKernelGGL((moe_route_kernel<DT, EPL>), grid, block, 0, s, router_logits, logits_row_stride, num_experts, topk_ids, \
+  hipLaunchKernelGGL((moe_route_kernel<DT, EPL>), grid, block, 0, s, router_logits, bias, logits_row_stride, num_experts, topk_ids, \
                      topk_weights, expert_counts, num_tokens, top_k, norm_topk_prob, weight_round_dtype)
 #define MI_ROUTE_E(DT)                                  \
   do {                                                  \
@@ -645,17 +605,6 @@ extern "C" int mi_moe_combine(void* out, const void* partial, const int32_t* row
     hipLaunchKernelGGL((moe_combine_kernel<f16_tag>), dim3(num_tokens), dim3(256), 0, s, o, pp, row_of_pair, topk_weights, sh, xx, gw, hidden, top_k, partial_row_stride, out_row_stride, x_row_stride, shared_row_stride);
   else
     return MI_ERR_UNSUPPORTED;
-  return launch_status();
-}
-
-extern "C" int mi_moe_router_logits(float* out, const void* h, const void* weight, const float* bias, int32_t rows,
-                                    int32_t num_experts, int32_t k, int64_t h_stride, void* stream) {
-  using namespace mi;
-  if (rows == 0) return MI_OK;
-  if (!out || !h || !weight || rows < 0 || num_experts <= 0 || k <= 0 || h_stride < k) return MI_ERR_INVALID_ARG;
-  if (k % 8 || h_stride % 8 || !aligned16(h) || !aligned16(weight)) return MI_ERR_UNSUPPORTED;
-  hipLaunchKernelGGL(moe_router_kernel, dim3((rows + 15) / 16, (num_experts + 15) / 16), dim3(256), 0, reinterpret_cast<hipStream_t>(stream),
-                     out, (const uint16_t*)h, (const uint16_t*)weight, bias, rows, num_experts, k, h_stride);
   return launch_status();
 }
 

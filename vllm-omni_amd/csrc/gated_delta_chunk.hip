@@ -20,17 +20,19 @@
 namespace mi {
 namespace {
 
-constexpr int kPrepThreads = 512;
+// threads of a prep workgroup: two workgroups a CU, or one (whose cumulative decays take the LDS of the second) of twice the size
+template <bool CHN>
+constexpr int prep_threads() { return CHN ? 1024 : 512; }
 
 // conv + silu of channels [ch0, ch0 + n) of the chunk's rows into buf [C][ld]; zeros in rows past len and columns past n
-template <typename T>
+template <typename T, int NT>
 __device__ __forceinline__ void conv_rows(const DeltaParams& p, float* buf, int ld, int np, int ch0, int n, int64_t row0, int i0,
                                           int len, int start, const T* ring) {
   const T* proj = reinterpret_cast<const T*>(p.proj);
   const T* cw = reinterpret_cast<const T*>(p.convw);
-  const int segs = kPrepThreads / np > 0 ? kPrepThreads / np : 1;      // row segments worked on side by side
+  const int segs = NT / np > 0 ? NT / np : 1;      // row segments worked on side by side
   const int rows_per = (kC + segs - 1) / segs;
-  for (int item = threadIdx.x; item < segs * np; item += kPrepThreads) {
+  for (int item = threadIdx.x; item < segs * np; item += NT) {
     const int c = item % np, seg = item / np;
     const int a = seg * rows_per, b = min(kC, a + rows_per);
     if (c >= n) {
@@ -71,65 +73,73 @@ __device__ __forceinline__ void conv_rows(const DeltaParams& p, float* buf, int 
   }
 }
 
-// the same, 8 channels a thread: every load of a thread is independent of the others.  Needs n, the channel offsets and the
-// row strides to be multiples of 8.
-template <typename T, int TAPS>
-__device__ __forceinline__ void conv_rows8(const DeltaParams& p, float* buf, int ld, int np, int ch0, int n, int64_t row0, int i0,
-                                           int len, int start, const T* ring) {
-  const T* proj = reinterpret_cast<const T*>(p.proj);
+// The same, 8 channels of two rows a thread, NB blocks of channels at once: all loads of a thread are unconditional (clamped
+// addresses, values selected afterwards) and independent, so a trip costs one memory latency.  Needs n, the channel offsets
+// and the row strides to be multiples of 8; the blocks share np and n.
+template <typename T, int NT, int TAPS, int NB>
+__device__ __forceinline__ void conv_rows8(const DeltaParams& p, float* const (&buf)[NB], const int (&ch0)[NB], int ld, int np, int n,
+                                           int64_t row0, int i0, int len, int start, const T* ring) {
+  const T* proj = reinterpret_cast<const T*>(p.proj) + row0 * p.ld;
   const T* cw = reinterpret_cast<const T*>(p.convw);
   const int per = np / 8;
-  for (int item = threadIdx.x; item < kC * per; item += kPrepThreads) {
-    const int c = (item % per) * 8, i = item / per;
-    float acc[8] = {};
-    if (c < n && i < len) {
-      const int ch = ch0 + c;
-      float w[TAPS][8], x[TAPS][8];
-      float wf[8 * TAPS];
+  for (int item = threadIdx.x; item < kC / 2 * per; item += NT) {
+    const int c = (item % per) * 8, i = item / per * 2;
+    float wf[NB][8 * TAPS], x[NB][TAPS + 1][8];
+    bool in[TAPS + 1];
 #pragma unroll
-      for (int t = 0; t < TAPS; ++t) Io<T>::template ldv<8>(cw + (int64_t)ch * TAPS + 8 * t, *reinterpret_cast<float(*)[8]>(wf + 8 * t));
+    for (int t = 0; t <= TAPS; ++t) {
+      const int k = min(i - (TAPS - 1) + t, len - 1), pos = start + i0 + k;
+      in[t] = pos >= 0;
+      const int64_t at = i0 + k >= 0 ? k * p.ld : 0, rat = (int64_t)(max(pos, 0) % TAPS) * p.CH;
 #pragma unroll
-      for (int t = 0; t < TAPS; ++t)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) w[t][j] = wf[j * TAPS + t];
-#pragma unroll
-      for (int t = 0; t < TAPS; ++t) {
-        const int k = i - (TAPS - 1) + t;
-        const int pos = start + i0 + k;
-        if (i0 + k >= 0) {
-          Io<T>::template ldv<8>(proj + (row0 + k) * p.ld + ch, x[t]);
-        } else if (pos >= 0) {
-          Io<T>::template ldv<8>(ring + (int64_t)(pos % TAPS) * p.CH + ch, x[t]);
-        } else {
-#pragma unroll
-          for (int j = 0; j < 8; ++j) x[t][j] = 0.f;
-        }
+      for (int b = 0; b < NB; ++b) {
+        const int ch = ch0[b] + min(c, n - 8);
+        Io<T>::template ldv<8>((i0 + k >= 0 ? proj + at : ring + rat) + ch, x[b][t]);
       }
+    }
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
 #pragma unroll
       for (int t = 0; t < TAPS; ++t)
+        Io<T>::template ldv<8>(cw + (int64_t)(ch0[b] + min(c, n - 8)) * TAPS + 8 * t, *reinterpret_cast<float(*)[8]>(wf[b] + 8 * t));
 #pragma unroll
-        for (int j = 0; j < 8; ++j) acc[j] += w[t][j] * x[t][j];
+    for (int b = 0; b < NB; ++b)
 #pragma unroll
-      for (int j = 0; j < 8; ++j) acc[j] = silu_f(acc[j]);
-    }
-    *reinterpret_cast<float4*>(buf + i * ld + c) = make_float4(acc[0], acc[1], acc[2], acc[3]);
-    *reinterpret_cast<float4*>(buf + i * ld + c + 4) = make_float4(acc[4], acc[5], acc[6], acc[7]);
+      for (int r = 0; r < 2; ++r) {
+        float acc[8] = {};
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) acc[j] += in[t + r] ? wf[b][j * TAPS + t] * x[b][t + r][j] : 0.f;
+        const bool live = c < n && i + r < len;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[j] = live ? silu_f(acc[j]) : 0.f;
+        Io<float>::stv<8>(buf[b] + (i + r) * ld + c, acc);
+      }
   }
 }
 
-template <typename T>
-__device__ __forceinline__ void conv_tile(const DeltaParams& p, bool vec, float* buf, int ld, int np, int ch0, int n, int64_t row0,
-                                          int i0, int len, int start, const T* ring) {
-  if (vec && p.taps == 4) conv_rows8<T, 4>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
-  else if (vec && p.taps == 3) conv_rows8<T, 3>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
-  else if (vec && p.taps == 2) conv_rows8<T, 2>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
-  else conv_rows<T>(p, buf, ld, np, ch0, n, row0, i0, len, start, ring);
+template <typename T, int NT, int NB>
+__device__ __forceinline__ void conv_tiles(const DeltaParams& p, bool vec, float* const (&buf)[NB], const int (&ch0)[NB], int ld, int np, int n,
+                                           int64_t row0, int i0, int len, int start, const T* ring) {
+  if constexpr (sizeof(T) == 4 && NB > 1) {      // twice the registers a value: one block at a time
+#pragma unroll
+    for (int b = 0; b < NB; ++b) conv_tiles<T, NT, 1>(p, vec, {buf[b]}, {ch0[b]}, ld, np, n, row0, i0, len, start, ring);
+    return;
+  }
+  if (vec && p.taps == 4) conv_rows8<T, NT, 4, NB>(p, buf, ch0, ld, np, n, row0, i0, len, start, ring);
+  else if (vec && p.taps == 3) conv_rows8<T, NT, 3, NB>(p, buf, ch0, ld, np, n, row0, i0, len, start, ring);
+  else if (vec && p.taps == 2) conv_rows8<T, NT, 2, NB>(p, buf, ch0, ld, np, n, row0, i0, len, start, ring);
+  else
+#pragma unroll
+    for (int b = 0; b < NB; ++b) conv_rows<T, NT>(p, buf[b], ld, np, ch0[b], n, row0, i0, len, start, ring);
 }
 
 // rows of buf made unit vectors (16 lanes a row), then times mul
+template <int NT>
 __device__ __forceinline__ void unit_rows(float* buf, int ld, int np, float mul) {
   const int sub = threadIdx.x & 15;
-  for (int i = threadIdx.x >> 4; i < kC; i += kPrepThreads / 16) {
+  for (int i = threadIdx.x >> 4; i < kC; i += NT / 16) {
     float ss = 0.f;
     for (int c = sub; c < np; c += 16) ss += buf[i * ld + c] * buf[i * ld + c];
     ss = group_allreduce_sum<16>(ss);
@@ -170,11 +180,11 @@ __device__ __forceinline__ void channel_tile(const float* kb, const float* qb, c
   }
 }
 
-// the same on the diagonal (ti == tj), in four levels of halving: pairs (i, j) whose highest differing bit is `half` are split
-// at the first row of the upper half of their block of 2 half rows.  A lane's token is in a row's role (upper half) or a
-// column's (lower half) on each level, so one exponential per level serves both.  dg: q_i . k_i of the lane's token.
-__device__ __forceinline__ void channel_diag(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti, int lane,
-                                             f32x4_t (&aA)[4], f32x4_t (&aP)[4], float& dg) {
+// the same on the diagonal (ti == tj), by levels of halving: pairs (i, j) whose highest differing bit is `half` are split at the
+// first row of the upper half of their block of 2 half rows.  A lane's token is in a row's role (upper half) or a column's
+// (lower half) on each level, so one exponential per level serves both.  Levels lv0 and lv0 + 1; dg: q_i . k_i of the lane's token.
+__device__ __forceinline__ void channel_diag(const float* kb, const float* qb, const float* gb, int ld, int Dp, int ti, int lv0, int lane,
+                                             f32x4_t (&aA)[2], f32x4_t (&aP)[2], float& dg) {
   const int t = lane & 15;
   const float* g0 = gb + ti * 16 * ld;
   dg = 0.f;
@@ -186,8 +196,8 @@ __device__ __forceinline__ void channel_diag(const float* kb, const float* qb, c
 #pragma unroll
     for (int s = 0; s < 4; ++s) dg += qf[s] * kf[s];
 #pragma unroll
-    for (int lv = 0; lv < 4; ++lv) {
-      const int half = 1 << lv, ref = (t & ~(2 * half - 1)) + half;
+    for (int l = 0; l < 2; ++l) {
+      const int half = 1 << (lv0 + l), ref = (t & ~(2 * half - 1)) + half;
       const bool up = t & half;
       const float4 rv = *reinterpret_cast<const float4*>(g0 + ref * ld + k + 4 * (lane >> 4));
       const float rf[4] = {rv.x, rv.y, rv.z, rv.w};
@@ -199,19 +209,31 @@ __device__ __forceinline__ void channel_diag(const float* kb, const float* qb, c
         rq[s] = up ? qf[s] * e : 0.f;
         ck[s] = up ? 0.f : kf[s] * e;
       }
-      aA[lv] = mma4(rk, ck, aA[lv]);
-      aP[lv] = mma4(rq, ck, aP[lv]);
+      aA[l] = mma4(rk, ck, aA[l]);
+      aP[l] = mma4(rq, ck, aP[l]);
     }
   }
   dg += __shfl_xor(dg, 16, 64);
   dg += __shfl_xor(dg, 32, 64);
 }
 
+// entry (4 (lane / 16) + s, lane % 16) of a diagonal tile belongs to the wave of levels lv0, lv0 + 1 (below the diagonal: their
+// pairs; the wave of the lower levels also has the diagonal and what is above)
+__device__ __forceinline__ bool diag_owner(int i, int j, int lv0) { return i > j ? ((i ^ j) >= 4) == (lv0 == 2) : lv0 == 0; }
+
+// ln(1 + e^x), hardware exponential and logarithm; a series where 1 + e^-|x| would round the small term away
+__device__ __forceinline__ float softplus_fast(float x) {
+  const float e = fast_exp2(-fabsf(x) * kLog2e);
+  const float s = e * (1.f - e * (0.5f - e * (0.33333334f - e * (0.25f - e * (0.2f - e * 0.16666667f)))));
+  return fmaxf(x, 0.f) + (e < 0.0625f ? s : __builtin_amdgcn_logf(1.f + e) * 0.69314718f);
+}
+
 // CHN: one decay per head and key channel
 template <typename T, bool CHN>
-__global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, bool vec) {
+__global__ __launch_bounds__(prep_threads<CHN>(), 4) void gated_delta_prep_kernel(const DeltaParams p, float* ws, const ChunkLayout lay, bool vec) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int NT = prep_threads<CHN>();
   const int r = p.req0 + blockIdx.z, h = blockIdx.y, ck = blockIdx.x;
   const int s0 = p.qsl[r], L = p.qsl[r + 1] - s0;
   const int i0 = ck * kC;
@@ -237,13 +259,15 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   const T* ring = reinterpret_cast<const T*>(p.ring) + (int64_t)p.slots[r] * p.taps * p.CH;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int kh = h / (p.H / p.K);
-  conv_tile<T>(p, vec, bufA, ldk, Dp, p.K * p.D + kh * p.D, p.D, row0, i0, len, start, ring);
-  conv_tile<T>(p, vec, bufB, ldk, Dp, kh * p.D, p.D, row0, i0, len, start, ring);
+  // what the gates take, asked for in front of the convolutions
+  const float raw_b = Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + min(lane, len - 1)) * p.ld_b + h);
+  const float raw_a = CHN ? 0.f : Io<T>::ld(reinterpret_cast<const T*>(p.a) + (row0 + min(lane, len - 1)) * p.ld_a + h);
+  conv_tiles<T, NT, 2>(p, vec, {bufA, bufB}, {p.K * p.D + kh * p.D, kh * p.D}, ldk, Dp, p.D, row0, i0, len, start, ring);
   if (!CHN && wave == 0) {   // gates: cumulative log decay over the 64 tokens of the chunk
     float lg = 0.f, b = 0.f;
     if (lane < len) {
-      lg = -expf(p.a_log[h]) * softplus_f(Io<T>::ld(reinterpret_cast<const T*>(p.a) + (row0 + lane) * p.ld_a + h) + p.dt_bias[h]);
-      b = sigmoid_f(Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + lane) * p.ld_b + h));
+      lg = -expf(p.a_log[h]) * softplus_f(raw_a + p.dt_bias[h]);
+      b = sigmoid_f(raw_b);
     }
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -262,17 +286,34 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   if constexpr (CHN) {
     const float neg_a = -expf(p.a_log[h]) * kLog2e;
     const T* ar = reinterpret_cast<const T*>(p.a) + row0 * p.ld_a + (int64_t)h * p.D;
-    for (int n = tid; n < kC * Dp; n += kPrepThreads) {
-      const int i = n / Dp, c = n % Dp;
-      const bool in = i < len && c < p.D;
-      const float v = Io<T>::ld(ar + (int64_t)min(i, len - 1) * p.ld_a + min(c, p.D - 1)) + p.dt_bias[h * p.D + min(c, p.D - 1)];
-      // (a decay below 2^-64 forgets as completely in 32 bits, and keeps the sums short)
-      bufG[i * ldk + c] = in ? fmaxf(neg_a * softplus_f(v), -64.f) : 0.f;
+    // (a decay below 2^-64 forgets as completely in 32 bits, and keeps the sums short)
+    if (vec) {
+      for (int n = tid; n < kC / 2 * Dp / 8; n += NT) {      // two rows a trip
+        const int i = n / (Dp / 8), c = n % (Dp / 8) * 8;
+        float v[2][8], dt[8];
+#pragma unroll
+        for (int r = 0; r < 2; ++r) Io<T>::template ldv<8>(ar + (int64_t)min(i + kC / 2 * r, len - 1) * p.ld_a + min(c, p.D - 8), v[r]);
+        Io<float>::ldv<8>(p.dt_bias + h * p.D + min(c, p.D - 8), dt);
+#pragma unroll
+        for (int r = 0; r < 2; ++r) {
+          const bool in = i + kC / 2 * r < len && c < p.D;
+#pragma unroll
+          for (int j = 0; j < 8; ++j) v[r][j] = in ? fmaxf(neg_a * softplus_fast(v[r][j] + dt[j]), -64.f) : 0.f;
+          Io<float>::stv<8>(bufG + (i + kC / 2 * r) * ldk + c, v[r]);
+        }
+      }
+    } else {
+      for (int n = tid; n < kC * Dp; n += NT) {
+        const int i = n / Dp, c = n % Dp;
+        const bool in = i < len && c < p.D;
+        const float v = Io<T>::ld(ar + (int64_t)min(i, len - 1) * p.ld_a + min(c, p.D - 1)) + p.dt_bias[h * p.D + min(c, p.D - 1)];
+        bufG[i * ldk + c] = in ? fmaxf(neg_a * softplus_fast(v), -64.f) : 0.f;
+      }
     }
-    if (wave == 0) sB[lane] = lane < len ? sigmoid_f(Io<T>::ld(reinterpret_cast<const T*>(p.b) + (row0 + min(lane, len - 1)) * p.ld_b + h)) : 0.f;
+    if (wave == 0) sB[lane] = lane < len ? sigmoid_f(raw_b) : 0.f;
     __syncthreads();
     // running sums over each 16-row tile, a segment of a tile's rows a thread, then the tile's segments in front
-    const int segs = kPrepThreads / Dp, c = tid % Dp, sg = tid / Dp, per = kC / segs;     // per <= 16: Dp <= 128
+    const int segs = NT / Dp, c = tid % Dp, sg = tid / Dp, per = kC / segs;     // per <= 16: Dp <= 128
     float acc = 0.f;
     for (int i = sg * per; i < (sg + 1) * per; ++i) acc += bufG[i * ldk + c], bufG[i * ldk + c] = acc;
     __syncthreads();
@@ -293,8 +334,8 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
     }
   }
   __syncthreads();
-  unit_rows(bufA, ldk, Dp, 1.0f);
-  unit_rows(bufB, ldk, Dp, 1.0f / sqrtf((float)p.D));
+  unit_rows<NT>(bufA, ldk, Dp, 1.0f);
+  unit_rows<NT>(bufB, ldk, Dp, 1.0f / sqrtf((float)p.D));
   __syncthreads();
   // A and P, 16 tiles each, lower ones only: P goes out, A waits in registers until Q is dead
   f32x4_t keep[2] = {};
@@ -304,35 +345,31 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
       out[lay.pm() + i * kC + j] = pv;
       kp[s] = a * sB[i];
     };
-    if (wave < 4) {          // a diagonal tile each, as much work as two others
-      f32x4_t aA[4] = {}, aP[4] = {};
+    if (wave < 8) {          // a diagonal tile for two waves
+      const int ti = wave & 3, lv0 = wave >> 2 << 1;
+      f32x4_t aA[2] = {}, aP[2] = {};
       float dg;
-      channel_diag(bufA, bufB, bufG, ldk, Dp, wave, lane, aA, aP, dg);
+      channel_diag(bufA, bufB, bufG, ldk, Dp, ti, lv0, lane, aA, aP, dg);
 #pragma unroll
       for (int s = 0; s < 4; ++s) {
         const int i = 4 * (lane >> 4) + s, j = lane & 15, x = i ^ j;
-        const float a = x >= 8 ? aA[3][s] : x >= 4 ? aA[2][s] : x >= 2 ? aA[1][s] : aA[0][s];
-        const float q = x >= 8 ? aP[3][s] : x >= 4 ? aP[2][s] : x >= 2 ? aP[1][s] : aP[0][s];
-        store(wave, wave, s, i > j ? a : 0.f, i > j ? q : i == j ? dg : 0.f, keep[0]);
+        const bool hi = x >= (lv0 ? 8 : 2);
+        if (diag_owner(i, j, lv0)) store(ti, ti, s, hi ? aA[1][s] : aA[0][s], i > j ? (hi ? aP[1][s] : aP[0][s]) : i == j ? dg : 0.f, keep[0]);
       }
-    } else {
+    } else if (wave < 14) {
+      const int t = wave - 8, ti = t < 1 ? 1 : t < 3 ? 2 : 3, tj = t - ti * (ti - 1) / 2;
+      f32x4_t aA = {}, aP = {};
+      channel_tile(bufA, bufB, bufG, ldk, Dp, ti, tj, lane, aA, aP);
 #pragma unroll
-      for (int n = 0; n < 2; ++n) {
-        const int t = wave - 4 + 4 * n, ti = t < 1 ? 1 : t < 3 ? 2 : 3, tj = t - ti * (ti - 1) / 2;
-        if (t >= 6) continue;
-        f32x4_t aA = {}, aP = {};
-        channel_tile(bufA, bufB, bufG, ldk, Dp, ti, tj, lane, aA, aP);
-#pragma unroll
-        for (int s = 0; s < 4; ++s) {
-          store(ti, tj, s, aA[s], aP[s], keep[n]);
-          out[lay.pm() + (tj * 16 + 4 * (lane >> 4) + s) * kC + ti * 16 + (lane & 15)] = 0.f;   // its mirror: whole rows of P are multiplied
-        }
+      for (int s = 0; s < 4; ++s) {
+        store(ti, tj, s, aA[s], aP[s], keep[0]);
+        out[lay.pm() + (tj * 16 + 4 * (lane >> 4) + s) * kC + ti * 16 + (lane & 15)] = 0.f;   // its mirror: whole rows of P are multiplied
       }
     }
   }
 #pragma unroll
   for (int n = 0; n < (CHN ? 0 : 4); ++n) {
-    const int t = wave + n * (kPrepThreads / 64);
+    const int t = wave + n * (NT / 64);
     const bool isP = n >= 2;
     const int ti = (t & 15) >> 2, tj = t & 3;
     if (!isP) keep[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -361,7 +398,7 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
     }
   }
   // diag(e^G) Q and the transposed, decayed keys
-  for (int n = tid; n < kC * Dp / 4; n += kPrepThreads) {
+  for (int n = tid; n < kC * Dp / 4; n += NT) {
     const int i = n / (Dp / 4), c = (n % (Dp / 4)) * 4;
     float4 v = *reinterpret_cast<const float4*>(bufB + i * ldk + c);
     if constexpr (CHN) {
@@ -373,28 +410,29 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
     }
     *reinterpret_cast<float4*>(out + lay.q() + (int64_t)i * Dp + c) = v;
   }
-  for (int n = tid; n < kC * Dp; n += kPrepThreads) {
+  for (int n = tid; n < kC * Dp; n += NT) {
     const int d = n / kC, j = n % kC;
     const float e = CHN ? fast_exp2((bufG[(j | 15) * ldk + d] - bufG[j * ldk + d]) + sSuf[(j >> 4) * Dp + d]) : sD[j];
     out[lay.kt() + n] = j < len ? bufA[j * ldk + d] * e : 0.f;
   }
   __syncthreads();   // Q is dead: A and T take its place
   if constexpr (CHN) {   // and nobody needs the plain keys again
-    for (int n = tid; n < kC * Dp; n += kPrepThreads) {
+    for (int n = tid; n < kC * Dp; n += NT) {
       const int i = n / Dp, c = n % Dp;
       bufA[i * ldk + c] *= fast_exp2(bufG[i * ldk + c] + sPre[(i >> 4) * Dp + c]);
     }
+    if (wave < 14) {
+      const int t = wave - 8, ti = wave < 8 ? wave & 3 : t < 1 ? 1 : t < 3 ? 2 : 3, tj = wave < 8 ? ti : t - ti * (ti - 1) / 2;
 #pragma unroll
-    for (int n = 0; n < 2; ++n) {
-      const int t = wave - 4 + 4 * n, ti = wave < 4 ? wave : t < 1 ? 1 : t < 3 ? 2 : 3, tj = wave < 4 ? wave : t - ti * (ti - 1) / 2;
-      if (wave < 4 ? n > 0 : t >= 6) continue;
-#pragma unroll
-      for (int s = 0; s < 4; ++s) mA[(ti * 16 + 4 * (lane >> 4) + s) * ldm + tj * 16 + (lane & 15)] = keep[n][s];
+      for (int s = 0; s < 4; ++s) {
+        const int i = 4 * (lane >> 4) + s, j = lane & 15;
+        if (wave >= 8 || (i > j && diag_owner(i, j, wave >> 2 << 1))) mA[(ti * 16 + i) * ldm + tj * 16 + j] = keep[0][s];
+      }
     }
   }
 #pragma unroll
   for (int n = 0; n < (CHN ? 0 : 2); ++n) {
-    const int t = wave + n * (kPrepThreads / 64);
+    const int t = wave + n * (NT / 64);
 #pragma unroll
     for (int s = 0; s < 4; ++s) mA[((t >> 2) * 16 + 4 * (lane >> 4) + s) * ldm + (t & 3) * 16 + (lane & 15)] = keep[n][s];
   }
@@ -435,7 +473,7 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   // T diag(f) X, X [C][n] in bufA
   auto times = [&](const float* f, int ld, int np, float* dst) {
     const int nt = np / 16;
-    for (int t = wave; t < 4 * nt; t += kPrepThreads / 64) {
+    for (int t = wave; t < 4 * nt; t += NT / 64) {
       const int ti = t / nt, tn = t % nt;
       f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
       for (int k = 0; k <= ti; ++k) {
@@ -452,7 +490,7 @@ __global__ __launch_bounds__(kPrepThreads, CHN ? 2 : 4) void gated_delta_prep_ke
   };
   times(CHN ? sB : sE, ldk, Dp, out + lay.w());
   __syncthreads();
-  conv_tile<T>(p, vec, bufA, ldv, Vp, 2 * p.K * p.D + h * p.V, p.V, row0, i0, len, start, ring);
+  conv_tiles<T, NT, 1>(p, vec, {bufA}, {2 * p.K * p.D + h * p.V}, ldv, Vp, p.V, row0, i0, len, start, ring);
   __syncthreads();
   times(sB, ldv, Vp, out + lay.u());
 }
@@ -550,19 +588,20 @@ extern "C" int mi_gated_delta_chunked(const mi_gated_delta_args* args, int32_t r
   const int ldk = lay.Dp + 4, ldv = lay.Vp + 4, ldm = kC + 4;
   const size_t lds = (size_t)(kC * (ldk > ldv ? ldk : ldv) + kC * (ldk > 2 * ldm ? ldk : 2 * ldm) + 5 * kC + (p.channel ? kC * ldk + 8 * lay.Dp : 0)) * 4;
   const int al = (dtype == MI_DTYPE_BF16 ? 8 : 4);
-  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && p.ld % al == 0 && CH % al == 0 && aligned16(p.proj) && aligned16(p.convw) && aligned16(p.ring);
+  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && p.ld % al == 0 && CH % al == 0 && aligned16(p.proj) && aligned16(p.convw) && aligned16(p.ring) &&
+                   (!p.channel || (p.ld_a % al == 0 && aligned16(p.a) && aligned16(p.dt_bias)));
   const dim3 pg((max_query_len + kC - 1) / kC, heads, num_reqs);
 #define MI_PREP(T)                                                                                                        \
   do {                                                                                                                    \
     auto kern = p.channel ? gated_delta_prep_kernel<T, true> : gated_delta_prep_kernel<T, false>;                                                                               \
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
       return MI_ERR_LAUNCH;                                                                                               \
-    hipLaunchKernelGGL(kern, pg, dim3(kPrepThreads), lds, s, p, ws, lay, vec);                                               \
+    hipLaunchKernelGGL(kern, pg, dim3(p.channel ? prep_threads<true>() : prep_threads<false>()), lds, s, p, ws, lay, vec);                                               \
   } while (0)
   if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
   else MI_PREP(float);
 #undef MI_PREP
-  const int sc = launch_scan<true>(ScanParams{p.state, p.slots, p.qsl, p.seq_lens, p.req0, heads, dim, vdim}, ws, lay, num_reqs, s);
+  const int sc = launch_scan<true, false>(ScanParams{p.state, p.slots, p.qsl, p.seq_lens, p.req0, heads, dim, vdim}, ws, lay, num_reqs, s);
   if (sc != MI_OK) return sc;
   const dim3 fg((unsigned)(((int64_t)rows * heads + 3) / 4)), rg((CH + 255) / 256, num_reqs);
   const dim3 f8((unsigned)(((int64_t)rows * heads + 15) / 16));

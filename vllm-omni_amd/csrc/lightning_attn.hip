@@ -7,6 +7,7 @@
 //     decode (HBM bound: the state is read and written once) and sizes outside the chunked form;
 //   * prompt portions in chunks of 64 tokens: prep here, the chain of chunks in chunk_scan.h (no delta term):
 //     O = diag(d^(i+1)) Q S0 + P V,  P_ij = d^(i-j) q_i . k_j (j <= i),  S1 = d^C S0 + sum_j d^(C-1-j) k_j v_j^T;
+//     few heads and requests: a request's chunks in segments side by side, their end states first;
 //   * finish: norm and gate, one workgroup per token.
 #include "chunk_scan.h"
 
@@ -107,25 +108,45 @@ __global__ __launch_bounds__(256) void lightning_step_kernel(const LightningPara
   }
 }
 
-// silu of columns [col, col + n) of the chunk's rows into dst [C][ld]; zeros in rows past len and columns [n, np)
+// silu of a chunk's q, k (to LDS) and v (to the workspace); zeros in rows past len and columns past dim / vdim
 template <typename T>
-__device__ __forceinline__ void silu_rows(const LightningParams& p, bool vec, float* dst, int ld, int np, int64_t col, int n, int64_t row0,
-                                          int len) {
-  const T* src = reinterpret_cast<const T*>(p.qkv) + row0 * p.ld + col;
-  if (vec) {      // n, the column and the row stride are multiples of 8
-    const int per = np / 8;
-    for (int item = threadIdx.x; item < kC * per; item += kPrep) {
-      const int i = item / per, c = (item % per) * 8;
-      float v[8];
-      Io<T>::template ldv<8>(src + (int64_t)min(i, len - 1) * p.ld + min(c, n - 8), v);
+__device__ __forceinline__ void silu_rows(const LightningParams& p, bool vec, float* bq, float* bk, float* bv, const ChunkLayout& lay, int h,
+                                          int64_t row0, int len) {
+  const int Dp = lay.Dp, Vp = lay.Vp, ldk = Dp + 4;
+  const T* base = reinterpret_cast<const T*>(p.qkv) + row0 * p.ld;
+  const int64_t cq = (int64_t)h * p.D, ck = (int64_t)(p.H + h) * p.D, cv = 2 * (int64_t)p.H * p.D + (int64_t)h * p.V;
+  if (vec) {      // sizes, columns and the row stride are multiples of 8: six loads of a thread in flight
+    const int per = (2 * Dp + Vp) / 8, total = kC * per;
+    for (int it0 = threadIdx.x; it0 < total; it0 += 6 * kPrep) {
+      float x[6][8];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = i < len && c < n ? silu_f(v[j]) : 0.f;
-      Io<float>::stv<8>(dst + i * ld + c, v);
+      for (int u = 0; u < 6; ++u) {
+        const int it = min(it0 + u * kPrep, total - 1), i = it / per, c = it % per * 8;
+        const int64_t col = c < Dp ? cq + min(c, p.D - 8) : c < 2 * Dp ? ck + min(c - Dp, p.D - 8) : cv + min(c - 2 * Dp, p.V - 8);
+        Io<T>::template ldv<8>(base + (int64_t)min(i, len - 1) * p.ld + col, x[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < 6; ++u) {
+        const int it = it0 + u * kPrep, i = it / per, c = it % per * 8;
+        if (it >= total) continue;
+        const int cc = c < Dp ? c : c < 2 * Dp ? c - Dp : c - 2 * Dp;
+        const bool in = i < len && cc < (c < 2 * Dp ? p.D : p.V);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[u][j] = in ? silu_f(x[u][j]) : 0.f;
+        float* dst = c < Dp ? bq + i * ldk + cc : c < 2 * Dp ? bk + i * ldk + cc : bv + i * Vp + cc;
+        Io<float>::stv<8>(dst, x[u]);
+      }
     }
   } else {
-    for (int item = threadIdx.x; item < kC * np; item += kPrep) {
-      const int i = item / np, c = item % np;
-      dst[i * ld + c] = i < len && c < n ? silu_f(Io<T>::ld(src + (int64_t)i * p.ld + c)) : 0.f;
+    for (int it = threadIdx.x; it < kC * Dp; it += kPrep) {
+      const int i = it / Dp, c = it % Dp;
+      const bool in = i < len && c < p.D;
+      bq[i * ldk + c] = in ? silu_f(Io<T>::ld(base + (int64_t)i * p.ld + cq + c)) : 0.f;
+      bk[i * ldk + c] = in ? silu_f(Io<T>::ld(base + (int64_t)i * p.ld + ck + c)) : 0.f;
+    }
+    for (int it = threadIdx.x; it < kC * Vp; it += kPrep) {
+      const int i = it / Vp, c = it % Vp;
+      bv[i * Vp + c] = i < len && c < p.V ? silu_f(Io<T>::ld(base + (int64_t)i * p.ld + cv + c)) : 0.f;
     }
   }
 }
@@ -145,9 +166,7 @@ __global__ __launch_bounds__(kPrep, 4) void lightning_prep_kernel(const Lightnin
   float* bufQ = bufK + kC * ldk;
   const float lg = p.log2_decay[h];
   float* out = ws + ((chunk_base(p, r) + ck) * p.H + h) * lay.size();
-  silu_rows<T>(p, vec, bufQ, ldk, Dp, (int64_t)h * p.D, p.D, row0, len);
-  silu_rows<T>(p, vec, bufK, ldk, Dp, (int64_t)(p.H + h) * p.D, p.D, row0, len);
-  silu_rows<T>(p, vec, out + lay.u(), lay.Vp, lay.Vp, 2 * (int64_t)p.H * p.D + (int64_t)h * p.V, p.V, row0, len);
+  silu_rows<T>(p, vec, bufQ, bufK, out + lay.u(), lay, h, row0, len);
   for (int d = tid; d < Dp; d += kPrep) out[lay.g() + d] = fast_exp2(lg * len);
   __syncthreads();
 #pragma unroll
@@ -287,7 +306,7 @@ extern "C" int64_t mi_lightning_workspace_bytes(int32_t rows, int32_t num_reqs, 
   if (!chunked) return (int64_t)rows * heads * vdim * 4;
   ChunkLayout lay;
   if (!chunk_layout(dim, vdim, &lay)) return 0;
-  return ((int64_t)rows / kC + num_reqs) * heads * lay.size() * 4;
+  return ((int64_t)rows / kC + num_reqs) * heads * lay.size() * 4 + (int64_t)num_reqs * kMaxSegments * heads * dim * vdim * 4;
 }
 
 extern "C" int mi_lightning_attn(const mi_lightning_args* a, int32_t row0, int32_t rows, int32_t max_query_len, int32_t chunked,
@@ -325,7 +344,10 @@ extern "C" int mi_lightning_attn(const mi_lightning_args* a, int32_t row0, int32
     if (dtype == MI_DTYPE_BF16) MI_PREP(uint16_t);
     else MI_PREP(float);
 #undef MI_PREP
-    rc = launch_scan<false>(ScanParams{p.state, p.slots, p.qsl, p.seq_lens, p.req0, H, D, V}, ws, lay, nreq, s);
+    ScanParams sp{p.state, p.slots, p.qsl, p.seq_lens, p.req0, H, D, V};
+    sp.log2_decay = p.log2_decay;
+    sp.seg_state = ws + ((int64_t)rows / kC + nreq) * H * lay.size();
+    rc = launch_linear_scan(sp, ws, lay, nreq, (max_query_len + kC - 1) / kC, s);
   }
   if (rc != MI_OK) return rc;
   const LightningFinish f{a->out, a->gate, a->norm_w, chunked ? nullptr : ws, ws, a->query_start_loc, a->out_stride, a->gate_stride,

@@ -108,7 +108,7 @@ SIGNATURES = {
                                        c_int32, c_int32, c_int32, c_int, _P]),
     "mi_moe_rows_per_tile": (c_int32, [c_int32, c_int32, c_int32]),
     "mi_moe_max_rows": (c_int64, [c_int32, c_int32, c_int32, c_int32]),
-    "mi_moe_route": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, c_int32, c_int, c_int, _P]),
+    "mi_moe_route": (c_int, [_P, _P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, c_int32, c_int, c_int, _P]),
     "mi_moe_align": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, _P]),
     "mi_moe_expert_gemm": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64,
                                    c_int64, c_int32, c_int, _P]),
@@ -179,7 +179,6 @@ SIGNATURES = {
                                              c_int32, _P, c_int64, _P]),
     "mi_lightning_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32]),
     "mi_lightning_attn": (c_int, [POINTER(LightningArgs), c_int32, c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
-    "mi_moe_router_logits": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int64, _P]),
     "mi_moe_pair_gemm": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64,
                                  c_int, _P]),
     "mi_head_gemm_nt": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, _P]),

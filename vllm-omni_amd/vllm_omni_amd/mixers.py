@@ -19,7 +19,7 @@ import torch.nn.functional as F
 
 from . import ops
 from .kv_cache import KVCacheSpec, LatentCacheSpec, normalize_layer_kv
-from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu
+from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu, tuned_linear
 from .state_cache import StateSpec
 
 
@@ -411,7 +411,7 @@ class ChannelDelta(Sublayer):
     def run(self, x, y, step, memory) -> None:
         c, md = self.cfg, step.md
         qkv, low, beta = x
-        both = F.linear(low, self.low)
+        both = tuned_linear(low, self.low)
         hd = c.heads * c.dim
         args = (qkv, self.conv_w, self.a_log, self.dt_bias, self.norm, *memory.states, md.state_rows, md.query_start_loc, md.seq_lens,
                 c.kv_heads, self.eps, y[0])
@@ -457,7 +457,7 @@ class SinkAttention(Sublayer):
         self.slopes = None if cfg.slopes is None else torch.tensor(cfg.slopes, dtype=torch.float32, device=device)
 
     def kv_cache_spec(self, block_size: int) -> KVCacheSpec:
-        return KVCacheSpec(block_size, self.cfg.kv_heads, self.head_dim, self.dtype)
+        return KVCacheSpec(block_size, self.cfg.kv_heads, self.head_dim, self.dtype, self.cfg.heads)
 
     def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
         yield p + "q.norm", self.q_norm

@@ -583,6 +583,10 @@ class GPUARModelRunner:
             caches = {i: allocate_layer_cache(num_blocks, s, self.device, self.kv_layout) for i, s in spec.items()}
             self.kv_caches = list(caches.values())
             self.model.bind_kv_caches(caches)
+            shapes = {(s.num_q_heads, s.num_kv_heads, s.head_dim) for s in spec.values() if isinstance(s, KVCacheSpec)
+                      and ops.paged_attn_bias_supported(s.dtype, s.head_dim, s.block_size)}
+            if shapes:      # layers on the paged decode kernel
+                self._alloc_decode_workspace(shapes)
             self.state_cache = StateCache(self.max_num_reqs, self.device)
             self.model.bind_states(self.state_cache.allocate(self.model.state_specs()))
             from .block_table import CpuGpuBuffer
@@ -601,20 +605,23 @@ class GPUARModelRunner:
         # need any batch size of this runner can have.  `_decode_part` (reporting only) = the full batch's choice.
         self._decode_part = ops.decode_auto_partition(self.max_num_reqs, a.num_kv_heads, self.max_model_len,
                                                        self.block_size, head_dim=a.head_dim)
-        nbytes = max(ops.decode_workspace_bytes(b, a.num_heads, a.head_dim, self.max_model_len,
-                                                ops.decode_auto_partition(b, a.num_kv_heads, self.max_model_len,
-                                                                          self.block_size, head_dim=a.head_dim))
-                     for b in range(1, self.max_num_reqs + 1))
-        if torch.device(self.device).type == "cuda":
-            self._decode_ws = ops.new_decode_workspace(nbytes, self.device)   # zeroed counters: fused partition merge
-        else:
-            self._decode_ws = torch.empty(max(nbytes, 16), dtype=torch.uint8, device=self.device)
+        self._alloc_decode_workspace({(a.num_heads, a.num_kv_heads, a.head_dim)})
         if self.enable_prefix_caching and self.engine_output_type != "text":
             from .prefix_cache import OmniTensorPrefixCache
 
             # host tensor on the KV cache's own (block, offset) grid (gpu_model_runner.py:79-85)
             self.omni_prefix_cache = OmniTensorPrefixCache(num_blocks=num_blocks, block_size=self.block_size,
                                                            hidden_size=self.config.hidden_size, hs_dtype=self.dtype)
+
+    def _alloc_decode_workspace(self, shapes) -> None:
+        """the largest need of any batch size, over the layers' (query heads, kv heads, head size)"""
+        nbytes = max(ops.decode_workspace_bytes(b, nq, hd, self.max_model_len,
+                                                ops.decode_auto_partition(b, nkv, self.max_model_len, self.block_size, head_dim=hd))
+                     for nq, nkv, hd in shapes for b in range(1, self.max_num_reqs + 1))
+        if torch.device(self.device).type == "cuda":
+            self._decode_ws = ops.new_decode_workspace(nbytes, self.device)   # zeroed counters: fused partition merge
+        else:
+            self._decode_ws = torch.empty(max(nbytes, 16), dtype=torch.uint8, device=self.device)
 
     def _zero_block_ids(self, block_ids: list[int]) -> None:
         idx = torch.as_tensor(block_ids, dtype=torch.int64, device=self.device)

@@ -129,6 +129,6 @@ class RoutedExperts:
             yield f"{p}e{i}.down", self.down[i, :, :self.ff]
 
     def __call__(self, h: torch.Tensor) -> ops.ExpertRows:
-        logits = ops.moe_router_logits(h, self.router, self.router_b)
-        ids, weights, _ = ops.moe_route(logits, self.top, True, want_counts=False)
+        logits = ops.moe_router_logits(h, self.router)
+        ids, weights, _ = ops.moe_route(logits, self.top, True, want_counts=False, bias=self.router_b)
         return ops.moe_expert_rows(h, ids, weights, self.gate_up.flatten(1, 2), self.down)

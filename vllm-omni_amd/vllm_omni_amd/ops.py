@@ -346,7 +346,7 @@ ROPE_DECODE_FUSION = os.environ.get("VLLM_OMNI_AMD_ROPE_DECODE_FUSION", "1") != 
 def _head_vectors(nq: int, *ts: Optional[torch.Tensor]) -> None:
     for t in ts:
         if t is not None and (t.dtype != torch.float32 or t.numel() != nq or not t.is_contiguous()):
-            raise ValueError(f"expected {nq} contiguous fp32 values, one per query head")
+            raise ValueError(f"expected {nq} contiguous fp32 values")
 
 
 def paged_attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -1036,15 +1036,17 @@ def int8_linear_silu_mul(x: torch.Tensor, wq: torch.Tensor, w_scale: torch.Tenso
 
 # --------------------------------------------------------------------------- N4: fused sparse MoE
 def moe_route(router_logits: torch.Tensor, top_k: int, norm_topk_prob: bool, round_to: Optional[torch.dtype] = None,
-              want_counts: bool = True):
+              want_counts: bool = True, bias: Optional[torch.Tensor] = None):
     """-> (topk_ids int32 [T, k], topk_weights fp32 [T, k], expert_counts int32 [E] or None).  ``want_counts=False``:
-    no per-expert counting and no launch to zero the counters (``fused_moe``: the grouping counts the ids itself)."""
-    _gpu(router_logits)
+    no per-expert counting and no launch to zero the counters (``fused_moe``: the grouping counts the ids itself).
+    ``bias`` (fp32 [E]) is added to the logits.  ``norm_topk_prob``: a softmax over the chosen logits only."""
+    _gpu(router_logits, bias)
     t, e = router_logits.shape
+    _head_vectors(e, bias)
     ids = torch.empty(t, top_k, dtype=torch.int32, device=router_logits.device)
     w = torch.empty(t, top_k, dtype=torch.float32, device=router_logits.device)
     counts = torch.empty(e, dtype=torch.int32, device=router_logits.device) if want_counts else None
-    check("mi_moe_route", lib.mi_moe_route(_p(ids), _p(w), _p(counts), _p(router_logits), t, e, router_logits.stride(0),
+    check("mi_moe_route", lib.mi_moe_route(_p(ids), _p(w), _p(counts), _p(router_logits), _p(bias), t, e, router_logits.stride(0),
                                            int(top_k), 1 if norm_topk_prob else 0, _dt(router_logits.dtype),
                                            -1 if round_to is None else _dt(round_to), _stream()))
     return ids, w, counts
@@ -1573,21 +1575,12 @@ def lightning_attn(qkv: torch.Tensor, gate: torch.Tensor, norm_w: torch.Tensor, 
     return out
 
 
-def moe_router_logits(h: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor]) -> torch.Tensor:
-    """fp32 logits h weight^T + bias of bf16 rows (fp32 sums; fp32 rows take the library product)"""
-    _gpu(h, weight, bias)
-    hs, k = _rows(h)
-    if h.dtype == torch.float32 or k % 8 or hs % 8:
-        y = torch.nn.functional.linear(h.float(), weight.float())
-        return y if bias is None else y + bias
-    if weight.dtype != h.dtype or h.dtype != torch.bfloat16 or not weight.is_contiguous() or weight.shape[1] != k:
-        raise ValueError("moe_router_logits: contiguous bf16 weight of the rows' width")
-    if bias is not None:
-        _head_vectors(weight.shape[0], bias)
-    out = torch.empty(h.shape[0], weight.shape[0], dtype=torch.float32, device=h.device)
-    check("mi_moe_router_logits", lib.mi_moe_router_logits(_p(out), _p(h), _p(weight), _p(bias), h.shape[0], weight.shape[0], k, hs,
-                                                           _stream()))
-    return out
+def moe_router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """h weight^T, sums and result in fp32 (a library product; ``moe_route`` adds a bias)"""
+    _gpu(h, weight)
+    if h.dtype == torch.float32:
+        return torch.nn.functional.linear(h, weight)
+    return torch.mm(h, weight.t(), out_dtype=torch.float32)
 
 
 def moe_expert_rows(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor,
