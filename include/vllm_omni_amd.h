@@ -23,7 +23,7 @@
 extern "C" {
 #endif
 
-#define MI_ABI_VERSION 4
+#define MI_ABI_VERSION 5
 
 /* dtype enum shared by every entry point */
 enum {
@@ -931,6 +931,84 @@ int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const i
                      int32_t num_pairs, int32_t num_experts, int32_t gated, int32_t n_out, int32_t k,
                      int32_t top_k, int64_t a_row_stride, int64_t out_row_stride,
                      int64_t weight_expert_stride, int dtype, void* stream);
+
+/* ------------------------------------------------------------------------
+ * Decoders with a filter in front of every sublayer and attention whose heads
+ * mix their softmax weights (Bodopel): bf16 or fp32 as above.
+ *
+ * The filter: out = h + sum_b conv_w[taps - 1 - b] * h of b rows ago, per
+ * channel, zeros before the sequence's start; conv_w [taps][width].  A
+ * sequence's last taps - 1 rows live in its ring [slots][taps - 1][width], row
+ * of position p in place p % (taps - 1).
+ * ---------------------------------------------------------------------- */
+/* mi_residual_add_norm for one-token rows: x += y (+ add_row [width]), norm,
+ * filter (conv_w == NULL: none; slots and positions per row), ring update. */
+int mi_residual_add_norm_conv(void* x, const void* y, int32_t split, const void* add_row,
+                              const void* w_pre, float w_shift, void* h, const void* conv_w, void* ring,
+                              const int32_t* slots, const int64_t* positions, int32_t taps, float eps,
+                              int32_t rows, int32_t width, int64_t x_stride, int64_t y_stride,
+                              int64_t h_stride, int dtype, void* stream);
+/* x = scale * table[id] + pos_table[position] + add_row; norm, filter and ring
+ * as above (each of pos_table, add_row, conv_w may be NULL). */
+int mi_embed_pos_norm(void* x, void* h, const void* table, float scale, const void* pos_table,
+                      const int64_t* positions, int32_t max_positions, const void* add_row,
+                      const void* w_pre, float w_shift, const int64_t* ids, const void* conv_w, void* ring,
+                      const int32_t* slots, int32_t taps, float eps, int32_t rows, int32_t width,
+                      int32_t vocab, int64_t x_stride, int64_t h_stride, int dtype, void* stream);
+/* The filter and the ring update over portions of any length; slots per
+ * request; taps <= 33. */
+int mi_input_conv(void* out, const void* h, const void* conv_w, void* ring, const int32_t* slots,
+                  const int32_t* query_start_loc, const int32_t* seq_lens, int32_t req0,
+                  int32_t num_reqs, int32_t max_query_len, int32_t taps, int32_t width,
+                  int64_t h_stride, int64_t out_stride, int dtype, void* stream);
+/* relu(z)^2 of rows of dtype (split == 0) or of fp32 slabs [split][rows][z_stride] */
+int mi_relu_squared(void* out, const void* z, int32_t split, int32_t rows, int32_t ff, int64_t z_stride,
+                    int64_t out_stride, int dtype, void* stream);
+/* Rows q (heads x dim) | k (kv x dim) | v (kv x vdim): q RMS-normed over all its
+ * heads at once, k likewise (weights [heads * dim], [kv * dim]; NULL: not); q to
+ * q_out, k and v to their cache rows, heads head_dim apart, zeros behind them. */
+int mi_row_norm_cache(const void* x, int64_t x_stride, const void* q_weight, const void* k_weight,
+                      void* q_out, int64_t q_stride, void* k_cache, void* v_cache,
+                      const int64_t* slot_mapping, int32_t rows, int32_t num_q_heads,
+                      int32_t num_kv_heads, int32_t dim, int32_t vdim, int32_t head_dim,
+                      int32_t block_size, int64_t cache_block_stride, int64_t cache_token_stride,
+                      int64_t cache_head_stride, float eps, int dtype, void* stream);
+/* Causal attention over the last `window` keys of every row; score = softcap
+ * tanh(scale q.k / softcap) (softcap <= 0: scale q.k) - r1_h ln(1 + r2_h
+ * distance); weights = softmax; head h then uses sum_g talk[h][g] weights_g on
+ * its own key/value head; out = that * sigmoid(gate).  Heads are head_dim apart
+ * in q and the caches, vdim apart in out and gate. */
+typedef struct {
+  void* out;
+  const void *q, *k_cache, *v_cache;
+  const int32_t *block_table, *seq_lens, *query_start_loc;
+  const float *r1, *r2;   /* [heads]; both NULL: no distance bias */
+  const float* talk;      /* [heads][heads] */
+  const void* gate;       /* NULL: none */
+  int64_t q_stride, out_stride, gate_stride;
+  int64_t cache_block_stride, cache_token_stride, cache_head_stride, table_stride;
+  int32_t heads, kv_heads, head_dim, vdim, block_size, window;
+  float scale, softcap;
+} mi_talking_attn_args;
+/* rows [row0, row0 + rows) of num_reqs requests, any sizes and types */
+int mi_talking_attn_rows(const mi_talking_attn_args* args, int32_t row0, int32_t rows,
+                         int32_t num_reqs, int dtype, void* stream);
+/* whether the two forms below are built for these sizes (bf16) */
+int mi_talking_attn_supported(int32_t heads, int32_t kv_heads, int32_t head_dim, int32_t vdim,
+                              int32_t block_size, float softcap);
+/* one row per request, requests [0, num_reqs) */
+int64_t mi_talking_decode_workspace_bytes(int32_t num_reqs, int32_t heads, int32_t kv_heads, int32_t vdim,
+                                          int32_t window, int32_t max_seq_len);
+int mi_talking_decode(const mi_talking_attn_args* args, int32_t num_reqs, int32_t max_seq_len,
+                      void* workspace, int64_t workspace_bytes, void* stream);
+/* prompt portions.  seq_lens, query_start_loc and block_table are the portions'
+ * own; ctx_start [num_reqs + 1]: where a portion's visible context starts among
+ * ctx_rows rows (multiples of 64). */
+int64_t mi_talking_prefill_workspace_bytes(int32_t rows, int32_t heads, int32_t kv_heads,
+                                           int32_t head_dim, int32_t ctx_rows);
+int mi_talking_prefill(const mi_talking_attn_args* args, const int32_t* ctx_start, int32_t ctx_rows,
+                       int32_t num_reqs, int32_t rows, int32_t max_query_len, void* workspace,
+                       int64_t workspace_bytes, void* stream);
 
 #ifdef __cplusplus
 }

@@ -19,7 +19,7 @@ MI_DTYPE_F16, MI_DTYPE_BF16, MI_DTYPE_F32 = 0, 1, 2
 MI_OK = 0
 MI_ERR_INVALID_ARG, MI_ERR_UNSUPPORTED, MI_ERR_WORKSPACE = -1, -2, -3
 MI_ERR_LAUNCH, MI_ERR_EXHAUSTED, MI_ERR_STATE = -4, -5, -6
-ABI_VERSION = 4
+ABI_VERSION = 5
 MI_LINEAR_PLAN_FULL, MI_LINEAR_PLAN_PARTIALS, MI_LINEAR_PLAN_GATED = 0, 1, 2
 MI_LINEAR_COUNTER_BYTES = 16 << 10
 MI_DECODE_PACKED_PV = 1
@@ -51,6 +51,17 @@ class LightningArgs(ctypes.Structure):
                                         "seq_lens", "out")] \
         + [(n, c_int64) for n in ("qkv_stride", "gate_stride", "out_stride")] \
         + [(n, c_int32) for n in ("req0", "num_reqs", "heads", "dim", "vdim")] + [("eps", c_float), ("mul", c_float)]
+
+
+class TalkingAttnArgs(ctypes.Structure):
+    """mi_talking_attn_args"""
+
+    _fields_ = [(n, c_void_p) for n in ("out", "q", "k_cache", "v_cache", "block_table", "seq_lens", "query_start_loc", "r1", "r2",
+                                        "talk", "gate")] \
+        + [(n, c_int64) for n in ("q_stride", "out_stride", "gate_stride", "cache_block_stride", "cache_token_stride",
+                                  "cache_head_stride", "table_stride")] \
+        + [(n, c_int32) for n in ("heads", "kv_heads", "head_dim", "vdim", "block_size", "window")] \
+        + [("scale", c_float), ("softcap", c_float)]
 
 
 # name -> (restype, argtypes); mirrors include/vllm_omni_amd.h declaration by declaration
@@ -181,6 +192,20 @@ SIGNATURES = {
     "mi_lightning_attn": (c_int, [POINTER(LightningArgs), c_int32, c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
     "mi_moe_pair_gemm": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64,
                                  c_int, _P]),
+    "mi_residual_add_norm_conv": (c_int, [_P, _P, c_int32, _P, _P, c_float, _P, _P, _P, _P, _P, c_int32, c_float, c_int32, c_int32, c_int64,
+                                          c_int64, c_int64, c_int, _P]),
+    "mi_embed_pos_norm": (c_int, [_P, _P, _P, c_float, _P, _P, c_int32, _P, _P, c_float, _P, _P, _P, _P, c_int32, c_float, c_int32, c_int32,
+                                  c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_input_conv": (c_int, [_P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_relu_squared": (c_int, [_P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_row_norm_cache": (c_int, [_P, c_int64, _P, _P, _P, c_int64, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32,
+                                  c_int32, c_int64, c_int64, c_int64, c_float, c_int, _P]),
+    "mi_talking_attn_rows": (c_int, [POINTER(TalkingAttnArgs), c_int32, c_int32, c_int32, c_int, _P]),
+    "mi_talking_attn_supported": (c_int, [c_int32, c_int32, c_int32, c_int32, c_int32, c_float]),
+    "mi_talking_decode_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32]),
+    "mi_talking_decode": (c_int, [POINTER(TalkingAttnArgs), c_int32, c_int32, _P, c_int64, _P]),
+    "mi_talking_prefill_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32]),
+    "mi_talking_prefill": (c_int, [POINTER(TalkingAttnArgs), _P, c_int32, c_int32, c_int32, c_int32, _P, c_int64, _P]),
     "mi_head_gemm_nt": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, _P]),
     "mi_latent_decode_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32]),
     "mi_latent_decode": (c_int, [_P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float, c_int64, c_int64,

@@ -51,6 +51,8 @@ class LLMEngine:
             weights = checkpoint_tensors(model) if weights is None else weights
         else:
             config = model
+        if getattr(config, "max_positions", None):      # a learned position per token: no sequence is longer than the table
+            max_model_len = min(max_model_len, config.max_positions)
         wc = WorkerConfig(model_config=config, dtype=torch_dtype(dtype), gpu_memory_utilization=gpu_memory_utilization,
                           block_size=block_size, max_num_seqs=max_num_seqs, max_model_len=max_model_len,
                           max_num_batched_tokens=max(max_num_batched_tokens, max_num_seqs), enforce_eager=enforce_eager,

@@ -595,7 +595,7 @@ class KVCacheSpec:
     num_kv_heads: int
     head_dim: int
     dtype: torch.dtype
-    num_q_heads: int = 0      # query heads of the layer that reads it (sizes the decode workspace); 0: not known
+    num_q_heads: int = 0      # query heads of the layer that reads it (sizes the paged decode kernel's workspace); 0: read by another kernel
 
     @property
     def page_bytes(self) -> int:

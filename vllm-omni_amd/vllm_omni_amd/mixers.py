@@ -1,9 +1,9 @@
 """Sequence mixers and small blocks of decoders with a 32-bit residual stream: latent attention without positions
 (its cache row shared by all heads, optionally by several layers), the gated delta rule with a decay per head or per key
-channel, attention with a distance bias and a sink, decayed linear attention, and several mixers side by side.  Constants
-that a design fixes are parameters here; the layers know nothing of the model they are in.
+channel, attention with a distance bias and a sink, decayed linear attention, several mixers side by side, attention whose
+heads mix their softmax weights, and a short filter in front of a sublayer.  Constants that a design fixes are parameters here; the layers know nothing of the model they are in.
 
-Two kinds: mixers that own their projections (``LatentAttention``, ``GatedDelta``: rows in, rows out), and mixers for layers
+Two kinds: mixers that own their projections (``LatentAttention``, ``GatedDelta``, ``TalkingAttention``: rows in, rows out), and mixers for layers
 whose sublayers all read one normed row and add up (``ChannelDelta``, ``SinkAttention``, ``LightningAttention``,
 ``ParallelMixers``, ``DenseGlu``): such a layer has ONE input product and ONE output product (``SharedProjections``), and a
 sublayer names its blocks of both, turning columns of the first into columns the second reads.
@@ -12,7 +12,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass, field
-from typing import Iterable, Optional, Sequence
+from typing import Iterable, Iterator, Optional, Sequence
 
 import torch
 import torch.nn.functional as F
@@ -29,25 +29,29 @@ def _pad16(n: int) -> int:
 
 class ReplicatedLinear:
     """y = x W^T, not sharded; routed like the decoder's other linears.  ``parts`` names row blocks of the weight that a
-    checkpoint stores apart; rows past their sum (padding to a multiple of 16) stay zero."""
+    checkpoint stores apart; rows past their sum (padding to a multiple of 16) stay zero.  ``biased``: the parts that have a
+    bias (stored as ``<part>.b``); the others' stays zero."""
 
-    def __init__(self, in_features: int, parts: dict[str, int], dtype, device, generator=None, pad: bool = False):
-        self.parts = parts
+    def __init__(self, in_features: int, parts: dict[str, int], dtype, device, generator=None, pad: bool = False,
+                 biased: Sequence[str] = ()):
+        self.parts, self.biased = parts, biased
         n = sum(parts.values())
         self.out_features = n
         self.weight = _init_weight(_pad16(n) if pad else n, in_features, dtype, device, generator, std=in_features ** -0.5)
         if pad:
             self.weight[n:].zero_()
-        self.bias = None
+        self.bias = torch.zeros(self.weight.shape[0], dtype=dtype, device=device) if biased else None
 
     def named(self, prefix: str) -> Iterable[tuple[str, torch.Tensor]]:
         r = 0
         for name, n in self.parts.items():
             yield prefix + name, self.weight[r:r + n]
+            if name in self.biased:
+                yield prefix + name + ".b", self.bias[r:r + n]
             r += n
 
     def __call__(self, x: torch.Tensor, defer_reduce: bool = False):
-        return _apply_linear(self, x, None, defer_reduce)
+        return _apply_linear(self, x, self.bias, defer_reduce)
 
 
 @dataclass
@@ -237,6 +241,109 @@ class TokenSideInput:
 
     def __call__(self, x: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, defer_reduce: bool = False):
         return self.proj(ops.gelu_lookup_mul(self.gate(x), table, ids, self.offset), defer_reduce)
+
+
+@dataclass
+class TalkingAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: Optional[int] = None      # tokens a query sees, itself included; None: all before it
+    softcap: float = 0.0              # 0: none
+
+
+class TalkingAttention:
+    """Grouped-query attention whose heads mix their softmax weights, with soft-capped scores, a distance bias of
+    r1 ln(1 + r2 distance), q and k each normed over all heads at once, and a gate on the concatenated heads
+    (``csrc/talking_attn.hip``, ``csrc/talking_attn_mfma.hip``)."""
+
+    def __init__(self, cfg: TalkingAttentionConfig, width: int, eps: float, dtype, device, generator=None):
+        if cfg.heads % cfg.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if cfg.window is not None and cfg.window < 1:
+            raise ValueError("a window holds at least the token itself")
+        if cfg.softcap < 0:
+            raise ValueError("the soft cap must be positive")
+        self.cfg, self.eps, self.dtype = cfg, eps, dtype
+        self.window = cfg.window if cfg.window is not None else 2**31 - 1
+        big = max(cfg.dim, cfg.vdim)
+        # heads are laid out to the sizes the matrix-core kernels are built for
+        self.head_dim = -(-big // 8) * 8 if dtype != torch.bfloat16 or big > 128 else 64 if big <= 64 else 128
+        nq, nk, nv, ng = cfg.heads * cfg.dim, cfg.kv_heads * cfg.dim, cfg.kv_heads * cfg.vdim, cfg.heads * cfg.vdim
+        self.qkv, self.gated = nq + nk + nv, ng
+        self.proj = ReplicatedLinear(width, {"q": nq, "k": nk, "v": nv, "g": ng}, dtype, device, generator, pad=True,
+                                     biased=("q", "k", "v"))
+        self.o = ReplicatedLinear(ng, {"o": width}, dtype, device, generator)
+        self.q_norm, self.k_norm = _vec(nq, dtype, device), _vec(nk, dtype, device)
+        self.r1, self.r2 = _vec(cfg.heads, torch.float32, device), _vec(cfg.heads, torch.float32, device)
+        self.talk = torch.eye(cfg.heads, dtype=torch.float32, device=device)
+        self.heads = ops.TalkingHeads(self.talk, self.r1, self.r2, cfg.scale, cfg.softcap, self.window, cfg.vdim)
+
+    def kv_cache_spec(self, block_size: int) -> KVCacheSpec:
+        return KVCacheSpec(block_size, self.cfg.kv_heads, self.head_dim, self.dtype)
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield from self.proj.named(p)
+        yield from self.o.named(p)
+        yield p + "q.norm", self.q_norm
+        yield p + "k.norm", self.k_norm
+        yield p + "r1", self.r1
+        yield p + "r2", self.r2
+        yield p + "talk", self.talk
+
+    def __call__(self, h: torch.Tensor, md: AttentionMetadata, memory: "LayerMemory", defer_reduce: bool = False):
+        c = self.cfg
+        kc, vc = memory.kv
+        x = self.proj(h)
+        q = ops.row_norm_cache(x[:, :self.qkv], self.q_norm, self.k_norm, kc, vc, md.slot_mapping, c.heads, c.dim, c.vdim, self.eps)
+        gate = x[:, self.qkv:self.qkv + self.gated]
+        out = torch.empty(h.shape[0], self.gated, dtype=self.dtype, device=h.device)
+        args = (out, q, kc, vc)
+        if not ops.talking_attn_supported(self.dtype, c.heads, c.kv_heads, self.head_dim, c.vdim, kc.shape[1], c.softcap):
+            ops.talking_attn_rows(*args, md.block_table, md.seq_lens, md.query_start_loc, self.heads, gate)
+            return self.o(out, defer_reduce)
+        nd, n = md.num_decodes, md.num_reqs
+        if nd:
+            ops.talking_decode(*args, md.block_table, md.seq_lens, md.query_start_loc, self.heads, md.max_seq_len, nd, gate)
+        if nd < n:      # the portions' row offsets count from the step's first row, so the operands go whole
+            start, rows = md.prefill_ctx[self.window]
+            ops.talking_prefill(*args, md.block_table[nd:n], md.seq_lens[nd:n], md.query_start_loc[nd:n + 1], self.heads, start, rows,
+                                md.max_query_len, gate)
+        return self.o(out, defer_reduce)
+
+
+class InputConv:
+    """h + a causal filter per channel over h: what a sublayer reads in place of h (``csrc/residual_norm.hip``)"""
+
+    def __init__(self, width: int, taps: int, dtype, device, generator=None):
+        if taps < 1:
+            raise ValueError("a filter has at least the tap of the row itself")
+        self.width, self.taps, self.dtype = width, taps, dtype
+        self.weight = _init_weight(taps, width, dtype, device, generator, std=0.5 * taps ** -0.5)
+
+    def state_specs(self) -> list[StateSpec]:
+        return [StateSpec((self.taps - 1, self.width), self.dtype)] if self.taps > 1 else []
+
+    def bind(self, it: Iterator[torch.Tensor]) -> ops.ConvRing:
+        """one layer run's filter, its ring taken from the run's state tensors"""
+        return ops.ConvRing(self.weight, next(it) if self.taps > 1 else None)
+
+
+class SquaredReluMLP:
+    """down(relu(up h)^2)"""
+
+    def __init__(self, width: int, ff: int, dtype, device, generator=None):
+        self.up = ReplicatedLinear(width, {"up": ff}, dtype, device, generator)
+        self.down = ReplicatedLinear(ff, {"down": width}, dtype, device, generator)
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield from self.up.named(p)
+        yield from self.down.named(p)
+
+    def __call__(self, h: torch.Tensor, defer_reduce: bool = False):
+        return self.down(ops.relu_squared(self.up(h, True)), defer_reduce)
 
 
 # ------------------------------------------------------------------------------------------ sublayers side by side

@@ -515,6 +515,9 @@ class GPUARModelRunner:
 
     # -------------------------------------------------------------------- model
     def load_model(self) -> None:
+        limit = getattr(self.config, "max_positions", None)
+        if limit and self.max_model_len > limit:
+            raise ValueError(f"max_model_len {self.max_model_len} exceeds the model's position table of {limit}")
         if torch.device(self.device).type == "cuda":
             from .tuned import enable_tuned_gemms
 
@@ -583,7 +586,7 @@ class GPUARModelRunner:
             caches = {i: allocate_layer_cache(num_blocks, s, self.device, self.kv_layout) for i, s in spec.items()}
             self.kv_caches = list(caches.values())
             self.model.bind_kv_caches(caches)
-            shapes = {(s.num_q_heads, s.num_kv_heads, s.head_dim) for s in spec.values() if isinstance(s, KVCacheSpec)
+            shapes = {(s.num_q_heads, s.num_kv_heads, s.head_dim) for s in spec.values() if isinstance(s, KVCacheSpec) and s.num_q_heads
                       and ops.paged_attn_bias_supported(s.dtype, s.head_dim, s.block_size)}
             if shapes:      # layers on the paged decode kernel
                 self._alloc_decode_workspace(shapes)
@@ -1215,6 +1218,11 @@ class GPUARModelRunner:
         if self._last_output is not None and not self._last_output.done and (
                 self._generic_hooks or not self._steady_decode(scheduler_output)):
             self._last_output.get_output()
+        # the previous step's host->device index copies read pinned buffers that are written from here on: the batch's own
+        # block-table rows (requests that come and go) as well as the step's arrays
+        if self._h2d_pending:
+            self._h2d_done.synchronize()
+            self._h2d_pending = False
         kv_done = None
         if scheduler_output.finished_requests_needing_kv_transfer:
             kv_done = self._extract_finished_kv(scheduler_output.finished_requests_needing_kv_transfer)
@@ -1223,9 +1231,6 @@ class GPUARModelRunner:
             if kv_done:
                 return OmniModelRunnerOutput([], {}, [], [], kv_extracted_req_ids=kv_done)
             return EMPTY_MODEL_RUNNER_OUTPUT
-        if self._h2d_pending:   # the previous step's host->device index copies read the pinned buffers written below
-            self._h2d_done.synchronize()
-            self._h2d_pending = False
         n, total, num_sched, max_seq_len, num_decodes = self._prepare_inputs(scheduler_output)
         use_graph = self._can_use_graph(n, total, num_decodes)
         if use_graph:

@@ -1616,3 +1616,237 @@ def moe_expert_rows(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w
         check("mi_moe_pair_gemm", lib.mi_moe_pair_gemm(_p(out), _p(a), _p(w), _p(ids), t * top, e, gated, n, kk, top, a.stride(0),
                                                        out.stride(0), w.stride(0), dt, _stream()))
     return ExpertRows(part, weights, None)
+
+
+# ------------------------------------------------- a filter in front of every sublayer, heads that mix their softmax weights
+class ConvRing:
+    """The filter of one sublayer in one layer run: ``weight`` [taps, width] (the last one for the row itself) and the ring of
+    every state slot's last taps - 1 rows [slots, taps - 1, width] (None when taps is 1)."""
+
+    def __init__(self, weight: torch.Tensor, ring: Optional[torch.Tensor]):
+        taps, width = weight.shape
+        if not weight.is_contiguous():
+            raise ValueError("filter weights must be contiguous")
+        if taps > 1 and (ring is None or tuple(ring.shape[1:]) != (taps - 1, width) or not ring.is_contiguous() or ring.dtype != weight.dtype):
+            raise ValueError("a ring of taps - 1 rows per slot, in the weights' dtype")
+        self.weight, self.ring, self.taps, self.width = weight, ring, taps, width
+
+
+def _conv_rows(conv: Optional[ConvRing], slots, positions, rows: int, width: int, dtype):
+    """C arguments (weight, ring, slots, positions, taps) of the one-token form"""
+    if conv is None:
+        return None, None, None, None, 0
+    _gpu(conv.weight, conv.ring, slots, positions)
+    _i32(slots)
+    _i64(positions)
+    if conv.width != width or conv.weight.dtype != dtype or slots.numel() < rows or positions.numel() < rows:
+        raise ValueError("filter of another width or dtype, or too few slots and positions")
+    return _p(conv.weight), _p(conv.ring), _p(slots), _p(positions), conv.taps
+
+
+def residual_add_norm_conv(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials"], w_pre: Optional[torch.Tensor], eps: float,
+                           h: torch.Tensor, w_shift: float = 0.0, add_row: Optional[torch.Tensor] = None,
+                           conv: Optional[ConvRing] = None, slots: Optional[torch.Tensor] = None,
+                           positions: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``residual_add_norm`` with a row ``add_row`` added to every row's stream, and the filter over ``h`` of rows that are
+    their sequences' only new ones (``slots``, ``positions`` per row)."""
+    part = isinstance(y, SplitKPartials)
+    if part:
+        y._live()
+        if y.bias is not None:
+            raise ValueError("partials of a linear without bias")
+    src = y.part if part else y
+    _gpu(x, src, w_pre, h, add_row)
+    xs, width = _rows(x)
+    hs, hw = _rows(h)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or hw != width or h.shape[0] < rows:
+        raise ValueError("residual_add_norm_conv: fp32 stream, h of its width")
+    for w in (w_pre, add_row):
+        if w is not None and (w.numel() != width or w.dtype != h.dtype or not w.is_contiguous()):
+            raise ValueError("residual_add_norm_conv: weights of the stream's width in h's dtype")
+    if part:
+        if (y.m, y.n) != (rows, width):
+            raise ValueError("partials of another shape")
+        split, ys = y.split, width
+    else:
+        ys, yw = _rows(y)
+        if y.shape[0] != rows or yw != width or y.dtype not in (h.dtype, torch.float32):
+            raise ValueError("layer output of another shape or dtype")
+        split = 1 if y.dtype == torch.float32 and h.dtype != torch.float32 else 0
+    cw, ring, sl, pos, taps = _conv_rows(conv, slots, positions, rows, width, h.dtype)
+    check("mi_residual_add_norm_conv", lib.mi_residual_add_norm_conv(
+        _p(x), _p(src), split, _p(add_row), _p(w_pre), float(w_shift), _p(h), cw, ring, sl, pos, taps, float(eps), rows, width, xs, ys, hs,
+        _dt(h.dtype), _stream()))
+    return h
+
+
+def embed_pos_norm(table: torch.Tensor, ids: torch.Tensor, x: torch.Tensor, w_pre: Optional[torch.Tensor], eps: float, h: torch.Tensor,
+                   positions: torch.Tensor, scale: float = 1.0, pos_table: Optional[torch.Tensor] = None,
+                   add_row: Optional[torch.Tensor] = None, w_shift: float = 0.0, conv: Optional[ConvRing] = None,
+                   slots: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x = scale * table[ids] + pos_table[positions] + add_row (fp32); ``h`` as in ``residual_add_norm_conv``"""
+    _gpu(table, ids, x, w_pre, h, positions, pos_table, add_row)
+    _i64(ids, positions)
+    xs, width = _rows(x)
+    hs, hw = _rows(h)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or not table.is_contiguous() or (table.shape[1], hw) != (width, width) or h.shape[0] < rows \
+            or ids.numel() != rows or positions.numel() < rows:
+        raise ValueError("embed_pos_norm: sizes do not fit")
+    for w in (w_pre, add_row):
+        if w is not None and (w.numel() != width or not w.is_contiguous()):
+            raise ValueError("embed_pos_norm: sizes do not fit")
+    if pos_table is not None and (pos_table.shape[1] != width or not pos_table.is_contiguous()):
+        raise ValueError("embed_pos_norm: position table of another width")
+    if any(t is not None and t.dtype != table.dtype for t in (h, w_pre, pos_table, add_row)):
+        raise TypeError("embed_pos_norm: one dtype")
+    cw, ring, sl, _, taps = _conv_rows(conv, slots, positions, rows, width, h.dtype)
+    check("mi_embed_pos_norm", lib.mi_embed_pos_norm(
+        _p(x), _p(h), _p(table), float(scale), _p(pos_table), _p(positions), pos_table.shape[0] if pos_table is not None else 0,
+        _p(add_row), _p(w_pre), float(w_shift), _p(ids), cw, ring, sl, taps, float(eps), rows, width, table.shape[0], xs, hs,
+        _dt(table.dtype), _stream()))
+    return h
+
+
+def input_conv(h: torch.Tensor, conv: ConvRing, slots: torch.Tensor, query_start_loc: torch.Tensor, seq_lens: torch.Tensor,
+               num_reqs: int, max_query_len: int, req0: int = 0) -> torch.Tensor:
+    """h plus the filter over it, for portions of any length; leaves each request's last rows in its ring"""
+    _gpu(h, conv.weight, conv.ring, slots, query_start_loc, seq_lens)
+    _i32(slots, query_start_loc, seq_lens)
+    hs, width = _rows(h)
+    if conv.width != width or conv.weight.dtype != h.dtype:
+        raise ValueError("filter of another width or dtype")
+    if min(slots.numel(), seq_lens.numel(), query_start_loc.numel() - 1) < req0 + num_reqs:
+        raise ValueError("input_conv: request range outside the metadata")
+    out = torch.empty(h.shape[0], width, dtype=h.dtype, device=h.device)
+    check("mi_input_conv", lib.mi_input_conv(
+        _p(out), _p(h), _p(conv.weight), _p(conv.ring), _p(slots), _p(query_start_loc), _p(seq_lens), req0, num_reqs, max_query_len,
+        conv.taps, width, hs, out.stride(0), _dt(h.dtype), _stream()))
+    return out
+
+
+def relu_squared(z: Union[torch.Tensor, "SplitKPartials"]) -> torch.Tensor:
+    """relu(z)^2; ``z`` may be the split-K partials of a linear without bias"""
+    if isinstance(z, SplitKPartials):
+        z._live()
+        if z.bias is not None:
+            raise ValueError("partials of a linear without bias")
+        src, split, rows, ff, zs, dtype = z.part, z.split, z.m, z.n, z.n, z.dtype
+    else:
+        zs, ff = _rows(z)
+        src, split, rows, dtype = z, 0, z.shape[0], z.dtype
+    _gpu(src)
+    out = torch.empty(rows, ff, dtype=dtype, device=src.device)
+    check("mi_relu_squared", lib.mi_relu_squared(_p(out), _p(src), split, rows, ff, zs, out.stride(0), _dt(dtype), _stream()))
+    return out
+
+
+def row_norm_cache(x: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], k_cache: torch.Tensor,
+                   v_cache: torch.Tensor, slot_mapping: torch.Tensor, num_q_heads: int, dim: int, vdim: int, eps: float) -> torch.Tensor:
+    """Rows q | k | v: q and k each normed over all heads at once, K / V cache write; returns q, heads laid out as in the cache."""
+    _gpu(x, q_weight, k_weight, k_cache, v_cache, slot_mapping)
+    _i64(slot_mapping)
+    xs, cols = _rows(x)
+    rows = x.shape[0]
+    _, bs, g, hd = k_cache.shape
+    cb, ct, ch = _cache_strides(k_cache, v_cache)
+    if cols != (num_q_heads + g) * dim + g * vdim or slot_mapping.numel() < rows or max(dim, vdim) > hd:
+        raise ValueError("row_norm_cache: sizes do not fit")
+    for w, n in ((q_weight, num_q_heads * dim), (k_weight, g * dim)):
+        if w is not None and (w.numel() != n or w.dtype != x.dtype):
+            raise ValueError("row_norm_cache: norm weights of the projection's size")
+    if x.dtype != k_cache.dtype:
+        raise TypeError("cache and activations share a dtype")
+    q = torch.empty(rows, num_q_heads * hd, dtype=x.dtype, device=x.device)
+    check("mi_row_norm_cache", lib.mi_row_norm_cache(
+        _p(x), xs, _p(q_weight), _p(k_weight), _p(q), q.stride(0), _p(k_cache), _p(v_cache), _p(slot_mapping), rows, num_q_heads, g, dim,
+        vdim, hd, bs, cb, ct, ch, float(eps), _dt(x.dtype), _stream()))
+    return q
+
+
+class TalkingHeads:
+    """What attention with mixed heads needs besides its operands: fp32 ``talk`` [H, H], ``r1`` / ``r2`` [H] (or None), scale,
+    soft cap (0: none), window, value size."""
+
+    def __init__(self, talk: torch.Tensor, r1: Optional[torch.Tensor], r2: Optional[torch.Tensor], scale: float, softcap: float,
+                 window: int, vdim: int):
+        h = talk.shape[0]
+        if talk.dtype != torch.float32 or tuple(talk.shape) != (h, h) or not talk.is_contiguous():
+            raise ValueError("talk: contiguous fp32 [heads, heads]")
+        if (r1 is None) != (r2 is None):
+            raise ValueError("r1 and r2 go together")
+        _head_vectors(h, r1, r2)
+        self.talk, self.r1, self.r2, self.scale, self.softcap, self.vdim = talk, r1, r2, float(scale), float(softcap), int(vdim)
+        self.heads, self.window = h, min(int(window), 2**31 - 1)
+
+
+def _talking_args(out, q, kc, vc, table, seq_lens, qsl, th: TalkingHeads, gate, n: int):
+    _gpu(out, q, kc, vc, table, seq_lens, qsl, th.talk, th.r1, th.r2, gate)
+    _i32(seq_lens, qsl)
+    _, bs, g, hd = kc.shape
+    cb, ct, ch = _cache_strides(kc, vc)
+    qs, qc = _rows(q)
+    os_, oc = _rows(out)
+    if qc != th.heads * hd or oc != th.heads * th.vdim or table.dtype != torch.int32 or table.stride(1) != 1:
+        raise ValueError("talking attention: sizes do not fit")
+    if not q.dtype == out.dtype == kc.dtype or (gate is not None and gate.dtype != q.dtype):
+        raise TypeError("talking attention: one dtype")
+    gs = 0
+    if gate is not None:
+        gs, gc = _rows(gate)
+        if gc != oc or gate.shape[0] < out.shape[0]:
+            raise ValueError("talking attention: a gate per output value")
+    if min(table.shape[0], seq_lens.numel(), qsl.numel() - 1) < n:
+        raise ValueError("talking attention: one metadata entry per request")
+    return _C.TalkingAttnArgs(_p(out), _p(q), _p(kc), _p(vc), _p(table), _p(seq_lens), _p(qsl), _p(th.r1), _p(th.r2), _p(th.talk), _p(gate),
+                              qs, os_, gs, cb, ct, ch, table.stride(0), th.heads, g, hd, th.vdim, bs, th.window, th.scale, th.softcap)
+
+
+def talking_attn_rows(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                      seq_lens: torch.Tensor, query_start_loc: torch.Tensor, th: TalkingHeads, gate: Optional[torch.Tensor] = None,
+                      row0: int = 0) -> torch.Tensor:
+    """Attention with mixed heads of rows [row0, T), any sizes and types"""
+    n = seq_lens.shape[0]
+    a = _talking_args(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, th, gate, n)
+    if out.shape[0] < q.shape[0]:
+        raise ValueError("talking_attn_rows: sizes do not fit")
+    check("mi_talking_attn_rows", lib.mi_talking_attn_rows(ctypes.byref(a), row0, q.shape[0] - row0, n, _dt(q.dtype), _stream()))
+    return out
+
+
+def talking_attn_supported(dtype: torch.dtype, heads: int, kv_heads: int, head_dim: int, vdim: int, block_size: int, softcap: float) -> bool:
+    """whether the matrix-core forms take these sizes"""
+    return dtype == torch.bfloat16 and bool(lib.mi_talking_attn_supported(heads, kv_heads, head_dim, vdim, block_size, float(softcap)))
+
+
+def talking_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                   seq_lens: torch.Tensor, query_start_loc: torch.Tensor, th: TalkingHeads, max_seq_len: int, num_reqs: int,
+                   gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """One row per request: rows and requests [0, num_reqs)"""
+    a = _talking_args(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, th, gate, num_reqs)
+    if min(q.shape[0], out.shape[0]) < num_reqs:
+        raise ValueError("talking_decode: sizes do not fit")
+    need = lib.mi_talking_decode_workspace_bytes(num_reqs, th.heads, k_cache.shape[2], th.vdim, th.window, max_seq_len)
+    ws = torch.empty(max(need, 1), dtype=torch.uint8, device=q.device)
+    check("mi_talking_decode", lib.mi_talking_decode(ctypes.byref(a), num_reqs, max_seq_len, _p(ws), need, _stream()))
+    return out
+
+
+def talking_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                    seq_lens: torch.Tensor, query_start_loc: torch.Tensor, th: TalkingHeads, ctx_start: torch.Tensor, ctx_rows: int,
+                    max_query_len: int, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Prompt portions: metadata of the portions alone, row offsets counted from the step's first row; ``ctx_start``: where a
+    portion's visible context starts among ``ctx_rows`` gathered rows (multiples of 64)."""
+    n = seq_lens.shape[0]
+    a = _talking_args(out, q, k_cache, v_cache, block_table, seq_lens, query_start_loc, th, gate, n)
+    _gpu(ctx_start)
+    _i32(ctx_start)
+    if out.shape[0] < q.shape[0] or ctx_start.numel() < n + 1:
+        raise ValueError("talking_prefill: sizes do not fit")
+    rows, g, hd = q.shape[0], k_cache.shape[2], k_cache.shape[3]
+    need = lib.mi_talking_prefill_workspace_bytes(rows, th.heads, g, hd, ctx_rows)
+    ws = torch.empty(max(need, 1), dtype=torch.uint8, device=q.device)
+    check("mi_talking_prefill", lib.mi_talking_prefill(ctypes.byref(a), _p(ctx_start), ctx_rows, n, rows, max_query_len, _p(ws), need,
+                                                       _stream()))
+    return out

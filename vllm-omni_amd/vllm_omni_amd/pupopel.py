@@ -23,7 +23,7 @@ from .mixers import (ChannelDelta, ChannelDeltaConfig, DenseGlu, LayerMemory, Li
                      SharedProjections, SinkAttention, SinkAttentionConfig, StepInfo, Sublayer)
 from .moe import RoutedExperts
 from .state_cache import StateSpec
-from .text_model import TokenDecoder
+from .text_model import LoopConfig, TokenDecoder, layer_runs
 
 NORM_SHIFT = 1.0        # norm weights of the stream are stored as their distance from one
 DENSE_ACT, EXPERT_ACT = "gelu_tanh", "silu"
@@ -56,13 +56,6 @@ class PupopelLayerConfig:
 
 
 @dataclass
-class LoopConfig:
-    start: int
-    stop: int
-    times: int
-
-
-@dataclass
 class PupopelConfig:
     vocab_size: int
     hidden_size: int
@@ -82,11 +75,7 @@ class PupopelConfig:
     @property
     def runs(self) -> list[tuple[int, bool]]:
         """(layer, whether a pass of the loop starts with it), in the order the layers run"""
-        n, lp = len(self.layers), self.loop
-        if lp is None:
-            return [(i, False) for i in range(n)]
-        one = [(i, i == lp.start) for i in range(lp.start, lp.stop)]
-        return [(i, False) for i in range(lp.start)] + one * lp.times + [(i, False) for i in range(lp.stop, n)]
+        return [(i, start is not None) for i, start in layer_runs(len(self.layers), self.loop)]
 
     @classmethod
     def from_dict(cls, d: dict, shapes: Optional[dict] = None) -> "PupopelConfig":
@@ -140,9 +129,8 @@ class PupopelConfig:
     def validate(self) -> None:
         if not self.layers:
             raise ValueError("a model has at least one layer")
-        lp = self.loop
-        if lp is not None and not (0 <= lp.start < lp.stop <= len(self.layers) and lp.times >= 1):
-            raise ValueError(f"loop {lp.start}..{lp.stop} x {lp.times} does not fit {len(self.layers)} layers")
+        if self.loop is not None:
+            self.loop.validate(len(self.layers))
 
 
 class PupopelDecoderLayer:

@@ -17,6 +17,7 @@ from .compat import _get
 ARCHITECTURES = {
     "Qwen2_5OmniTalkerForConditionalGeneration": ("talker", "TalkerConfig", "Qwen2_5OmniTalkerForConditionalGeneration"),
     "Dogulorn": ("dogulorn", "DogulornConfig", "DogulornForCausalLM"),
+    "Bodopel": ("bodopel", "BodopelConfig", "BodopelForCausalLM"),
     "Pupopel": ("pupopel", "PupopelConfig", "PupopelForCausalLM"),
 }
 DEFAULT_ARCHITECTURE = "Qwen2_5OmniTalkerForConditionalGeneration"

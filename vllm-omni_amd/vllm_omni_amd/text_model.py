@@ -1,12 +1,34 @@
-"""What decoders that take token ids share: the runner's view of such a model, logits, checkpoint loading."""
+"""What decoders that take token ids share: the runner's view of such a model, logits, checkpoint loading, looped layers."""
 from __future__ import annotations
 
+from dataclasses import dataclass
 from typing import Any, Iterable, Optional
 
 import torch
 
 from . import ops
 from .layers import tuned_linear
+
+
+@dataclass
+class LoopConfig:
+    """layers start .. stop - 1 run ``times`` times in a row"""
+
+    start: int
+    stop: int
+    times: int
+
+    def validate(self, layers: int) -> None:
+        if not (0 <= self.start < self.stop <= layers and self.times >= 1):
+            raise ValueError(f"loop {self.start}..{self.stop} x {self.times} does not fit {layers} layers")
+
+
+def layer_runs(n: int, loop: Optional[LoopConfig]) -> list[tuple[int, Optional[int]]]:
+    """(layer, pass of the loop that starts with it or None), in the order ``n`` layers run"""
+    if loop is None:
+        return [(i, None) for i in range(n)]
+    passes = [(i, t if i == loop.start else None) for t in range(loop.times) for i in range(loop.start, loop.stop)]
+    return [(i, None) for i in range(loop.start)] + passes + [(i, None) for i in range(loop.stop, n)]
 
 
 class TokenDecoder:
