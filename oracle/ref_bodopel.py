@@ -53,14 +53,14 @@ def head_weights(q, k, scale, cap, r1, r2, window):
     """q [T, H, D], k [T, G, D] -> every head's softmax weights [H, T, T], zero where a key is not visible"""
     T, H, _ = q.shape
     per = H // k.shape[1]
+    d = (torch.arange(T)[:, None] - torch.arange(T)[None]).to(q.dtype)
+    seen = (d >= 0) if window is None else (d >= 0) & (d < window)
     out = torch.zeros(H, T, T, dtype=q.dtype)
     for h in range(H):
-        for i in range(T):
-            lo = 0 if window is None else max(0, i - window + 1)
-            j = torch.arange(lo, i + 1)
-            s = soft_cap((k[lo:i + 1, h // per] @ q[i, h]) * scale, cap) - log_distance(r1[h], r2[h], (i - j).to(q.dtype))
-            e = torch.exp(s - s.max())
-            out[h, i, lo:i + 1] = e / e.sum()
+        s = soft_cap((q[:, h] @ k[:, h // per].T) * scale, cap) - log_distance(r1[h], r2[h], d.clamp(min=0))
+        s = s.masked_fill(~seen, float("-inf"))
+        e = torch.exp(s - s.max(-1, keepdim=True).values)
+        out[h] = e / e.sum(-1, keepdim=True)
     return out
 
 
