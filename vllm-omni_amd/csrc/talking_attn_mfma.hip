@@ -31,16 +31,20 @@ struct ScoreMul {
 
 __device__ __forceinline__ float fast_log2(float x) { return __builtin_amdgcn_logf(x); }
 
-// score in log2 units, distance d as a float (>= 0 where the result counts)
+// score in log2 units plus base - out, distance d as a float (>= 0 where the result counts)
 template <bool CAP>
-__device__ __forceinline__ float score_of(float s, float d, float r1, float r2, const ScoreMul& m) {
-  const float bias = r1 * fast_log2(fmaf(r2, d, 1.f));
+__device__ __forceinline__ float score_from(float base, float s, float d, float r1, float r2, const ScoreMul& m) {
+  const float b = fmaf(-r1, fast_log2(fmaf(r2, d, 1.f)), base);
   if constexpr (CAP) {
     const float t = __builtin_amdgcn_rcpf(fast_exp2(s * m.in) + 1.f);
-    return fmaf(-2.f * m.out, t, m.out - bias);
+    return fmaf(-2.f * m.out, t, b);
   } else {
-    return fmaf(s, m.in, -bias);
+    return fmaf(s, m.in, b);
   }
+}
+template <bool CAP>
+__device__ __forceinline__ float score_of(float s, float d, float r1, float r2, const ScoreMul& m) {
+  return score_from<CAP>(m.out, s, d, r1, r2, m);
 }
 
 constexpr float kFloor = -1e30f;     // stands in for the maximum of no scores
@@ -445,30 +449,25 @@ __device__ __forceinline__ void store_heads(char* at, const uint32_t (&w)[(HW + 
   else *reinterpret_cast<uint4*>(at) = make_uint4(w[0], w[1], w[2], w[3]);
 }
 
-// LDS layout of the exchange (bytes): weights [hi, lo][16 keys][16 rows][KP heads], mixed weights [H][16 rows][16 keys hi | lo],
-// talk [16 HT][KP]
+// LDS layout of the exchange (bytes): weights [hi, lo][16 keys][16 rows][KP heads], mixed weights [16 HT heads][16 rows][16 keys
+// hi | lo], talk [16 HT][KP]; then the query operands that find no room in registers
+template <int HD, int HW>
 struct MixLds {
-  int kp, pq, pk, half, mixed, talk, talk_pitch, bytes;
+  static constexpr int HT = HW == 8 ? 4 : HW == 4 ? 2 : 1, KP = HW == 8 ? 64 : 32;      // at most 8 HW heads
+  static constexpr int PQ = KP * 2 + 16, PK = 16 * PQ + 16, kHalf = 16 * PK;
+  static constexpr int kMixedPitch = 16 * 64 + 16, kMixed = 2 * kHalf;
+  static constexpr int kTalkPitch = KP * 2 + 16, kTalk = kMixed + 16 * HT * kMixedPitch;
+  static constexpr int QL = HD == 128 && HW == 4 ? 2 : 0;                                // heads of a wave with their q here
+  static constexpr int kQ = kTalk + 16 * HT * kTalkPitch, kQWave = QL * (HD / 32) * 1024;
+  static constexpr int bytes(int waves) { return kQ + waves * kQWave; }
 };
-constexpr int kMixedPitch = 16 * 64 + 16;
-__host__ __device__ inline MixLds mix_lds(int H) {
-  MixLds m;
-  m.kp = (H + 31) / 32 * 32;
-  m.pq = m.kp * 2 + 16;
-  m.pk = 16 * m.pq + 16;
-  m.half = 16 * m.pk;
-  m.mixed = 2 * m.half;
-  m.talk = m.mixed + H * kMixedPitch;
-  m.talk_pitch = m.kp * 2 + 16;
-  m.bytes = m.talk + (H + 15) / 16 * 16 * m.talk_pitch;
-  return m;
-}
 
 template <int HD, int HW, bool ONE, bool CAP>
 __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams p) {
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  constexpr int KS = HD / 32, VN = HD / 16, HT = HW == 8 ? 4 : 2;
+  using M = MixLds<HD, HW>;
+  constexpr int KS = HD / 32, VN = HD / 16, HT = M::HT, QR = HW - M::QL;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int NW = blockDim.x >> 6, R = p.H / p.G, r = blockIdx.y;
   // workgroups go to the 8 XCDs in turn: up to 32 neighbouring tiles on one, where they walk the same keys; late tiles (long
@@ -478,26 +477,31 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
   const int tile = gridDim.x - 1 - (whole ? b / set * set + (b & 7) * per + (b % set >> 3) : b);
   const TileSpan t = tile_span(p, r, tile * 16);
   if (!t.any) return;
-  const MixLds ml = mix_lds(p.H);
-  for (int i = tid; i < ml.mixed / 16; i += blockDim.x) reinterpret_cast<uint4*>(smem)[i] = make_uint4(0, 0, 0, 0);
-  for (int i = tid; i < (p.H + 15) / 16 * 16 * ml.kp; i += blockDim.x) {
-    const int h = i / ml.kp, g = i % ml.kp;
-    reinterpret_cast<uint16_t*>(smem + ml.talk + h * ml.talk_pitch)[g] = h < p.H && g < p.H ? E16::to_bits(p.talk[h * p.H + g]) : 0;
+  for (int i = tid; i < M::kMixed / 16; i += blockDim.x) reinterpret_cast<uint4*>(smem)[i] = make_uint4(0, 0, 0, 0);
+  for (int i = tid; i < 16 * HT * M::KP; i += blockDim.x) {
+    const int h = i / M::KP, g = i % M::KP;
+    reinterpret_cast<uint16_t*>(smem + M::kTalk + h * M::kTalkPitch)[g] = h < p.H && g < p.H ? E16::to_bits(p.talk[h * p.H + g]) : 0;
   }
   const int h0 = wave * HW, qi = min(t.tile0 + lr, t.ql - 1), qpos = t.start + t.tile0 + lr;
   const uint16_t* q = p.q + (int64_t)(t.s0 + qi) * p.q_stride + 8 * lg;
-  uint4 qf[HW][KS];
-  float lse[HW], r1[HW], r2[HW];
+  uint4 qf[QR][KS];
+  uint4* ql = reinterpret_cast<uint4*>(smem + M::kQ + wave * M::kQWave) + lane;
+  float base[HW], r1[HW], r2[HW];      // base: what of the exponent depends on the row alone
   f32x4_t o[HW][VN] = {};
 #pragma unroll
   for (int i = 0; i < HW; ++i) {
     const int h = min(h0 + i, p.H - 1);
 #pragma unroll
-    for (int k = 0; k < KS; ++k) qf[i][k] = *reinterpret_cast<const uint4*>(q + h * HD + 32 * k);
-    lse[i] = p.lse[(int64_t)h * p.rows + t.s0 + qi];
+    for (int k = 0; k < KS; ++k) {
+      const uint4 v = *reinterpret_cast<const uint4*>(q + h * HD + 32 * k);
+      if (i < QR) qf[i][k] = v;
+      else ql[((i - QR) * KS + k) * 64] = v;
+    }
+    const float lse = p.lse[(int64_t)h * p.rows + t.s0 + qi];
+    base[i] = h0 + i < p.H ? p.mul.out - lse : -INFINITY;      // heads past the last: no weight
     r1[i] = p.r1 ? p.r1[h] : 0.f, r2[i] = p.r1 ? p.r2[h] : 0.f;
   }
-  char* wr = smem + (4 * lg) * ml.pk + lr * ml.pq + h0 * 2;
+  char* wr = smem + (4 * lg) * M::PK + lr * M::PQ + h0 * 2;
   const int kv0 = min(h0, p.H - 1) / R;
   uint4 kf[KS];
   load_k<HD>(kf, p, kv0, t.c0 + t.kb, lr, lg);
@@ -508,21 +512,36 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
 #pragma unroll
     for (int i = 0; i < HW; ++i) {
       if (!ONE && i > 0) load_k<HD>(kf, p, min(h0 + i, p.H - 1) / R, t.c0 + k0, lr, lg);
-      s[i] = qk<HD>(kf, qf[i]);
+      if (i < QR) {
+        s[i] = qk<HD>(kf, qf[i < QR ? i : 0]);
+      } else {
+        uint4 x[KS];
+#pragma unroll
+        for (int k = 0; k < KS; ++k) x[k] = ql[((i - QR) * KS + k) * 64];
+        s[i] = qk<HD>(kf, x);
+      }
     }
     if (k0 + 16 <= t.ke) load_k<HD>(kf, p, kv0, t.c0 + k0 + 16, lr, lg);
     const int key0 = t.first + k0, d0 = qpos - key0 - 4 * lg;
     const bool inside = key0 + 15 <= t.start + t.tile0 && t.start + t.tile0 + 15 - key0 < p.window;
     const float fd = (float)d0;
 #pragma unroll
+    for (int i = 0; i < HW; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) s[i][j] = score_from<CAP>(base[i], s[i][j], fd - (float)j, r1[i], r2[i], p.mul);
+    if (!inside) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const bool seen = (unsigned)(d0 - j) < (unsigned)p.window;
+#pragma unroll
+        for (int i = 0; i < HW; ++i) s[i][j] = seen ? s[i][j] : -INFINITY;
+      }
+    }
+#pragma unroll
     for (int j = 0; j < 4; ++j) {
       float w[HW];
 #pragma unroll
-      for (int i = 0; i < HW; ++i) {
-        float u = score_of<CAP>(s[i][j], fd - (float)j, r1[i], r2[i], p.mul);
-        if (!inside) u = (unsigned)(d0 - j) < (unsigned)p.window ? u : -INFINITY;
-        w[i] = h0 + i < p.H ? fast_exp2(u - lse[i]) : 0.f;
-      }
+      for (int i = 0; i < HW; ++i) w[i] = fast_exp2(s[i][j]);
       uint32_t hi[(HW + 1) / 2], lo[(HW + 1) / 2];
       if constexpr (HW == 1) {
         hi[0] = E16::to_bits(w[0]);
@@ -534,61 +553,82 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
           lo[i] = E16::pack(w[2 * i] - E16::lo(hi[i]), w[2 * i + 1] - E16::hi(hi[i]));
         }
       }
-      store_heads<HW>(wr + j * ml.pk, hi);
-      store_heads<HW>(wr + j * ml.pk + ml.half, lo);
+      store_heads<HW>(wr + j * M::PK, hi);
+      store_heads<HW>(wr + j * M::PK + M::kHalf, lo);
+    }
+    // value operands (columns past the values' size are zeros): the first half arrives while the weights are mixed
+    auto v_at = [&](int kv) {
+      return p.vt + ((int64_t)kv * p.ctx_rows + t.c0 + k0) * HD + lr * 16 + (lg & 1) * 8;
+    };
+    const uint16_t* vt = v_at(kv0);
+    uint4 va[VN / 2], vb[VN / 2];
+    if constexpr (ONE) {
+#pragma unroll
+      for (int n = 0; n < VN / 2; ++n) va[n] = *reinterpret_cast<const uint4*>(vt + n * 256);
     }
     __syncthreads();
     // mixed weights of all heads, rows of the tile in turn
-    for (int qq = wave; qq < 16; qq += NW) {
-      f32x4_t a[HT] = {};
-      const char* pr = smem + lr * ml.pk + qq * ml.pq + lg * 16;
-      for (int k = 0; k < ml.kp / 32; ++k) {
-        const uint4 hi = *reinterpret_cast<const uint4*>(pr + 64 * k), lo = *reinterpret_cast<const uint4*>(pr + 64 * k + ml.half);
+    for (int q0 = wave; q0 < 16; q0 += 2 * NW) {
+      const int qq[2] = {q0, q0 + NW < 16 ? q0 + NW : q0};      // two rows side by side (the last one may be alone)
+      f32x4_t a[2][HT] = {};
+#pragma unroll
+      for (int k = 0; k < M::KP / 32; ++k) {
+        uint4 hi[2], lo[2];
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+          const char* pr = smem + lr * M::PK + qq[x] * M::PQ + lg * 16 + 64 * k;
+          hi[x] = *reinterpret_cast<const uint4*>(pr), lo[x] = *reinterpret_cast<const uint4*>(pr + M::kHalf);
+        }
 #pragma unroll
         for (int h = 0; h < HT; ++h) {
-          if (16 * h >= p.H) continue;
-          const uint4 tk = *reinterpret_cast<const uint4*>(smem + ml.talk + (16 * h + lr) * ml.talk_pitch + 64 * k + lg * 16);
-          a[h] = mfma16<bf16_tag>(hi, tk, a[h]);
-          a[h] = mfma16<bf16_tag>(lo, tk, a[h]);
+          const uint4 tk = *reinterpret_cast<const uint4*>(smem + M::kTalk + (16 * h + lr) * M::kTalkPitch + 64 * k + lg * 16);
+#pragma unroll
+          for (int x = 0; x < 2; ++x) a[x][h] = mfma16<bf16_tag>(hi[x], tk, a[x][h]);
+#pragma unroll
+          for (int x = 0; x < 2; ++x) a[x][h] = mfma16<bf16_tag>(lo[x], tk, a[x][h]);
         }
       }
 #pragma unroll
-      for (int h = 0; h < HT; ++h) {
-        if (16 * h + lr >= p.H) continue;
-        char* at = smem + ml.mixed + (16 * h + lr) * kMixedPitch + qq * 64 + lg * 8;
-        const uint2 hi = make_uint2(E16::pack(a[h][0], a[h][1]), E16::pack(a[h][2], a[h][3]));
-        *reinterpret_cast<uint2*>(at) = hi;
-        *reinterpret_cast<uint2*>(at + 32) = make_uint2(E16::pack(a[h][0] - E16::lo(hi.x), a[h][1] - E16::hi(hi.x)),
-                                                        E16::pack(a[h][2] - E16::lo(hi.y), a[h][3] - E16::hi(hi.y)));
-      }
+      for (int x = 0; x < 2; ++x)
+#pragma unroll
+        for (int h = 0; h < HT; ++h) {
+          char* at = smem + M::kMixed + (16 * h + lr) * M::kMixedPitch + qq[x] * 64 + lg * 8;
+          const f32x4_t& v = a[x][h];
+          const uint2 hi = make_uint2(E16::pack(v[0], v[1]), E16::pack(v[2], v[3]));
+          *reinterpret_cast<uint2*>(at) = hi;
+          *reinterpret_cast<uint2*>(at + 32) = make_uint2(E16::pack(v[0] - E16::lo(hi.x), v[1] - E16::hi(hi.x)),
+                                                          E16::pack(v[2] - E16::lo(hi.y), v[3] - E16::hi(hi.y)));
+        }
     }
     __syncthreads();
     // values
     uint4 pa[HW];
 #pragma unroll
     for (int i = 0; i < HW; ++i)
-      pa[i] = *reinterpret_cast<const uint4*>(smem + ml.mixed + min(h0 + i, p.H - 1) * kMixedPitch + lr * 64 + lg * 16);
-    auto v_at = [&](int kv) {
-      return p.vt + ((int64_t)kv * p.ctx_rows + t.c0 + k0) * HD + lr * 16 + (lg & 1) * 8;
-    };
+      pa[i] = *reinterpret_cast<const uint4*>(smem + M::kMixed + min(h0 + i, 16 * HT - 1) * M::kMixedPitch + lr * 64 + lg * 16);
     if constexpr (ONE) {
-      const uint16_t* vt = v_at(kv0);
 #pragma unroll
-      for (int n = 0; n < VN; ++n) {
-        if (16 * n >= p.V) continue;
-        const uint4 v = *reinterpret_cast<const uint4*>(vt + n * 256);
+      for (int n = 0; n < VN / 2; ++n) vb[n] = *reinterpret_cast<const uint4*>(vt + (n + VN / 2) * 256);
 #pragma unroll
-        for (int i = 0; i < HW; ++i) o[i][n] = mfma16<bf16_tag>(pa[i], v, o[i][n]);
-      }
+      for (int n = 0; n < VN / 2; ++n)
+#pragma unroll
+        for (int i = 0; i < HW; ++i) o[i][n] = mfma16<bf16_tag>(pa[i], va[n], o[i][n]);
+#pragma unroll
+      for (int n = 0; n < VN / 2; ++n)
+#pragma unroll
+        for (int i = 0; i < HW; ++i) o[i][n + VN / 2] = mfma16<bf16_tag>(pa[i], vb[n], o[i][n + VN / 2]);
     } else {
 #pragma unroll
       for (int i = 0; i < HW; ++i) {
-        const uint16_t* vt = v_at(min(h0 + i, p.H - 1) / R);
+        vt = v_at(min(h0 + i, p.H - 1) / R);
 #pragma unroll
-        for (int n = 0; n < VN; ++n) {
-          if (16 * n >= p.V) continue;
-          o[i][n] = mfma16<bf16_tag>(pa[i], *reinterpret_cast<const uint4*>(vt + n * 256), o[i][n]);
-        }
+        for (int n = 0; n < VN / 2; ++n) va[n] = *reinterpret_cast<const uint4*>(vt + n * 256);
+#pragma unroll
+        for (int n = 0; n < VN / 2; ++n) vb[n] = *reinterpret_cast<const uint4*>(vt + (n + VN / 2) * 256);
+#pragma unroll
+        for (int n = 0; n < VN / 2; ++n) o[i][n] = mfma16<bf16_tag>(pa[i], va[n], o[i][n]);
+#pragma unroll
+        for (int n = 0; n < VN / 2; ++n) o[i][n + VN / 2] = mfma16<bf16_tag>(pa[i], vb[n], o[i][n + VN / 2]);
       }
     }
   }
@@ -712,10 +752,10 @@ template <int HD, int HW, bool ONE, bool CAP>
 int launch_prefill(const PrefillParams& p, int reqs, int max_q, hipStream_t s) {
   hipLaunchKernelGGL((prefill_sums_kernel<HD, HW, ONE, CAP>), dim3(ceil_div(p.H, HW) * ceil_div(max_q, 64), reqs), dim3(256), 0, s, p);
   if (int e = launch_status()) return e;
-  const int bytes = mix_lds(p.H).bytes;
+  const int waves = ceil_div(p.H, HW), bytes = MixLds<HD, HW>::bytes(waves);
   auto kern = prefill_mix_kernel<HD, HW, ONE, CAP>;
   if (int e = allow_lds(kern, bytes)) return e;
-  hipLaunchKernelGGL(kern, dim3(ceil_div(max_q, 16), reqs), dim3(64 * ceil_div(p.H, HW)), bytes, s, p);
+  hipLaunchKernelGGL(kern, dim3(ceil_div(max_q, 16), reqs), dim3(64 * waves), bytes, s, p);
   return launch_status();
 }
 
