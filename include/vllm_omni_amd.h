@@ -956,7 +956,7 @@ int mi_embed_pos_norm(void* x, void* h, const void* table, float scale, const vo
                       const int32_t* slots, int32_t taps, float eps, int32_t rows, int32_t width,
                       int32_t vocab, int64_t x_stride, int64_t h_stride, int dtype, void* stream);
 /* The filter and the ring update over portions of any length; slots per
- * request; taps <= 33. */
+ * request; taps <= 17. */
 int mi_input_conv(void* out, const void* h, const void* conv_w, void* ring, const int32_t* slots,
                   const int32_t* query_start_loc, const int32_t* seq_lens, int32_t req0,
                   int32_t num_reqs, int32_t max_query_len, int32_t taps, int32_t width,

@@ -248,7 +248,7 @@ struct InputConvParams {
   int req0, width;
 };
 
-constexpr int kConvRows = 32;
+constexpr int kConvRows = 16;
 
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void input_conv_kernel(const InputConvParams p) {

@@ -47,6 +47,10 @@ __device__ __forceinline__ float score_of(float s, float d, float r1, float r2, 
   return score_from<CAP>(m.out, s, d, r1, r2, m);
 }
 
+__device__ __forceinline__ float uniform(float v) {      // the same in all lanes: a scalar register
+  return __builtin_bit_cast(float, __builtin_amdgcn_readfirstlane(__builtin_bit_cast(int, v)));
+}
+
 constexpr float kFloor = -1e30f;     // stands in for the maximum of no scores
 
 // ------------------------------------------------------------------------------------------------ decode
@@ -403,7 +407,7 @@ __global__ __launch_bounds__(256) void prefill_sums_kernel(const PrefillParams p
 #pragma unroll
     for (int k = 0; k < KS; ++k) qf[i][k] = *reinterpret_cast<const uint4*>(q + h * HD + 32 * k);
     m[i] = kFloor, l[i] = 0.f;
-    r1[i] = p.r1 ? p.r1[h] : 0.f, r2[i] = p.r1 ? p.r2[h] : 0.f;
+    r1[i] = uniform(p.r1 ? p.r1[h] : 0.f), r2[i] = uniform(p.r1 ? p.r2[h] : 0.f);
   }
   uint4 kf[KS];
   load_k<HD>(kf, p, h0 / R, t.c0 + t.kb, lr, lg);
@@ -449,14 +453,16 @@ __device__ __forceinline__ void store_heads(char* at, const uint32_t (&w)[(HW + 
   else *reinterpret_cast<uint4*>(at) = make_uint4(w[0], w[1], w[2], w[3]);
 }
 
-// LDS layout of the exchange (bytes): weights [hi, lo][16 keys][16 rows][KP heads], mixed weights [16 HT heads][16 rows][16 keys
-// hi | lo], talk [16 HT][KP]; then the query operands that find no room in registers
+// LDS layout of the exchange (bytes).  A buffer has a region per row: the weights [hi, lo][16 keys][KP heads], which the one
+// wave that mixes the row replaces by the mixed weights [16 HT heads][16 keys hi | lo].  Then talk [16 HT][KP] and the query
+// operands that find no room in registers.
 template <int HD, int HW>
 struct MixLds {
   static constexpr int HT = HW == 8 ? 4 : HW == 4 ? 2 : 1, KP = HW == 8 ? 64 : 32;      // at most 8 HW heads
-  static constexpr int PQ = KP * 2 + 16, PK = 16 * PQ + 16, kHalf = 16 * PK;
-  static constexpr int kMixedPitch = 16 * 64 + 16, kMixed = 2 * kHalf;
-  static constexpr int kTalkPitch = KP * 2 + 16, kTalk = kMixed + 16 * HT * kMixedPitch;
+  static constexpr int kBufs = HW < 8 ? 2 : 1;         // two: values of a tile and weights of the next between the same barriers
+  static constexpr int kKey = KP * 2 + 16, kHalf = 16 * kKey, kHead = 64 + 16;
+  static constexpr int kRow = (2 * kHalf > 16 * HT * kHead ? 2 * kHalf : 16 * HT * kHead) + 16, kBuf = 16 * kRow;
+  static constexpr int kTalkPitch = KP * 2 + 16, kTalk = kBufs * kBuf;
   static constexpr int QL = HD == 128 && HW == 4 ? 2 : 0;                                // heads of a wave with their q here
   static constexpr int kQ = kTalk + 16 * HT * kTalkPitch, kQWave = QL * (HD / 32) * 1024;
   static constexpr int bytes(int waves) { return kQ + waves * kQWave; }
@@ -467,7 +473,7 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
   scalar_cache_acquire();
   extern __shared__ __attribute__((aligned(16))) char smem[];
   using M = MixLds<HD, HW>;
-  constexpr int KS = HD / 32, VN = HD / 16, HT = M::HT, QR = HW - M::QL;
+  constexpr int KS = HD / 32, VN = HD / 16, VH = VN / 2, HT = M::HT, QR = HW - M::QL;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
   const int NW = blockDim.x >> 6, R = p.H / p.G, r = blockIdx.y;
   // workgroups go to the 8 XCDs in turn: up to 32 neighbouring tiles on one, where they walk the same keys; late tiles (long
@@ -477,7 +483,7 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
   const int tile = gridDim.x - 1 - (whole ? b / set * set + (b & 7) * per + (b % set >> 3) : b);
   const TileSpan t = tile_span(p, r, tile * 16);
   if (!t.any) return;
-  for (int i = tid; i < M::kMixed / 16; i += blockDim.x) reinterpret_cast<uint4*>(smem)[i] = make_uint4(0, 0, 0, 0);
+  for (int i = tid; i < M::kTalk / 16; i += blockDim.x) reinterpret_cast<uint4*>(smem)[i] = make_uint4(0, 0, 0, 0);
   for (int i = tid; i < 16 * HT * M::KP; i += blockDim.x) {
     const int h = i / M::KP, g = i % M::KP;
     reinterpret_cast<uint16_t*>(smem + M::kTalk + h * M::kTalkPitch)[g] = h < p.H && g < p.H ? E16::to_bits(p.talk[h * p.H + g]) : 0;
@@ -494,20 +500,19 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
       const uint4 v = *reinterpret_cast<const uint4*>(q + h * HD + 32 * k);
-      if (i < QR) qf[i][k] = v;
+      if (i < QR) qf[i < QR ? i : 0][k] = v;
       else ql[((i - QR) * KS + k) * 64] = v;
     }
     const float lse = p.lse[(int64_t)h * p.rows + t.s0 + qi];
     base[i] = h0 + i < p.H ? p.mul.out - lse : -INFINITY;      // heads past the last: no weight
-    r1[i] = p.r1 ? p.r1[h] : 0.f, r2[i] = p.r1 ? p.r2[h] : 0.f;
+    r1[i] = uniform(p.r1 ? p.r1[h] : 0.f), r2[i] = uniform(p.r1 ? p.r2[h] : 0.f);
   }
-  char* wr = smem + (4 * lg) * M::PK + lr * M::PQ + h0 * 2;
   const int kv0 = min(h0, p.H - 1) / R;
-  uint4 kf[KS];
+  uint4 kf[KS], va[VH], vb[VH];
   load_k<HD>(kf, p, kv0, t.c0 + t.kb, lr, lg);
-  __syncthreads();
-  for (int k0 = t.kb; k0 <= t.ke; k0 += 16) {
-    // weights of this wave's heads
+
+  // this wave's heads: weights of the keys at k0 (its K operands, and then those of the next tile, are in kf)
+  auto weights = [&](int k0, char* buf) {
     f32x4_t s[HW];
 #pragma unroll
     for (int i = 0; i < HW; ++i) {
@@ -521,7 +526,7 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
         s[i] = qk<HD>(kf, x);
       }
     }
-    if (k0 + 16 <= t.ke) load_k<HD>(kf, p, kv0, t.c0 + k0 + 16, lr, lg);
+    load_k<HD>(kf, p, kv0, t.c0 + min(k0 + 16, t.ke & ~15), lr, lg);
     const int key0 = t.first + k0, d0 = qpos - key0 - 4 * lg;
     const bool inside = key0 + 15 <= t.start + t.tile0 && t.start + t.tile0 + 15 - key0 < p.window;
     const float fd = (float)d0;
@@ -537,6 +542,7 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
         for (int i = 0; i < HW; ++i) s[i][j] = seen ? s[i][j] : -INFINITY;
       }
     }
+    char* wr = buf + lr * M::kRow + 4 * lg * M::kKey + h0 * 2;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       float w[HW];
@@ -553,84 +559,88 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
           lo[i] = E16::pack(w[2 * i] - E16::lo(hi[i]), w[2 * i + 1] - E16::hi(hi[i]));
         }
       }
-      store_heads<HW>(wr + j * M::PK, hi);
-      store_heads<HW>(wr + j * M::PK + M::kHalf, lo);
+      store_heads<HW>(wr + j * M::kKey, hi);
+      store_heads<HW>(wr + j * M::kKey + M::kHalf, lo);
     }
-    // value operands (columns past the values' size are zeros): the first half arrives while the weights are mixed
-    auto v_at = [&](int kv) {
-      return p.vt + ((int64_t)kv * p.ctx_rows + t.c0 + k0) * HD + lr * 16 + (lg & 1) * 8;
-    };
-    const uint16_t* vt = v_at(kv0);
-    uint4 va[VN / 2], vb[VN / 2];
-    if constexpr (ONE) {
-#pragma unroll
-      for (int n = 0; n < VN / 2; ++n) va[n] = *reinterpret_cast<const uint4*>(vt + n * 256);
-    }
-    __syncthreads();
-    // mixed weights of all heads, rows of the tile in turn
-    for (int q0 = wave; q0 < 16; q0 += 2 * NW) {
-      const int qq[2] = {q0, q0 + NW < 16 ? q0 + NW : q0};      // two rows side by side (the last one may be alone)
-      f32x4_t a[2][HT] = {};
+  };
+  // rows of the tile in turn: all heads' weights mixed, in place
+  auto mix = [&](char* buf) {
+    for (int row = wave; row < 16; row += NW) {
+      char* at = buf + row * M::kRow;
+      f32x4_t a[HT] = {};
 #pragma unroll
       for (int k = 0; k < M::KP / 32; ++k) {
-        uint4 hi[2], lo[2];
+        const char* pr = at + lr * M::kKey + lg * 16 + 64 * k;
+        const uint4 hi = *reinterpret_cast<const uint4*>(pr), lo = *reinterpret_cast<const uint4*>(pr + M::kHalf);
+        uint4 tk[HT];
 #pragma unroll
-        for (int x = 0; x < 2; ++x) {
-          const char* pr = smem + lr * M::PK + qq[x] * M::PQ + lg * 16 + 64 * k;
-          hi[x] = *reinterpret_cast<const uint4*>(pr), lo[x] = *reinterpret_cast<const uint4*>(pr + M::kHalf);
-        }
+        for (int h = 0; h < HT; ++h)
+          tk[h] = *reinterpret_cast<const uint4*>(smem + M::kTalk + (16 * h + lr) * M::kTalkPitch + 64 * k + lg * 16);
 #pragma unroll
-        for (int h = 0; h < HT; ++h) {
-          const uint4 tk = *reinterpret_cast<const uint4*>(smem + M::kTalk + (16 * h + lr) * M::kTalkPitch + 64 * k + lg * 16);
+        for (int h = 0; h < HT; ++h) a[h] = mfma16<bf16_tag>(hi, tk[h], a[h]);
 #pragma unroll
-          for (int x = 0; x < 2; ++x) a[x][h] = mfma16<bf16_tag>(hi[x], tk, a[x][h]);
-#pragma unroll
-          for (int x = 0; x < 2; ++x) a[x][h] = mfma16<bf16_tag>(lo[x], tk, a[x][h]);
-        }
+        for (int h = 0; h < HT; ++h) a[h] = mfma16<bf16_tag>(lo, tk[h], a[h]);
       }
 #pragma unroll
-      for (int x = 0; x < 2; ++x)
-#pragma unroll
-        for (int h = 0; h < HT; ++h) {
-          char* at = smem + M::kMixed + (16 * h + lr) * M::kMixedPitch + qq[x] * 64 + lg * 8;
-          const f32x4_t& v = a[x][h];
-          const uint2 hi = make_uint2(E16::pack(v[0], v[1]), E16::pack(v[2], v[3]));
-          *reinterpret_cast<uint2*>(at) = hi;
-          *reinterpret_cast<uint2*>(at + 32) = make_uint2(E16::pack(v[0] - E16::lo(hi.x), v[1] - E16::hi(hi.x)),
-                                                          E16::pack(v[2] - E16::lo(hi.y), v[3] - E16::hi(hi.y)));
-        }
+      for (int h = 0; h < HT; ++h) {
+        const f32x4_t& v = a[h];
+        char* to = at + (16 * h + lr) * M::kHead + lg * 8;
+        const uint2 hi = make_uint2(E16::pack(v[0], v[1]), E16::pack(v[2], v[3]));
+        *reinterpret_cast<uint2*>(to) = hi;
+        *reinterpret_cast<uint2*>(to + 32) = make_uint2(E16::pack(v[0] - E16::lo(hi.x), v[1] - E16::hi(hi.x)),
+                                                        E16::pack(v[2] - E16::lo(hi.y), v[3] - E16::hi(hi.y)));
+      }
     }
-    __syncthreads();
-    // values
-    uint4 pa[HW];
+  };
+  // value operands (columns past the values' size are zeros)
+  auto load_v = [&](uint4 (&v)[VH], int kv, int k0, int n0) {
+    const uint16_t* vt = p.vt + ((int64_t)kv * p.ctx_rows + t.c0 + k0) * HD + lr * 16 + (lg & 1) * 8 + n0 * 256;
 #pragma unroll
-    for (int i = 0; i < HW; ++i)
-      pa[i] = *reinterpret_cast<const uint4*>(smem + M::kMixed + min(h0 + i, 16 * HT - 1) * M::kMixedPitch + lr * 64 + lg * 16);
-    if constexpr (ONE) {
+    for (int n = 0; n < VH; ++n) v[n] = *reinterpret_cast<const uint4*>(vt + n * 256);
+  };
+  auto values = [&](int k0, const char* buf) {
+    const char* rd = buf + lr * M::kRow + h0 * M::kHead + lg * 16;
+    if constexpr (ONE) {       // the operands are in va and vb
 #pragma unroll
-      for (int n = 0; n < VN / 2; ++n) vb[n] = *reinterpret_cast<const uint4*>(vt + (n + VN / 2) * 256);
+      for (int i = 0; i < HW; ++i) {
+        const uint4 w = *reinterpret_cast<const uint4*>(rd + i * M::kHead);
 #pragma unroll
-      for (int n = 0; n < VN / 2; ++n)
+        for (int n = 0; n < VH; ++n) o[i][n] = mfma16<bf16_tag>(w, va[n], o[i][n]);
+      }
 #pragma unroll
-        for (int i = 0; i < HW; ++i) o[i][n] = mfma16<bf16_tag>(pa[i], va[n], o[i][n]);
+      for (int i = 0; i < HW; ++i) {
+        const uint4 w = *reinterpret_cast<const uint4*>(rd + i * M::kHead);
 #pragma unroll
-      for (int n = 0; n < VN / 2; ++n)
-#pragma unroll
-        for (int i = 0; i < HW; ++i) o[i][n + VN / 2] = mfma16<bf16_tag>(pa[i], vb[n], o[i][n + VN / 2]);
+        for (int n = 0; n < VH; ++n) o[i][n + VH] = mfma16<bf16_tag>(w, vb[n], o[i][n + VH]);
+      }
     } else {
 #pragma unroll
       for (int i = 0; i < HW; ++i) {
-        vt = v_at(min(h0 + i, p.H - 1) / R);
+        const uint4 w = *reinterpret_cast<const uint4*>(rd + i * M::kHead);
+        const int kv = min(h0 + i, p.H - 1) / R;
+        load_v(va, kv, k0, 0);
+        load_v(vb, kv, k0, VH);
 #pragma unroll
-        for (int n = 0; n < VN / 2; ++n) va[n] = *reinterpret_cast<const uint4*>(vt + n * 256);
+        for (int n = 0; n < VH; ++n) o[i][n] = mfma16<bf16_tag>(w, va[n], o[i][n]);
 #pragma unroll
-        for (int n = 0; n < VN / 2; ++n) vb[n] = *reinterpret_cast<const uint4*>(vt + (n + VN / 2) * 256);
-#pragma unroll
-        for (int n = 0; n < VN / 2; ++n) o[i][n] = mfma16<bf16_tag>(pa[i], va[n], o[i][n]);
-#pragma unroll
-        for (int n = 0; n < VN / 2; ++n) o[i][n + VN / 2] = mfma16<bf16_tag>(pa[i], vb[n], o[i][n + VN / 2]);
+        for (int n = 0; n < VH; ++n) o[i][n + VH] = mfma16<bf16_tag>(w, vb[n], o[i][n + VH]);
       }
     }
+  };
+  __syncthreads();
+  int at = 0;
+  for (int k0 = t.kb; k0 <= t.ke; k0 += 16) {
+    char* buf = smem + at;
+    weights(k0, buf);
+    if constexpr (ONE) load_v(va, kv0, k0, 0);
+    __syncthreads();
+    mix(buf);
+    if constexpr (ONE) load_v(vb, kv0, k0, VH);
+    __builtin_amdgcn_sched_barrier(0);      // the loads are on their way before the wait
+    __syncthreads();
+    values(k0, buf);
+    if constexpr (M::kBufs == 2) at = M::kBuf - at;
+    else __syncthreads();
   }
 #pragma unroll
   for (int i = 0; i < HW; ++i) {
