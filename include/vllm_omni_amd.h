@@ -964,6 +964,10 @@ int mi_input_conv(void* out, const void* h, const void* conv_w, void* ring, cons
 /* relu(z)^2 of rows of dtype (split == 0) or of fp32 slabs [split][rows][z_stride] */
 int mi_relu_squared(void* out, const void* z, int32_t split, int32_t rows, int32_t ff, int64_t z_stride,
                     int64_t out_stride, int dtype, void* stream);
+/* relu(x W^T)^2 for a decode batch (shapes and workspace as mi_linear, bf16) */
+int mi_linear_relu_squared(void* out, const void* x, const void* weight, int32_t m, int32_t n, int32_t k,
+                           int64_t x_row_stride, int64_t out_row_stride, void* workspace,
+                           int64_t workspace_bytes, int dtype, void* stream);
 /* Rows q (heads x dim) | k (kv x dim) | v (kv x vdim): q RMS-normed over all its
  * heads at once, k likewise (weights [heads * dim], [kv * dim]; NULL: not); q to
  * q_out, k and v to their cache rows, heads head_dim apart, zeros behind them. */

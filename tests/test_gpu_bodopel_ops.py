@@ -105,6 +105,15 @@ def test_squared_relu(dev, dtype, ff):
     close(ops.relu_squared(z.to(dev)), ref.relu_squared(z.double()), **tol(dtype))
 
 
+@pytest.mark.parametrize("m,n,k", [(1, 256, 256), (7, 48, 512), (32, 6144, 2048), (200, 1024, 128), (5, 64, 16384)])
+def test_up_projection_with_squared_relu(dev, m, n, k):
+    """with and without slabs to sum"""
+    from vllm_omni_amd import ops
+
+    x, w = rnd(m, k, dtype=torch.bfloat16, seed=1), rnd(n, k, dtype=torch.bfloat16, std=k ** -0.5, seed=2)
+    close(ops.linear_relu_squared(x.to(dev), w.to(dev)), ref.relu_squared(x.double() @ w.double().T), **tol(torch.bfloat16))
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("width", [48, 50])
 def test_embedding_with_positions(dev, dtype, width):

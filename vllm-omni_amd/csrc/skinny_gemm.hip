@@ -719,6 +719,36 @@ extern "C" int mi_linear(void* out, const void* x, const void* weight, const voi
   return launch_status();
 }
 
+// relu(x W^T)^2: in the epilogue when the plan does not split K, else in the launch that sums the slabs
+extern "C" int mi_linear_relu_squared(void* out, const void* x, const void* weight, int32_t m, int32_t n, int32_t k,
+                                      int64_t x_row_stride, int64_t out_row_stride, void* workspace, int64_t workspace_bytes,
+                                      int dtype, void* stream) {
+  using namespace mi;
+  if (m == 0 || n == 0) return MI_OK;
+  if (!out || !x || !weight || m < 0 || n < 0 || k <= 0) return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 || m > 512 || k % 64 || n % 16 || x_row_stride % 8 || out_row_stride % 4) return MI_ERR_UNSUPPORTED;
+  if ((int64_t)m * x_row_stride * 2 >= ((int64_t)1 << 31)) return MI_ERR_UNSUPPORTED;
+  if (((uintptr_t)x | (uintptr_t)weight) & 15 || ((uintptr_t)out & 7)) return MI_ERR_INVALID_ARG;
+  const SkinnyPlan pl = linear_plan(m, n, k);
+  if (pl.split > 1 && (!workspace || ((uintptr_t)workspace & 15))) return MI_ERR_INVALID_ARG;
+  if (pl.split > 1 && workspace_bytes < (int64_t)pl.split * m * n * (int64_t)sizeof(float)) return MI_ERR_WORKSPACE;
+  SkinnyParams p;
+  p.x = reinterpret_cast<const uint16_t*>(x);
+  p.w = reinterpret_cast<const uint16_t*>(weight);
+  p.bias = nullptr;
+  p.out = reinterpret_cast<uint16_t*>(out);
+  p.part = reinterpret_cast<float*>(workspace);
+  p.xs = p.ws = nullptr;
+  p.M = m; p.N = n; p.K = k; p.S = pl.split;
+  p.dbg = linear_dbg();
+  p.ldx = x_row_stride;
+  p.ldo = out_row_stride;
+  p.relu_squared = 1;
+  const int rc = launch_skinny(p, pl, false, dtype, reinterpret_cast<hipStream_t>(stream));
+  if (rc != MI_OK || pl.split == 1) return rc != MI_OK ? rc : launch_status();
+  return mi_relu_squared(out, workspace, pl.split, m, n, n, out_row_stride, dtype, stream);
+}
+
 // mi_linear with the split-K reduce inside the launch (first-generation kernel, <= 8 slices): the slice of a (tile, row
 // block) that arrives last sums the slabs in slice order — the bits of mi_linear, one launch less.  `counters`: >=
 // MI_LINEAR_COUNTER_BYTES of int32, zero before the first launch (every launch leaves them zero).

@@ -57,6 +57,7 @@ struct SkinnyParams {
   int32_t* cnt = nullptr;
   // GATED: 0 = silu(gate) * up; > 0 = the clamped form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit)
   float glu_alpha = 0.f, glu_limit = 0.f;
+  int32_t relu_squared = 0;    // not GATED, S == 1: the output is relu(sum)^2
   // GROUPED (sparse-MoE expert GEMMs, fused_moe.hip): grid.y = one tile of `rpt` token rows that share one expert
   const int32_t* row_map;      // [max_rows] pair index per row or -1
   const int32_t* tile_expert;  // [max_tiles]
@@ -98,6 +99,10 @@ __device__ __forceinline__ void finish_quad(const SkinnyParams& p, const typenam
   } else {
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = a[r] + bv[r];
+    if (p.relu_squared) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = fmaxf(v[r], 0.f) * fmaxf(v[r], 0.f);
+    }
   }
 }
 

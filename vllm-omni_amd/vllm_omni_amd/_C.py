@@ -198,6 +198,7 @@ SIGNATURES = {
                                   c_int32, c_int64, c_int64, c_int, _P]),
     "mi_input_conv": (c_int, [_P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int, _P]),
     "mi_relu_squared": (c_int, [_P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_int, _P]),
+    "mi_linear_relu_squared": (c_int, [_P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, _P, c_int64, c_int, _P]),
     "mi_row_norm_cache": (c_int, [_P, c_int64, _P, _P, _P, c_int64, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32,
                                   c_int32, c_int64, c_int64, c_int64, c_float, c_int, _P]),
     "mi_talking_attn_rows": (c_int, [POINTER(TalkingAttnArgs), c_int32, c_int32, c_int32, c_int, _P]),

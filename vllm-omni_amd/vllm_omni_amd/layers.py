@@ -411,6 +411,20 @@ def fused_gate_up_silu(layer, x: torch.Tensor, clamped: Optional[tuple[float, fl
     return ops.linear_silu_mul(x, w, clamped)
 
 
+def fused_up_relu_squared(layer, x: torch.Tensor) -> Optional[torch.Tensor]:
+    """``relu(up(x))^2`` with the activation behind the sums of the streaming kernel (``ops.linear_relu_squared``) where the
+    policy of ``_apply_linear`` picks that kernel for this shape, else None.  No bias, 16-bit weights only."""
+    if layer.bias is not None or getattr(layer, "qweight", None) is not None or not x.is_cuda or _LINEAR_MODE == "library":
+        return None
+    (n, k), m = layer.weight.shape, x.shape[0]
+    if x.dtype != torch.bfloat16 or not ops.linear_supported(m, n, k, x.dtype):
+        return None
+    e = _tuned(m, n, k)
+    if e["full"]["us"] < e["library_us"] if e is not None and e.get("full") else (_LINEAR_MODE == "kernel" or _streaming_kernel_wins(m, n, k)):
+        return ops.linear_relu_squared(x, layer.weight)
+    return None
+
+
 def _deferred_kernel_wins(m: int, n: int, k: int) -> bool:
     # square-ish projections (o_proj 3584 x 3584) when the split-K reduce rides in the fused-add RMSNorm behind them:
     # level with the library at 256 rows, 1-1.5 % of the step ahead at 32-128 rows (same measurements)

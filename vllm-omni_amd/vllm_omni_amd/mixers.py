@@ -19,7 +19,7 @@ import torch.nn.functional as F
 
 from . import ops
 from .kv_cache import KVCacheSpec, LatentCacheSpec, normalize_layer_kv
-from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu, tuned_linear
+from .layers import AttentionMetadata, _apply_linear, _init_weight, fused_gate_up_silu, fused_up_relu_squared, tuned_linear
 from .state_cache import StateSpec
 
 
@@ -343,7 +343,10 @@ class SquaredReluMLP:
         yield from self.down.named(p)
 
     def __call__(self, h: torch.Tensor, defer_reduce: bool = False):
-        return self.down(ops.relu_squared(self.up(h, True)), defer_reduce)
+        act = fused_up_relu_squared(self.up, h)       # decode batches: no launch of its own for the activation
+        if act is None:
+            act = ops.relu_squared(self.up(h))
+        return self.down(act, defer_reduce)
 
 
 # ------------------------------------------------------------------------------------------ sublayers side by side

@@ -1742,6 +1742,21 @@ def relu_squared(z: Union[torch.Tensor, "SplitKPartials"]) -> torch.Tensor:
     return out
 
 
+def linear_relu_squared(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """relu(x W^T)^2 for a decode batch by the weight-streaming kernel of ``linear``"""
+    _gpu(x, weight)
+    xs, k = _rows(x)
+    m, n = x.shape[0], weight.shape[0]
+    if weight.shape[1] != k or not weight.is_contiguous() or weight.dtype != x.dtype:
+        raise ValueError("weight must be a contiguous [n, k] tensor of x's dtype")
+    out = torch.empty(m, n, dtype=x.dtype, device=x.device)
+    need = lib.mi_linear_workspace_bytes(m, n, k)
+    ws = _linear_workspace(x.device, need) if need else None
+    check("mi_linear_relu_squared", lib.mi_linear_relu_squared(_p(out), _p(x), _p(weight), m, n, k, xs, out.stride(0), _p(ws),
+                                                               ws.numel() if need else 0, _dt(x.dtype), _stream()))
+    return out
+
+
 def row_norm_cache(x: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], k_cache: torch.Tensor,
                    v_cache: torch.Tensor, slot_mapping: torch.Tensor, num_q_heads: int, dim: int, vdim: int, eps: float) -> torch.Tensor:
     """Rows q | k | v: q and k each normed over all heads at once, K / V cache write; returns q, heads laid out as in the cache."""
