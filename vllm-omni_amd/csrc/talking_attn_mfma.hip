@@ -51,6 +51,11 @@ __device__ __forceinline__ float uniform(float v) {      // the same in all lane
   return __builtin_bit_cast(float, __builtin_amdgcn_readfirstlane(__builtin_bit_cast(int, v)));
 }
 
+// 16 bytes that are read once
+__device__ __forceinline__ uint4 load_once(const uint16_t* p) {
+  return __builtin_bit_cast(uint4, __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(p)));
+}
+
 constexpr float kFloor = -1e30f;     // stands in for the maximum of no scores
 
 // ------------------------------------------------------------------------------------------------ decode
@@ -73,69 +78,71 @@ struct DecodeParams {
   ScoreMul mul;
 };
 
-template <int HD, int NT, bool CAP>
+// A wave has 16 NT keys of one kv head; neighbouring waves have neighbouring kv heads.  A group of at most CW heads stands in
+// the products' 16 columns 16 / CW times, and a column's lanes go on with one of 16 / CW tiles: no score is formed twice.
+template <int HD, int NT, int CW, bool CAP>
 __global__ __launch_bounds__(256) void decode_scores_kernel(const DecodeParams p) {
   scalar_cache_acquire();
-  constexpr int KS = HD / 32;
-  __shared__ float2 sml[4][16];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
-  const int part = blockIdx.x, kv = blockIdx.y, req = blockIdx.z;
+  constexpr int KS = HD / 32, NG = 16 / CW, NP = NT / NG;
+  const int lane = threadIdx.x & 63, lr = lane & 15, lg = lane >> 4, col = lr % CW, group = lr / CW;
+  const int unit = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6)), req = blockIdx.y;
+  const int part = unit / p.G, kv = unit % p.G;
   const int L = p.seq_lens[req], lo = max(0, L - p.window), n = L - lo;
-  const int t0 = part * (64 * NT) + wave * (16 * NT);
-  if (part * (64 * NT) >= n) return;
+  const int t0 = part * (16 * NT);
+  if (t0 >= n) return;
   const int R = p.H / p.G;
   const int32_t* tab = p.table + (int64_t)req * p.table_stride;
-  const uint16_t* kc = p.kc + kv * p.head_stride;
+  const uint16_t* kc = p.kc + kv * p.head_stride + 8 * lg;
   uint4 kf[NT][KS];
 #pragma unroll
   for (int u = 0; u < NT; ++u) {
     const int key = lo + min(t0 + 16 * u + lr, n - 1);
     const uint16_t* row = kc + (int64_t)tab[key >> p.bs_log2] * p.block_stride + (int64_t)(key & ((1 << p.bs_log2) - 1)) * p.token_stride;
 #pragma unroll
-    for (int k = 0; k < KS; ++k) kf[u][k] = *reinterpret_cast<const uint4*>(row + 32 * k + 8 * lg);
+    for (int k = 0; k < KS; ++k) kf[u][k] = *reinterpret_cast<const uint4*>(row + 32 * k);
   }
-  for (int c0 = 0; c0 < R; c0 += 16) {
-    const bool used = c0 + lr < R;
-    const int h = kv * R + min(c0 + lr, R - 1);
+  for (int c0 = 0; c0 < R; c0 += CW) {
+    const bool used = c0 + col < R;
+    const int h = kv * R + min(c0 + col, R - 1);
     const uint16_t* q = p.q + req * p.q_stride + (int64_t)h * HD;
     uint4 qf[KS];
 #pragma unroll
     for (int k = 0; k < KS; ++k) qf[k] = *reinterpret_cast<const uint4*>(q + 32 * k + 8 * lg);
     const float r1 = p.r1 ? p.r1[h] : 0.f, r2 = p.r1 ? p.r2[h] : 0.f;
     float* out = p.scores + ((int64_t)req * p.H + h) * p.pitch;
-    float s[NT][4];
+    float s[NP][4];
     float m = kFloor;
 #pragma unroll
-    for (int u = 0; u < NT; ++u) {
-      f32x4_t a = {};
+    for (int u = 0; u < NP; ++u) {
 #pragma unroll
-      for (int k = 0; k < KS; ++k) a = mfma16<bf16_tag>(kf[u][k], qf[k], a);
+      for (int g = 0; g < NG; ++g) {
+        f32x4_t a = {};
+#pragma unroll
+        for (int k = 0; k < KS; ++k) a = mfma16<bf16_tag>(kf[u * NG + g][k], qf[k], a);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[u][j] = g == 0 || group == g ? a[j] : s[u][j];
+      }
+      const int at = t0 + 16 * (u * NG + group) + 4 * lg;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const int idx = t0 + 16 * u + 4 * lg + j, d = n - 1 - idx;
-        s[u][j] = d >= 0 ? score_of<CAP>(a[j], (float)d, r1, r2, p.mul) : -INFINITY;
+        const int d = n - 1 - at - j;
+        s[u][j] = d >= 0 ? score_of<CAP>(s[u][j], (float)d, r1, r2, p.mul) : -INFINITY;
         m = max2f(m, s[u][j]);
       }
-      if (used) *reinterpret_cast<float4*>(out + t0 + 16 * u + 4 * lg) = make_float4(s[u][0], s[u][1], s[u][2], s[u][3]);
+      if (used) *reinterpret_cast<float4*>(out + at) = make_float4(s[u][0], s[u][1], s[u][2], s[u][3]);
     }
     m = rows_allreduce_max(m);
+#pragma unroll
+    for (int o = CW; o < 16; o <<= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
     float l = 0.f;
 #pragma unroll
-    for (int u = 0; u < NT; ++u)
+    for (int u = 0; u < NP; ++u)
 #pragma unroll
       for (int j = 0; j < 4; ++j) l += fast_exp2(s[u][j] - m);
     l = rows_allreduce_sum(l);
-    if (lg == 0) sml[wave][lr] = make_float2(m, l);
-    __syncthreads();
-    if (wave == 0 && lg == 0 && used) {
-      float mm = m, ll = 0.f;
 #pragma unroll
-      for (int w = 1; w < 4; ++w) mm = fmaxf(mm, sml[w][lr].x);
-#pragma unroll
-      for (int w = 0; w < 4; ++w) ll += sml[w][lr].y * fast_exp2(sml[w][lr].x - mm);
-      p.ml[((int64_t)req * p.parts1 + part) * p.H + h] = make_float2(mm, ll);
-    }
-    __syncthreads();
+    for (int o = CW; o < 16; o <<= 1) l += __shfl_xor(l, o, 64);
+    if (lane < CW && used) p.ml[((int64_t)req * p.parts1 + part) * p.H + h] = make_float2(m, l);
   }
 }
 
@@ -156,11 +163,11 @@ __global__ __launch_bounds__(256) void decode_values_kernel(const DecodeParams p
   float* pm = lds;                                     // [keys2][pad]
   float* st = pm + p.keys2 * pad + 16;                 // [16 HT][tp]
   float* lse = st + 16 * HT * tp;                      // [4 kq]
-  int* pages = reinterpret_cast<int*>(lse + 4 * kq);   // pages of the part
+  int64_t* pages = reinterpret_cast<int64_t*>(lse + 4 * kq);      // where the part's pages start in the cache
   const int first_page = (lo + k0) >> p.bs_log2, nk = min(p.keys2, n - k0);
   const int last_page = (lo + k0 + nk - 1) >> p.bs_log2;
   const int32_t* tab = p.table + (int64_t)req * p.table_stride;
-  for (int i = tid; i <= last_page - first_page; i += 256) pages[i] = tab[first_page + i];
+  for (int i = tid; i <= last_page - first_page; i += 256) pages[i] = (int64_t)tab[first_page + i] * p.block_stride;
   for (int i = tid; i < 16 * HT * 4 * kq; i += 256) {
     const int h = i / (4 * kq), g = i % (4 * kq);
     st[h * tp + g] = h < H && g < H ? p.talk[h * H + g] : 0.f;
@@ -216,22 +223,20 @@ __global__ __launch_bounds__(256) void decode_values_kernel(const DecodeParams p
 #pragma unroll
       for (int u = 0; u < UN; ++u) {
         const int key = lo + k0 + min(j0 + u * KPI + sub, nk - 1);
-        v[u] = *reinterpret_cast<const uint4*>(vc + (int64_t)pages[(key >> p.bs_log2) - first_page] * p.block_stride +
-                                               (int64_t)(key & ((1 << p.bs_log2) - 1)) * p.token_stride);
+        v[u] = load_once(vc + pages[(key >> p.bs_log2) - first_page] + (int64_t)(key & ((1 << p.bs_log2) - 1)) * p.token_stride);
       }
 #pragma unroll
       for (int u = 0; u < UN; ++u) {
-        const int j = j0 + u * KPI + sub;
-        const float* w = pm + min(j, p.keys2 - 1) * pad + h0;
+        // (mixed weights of keys past the last are zeros; splits of the part are multiples of a round of loads)
+        const float* w = pm + (j0 + u * KPI + sub) * pad + h0;
         const uint32_t a[4] = {v[u].x, v[u].y, v[u].z, v[u].w};
         float x[8];
 #pragma unroll
         for (int i = 0; i < 4; ++i) x[2 * i] = E16::lo(a[i]), x[2 * i + 1] = E16::hi(a[i]);
 #pragma unroll
         for (int r = 0; r < RM; ++r) {
-          const float ww = j < je ? w[r] : 0.f;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) acc[r][i] = fmaf(ww, x[i], acc[r][i]);
+          for (int i = 0; i < 8; ++i) acc[r][i] = fmaf(w[r], x[i], acc[r][i]);
         }
       }
     }
@@ -428,6 +433,7 @@ __global__ __launch_bounds__(256) void prefill_sums_kernel(const PrefillParams p
 #pragma unroll
       for (int j = 0; j < 4; ++j) u[j] = score_of<CAP>(s[i][j], fd - (float)j, r1[i], r2[i], p.mul);
       if (!inside) {
+        asm volatile("");      // stays a branch
 #pragma unroll
         for (int j = 0; j < 4; ++j) u[j] = (unsigned)(d0 - j) < (unsigned)p.window ? u[j] : -INFINITY;
       }
@@ -535,6 +541,7 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
 #pragma unroll
       for (int j = 0; j < 4; ++j) s[i][j] = score_from<CAP>(base[i], s[i][j], fd - (float)j, r1[i], r2[i], p.mul);
     if (!inside) {
+      asm volatile("");      // stays a branch: sixteen selects a tile for its edges only
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const bool seen = (unsigned)(d0 - j) < (unsigned)p.window;
@@ -675,16 +682,16 @@ DecodePlan decode_plan(int reqs, int H, int G, int V, int window, int max_seq_le
   const int R = H / G;
   d.span = window < max_seq_len ? window : max_seq_len;
   if (d.span < 1) d.span = 1;
-  d.pitch = ceil_div(d.span, 256) * 256;
-  d.keys1 = (int64_t)reqs * G * ceil_div(d.span, 256) >= 512 ? 256 : 64;
+  d.pitch = ceil_div(d.span, 64) * 64;
+  d.keys1 = (int64_t)reqs * G * ceil_div(d.span, 64) >= 1024 ? 64 : 16;
   d.parts1 = ceil_div(d.span, d.keys1);
-  d.keys2 = 64;
-  for (int k = 256; k > 64; k >>= 1)
-    if ((int64_t)reqs * ceil_div(d.span, k) >= 1024 && (k <= 128 || H <= 32)) { d.keys2 = k; break; }
-  d.parts2 = ceil_div(d.span, d.keys2);
   d.rm = R <= 1 ? 1 : R <= 2 ? 2 : R <= 4 ? 4 : 8;
   const int units = G * ceil_div(R, d.rm);
   d.ksplit = units == 1 ? 4 : units == 2 ? 2 : 1;
+  d.keys2 = d.ksplit == 4 ? 128 : 64;      // a split is a multiple of 32 keys
+  for (int k = 256; k > d.keys2; k >>= 1)
+    if ((int64_t)reqs * ceil_div(d.span, k) >= 1024 && (k <= 128 || H <= 32)) { d.keys2 = k; break; }
+  d.parts2 = ceil_div(d.span, d.keys2);
   auto up = [](int64_t n) { return (n + 255) / 256 * 256; };
   d.scores = up((int64_t)reqs * H * d.pitch * 4);
   d.ml = up((int64_t)reqs * d.parts1 * H * 8);
@@ -728,7 +735,7 @@ int allow_lds(K kern, int bytes) {
 template <int HD, int RM, int HT>
 int launch_values(const DecodeParams& p, int reqs, hipStream_t s) {
   const int kq = (p.H + 3) / 4;
-  const int bytes = (p.keys2 * decode_pad(p.H) + 16 + 16 * HT * (4 * kq + 1) + 4 * kq + (p.keys2 >> p.bs_log2) + 2) * 4;
+  const int bytes = (p.keys2 * decode_pad(p.H) + 16 + 16 * HT * (4 * kq + 1) + 4 * kq + 2 * ((p.keys2 >> p.bs_log2) + 2)) * 4;
   auto kern = decode_values_kernel<HD, RM, HT>;
   if (int e = allow_lds(kern, bytes)) return e;
   hipLaunchKernelGGL(kern, dim3(p.parts2, reqs), dim3(256), bytes, s, p);
@@ -737,14 +744,18 @@ int launch_values(const DecodeParams& p, int reqs, hipStream_t s) {
 
 template <int HD>
 int launch_decode(const DecodeParams& p, int reqs, int rm, bool cap, hipStream_t s) {
-  const dim3 g1(p.parts1, p.G, reqs), block(256);
-  if (p.keys1 == 256) {
-    if (cap) hipLaunchKernelGGL((decode_scores_kernel<HD, 4, true>), g1, block, 0, s, p);
-    else hipLaunchKernelGGL((decode_scores_kernel<HD, 4, false>), g1, block, 0, s, p);
-  } else {
-    if (cap) hipLaunchKernelGGL((decode_scores_kernel<HD, 1, true>), g1, block, 0, s, p);
-    else hipLaunchKernelGGL((decode_scores_kernel<HD, 1, false>), g1, block, 0, s, p);
-  }
+  const dim3 g1(ceil_div(p.parts1 * p.G, 4), reqs), block(256);
+#define MI_DS(NT, CW)                                                                                 \
+  do {                                                                                                \
+    if (cap) hipLaunchKernelGGL((decode_scores_kernel<HD, NT, CW, true>), g1, block, 0, s, p);        \
+    else hipLaunchKernelGGL((decode_scores_kernel<HD, NT, CW, false>), g1, block, 0, s, p);           \
+  } while (0)
+  const int R = p.H / p.G;
+  if (p.keys1 == 16) MI_DS(1, 16);
+  else if (R <= 4) MI_DS(4, 4);
+  else if (R <= 8) MI_DS(4, 8);
+  else MI_DS(4, 16);
+#undef MI_DS
   int e = launch_status();
   if (e) return e;
   if (p.H <= 32)
