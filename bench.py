@@ -94,7 +94,7 @@ def parse_args():
     ap.add_argument("--pupopel-ctx", type=int, default=4096, help="context of the decode cases")
     ap.add_argument("--pupopel-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
     ap.add_argument("--bodopel", action="store_true",
-                    help="instead of the headline workload: prefill and decode throughput of the Bodopel stack beside the Dogulorn "
+                    help="instead of the headline workload: prefill and decode throughput of the Bodopel stack beside the Pupopel "
                          "and talker stacks of equal size (tools/bench_bodopel.py; one JSON line per case)")
     ap.add_argument("--bodopel-size", default="2k,4k")
     ap.add_argument("--bodopel-mode", default="decode,prefill")

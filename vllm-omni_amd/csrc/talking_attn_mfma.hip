@@ -299,7 +299,7 @@ struct PrefillParams {
   const uint16_t* gate;    // nullptr: none
   uint16_t* out;
   int64_t q_stride, out_stride, gate_stride;
-  int H, G, V, window, rows, ctx_rows;
+  int H, G, V, window, rows, ctx_rows, reqs, max_q;
   ScoreMul mul;
 };
 
@@ -398,9 +398,10 @@ __global__ __launch_bounds__(256) void prefill_sums_kernel(const PrefillParams p
   scalar_cache_acquire();
   constexpr int KS = HD / 32;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
-  const int groups = (p.H + HW - 1) / HW;
-  const int h0 = (blockIdx.x % groups) * HW, r = blockIdx.y, R = p.H / p.G;
-  const TileSpan t = tile_span(p, r, (blockIdx.x / groups) * 64 + wave * 16);
+  // late tiles (long rows) of all portions first; a group of heads stays on its XCD
+  const int groups = (p.H + HW - 1) / HW, at = blockIdx.x / groups;
+  const int h0 = (blockIdx.x % groups) * HW, r = at % p.reqs, R = p.H / p.G;
+  const TileSpan t = tile_span(p, r, ((p.max_q + 63) / 64 - 1 - at / p.reqs) * 64 + wave * 16);
   if (!t.any) return;
   const int qi = min(t.tile0 + lr, t.ql - 1), qpos = t.start + t.tile0 + lr;
   const uint16_t* q = p.q + (int64_t)(t.s0 + qi) * p.q_stride + 8 * lg;
@@ -459,6 +460,12 @@ __device__ __forceinline__ void store_heads(char* at, const uint32_t (&w)[(HW + 
   else *reinterpret_cast<uint4*>(at) = make_uint4(w[0], w[1], w[2], w[3]);
 }
 
+// tiles of a portion that stay together
+__host__ __device__ inline int mix_run(int reqs, int max_q) {
+  const int n = (int)(((int64_t)reqs * ((max_q + 15) / 16)) >> 6);
+  return n < 1 ? 1 : n > 16 ? 16 : n;
+}
+
 // LDS layout of the exchange (bytes).  A buffer has a region per row: the weights [hi, lo][16 keys][KP heads], which the one
 // wave that mixes the row replaces by the mixed weights [16 HT heads][16 keys hi | lo].  Then talk [16 HT][KP] and the query
 // operands that find no room in registers.
@@ -481,12 +488,13 @@ __global__ __launch_bounds__(512, 2) void prefill_mix_kernel(const PrefillParams
   using M = MixLds<HD, HW>;
   constexpr int KS = HD / 32, VN = HD / 16, VH = VN / 2, HT = M::HT, QR = HW - M::QL;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
-  const int NW = blockDim.x >> 6, R = p.H / p.G, r = blockIdx.y;
-  // workgroups go to the 8 XCDs in turn: up to 32 neighbouring tiles on one, where they walk the same keys; late tiles (long
-  // rows) first
-  const int b = blockIdx.x, per = min(32, (int)gridDim.x >> 3), set = 8 * per;
-  const bool whole = per > 0 && b < (int)gridDim.x / max(set, 1) * set;
-  const int tile = gridDim.x - 1 - (whole ? b / set * set + (b & 7) * per + (b % set >> 3) : b);
+  const int NW = blockDim.x >> 6, R = p.H / p.G;
+  // Workgroups go to the 8 XCDs in turn: `run` neighbouring tiles of a portion on one, where they walk the same keys; late
+  // tiles (long rows) of all portions first.
+  const int run = mix_run(p.reqs, p.max_q), tiles = (p.max_q + 15) / 16, b = blockIdx.x;
+  const int unit = b / (8 * run) * 8 + (b & 7), r = unit % p.reqs;
+  const int tile = tiles - 1 - (unit / p.reqs * run + (b >> 3) % run);
+  if (tile < 0) return;
   const TileSpan t = tile_span(p, r, tile * 16);
   if (!t.any) return;
   for (int i = tid; i < M::kTalk / 16; i += blockDim.x) reinterpret_cast<uint4*>(smem)[i] = make_uint4(0, 0, 0, 0);
@@ -771,12 +779,13 @@ int launch_decode(const DecodeParams& p, int reqs, int rm, bool cap, hipStream_t
 
 template <int HD, int HW, bool ONE, bool CAP>
 int launch_prefill(const PrefillParams& p, int reqs, int max_q, hipStream_t s) {
-  hipLaunchKernelGGL((prefill_sums_kernel<HD, HW, ONE, CAP>), dim3(ceil_div(p.H, HW) * ceil_div(max_q, 64), reqs), dim3(256), 0, s, p);
+  hipLaunchKernelGGL((prefill_sums_kernel<HD, HW, ONE, CAP>), dim3(ceil_div(p.H, HW) * ceil_div(max_q, 64) * reqs), dim3(256), 0, s, p);
   if (int e = launch_status()) return e;
   const int waves = ceil_div(p.H, HW), bytes = MixLds<HD, HW>::bytes(waves);
   auto kern = prefill_mix_kernel<HD, HW, ONE, CAP>;
   if (int e = allow_lds(kern, bytes)) return e;
-  hipLaunchKernelGGL(kern, dim3(ceil_div(max_q, 16), reqs), dim3(64 * waves), bytes, s, p);
+  const int run = mix_run(reqs, max_q), units = ceil_div(ceil_div(max_q, 16), run) * reqs;
+  hipLaunchKernelGGL(kern, dim3(ceil_div(units, 8) * 8 * run), dim3(64 * waves), bytes, s, p);
   return launch_status();
 }
 
@@ -850,7 +859,7 @@ extern "C" int mi_talking_prefill(const mi_talking_attn_args* args, const int32_
   if (int e = launch_status()) return e;
   const PrefillParams p{(const uint16_t*)a.q, (const uint16_t*)ws, (const uint16_t*)(ws + kb), (float*)(ws + 2 * kb), ctx_start, a.seq_lens,
                         a.query_start_loc, a.r1, a.r2, a.talk, (const uint16_t*)a.gate, (uint16_t*)a.out, a.q_stride, a.out_stride,
-                        a.gate_stride, a.heads, a.kv_heads, a.vdim, a.window, rows, ctx_rows, score_mul(a.scale, a.softcap)};
+                        a.gate_stride, a.heads, a.kv_heads, a.vdim, a.window, rows, ctx_rows, num_reqs, max_query_len, score_mul(a.scale, a.softcap)};
   const bool cap = a.softcap > 0.f;
   const int hw = heads_per_wave(a.heads);
   if (a.head_dim == 64) {
