@@ -23,7 +23,7 @@
 extern "C" {
 #endif
 
-#define MI_ABI_VERSION 5
+#define MI_ABI_VERSION 6
 
 /* dtype enum shared by every entry point */
 enum {
@@ -365,37 +365,42 @@ int mi_mask_logits_argmax(void* logits, int64_t* ids, int32_t num_tokens, int32_
  *                  weights (fp32, optionally renormalised, optionally rounded to
  *                  weight_round_dtype as HF does; -1 = keep fp32); per-expert
  *                  pair counts (zeroed inside; expert_counts may be NULL: no counting,
- *                  one launch less).  num_experts in {64, 128, 256}.
+ *                  one launch less).  At most 256 experts.  sigmoid != 0: p =
+ *                  sigmoid of each logit, the largest chosen by their logits.
  *   mi_moe_align   groups the T*k (token, slot) pairs by expert, each group padded
  *                  to a multiple of rows_per_tile (32, 64, 128 or 256; mi_moe_rows_per_tile()
  *                  picks by mean pairs per expert): sorted_pairs[row] = pair or -1,
  *                  row_of_pair[pair], tile_expert[row / rows_per_tile], num_tiles[0].
  *                  Buffers sized by mi_moe_max_rows().  expert_counts NULL: counted
  *                  from topk_ids inside the launch.
- *   mi_moe_expert_gemm  gated != 0: out[row, :n_out] = silu(a[tok] . Wg_e^T) *
+ *   mi_moe_expert_gemm  form MI_MOE_GATED: out[row, :n_out] = silu(a[tok] . Wg_e^T) *
  *                  (a[tok] . Wu_e^T), weights [E, 2*n_out, k] (gate rows then up
  *                  rows), a = x [T, k], tok = sorted_pairs[row] / top_k;
- *                  gated == 0: out[row, :n_out] = a[row] . W_e^T, weights
- *                  [E, n_out, k], a = the gated output.  max_tiles bounds the
- *                  grid; tiles >= num_tiles[0] exit.  k % 64 == 0; n_out % 64
+ *                  MI_MOE_RELU_SQUARED: relu(s a[tok] . W_e^T)^2, weights [E, n_out,
+ *                  k], s = pair_weights[sorted_pairs[row]] (NULL: 1);
+ *                  MI_MOE_PLAIN: out[row, :n_out] = a[row] . W_e^T, weights
+ *                  [E, n_out, k], a = the output of one of the other forms.
+ *                  pair_weights goes with MI_MOE_RELU_SQUARED only.  max_tiles bounds
+ *                  the grid; tiles >= num_tiles[0] exit.  k % 64 == 0; n_out % 64
  *                  (gated) / % 128 == 0; bf16 and at most 64 rows per tile also
  *                  k % 8 == 0, n_out % 4 == 0.
  *   mi_moe_combine out[t] = sum_j w[t, j] * partial[row_of_pair[t*k + j]]
  *                  (+ g * shared_out[t], g = sigmoid(x[t] . shared_gate_weight) or 1).
  * ---------------------------------------------------------------------- */
+enum { MI_MOE_PLAIN = 0, MI_MOE_GATED = 1, MI_MOE_RELU_SQUARED = 2 };
 int32_t mi_moe_rows_per_tile(int32_t num_tokens, int32_t top_k, int32_t num_experts); /* 32, 64 or (prefill chunks) 256 */
 int64_t mi_moe_max_rows(int32_t num_tokens, int32_t top_k, int32_t num_experts, int32_t rows_per_tile);
 int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* expert_counts, const void* router_logits,
                  const float* bias /* [num_experts], added to the logits, or NULL */, int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
-                 int32_t norm_topk_prob, int logits_dtype, int weight_round_dtype, void* stream);
+                 int32_t norm_topk_prob, int32_t sigmoid, int logits_dtype, int weight_round_dtype, void* stream);
 int mi_moe_align(int32_t* sorted_pairs, int32_t* row_of_pair, int32_t* tile_expert, int32_t* num_tiles,
                  const int32_t* topk_ids, const int32_t* expert_counts, int32_t num_pairs,
                  int32_t num_experts, int64_t max_rows, int32_t rows_per_tile, void* stream);
 int mi_moe_expert_gemm(void* out, const void* a_rows, const void* weights, const int32_t* sorted_pairs,
                        const int32_t* tile_expert, const int32_t* num_tiles, int32_t max_tiles,
-                       int32_t gated, int32_t n_out, int32_t k, int32_t top_k, int64_t a_row_stride,
-                       int64_t out_row_stride, int64_t weight_expert_stride, int32_t rows_per_tile, int dtype,
-                       void* stream);
+                       int32_t form, const float* pair_weights, int32_t n_out, int32_t k, int32_t top_k,
+                       int64_t a_row_stride, int64_t out_row_stride, int64_t weight_expert_stride,
+                       int32_t rows_per_tile, int dtype, void* stream);
 int mi_moe_combine(void* out, const void* partial, const int32_t* row_of_pair, const float* topk_weights,
                    const void* shared_out, const void* x, const void* shared_gate_weight,
                    int32_t num_tokens, int32_t hidden, int32_t top_k, int64_t partial_row_stride,
@@ -926,10 +931,10 @@ int mi_lightning_attn(const mi_lightning_args* args, int32_t row0, int32_t rows,
                       int32_t max_query_len, int32_t chunked, void* workspace,
                       int64_t workspace_bytes, int dtype, void* stream);
 /* mi_moe_expert_gemm for any sizes and for fp32, pairs ungrouped: row p of out
- * (and of a_rows, gated == 0) belongs to pair p = token * top_k + j. */
+ * (and of a_rows, MI_MOE_PLAIN) belongs to pair p = token * top_k + j. */
 int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const int32_t* topk_ids,
-                     int32_t num_pairs, int32_t num_experts, int32_t gated, int32_t n_out, int32_t k,
-                     int32_t top_k, int64_t a_row_stride, int64_t out_row_stride,
+                     int32_t num_pairs, int32_t num_experts, int32_t form, const float* pair_weights,
+                     int32_t n_out, int32_t k, int32_t top_k, int64_t a_row_stride, int64_t out_row_stride,
                      int64_t weight_expert_stride, int dtype, void* stream);
 
 /* ------------------------------------------------------------------------
@@ -1013,6 +1018,75 @@ int64_t mi_talking_prefill_workspace_bytes(int32_t rows, int32_t heads, int32_t 
 int mi_talking_prefill(const mi_talking_attn_args* args, const int32_t* ctx_start, int32_t ctx_rows,
                        int32_t num_reqs, int32_t rows, int32_t max_query_len, void* workspace,
                        int64_t workspace_bytes, void* stream);
+
+/* ------------------------------------------------------------------------
+ * Decoders of state-space layers and attention whose values are its keys,
+ * mixer and feed-forward side by side, each behind a norm of its own (Lifuzen):
+ * bf16 or fp32 as above.
+ * ---------------------------------------------------------------------- */
+/* x[row] += mult (y[row] + sum_j weights[row][j] part[row_of_pair[row][j]]), or
+ * x[row] = 0 when y == NULL;  x += table[id] (table != NULL; zeros for ids
+ * outside it) + add_row [width] (NULL: none);  h1, h2 = x / rms(x) * (w +
+ * w_shift) with w1 and w2 (NULL: no h2).  y, part, row_of_pair as in
+ * mi_residual_add_norm; weights NULL: 1. */
+int mi_stream_norm2(void* x, const void* y, int32_t split, const void* part, const int32_t* row_of_pair,
+                    const float* weights, int32_t top, float mult, const void* table,
+                    const int64_t* ids, int32_t vocab, const void* add_row, const void* w1,
+                    const void* w2, float w_shift, void* h1, void* h2, float eps, int32_t rows,
+                    int32_t width, int64_t x_stride, int64_t y_stride, int64_t part_stride,
+                    int64_t h1_stride, int64_t h2_stride, int dtype, void* stream);
+/* Rows q (heads x dim) | k (kv x dim): each channel through a causal filter over
+ * the sequence (conv_w [(heads + kv) dim][taps], the last tap for the row
+ * itself, zeros before the start); v = that k; then the pairs (2i, 2i + 1), i <
+ * rot_dims / 2, of q's and k's heads turned by position * inv_freq[i]; then both
+ * divided by their root mean square over dim, per head.  q to q_out (rows of the
+ * whole step), k and v to their cache rows, heads head_dim apart, zeros behind
+ * them.  ring [slots][taps][(heads + kv) dim]: a request's last inputs, the one
+ * of position p in place p % taps; update_ring: also those of portions of more
+ * than one row (a one-row portion's is always left there).  slots per request;
+ * requests [req0, req0 + num_reqs). */
+typedef struct {
+  const void *x, *conv_w;
+  void *ring, *q_out, *k_cache, *v_cache;
+  const float* inv_freq; /* [rot_dims / 2] */
+  const int32_t *slots, *query_start_loc, *seq_lens;
+  const int64_t* slot_mapping; /* per row; < 0: not written */
+  int64_t x_stride, q_stride, cache_block_stride, cache_token_stride, cache_head_stride;
+  int32_t req0, num_reqs, max_query_len, heads, kv_heads, dim, head_dim, block_size, rot_dims, taps;
+  int32_t update_ring;
+  float eps;
+} mi_conv_rope_cache_args;
+int mi_conv_rope_cache(const mi_conv_rope_cache_args* args, int dtype, void* stream);
+/* State-space recurrence of requests [req0, req0 + num_reqs), which own rows
+ * [row0, row0 + rows): x (heads x vdim) | B (groups x state) | C (groups x
+ * state) of a row through causal filters (conv_w [channels][taps], conv_b
+ * [channels]) and silu; dt = softplus(dt + dt_bias); per head, with B and C of
+ * its group, S = exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + d x; out[row] =
+ * y silu(z), RMS-normed in norm_groups equal parts, times norm_w.  S
+ * [slots][heads][state][vdim] fp32; ring [slots][taps][channels] as above. */
+typedef struct {
+  const void *xbc, *z, *dt; /* rows of the model's dtype, `stride` apart */
+  const void *conv_w, *conv_b, *norm_w;
+  const float *dt_bias, *a_log, *d; /* [heads] */
+  float* state;
+  void* ring;
+  const int32_t *slots, *query_start_loc, *seq_lens;
+  void* out;
+  int64_t stride, out_stride;
+  int32_t req0, num_reqs, heads, groups, state_dim, vdim, taps, norm_groups;
+  float eps;
+} mi_state_space_args;
+/* chunked: 64 tokens at a time on the matrix cores (bf16; state_dim, vdim <=
+ * 256), else token by token.  The workspace is scratch; 0 bytes = sizes not
+ * built. */
+int64_t mi_state_space_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t groups,
+                                       int32_t state_dim, int32_t vdim, int32_t chunked, int dtype);
+int mi_state_space(const mi_state_space_args* args, int32_t row0, int32_t rows, int32_t max_query_len,
+                   int32_t chunked, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
+/* logits = cap tanh(logits / cap) in place, then mi_mask_logits_argmax's greedy
+ * ids of them (ids NULL: none) */
+int mi_soft_cap_argmax(void* logits, int64_t* ids, float cap, int32_t num_tokens, int32_t vocab,
+                       int64_t row_stride, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

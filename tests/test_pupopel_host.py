@@ -181,8 +181,8 @@ def test_argument_validation_without_gpu():
     assert call(1 << 30, qkv_stride=90) == bad and call(1 << 30, dim=300, qkv_stride=2000) == no
     assert call(lib.mi_lightning_workspace_bytes(64, 1, 2, 16, 16, 1) - 1) == _C.MI_ERR_WORKSPACE
     assert lib.mi_lightning_workspace_bytes(64, 1, 2, 300, 16, 1) == 0
-    assert lib.mi_moe_route(p, p, None, p, p, 2, 257, 257, 2, 1, _C.MI_DTYPE_F32, -1, None) == no
-    assert lib.mi_moe_pair_gemm(p, p, p, p, 4, 2, 1, 8, 16, 2, 16, 8, 100, 1, None) == bad
+    assert lib.mi_moe_route(p, p, None, p, p, 2, 257, 257, 2, 1, 0, _C.MI_DTYPE_F32, -1, None) == no
+    assert lib.mi_moe_pair_gemm(p, p, p, p, 4, 2, _C.MI_MOE_GATED, None, 8, 16, 2, 16, 8, 100, 1, None) == bad
 
 
 # ------------------------------------------------------------------------------------------------ the restatement itself

@@ -44,7 +44,7 @@ __device__ __forceinline__ float wave_max_valu(float v) {
   return rows_allreduce_max(v);
 }
 
-template <int DT, int EPL>  // EPL = experts per lane = E / 64, rounded up
+template <int DT, int EPL, bool SIG>  // EPL = experts per lane = E / 64, rounded up; SIG: scores are sigmoids, ranked by their logits
 __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict__ logits, const float* __restrict__ bias,
                                                          int64_t row_stride, int num_experts,
                                                          int32_t* __restrict__ ids, float* __restrict__ weights,
@@ -58,6 +58,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   for (int e = threadIdx.x; e < 64 * EPL; e += 1024) hist[e] = 0;
   __syncthreads();
+  constexpr float kNone = SIG ? -INFINITY : -1.f;     // below every score
   for (int t = blockIdx.x * 16 + wid; t < T; t += gridDim.x * 16) {
     float p[EPL];
     float mx = -INFINITY;
@@ -75,22 +76,22 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
     float s = 0.f;
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
-      p[i] = __expf(p[i] - mx);
-      if (lane + 64 * i >= num_experts) p[i] = -1.f;   // not an expert
+      if constexpr (!SIG) p[i] = __expf(p[i] - mx);
+      if (lane + 64 * i >= num_experts) p[i] = kNone;   // not an expert
       else s += p[i];
     }
-    s = wave_allreduce_sum(s);
-    const float inv = 1.f / s;
+    float inv = 1.f;
+    if constexpr (!SIG) inv = 1.f / wave_allreduce_sum(s);
     float wsum = 0.f, myw = 0.f;
     int mye = 0;
     for (int j = 0; j < top_k; ++j) {  // k rounds of wave arg-max, lowest expert id on ties
       // the largest remaining probability, then the lowest expert id that holds it
-      float best = -1.f;
+      float best = kNone;
 #pragma unroll
       for (int i = 0; i < EPL; ++i) best = p[i] > best ? p[i] : best;   // NaN never wins
       best = wave_max_valu(best);
       int bi = 0x7fffffff;
-      if (best >= 0.f) {
+      if (best > kNone) {
 #pragma unroll
         for (int i = EPL - 1; i >= 0; --i) {
           const uint64_t m = __ballot(p[i] == best);
@@ -99,12 +100,12 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const void* __restrict_
       }
 #pragma unroll
       for (int i = 0; i < EPL; ++i)
-        if (lane + 64 * i == bi) p[i] = -1.f;  // taken
+        if (lane + 64 * i == bi) p[i] = kNone;  // taken
       if (bi == 0x7fffffff) {  // NaN logits: no comparison succeeds.  Never let an out-of-range id reach the
         bi = j;                // counters or the grouping; experts 0..k-1 with weight NaN keep the poison visible
         best = __builtin_nanf("");
       }
-      const float w = best * inv;
+      const float w = SIG ? sigmoid_f(best) : best * inv;
       wsum += w;
       if (lane == j) { myw = w; mye = bi; }
     }
@@ -236,13 +237,15 @@ struct MoeGemmParams {
   const int32_t* num_tiles;
   int32_t K, N_out, top_k;
   int64_t a_stride, out_stride, w_expert_stride;
+  const float* pair_weights;     // MI_MOE_RELU_SQUARED: what a pair's row is multiplied by, or nullptr
 };
 
-// GATED: gemm 1 — a wave owns 16 gate rows and the 16 matching up rows; WG = 4 waves = 64 outputs.
-// !GATED: gemm 2 — a wave owns 32 weight rows; WG = 4 waves = 128 outputs.
+// FORM: MI_MOE_GATED: gemm 1 — a wave owns 16 gate rows and the 16 matching up rows; WG = 4 waves = 64 outputs.
+// Else a wave owns 32 weight rows, WG = 4 waves = 128 outputs: gemm 2 (MI_MOE_PLAIN), or gemm 1 of experts without a gate.
 // GUARD: any n_out that is a multiple of 4 and any K that is a multiple of 8 (weight rows and k past the end are blanked out)
-template <typename Tag, bool GATED, int MT, bool GUARD = false>  // MT = 16-row token tiles per workgroup tile (2 or 4)
+template <typename Tag, int FORM, int MT, bool GUARD = false>  // MT = 16-row token tiles per workgroup tile (2 or 4)
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
+  constexpr bool GATED = FORM == MI_MOE_GATED;
   constexpr int kMoeRows = 16 * MT;
   scalar_cache_acquire();
   using E = Elem<Tag>;
@@ -263,7 +266,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
 #pragma unroll
   for (int mt = 0; mt < MT; ++mt) {
     const int row = row0 + 16 * mt + r16;
-    if constexpr (GATED) {
+    if constexpr (FORM != MI_MOE_PLAIN) {
       const int pair = p.sorted_pairs[row];
       brow[mt] = p.a_rows + (int64_t)(pair < 0 ? 0 : pair / p.top_k) * p.a_stride + 16 * kg;
     } else {
@@ -342,6 +345,17 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
       q.y = E::pack(v[2], v[3]);
       if (!GUARD || n_base + 4 * kg < p.N_out) *reinterpret_cast<uint2*>(o + n_base + 4 * kg) = q;
     } else {
+      if constexpr (FORM == MI_MOE_RELU_SQUARED) {
+        const int pair = p.sorted_pairs[row];
+        const float s = p.pair_weights && pair >= 0 ? p.pair_weights[pair] : 1.f;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float v = fmaxf(s * acc[i][mt][r], 0.f);
+            acc[i][mt][r] = v * v;
+          }
+      }
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
         uint2 q;
@@ -355,17 +369,18 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const MoeGemmParams p) {
 
 // ---------------------------------------------------------------- any sizes and types
 // One workgroup per (pair, 16 outputs), a wave per four of them, pairs in their own order (no grouping): 32-bit models and
-// sizes the matrix-core kernels do not take.  GATED: out[pair] = silu(x[tok] Wg^T) * (x[tok] Wu^T), else out[pair] = a[pair] W^T.
-template <typename T, bool GATED>
+// sizes the matrix-core kernels do not take.  FORM as above, row p of out (and of a, MI_MOE_PLAIN) is pair p's.
+template <typename T, int FORM>
 __global__ __launch_bounds__(256) void moe_pair_gemm_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ w,
-                                                            const int32_t* __restrict__ ids, int n_out, int K, int top_k, int E,
+                                                            const int32_t* __restrict__ ids, const float* pair_weights, int n_out, int K, int top_k, int E,
                                                             int64_t a_stride, int64_t out_stride, int64_t w_stride) {
   scalar_cache_acquire();
+  constexpr bool GATED = FORM == MI_MOE_GATED;
   const int64_t pair = blockIdx.x;
   const int lane = threadIdx.x & 63, n0 = blockIdx.y * 16 + (threadIdx.x >> 6) * 4;
   const int e = ids[pair];
   const bool known = e >= 0 && e < E;
-  const T* x = a + (GATED ? pair / top_k : pair) * a_stride;
+  const T* x = a + (FORM != MI_MOE_PLAIN ? pair / top_k : pair) * a_stride;
   const T* we = w + (known ? e : 0) * w_stride;
   for (int n = n0; n < min(n0 + 4, n_out); ++n) {
     float g = 0.f, u = 0.f;
@@ -376,6 +391,10 @@ __global__ __launch_bounds__(256) void moe_pair_gemm_kernel(T* __restrict__ out,
     }
     g = wave_allreduce_sum(g);
     if constexpr (GATED) g = silu_f(g) * wave_allreduce_sum(u);
+    if constexpr (FORM == MI_MOE_RELU_SQUARED) {
+      g = fmaxf(pair_weights ? pair_weights[pair] * g : g, 0.f);
+      g *= g;
+    }
     if (lane == 0) Io<T>::st(out + pair * out_stride + n, known ? g : 0.f);
   }
 }
@@ -457,7 +476,7 @@ extern "C" int64_t mi_moe_max_rows(int32_t num_tokens, int32_t top_k, int32_t nu
 
 extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* expert_counts, const void* router_logits,
                             const float* bias, int32_t num_tokens, int32_t num_experts, int64_t logits_row_stride, int32_t top_k,
-                            int32_t norm_topk_prob, int logits_dtype, int weight_round_dtype, void* stream) {
+                            int32_t norm_topk_prob, int32_t sigmoid, int logits_dtype, int weight_round_dtype, void* stream) {
   using namespace mi;
   if (num_tokens == 0) return MI_OK;
   if (!topk_ids || !topk_weights || !router_logits || num_tokens < 0) return MI_ERR_INVALID_ARG;
@@ -471,14 +490,19 @@ extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* exp
   // tokens per wave: 1 for decode batches (latency), up to 4 for prefill chunks (fewer, fuller count flushes)
   const int tpw = num_tokens >= 8192 ? 4 : num_tokens >= 1024 ? 2 : 1;
   const dim3 grid((num_tokens + 16 * tpw - 1) / (16 * tpw)), block(1024);
-#define MI_ROUTE(DT, EPL)                                                                                        \
-  hipLaunchKernelGGL((moe_route_kernel<DT, EPL>), grid, block, 0, s, router_logits, bias, logits_row_stride, num_experts, topk_ids, \
+#define MI_ROUTE(DT, EPL, SIG)                                                                                   \
+  hipLaunchKernelGGL((moe_route_kernel<DT, EPL, SIG>), grid, block, 0, s, router_logits, bias, logits_row_stride, num_experts, topk_ids, \
                      topk_weights, expert_counts, num_tokens, top_k, norm_topk_prob, weight_round_dtype)
+#define MI_ROUTE_S(DT, SIG)                             \
+  do {                                                  \
+    if (num_experts <= 64) MI_ROUTE(DT, 1, SIG);        \
+    else if (num_experts <= 128) MI_ROUTE(DT, 2, SIG);  \
+    else MI_ROUTE(DT, 4, SIG);                          \
+  } while (0)
 #define MI_ROUTE_E(DT)                                  \
   do {                                                  \
-    if (num_experts <= 64) MI_ROUTE(DT, 1);             \
-    else if (num_experts <= 128) MI_ROUTE(DT, 2);       \
-    else MI_ROUTE(DT, 4);                               \
+    if (sigmoid) MI_ROUTE_S(DT, true);                  \
+    else MI_ROUTE_S(DT, false);                         \
   } while (0)
   switch (logits_dtype) {
     case MI_DTYPE_F32: MI_ROUTE_E(MI_DTYPE_F32); break;
@@ -487,6 +511,7 @@ extern "C" int mi_moe_route(int32_t* topk_ids, float* topk_weights, int32_t* exp
     default: return MI_ERR_UNSUPPORTED;
   }
 #undef MI_ROUTE_E
+#undef MI_ROUTE_S
 #undef MI_ROUTE
   return launch_status();
 }
@@ -511,10 +536,13 @@ extern "C" int mi_moe_align(int32_t* sorted_pairs, int32_t* row_of_pair, int32_t
 
 extern "C" int mi_moe_expert_gemm(void* out, const void* a_rows, const void* weights, const int32_t* sorted_pairs,
                                   const int32_t* tile_expert, const int32_t* num_tiles, int32_t max_tiles,
-                                  int32_t gated, int32_t n_out, int32_t k, int32_t top_k, int64_t a_row_stride,
-                                  int64_t out_row_stride, int64_t weight_expert_stride, int32_t rows_per_tile,
-                                  int dtype, void* stream) {
+                                  int32_t form, const float* pair_weights, int32_t n_out, int32_t k, int32_t top_k,
+                                  int64_t a_row_stride, int64_t out_row_stride, int64_t weight_expert_stride,
+                                  int32_t rows_per_tile, int dtype, void* stream) {
   using namespace mi;
+  const bool gated = form == MI_MOE_GATED;
+  if (form < MI_MOE_PLAIN || form > MI_MOE_RELU_SQUARED || (pair_weights && form != MI_MOE_RELU_SQUARED) || top_k <= 0)
+    return MI_ERR_INVALID_ARG;
   if (max_tiles == 0) return MI_OK;
   if (!out || !a_rows || !weights || !sorted_pairs || !tile_expert || !num_tiles || max_tiles < 0)
     return MI_ERR_INVALID_ARG;
@@ -534,7 +562,7 @@ extern "C" int mi_moe_expert_gemm(void* out, const void* a_rows, const void* wei
       GroupedGemmArgs ga;
       ga.out = out; ga.a_rows = a_rows; ga.weights = weights;
       ga.sorted_pairs = sorted_pairs; ga.tile_expert = tile_expert; ga.num_tiles = num_tiles;
-      ga.max_tiles = max_tiles; ga.gated = gated; ga.n_out = n_out; ga.k = k; ga.top_k = top_k;
+      ga.max_tiles = max_tiles; ga.form = form; ga.pair_weights = pair_weights; ga.n_out = n_out; ga.k = k; ga.top_k = top_k;
       ga.rows_per_tile = rows_per_tile;
       ga.a_row_stride = a_row_stride; ga.out_row_stride = out_row_stride; ga.weight_expert_stride = weight_expert_stride;
       ga.dtype = dtype;
@@ -556,27 +584,30 @@ extern "C" int mi_moe_expert_gemm(void* out, const void* a_rows, const void* wei
   p.a_stride = a_row_stride;
   p.out_stride = out_row_stride;
   p.w_expert_stride = weight_expert_stride;
+  p.pair_weights = pair_weights;
   const dim3 grid((max_tiles + 7) / 8 * 8, gated ? (n_out + 63) / 64 : (n_out + 127) / 128), block(256);
   if (guard) {
 #define MI_MOE_GUARD(G, M) hipLaunchKernelGGL((moe_gemm_kernel<bf16_tag, G, M, true>), grid, block, 0, s, p)
-    if (gated && rows_per_tile == 32) MI_MOE_GUARD(true, 2);
-    else if (gated) MI_MOE_GUARD(true, 4);
-    else if (rows_per_tile == 32) MI_MOE_GUARD(false, 2);
-    else MI_MOE_GUARD(false, 4);
+#define MI_MOE_GUARD_F(G) do { if (rows_per_tile == 32) MI_MOE_GUARD(G, 2); else MI_MOE_GUARD(G, 4); } while (0)
+    if (gated) MI_MOE_GUARD_F(MI_MOE_GATED);
+    else if (form == MI_MOE_PLAIN) MI_MOE_GUARD_F(MI_MOE_PLAIN);
+    else MI_MOE_GUARD_F(MI_MOE_RELU_SQUARED);
+#undef MI_MOE_GUARD_F
 #undef MI_MOE_GUARD
     return launch_status();
   }
 #define MI_MOE_GEMM(TAG, G, M) hipLaunchKernelGGL((moe_gemm_kernel<TAG, G, M>), grid, block, 0, s, p)
 #define MI_MOE_GEMM_T(TAG)                                \
   do {                                                    \
-    if (gated && rows_per_tile == 32) MI_MOE_GEMM(TAG, true, 2);        \
-    else if (gated) MI_MOE_GEMM(TAG, true, 4);            \
-    else if (rows_per_tile == 32) MI_MOE_GEMM(TAG, false, 2);           \
-    else MI_MOE_GEMM(TAG, false, 4);                      \
+    if (gated) MI_MOE_GEMM_F(TAG, MI_MOE_GATED);          \
+    else if (form == MI_MOE_PLAIN) MI_MOE_GEMM_F(TAG, MI_MOE_PLAIN);    \
+    else MI_MOE_GEMM_F(TAG, MI_MOE_RELU_SQUARED);         \
   } while (0)
+#define MI_MOE_GEMM_F(TAG, G) do { if (rows_per_tile == 32) MI_MOE_GEMM(TAG, G, 2); else MI_MOE_GEMM(TAG, G, 4); } while (0)
   if (dtype == MI_DTYPE_BF16) MI_MOE_GEMM_T(bf16_tag);
   else if (dtype == MI_DTYPE_F16) MI_MOE_GEMM_T(f16_tag);
   else return MI_ERR_UNSUPPORTED;
+#undef MI_MOE_GEMM_F
 #undef MI_MOE_GEMM_T
 #undef MI_MOE_GEMM
   return launch_status();
@@ -609,25 +640,29 @@ extern "C" int mi_moe_combine(void* out, const void* partial, const int32_t* row
 }
 
 extern "C" int mi_moe_pair_gemm(void* out, const void* a_rows, const void* weights, const int32_t* topk_ids, int32_t num_pairs,
-                                int32_t num_experts, int32_t gated, int32_t n_out, int32_t k, int32_t top_k, int64_t a_row_stride,
-                                int64_t out_row_stride, int64_t weight_expert_stride, int dtype, void* stream) {
+                                int32_t num_experts, int32_t form, const float* pair_weights, int32_t n_out, int32_t k, int32_t top_k,
+                                int64_t a_row_stride, int64_t out_row_stride, int64_t weight_expert_stride, int dtype, void* stream) {
   using namespace mi;
   if (num_pairs == 0) return MI_OK;
   if (!out || !a_rows || !weights || !topk_ids || num_pairs < 0 || num_experts <= 0 || n_out <= 0 || k <= 0 || top_k <= 0 ||
-      a_row_stride < k || out_row_stride < n_out || weight_expert_stride < (int64_t)(gated ? 2 : 1) * n_out * k)
+      form < MI_MOE_PLAIN || form > MI_MOE_RELU_SQUARED || (pair_weights && form != MI_MOE_RELU_SQUARED) ||
+      a_row_stride < k || out_row_stride < n_out || weight_expert_stride < (int64_t)(form == MI_MOE_GATED ? 2 : 1) * n_out * k)
     return MI_ERR_INVALID_ARG;
   const dim3 grid(num_pairs, (n_out + 15) / 16), block(256);
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-#define MI_PAIR(T)                                                                                                                  \
-  do {                                                                                                                              \
-    if (gated) hipLaunchKernelGGL((moe_pair_gemm_kernel<T, true>), grid, block, 0, s, (T*)out, (const T*)a_rows, (const T*)weights, \
-                                  topk_ids, n_out, k, top_k, num_experts, a_row_stride, out_row_stride, weight_expert_stride);      \
-    else hipLaunchKernelGGL((moe_pair_gemm_kernel<T, false>), grid, block, 0, s, (T*)out, (const T*)a_rows, (const T*)weights,      \
-                            topk_ids, n_out, k, top_k, num_experts, a_row_stride, out_row_stride, weight_expert_stride);            \
+#define MI_PAIR_F(T, G)                                                                                                         \
+  hipLaunchKernelGGL((moe_pair_gemm_kernel<T, G>), grid, block, 0, s, (T*)out, (const T*)a_rows, (const T*)weights, topk_ids,   \
+                     pair_weights, n_out, k, top_k, num_experts, a_row_stride, out_row_stride, weight_expert_stride)
+#define MI_PAIR(T)                                              \
+  do {                                                          \
+    if (form == MI_MOE_GATED) MI_PAIR_F(T, MI_MOE_GATED);       \
+    else if (form == MI_MOE_PLAIN) MI_PAIR_F(T, MI_MOE_PLAIN);  \
+    else MI_PAIR_F(T, MI_MOE_RELU_SQUARED);                     \
   } while (0)
   if (dtype == MI_DTYPE_BF16) MI_PAIR(uint16_t);
   else if (dtype == MI_DTYPE_F32) MI_PAIR(float);
   else return MI_ERR_UNSUPPORTED;
 #undef MI_PAIR
+#undef MI_PAIR_F
   return launch_status();
 }

@@ -8,7 +8,7 @@
 #include <cstdlib>
 #include <type_traits>
 
-#include "common.h"
+#include "row_io.h"
 
 namespace mi {
 namespace {
@@ -454,6 +454,46 @@ reduce:
   }
 }
 
+// logits row: cap * tanh(logit / cap) in place, then (ids) the first index of the maximum of what was stored
+template <typename T, int VEC>
+__global__ __launch_bounds__(1024) void soft_cap_argmax_kernel(T* logits, int64_t* ids, float cap, int vocab, int64_t row_stride) {
+  scalar_cache_acquire();
+  __shared__ float sv[16];
+  __shared__ int si[16];
+  T* row = logits + blockIdx.x * row_stride;
+  const float inv = 1.f / cap;
+  float best = -INFINITY;
+  int besti = 0x7fffffff;
+  for (int c = threadIdx.x * VEC; c < vocab; c += 1024 * VEC) {
+    float v[VEC];
+    Io<T>::template ldv<VEC>(row + c, v);
+    T h[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] = cap * tanhf(v[j] * inv);
+    Io<T>::template stv<VEC>(row + c, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      Io<T>::st(h + j, v[j]);
+      const float s = Io<T>::ld(h + j);
+      if (s > best) best = s, besti = c + j;      // columns of a thread ascend: the first one of a value stays
+    }
+  }
+  if (ids == nullptr) return;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ov = __shfl_xor(best, o, 64);
+    const int oi = __shfl_xor(besti, o, 64);
+    if (ov > best || (ov == best && oi < besti)) { best = ov; besti = oi; }
+  }
+  if ((threadIdx.x & 63) == 0) { sv[threadIdx.x >> 6] = best; si[threadIdx.x >> 6] = besti; }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int i = 1; i < 16; ++i)
+      if (sv[i] > best || (sv[i] == best && si[i] < besti)) { best = sv[i]; besti = si[i]; }
+    ids[blockIdx.x] = besti == 0x7fffffff ? 0 : besti;
+  }
+}
+
 // out[t] = embed[ids[t]] (+ reply[idx[t]]): one workgroup per token, 16 B per lane.
 template <typename Tag>
 __global__ __launch_bounds__(256) void talker_embeds_kernel(uint16_t* __restrict__ out,
@@ -762,6 +802,22 @@ extern "C" int mi_mask_logits_argmax(void* logits, int64_t* ids, int32_t num_tok
     default:
       return MI_ERR_UNSUPPORTED;
   }
+  return launch_status();
+}
+
+extern "C" int mi_soft_cap_argmax(void* logits, int64_t* ids, float cap, int32_t num_tokens, int32_t vocab, int64_t row_stride,
+                                  int dtype, void* stream) {
+  using namespace mi;
+  if (num_tokens == 0) return MI_OK;
+  if (!logits || !(cap > 0.f) || num_tokens < 0 || vocab <= 0 || row_stride < vocab) return MI_ERR_INVALID_ARG;
+  hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  const dim3 grid(num_tokens), block(1024);
+  const bool vec = vocab % 8 == 0 && row_stride % 8 == 0 && aligned16(logits);
+#define MI_SC(T, V) hipLaunchKernelGGL((soft_cap_argmax_kernel<T, V>), grid, block, 0, s, (T*)logits, ids, cap, vocab, row_stride)
+  if (dtype == MI_DTYPE_BF16) { if (vec) MI_SC(uint16_t, 8); else MI_SC(uint16_t, 1); }
+  else if (dtype == MI_DTYPE_F32) { if (vec) MI_SC(float, 8); else MI_SC(float, 1); }
+  else return MI_ERR_UNSUPPORTED;
+#undef MI_SC
   return launch_status();
 }
 

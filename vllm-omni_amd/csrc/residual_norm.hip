@@ -4,6 +4,8 @@
 //   * residual_add_norm: residual add of a layer's output (and of its routed experts' rows, weighted) + pre-norm or cast
 //     for what follows; also starts a stream from a projection (no add)
 //   * embed_norm:      token embedding + the first pre-norm or cast
+//   * stream_norm2:    residual add times a multiplier, what a pass of looped layers adds, and TWO norms of the sum (mixer and
+//     feed-forward each read a norm of their own); also starts a stream from the embedding
 //   * pair_embed_norm: scaled token embedding + the row of the (previous, current) token pair + the first pre-norm
 //   * gelu_lookup_mul: gelu_tanh(z) * (a slice of a per-token table row)
 //   * clamped_glu:     g sigmoid(alpha g) (u + 1) on clamped g, u
@@ -395,6 +397,100 @@ __global__ __launch_bounds__(256) void embed_pos_norm_kernel(const EmbedNormPara
   embed_norm_row<T, VEC, MAXC, true>(p);
 }
 
+struct StreamParams {
+  float* x;
+  const void* y;                // T rows, or fp32 slabs [split][rows][y_stride]; nullptr: x = table[id]
+  const void* part;             // routed experts' output rows, T; nullptr: none
+  const int32_t* row_of_pair;   // nullptr: pair t * top + j is its row t * top + j
+  const float* weights;         // [rows][top]; nullptr: 1
+  const void* table;            // nullptr: none; with y: table[id] is added once more
+  const int64_t* ids;
+  const void* add_row;          // [width] added to every row; nullptr: none
+  const void* w1;
+  const void* w2;               // nullptr: one norm only
+  void* h1;
+  void* h2;
+  int64_t x_stride, y_stride, part_stride, h1_stride, h2_stride;
+  int rows, width, split, top, vocab;
+  float mult, w_shift, eps;
+};
+
+template <typename T, int VEC, int MAXC>
+__global__ __launch_bounds__(256) void stream_norm2_kernel(const StreamParams p) {
+  scalar_cache_acquire();
+  __shared__ float smem[16];
+  const int64_t row = blockIdx.x;
+  const int64_t id = p.table ? p.ids[row] : 0;
+  const bool known = id >= 0 && id < p.vocab;   // an id outside the table reads as a zero row
+  const T* er = reinterpret_cast<const T*>(p.table) + (known ? id : 0) * p.width;
+  float* xr = p.x + row * p.x_stride;
+  float x[MAXC][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float t[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) x[k][j] = 0.f;
+    if (p.y) {
+      if (p.split) {
+        const float* yp = reinterpret_cast<const float*>(p.y) + row * p.y_stride + c;
+        for (int s = 0; s < p.split; ++s) {
+          Io<float>::ldv<VEC>(yp + (int64_t)s * p.rows * p.y_stride, t);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) x[k][j] += t[j];
+        }
+      } else {
+        Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.y) + row * p.y_stride + c, x[k]);
+      }
+      if (p.part) {
+        for (int j0 = 0; j0 < p.top; ++j0) {
+          const int64_t pair = row * p.top + j0;
+          const int64_t pr = p.row_of_pair ? p.row_of_pair[pair] : pair;
+          const float w = p.weights ? p.weights[pair] : 1.f;
+          Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.part) + pr * p.part_stride + c, t);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) x[k][j] += w * t[j];
+        }
+      }
+      Io<float>::ldv<VEC>(xr + c, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] = t[j] + p.mult * x[k][j];
+    }
+    if (p.table) {
+      Io<T>::template ldv<VEC>(er + c, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] += known ? t[j] : 0.f;
+    }
+    if (p.add_row) {
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.add_row) + c, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) x[k][j] += t[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss += x[k][j] * x[k][j];
+    Io<float>::stv<VEC>(xr + c, x[k]);
+  }
+  const float inv = inv_rms(wg_sum(ss, smem), p.width, p.eps);
+#pragma unroll
+  for (int k = 0; k < MAXC; ++k) {
+    const int c = (threadIdx.x + k * 256) * VEC;
+    if (c >= p.width) continue;
+    float w[VEC], v[VEC];
+    Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.w1) + c, w);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] = x[k][j] * inv * (w[j] + p.w_shift);
+    Io<T>::template stv<VEC>(reinterpret_cast<T*>(p.h1) + row * p.h1_stride + c, v);
+    if (p.w2) {
+      Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.w2) + c, w);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] = x[k][j] * inv * (w[j] + p.w_shift);
+      Io<T>::template stv<VEC>(reinterpret_cast<T*>(p.h2) + row * p.h2_stride + c, v);
+    }
+  }
+}
+
 struct PairEmbedParams {
   float* x;
   void* h;
@@ -764,6 +860,30 @@ extern "C" int mi_embed_norm(void* x, void* h, void* copy, const void* table, co
   hipStream_t s = (hipStream_t)stream;
   if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(embed_norm_kernel, uint16_t, width, vec, p);
   else MI_ROW_DISPATCH(embed_norm_kernel, float, width, vec, p);
+  return launch_status();
+}
+
+extern "C" int mi_stream_norm2(void* x, const void* y, int32_t split, const void* part, const int32_t* row_of_pair, const float* weights,
+                               int32_t top, float mult, const void* table, const int64_t* ids, int32_t vocab, const void* add_row,
+                               const void* w1, const void* w2, float w_shift, void* h1, void* h2, float eps, int32_t rows, int32_t width,
+                               int64_t x_stride, int64_t y_stride, int64_t part_stride, int64_t h1_stride, int64_t h2_stride, int dtype,
+                               void* stream) {
+  if (rows == 0) return MI_OK;
+  if (!x || !w1 || !h1 || rows < 0 || width <= 0 || split < 0 || x_stride < width || h1_stride < width) return MI_ERR_INVALID_ARG;
+  if (!y && !table) return MI_ERR_INVALID_ARG;
+  if ((y && y_stride < width) || (part && (!y || top <= 0 || part_stride < width)) || (table && (!ids || vocab <= 0)) ||
+      (w2 && (!h2 || h2_stride < width)))
+    return MI_ERR_INVALID_ARG;
+  if (dtype != MI_DTYPE_BF16 && dtype != MI_DTYPE_F32) return MI_ERR_UNSUPPORTED;
+  const StreamParams p{(float*)x, y, part, row_of_pair, weights, table, ids, add_row, w1, w2, h1, h2, x_stride, y_stride, part_stride,
+                       h1_stride, h2_stride, rows, width, split, part ? top : 0, vocab, mult, w_shift, eps};
+  const bool vec = width % 8 == 0 && x_stride % 8 == 0 && (!y || y_stride % 8 == 0) && (!part || part_stride % 8 == 0) &&
+                   h1_stride % 8 == 0 && (!w2 || h2_stride % 8 == 0) && aligned16(x) && aligned16(y) && aligned16(part) &&
+                   aligned16(table) && aligned16(add_row) && aligned16(w1) && aligned16(w2) && aligned16(h1) && aligned16(h2);
+  const dim3 grid(rows), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MI_DTYPE_BF16) MI_ROW_DISPATCH(stream_norm2_kernel, uint16_t, width, vec, p);
+  else MI_ROW_DISPATCH(stream_norm2_kernel, float, width, vec, p);
   return launch_status();
 }
 

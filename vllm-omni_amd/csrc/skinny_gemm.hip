@@ -998,7 +998,8 @@ extern "C" int mi_int8_linear_silu_mul(void* out, const int8_t* xq, const float*
 // ---------------------------------------------------------------------------------- grouped form (sparse-MoE experts)
 namespace mi {
 int launch_grouped_skinny(const GroupedGemmArgs& a, hipStream_t s) {
-  if (a.k % 64 || a.n_out % (a.gated ? 64 : 128) || a.rows_per_tile > 256 || a.rows_per_tile <= 0) return MI_ERR_UNSUPPORTED;
+  const bool gated = a.form == MI_MOE_GATED;
+  if (a.k % 64 || a.n_out % (gated ? 64 : 128) || a.rows_per_tile > 256 || a.rows_per_tile <= 0) return MI_ERR_UNSUPPORTED;
   if (a.dtype != MI_DTYPE_BF16 && a.dtype != MI_DTYPE_F16) return MI_ERR_UNSUPPORTED;
   if (a.a_row_stride % 8 || a.out_row_stride % 4 || a.weight_expert_stride % 8) return MI_ERR_UNSUPPORTED;
   SkinnyParams p;
@@ -1016,17 +1017,19 @@ int launch_grouped_skinny(const GroupedGemmArgs& a, hipStream_t s) {
   p.tile_expert = a.tile_expert;
   p.num_tiles = a.num_tiles;
   p.rpt = a.rows_per_tile;
-  p.gather_div = a.gated ? a.top_k : 0;
+  p.gather_div = a.form != MI_MOE_PLAIN ? a.top_k : 0;
+  p.relu_squared = a.form == MI_MOE_RELU_SQUARED;
+  p.pair_weights = a.pair_weights;
   p.w_expert_stride = a.weight_expert_stride;
   p.dbg = 0;
   p.ldx = a.a_row_stride;
   p.ldo = a.out_row_stride;
   // Weight tiles of one row tile chained into one workgroup (one ring through all of them: SkinnyParams::chain): as many as
   // still leave about two workgroups per CU.  MI_MOE_CHAIN_GATED / MI_MOE_CHAIN_DOWN = <tiles per workgroup> override (A/B).
-  const int n_tiles = a.gated ? a.n_out / 64 : a.n_out / 128;
+  const int n_tiles = gated ? a.n_out / 64 : a.n_out / 128;
   int chain = 1;
   {
-    const char* e = getenv(a.gated ? "MI_MOE_CHAIN_GATED" : "MI_MOE_CHAIN_DOWN");
+    const char* e = getenv(gated ? "MI_MOE_CHAIN_GATED" : "MI_MOE_CHAIN_DOWN");
     if (e && atoi(e) > 0) {
       chain = atoi(e);
     } else {
@@ -1042,7 +1045,7 @@ int launch_grouped_skinny(const GroupedGemmArgs& a, hipStream_t s) {
   const dim3 grid(n_tiles / chain, a.max_tiles);
   const int rpt = a.rows_per_tile;
   if (a.dtype == MI_DTYPE_BF16)
-    return a.gated ? launch_grouped_rows<bf16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<bf16_tag, false>(p, grid, rpt, s);
-  return a.gated ? launch_grouped_rows<f16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<f16_tag, false>(p, grid, rpt, s);
+    return gated ? launch_grouped_rows<bf16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<bf16_tag, false>(p, grid, rpt, s);
+  return gated ? launch_grouped_rows<f16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<f16_tag, false>(p, grid, rpt, s);
 }
 }  // namespace mi

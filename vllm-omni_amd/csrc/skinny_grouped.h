@@ -9,12 +9,13 @@ namespace mi {
 
 struct GroupedGemmArgs {
   void* out;                    // [max_rows, n_out]
-  const void* a_rows;           // gated: x [T, k] (row = sorted_pairs[r] / top_k); else the gated output [max_rows, k]
-  const void* weights;          // [E, (gated ? 2 : 1) * n_out, k]
+  const void* a_rows;           // MI_MOE_PLAIN: rows [max_rows, k]; else x [T, k] (row = sorted_pairs[r] / top_k)
+  const void* weights;          // [E, (MI_MOE_GATED ? 2 : 1) * n_out, k]
   const int32_t* sorted_pairs;  // [max_rows]: pair index or -1 (padding)
   const int32_t* tile_expert;   // [max_tiles]
   const int32_t* num_tiles;     // [1], device
-  int32_t max_tiles, gated, n_out, k, top_k, rows_per_tile;
+  const float* pair_weights;    // MI_MOE_RELU_SQUARED: what a pair's row is multiplied by, or nullptr
+  int32_t max_tiles, form, n_out, k, top_k, rows_per_tile;
   int64_t a_row_stride, out_row_stride, weight_expert_stride;
   int dtype;
 };

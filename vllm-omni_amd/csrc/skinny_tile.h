@@ -67,6 +67,7 @@ struct SkinnyParams {
   // go on to the next tile's stages while the consumers store the last one (a K of 384 is six steps: a workgroup per tile
   // spent more time filling and draining its ring than streaming)
   int32_t chain = 1;
+  const float* pair_weights = nullptr;   // GROUPED, not GATED: the sums of a pair's row times this, in front of the activation
   int64_t w_expert_stride;     // elements
   int32_t dbg;            // MI_LINEAR_DBG (timing experiments only): 1 = no DMA, 2 = no fragment reads / MFMAs, 4 = no reduce launch, 8 = no output stores
   int64_t ldx, ldo;
@@ -418,6 +419,12 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
       if constexpr (GROUPED) m += blockIdx.y * p.rpt;
       if (!slabs) {
         float v[4];
+        if constexpr (GROUPED) {
+          if (p.pair_weights) {
+            const int pr = p.row_map[m];
+            acc[g][j] *= pr < 0 ? 0.f : p.pair_weights[pr];
+          }
+        }
         finish_quad<Tag>(p, acc[g][j], m, n, bv, v);
         uint2 q;
         q.x = E::pack(v[0], v[1]);

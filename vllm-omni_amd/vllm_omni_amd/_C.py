@@ -19,7 +19,7 @@ MI_DTYPE_F16, MI_DTYPE_BF16, MI_DTYPE_F32 = 0, 1, 2
 MI_OK = 0
 MI_ERR_INVALID_ARG, MI_ERR_UNSUPPORTED, MI_ERR_WORKSPACE = -1, -2, -3
 MI_ERR_LAUNCH, MI_ERR_EXHAUSTED, MI_ERR_STATE = -4, -5, -6
-ABI_VERSION = 5
+ABI_VERSION = 6
 MI_LINEAR_PLAN_FULL, MI_LINEAR_PLAN_PARTIALS, MI_LINEAR_PLAN_GATED = 0, 1, 2
 MI_LINEAR_COUNTER_BYTES = 16 << 10
 MI_DECODE_PACKED_PV = 1
@@ -32,6 +32,7 @@ MI_DECODE_COUNTER_BYTES = 1 << 20
 MI_ALLREDUCE_MAX_RANKS, MI_ALLREDUCE_HANDLE_BYTES = 8, 64
 
 MI_ACT_SILU, MI_ACT_GELU_TANH = 0, 1
+MI_MOE_PLAIN, MI_MOE_GATED, MI_MOE_RELU_SQUARED = 0, 1, 2
 
 
 class GatedDeltaArgs(ctypes.Structure):
@@ -51,6 +52,25 @@ class LightningArgs(ctypes.Structure):
                                         "seq_lens", "out")] \
         + [(n, c_int64) for n in ("qkv_stride", "gate_stride", "out_stride")] \
         + [(n, c_int32) for n in ("req0", "num_reqs", "heads", "dim", "vdim")] + [("eps", c_float), ("mul", c_float)]
+
+
+class ConvRopeCacheArgs(ctypes.Structure):
+    """mi_conv_rope_cache_args"""
+
+    _fields_ = [(n, c_void_p) for n in ("x", "conv_w", "ring", "q_out", "k_cache", "v_cache", "inv_freq", "slots", "query_start_loc",
+                                        "seq_lens", "slot_mapping")] \
+        + [(n, c_int64) for n in ("x_stride", "q_stride", "cache_block_stride", "cache_token_stride", "cache_head_stride")] \
+        + [(n, c_int32) for n in ("req0", "num_reqs", "max_query_len", "heads", "kv_heads", "dim", "head_dim", "block_size", "rot_dims",
+                                  "taps", "update_ring")] + [("eps", c_float)]
+
+
+class StateSpaceArgs(ctypes.Structure):
+    """mi_state_space_args"""
+
+    _fields_ = [(n, c_void_p) for n in ("xbc", "z", "dt", "conv_w", "conv_b", "norm_w", "dt_bias", "a_log", "d", "state", "ring", "slots",
+                                        "query_start_loc", "seq_lens", "out")] \
+        + [(n, c_int64) for n in ("stride", "out_stride")] \
+        + [(n, c_int32) for n in ("req0", "num_reqs", "heads", "groups", "state_dim", "vdim", "taps", "norm_groups")] + [("eps", c_float)]
 
 
 class TalkingAttnArgs(ctypes.Structure):
@@ -119,9 +139,9 @@ SIGNATURES = {
                                        c_int32, c_int32, c_int32, c_int, _P]),
     "mi_moe_rows_per_tile": (c_int32, [c_int32, c_int32, c_int32]),
     "mi_moe_max_rows": (c_int64, [c_int32, c_int32, c_int32, c_int32]),
-    "mi_moe_route": (c_int, [_P, _P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, c_int32, c_int, c_int, _P]),
+    "mi_moe_route": (c_int, [_P, _P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, c_int32, c_int32, c_int, c_int, _P]),
     "mi_moe_align": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int64, c_int32, _P]),
-    "mi_moe_expert_gemm": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64,
+    "mi_moe_expert_gemm": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, _P, c_int32, c_int32, c_int32, c_int64, c_int64,
                                    c_int64, c_int32, c_int, _P]),
     "mi_moe_combine": (c_int, [_P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, c_int64,
                                c_int, _P]),
@@ -190,7 +210,7 @@ SIGNATURES = {
                                              c_int32, _P, c_int64, _P]),
     "mi_lightning_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32]),
     "mi_lightning_attn": (c_int, [POINTER(LightningArgs), c_int32, c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
-    "mi_moe_pair_gemm": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64,
+    "mi_moe_pair_gemm": (c_int, [_P, _P, _P, _P, c_int32, c_int32, c_int32, _P, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64,
                                  c_int, _P]),
     "mi_residual_add_norm_conv": (c_int, [_P, _P, c_int32, _P, _P, c_float, _P, _P, _P, _P, _P, c_int32, c_float, c_int32, c_int32, c_int64,
                                           c_int64, c_int64, c_int, _P]),
@@ -214,6 +234,12 @@ SIGNATURES = {
     "mi_latent_gather": (c_int, [_P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int64, c_int64, c_int64, _P]),
     "mi_latent_prefill": (c_int, [_P, _P, _P, _P, _P, _P, _P, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_float, c_int64,
                                   c_int64, c_int64, c_int64, _P]),
+    "mi_stream_norm2": (c_int, [_P, _P, c_int32, _P, _P, _P, c_int32, c_float, _P, _P, c_int32, _P, _P, _P, c_float, _P, _P, c_float, c_int32,
+                                c_int32, c_int64, c_int64, c_int64, c_int64, c_int64, c_int, _P]),
+    "mi_conv_rope_cache": (c_int, [POINTER(ConvRopeCacheArgs), c_int, _P]),
+    "mi_state_space_workspace_bytes": (c_int64, [c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int32, c_int]),
+    "mi_state_space": (c_int, [POINTER(StateSpaceArgs), c_int32, c_int32, c_int32, c_int32, _P, c_int64, c_int, _P]),
+    "mi_soft_cap_argmax": (c_int, [_P, _P, c_float, c_int32, c_int32, c_int64, c_int, _P]),
     "mi_blockpool_create": (_P, [c_int32]),
     "mi_blockpool_destroy": (None, [_P]),
     "mi_blockpool_num_free": (c_int32, [_P]),

@@ -503,13 +503,13 @@ class _Weights:
         self.weight, self.bias, self.qweight = weight, bias, None
 
 
-def tuned_linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+def tuned_linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None, defer_reduce: bool = False):
     """``F.linear`` for the step's un-sharded extras (``thinker_to_talker_proj``, the vocab-parallel ``lm_head``), routed
     like the decoder's projections: the streaming kernel where the tuned table (or the round-3 rule) has it ahead of
-    the library GEMM at this shape."""
+    the library GEMM at this shape.  ``defer_reduce``: as in ``_apply_linear``."""
     if x.dim() > 2 or not x.is_cuda:
         return F.linear(x, weight, bias)
-    return _apply_linear(_Weights(weight, bias), x, bias)
+    return _apply_linear(_Weights(weight, bias), x, bias, defer_reduce)
 
 
 def quantize_int8_(layer) -> None:

@@ -1,10 +1,11 @@
 """Sequence mixers and small blocks of decoders with a 32-bit residual stream: latent attention without positions
 (its cache row shared by all heads, optionally by several layers), the gated delta rule with a decay per head or per key
 channel, attention with a distance bias and a sink, decayed linear attention, several mixers side by side, attention whose
-heads mix their softmax weights, and a short filter in front of a sublayer.  Constants that a design fixes are parameters here; the layers know nothing of the model they are in.
+heads mix their softmax weights, a short filter in front of a sublayer, a state-space recurrence, and attention whose values are its
+keys.  Constants that a design fixes are parameters here; the layers know nothing of the model they are in.
 
-Two kinds: mixers that own their projections (``LatentAttention``, ``GatedDelta``, ``TalkingAttention``: rows in, rows out), and mixers for layers
-whose sublayers all read one normed row and add up (``ChannelDelta``, ``SinkAttention``, ``LightningAttention``,
+Two kinds: mixers that own their projections (``LatentAttention``, ``GatedDelta``, ``TalkingAttention``, ``StateSpace``,
+``KeyValueAttention``: rows in, rows out), and mixers for layers whose sublayers all read one normed row and add up (``ChannelDelta``, ``SinkAttention``, ``LightningAttention``,
 ``ParallelMixers``, ``DenseGlu``): such a layer has ONE input product and ONE output product (``SharedProjections``), and a
 sublayer names its blocks of both, turning columns of the first into columns the second reads.
 """
@@ -312,6 +313,150 @@ class TalkingAttention:
             ops.talking_prefill(*args, md.block_table[nd:n], md.seq_lens[nd:n], md.query_start_loc[nd:n + 1], self.heads, start, rows,
                                 md.max_query_len, gate)
         return self.o(out, defer_reduce)
+
+
+@dataclass
+class StateSpaceConfig:
+    heads: int
+    groups: int                       # of heads that share B and C
+    state: int
+    vdim: int
+    conv: int                         # taps of the short filters
+    norm_groups: int                  # equal parts of the gated row that are normed apart
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+class StateSpace:
+    """State-space recurrence with a scalar decay per head and token, short filters in front of it and a gated norm behind it
+    (``csrc/state_space.hip``)."""
+
+    def __init__(self, cfg: StateSpaceConfig, width: int, eps: float, dtype, device, generator=None):
+        if cfg.heads % cfg.groups or cfg.inner % cfg.norm_groups:
+            raise ValueError("heads must be a multiple of groups, and their columns of norm_groups")
+        if cfg.conv < 1:
+            raise ValueError("a filter has at least the tap of the row itself")
+        self.cfg, self.eps, self.dtype = cfg, eps, dtype
+        # z | x | B | C | step sizes
+        self.proj = ReplicatedLinear(width, {"in": cfg.inner + cfg.channels + cfg.heads}, dtype, device, generator, pad=True)
+        self.o = ReplicatedLinear(cfg.inner, {"o": width}, dtype, device, generator)
+        self.conv_w = _init_weight(cfg.channels, cfg.conv, dtype, device, generator, std=0.5)
+        self.conv_b = _vec(cfg.channels, dtype, device, 0.0)
+        self.dt_bias, self.a_log = _vec(cfg.heads, torch.float32, device, 0.0), _vec(cfg.heads, torch.float32, device, 0.0)
+        self.d = _vec(cfg.heads, torch.float32, device)
+        self.norm = _vec(cfg.inner, dtype, device)
+
+    def kv_cache_spec(self, block_size: int) -> Optional[KVCacheSpec]:
+        return None
+
+    def state_specs(self) -> list[StateSpec]:
+        c = self.cfg
+        return [StateSpec((c.heads, c.state, c.vdim), torch.float32), StateSpec((c.conv, c.channels), self.dtype)]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield from self.proj.named(p)
+        yield from self.o.named(p)
+        yield p + "conv", self.conv_w
+        yield p + "conv.b", self.conv_b
+        yield p + "dt_bias", self.dt_bias
+        yield p + "A_log", self.a_log
+        yield p + "D", self.d
+        yield p + "norm", self.norm
+
+    def __call__(self, h: torch.Tensor, md: AttentionMetadata, memory: "LayerMemory", defer_reduce: bool = False):
+        c = self.cfg
+        x = self.proj(h)
+        out = torch.empty(h.shape[0], c.inner, dtype=self.dtype, device=h.device)
+        at = c.inner + c.channels
+        args = (x[:, c.inner:at], x[:, :c.inner], x[:, at:at + c.heads], self.conv_w, self.conv_b, self.dt_bias, self.a_log, self.d,
+                self.norm, *memory.states, md.state_rows, md.query_start_loc, md.seq_lens, c.groups, c.norm_groups, self.eps, out)
+        nd = md.num_decodes
+        if nd:
+            ops.state_space(*args, 0, nd, 0, nd, 1, chunked=False)
+        if nd < md.num_reqs:
+            ops.state_space(*args, nd, md.num_reqs - nd, nd, h.shape[0] - nd, md.max_query_len)
+        return self.o(out, defer_reduce)
+
+
+@dataclass
+class KeyValueAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int
+    conv: int                         # taps of the short filters
+    scale: float
+    rot_dims: int = 0                 # leading dimensions of a head that turn with the position, in neighbouring pairs
+    rot_base: float = 10000.0
+    sink: Optional[float] = None      # score of one more term of the softmax's denominator; None: no such term
+
+
+class KeyValueAttention:
+    """Grouped-query attention whose values are its keys as the short filter leaves them; queries and keys turn with the position
+    and are then normed per head, without weights (``csrc/conv_rope.hip`` and the paged-attention kernels)."""
+
+    def __init__(self, cfg: KeyValueAttentionConfig, width: int, eps: float, dtype, device, generator=None):
+        if cfg.heads % cfg.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if cfg.scale <= 0:
+            raise ValueError("the score scale must be positive")
+        if cfg.conv < 1:
+            raise ValueError("a filter has at least the tap of the row itself")
+        if cfg.rot_dims % 2 or not 0 <= cfg.rot_dims <= cfg.dim:
+            raise ValueError("rotary dimensions come in pairs, no more than a head has")
+        self.cfg, self.eps, self.dtype = cfg, eps, dtype
+        # heads are laid out to the sizes the matrix-core kernels are built for
+        self.head_dim = -(-cfg.dim // 8) * 8 if dtype != torch.bfloat16 or cfg.dim > 128 else 64 if cfg.dim <= 64 else 128
+        nq, nk = cfg.heads * cfg.dim, cfg.kv_heads * cfg.dim
+        self.nq, self.channels = nq, nq + nk
+        self.proj = ReplicatedLinear(width, {"q": nq, "k": nk}, dtype, device, generator, pad=True)
+        self.conv_w = _init_weight(self.channels, cfg.conv, dtype, device, generator, std=0.5)
+        self.o = _init_weight(width, cfg.heads * self.head_dim, dtype, device, generator, std=nq ** -0.5)
+        self.o.view(width, cfg.heads, self.head_dim)[:, :, cfg.dim:].zero_()
+        freq = [cfg.rot_base ** (-2.0 * i / cfg.rot_dims) for i in range(cfg.rot_dims // 2)]
+        self.inv_freq = torch.tensor(freq, dtype=torch.float32, device=device) if freq else None
+        self.sinks = None if cfg.sink is None else _vec(cfg.heads, torch.float32, device, cfg.sink)
+
+    def kv_cache_spec(self, block_size: int) -> Optional[KVCacheSpec]:
+        return KVCacheSpec(block_size, self.cfg.kv_heads, self.head_dim, self.dtype, self.cfg.heads)
+
+    def state_specs(self) -> list[StateSpec]:
+        return [StateSpec((self.cfg.conv, self.channels), self.dtype)]
+
+    def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
+        yield from self.proj.named(p)
+        yield p + "q.conv", self.conv_w[:self.nq]
+        yield p + "k.conv", self.conv_w[self.nq:]
+        w = self.o.view(self.o.shape[0], self.cfg.heads, self.head_dim)[:, :, :self.cfg.dim]
+        yield p + "o", self.o if self.head_dim == self.cfg.dim else w
+
+    def __call__(self, h: torch.Tensor, md: AttentionMetadata, memory: "LayerMemory", defer_reduce: bool = False):
+        c, (kc, vc) = self.cfg, memory.kv
+        x = self.proj(h)[:, :self.channels]
+        q = torch.empty(h.shape[0], c.heads * self.head_dim, dtype=self.dtype, device=h.device)
+        args = (x, self.conv_w, memory.states[0], q, kc, vc, self.inv_freq, md.state_rows, md.query_start_loc, md.seq_lens, md.slot_mapping,
+                c.heads, c.dim, self.eps)
+        nd, n = md.num_decodes, md.num_reqs
+        if nd:
+            ops.conv_rope_cache(*args, 0, nd, 1)
+        if nd < n:
+            ops.conv_rope_cache(*args, nd, n - nd, md.max_query_len)
+        out = torch.empty_like(q)
+        if not ops.paged_attn_bias_supported(self.dtype, self.head_dim, kc.shape[1]):
+            ops.attn_rows(out, q, kc, vc, md.block_table, md.seq_lens, md.query_start_loc, c.scale, sinks=self.sinks)
+        else:
+            if nd:
+                ops.paged_attn_decode(out[:nd], q[:nd], kc, vc, md.block_table[:nd], md.seq_lens[:nd], md.max_seq_len, c.scale,
+                                      workspace=md.decode_workspace, sinks=self.sinks)
+            if nd < n:      # the portions' row offsets count from the step's first row, so q and out go whole
+                ops.paged_attn_prefill(out, q, kc, vc, md.block_table[nd:n], md.seq_lens[nd:n], md.query_start_loc[nd:n + 1],
+                                       md.max_query_len, c.scale, max_seq_len=md.max_seq_len, sinks=self.sinks)
+        return tuned_linear(out, self.o, defer_reduce=defer_reduce)
 
 
 class InputConv:

@@ -103,32 +103,42 @@ class Qwen3OmniMoeSparseMoeBlock:
 
 
 class RoutedExperts:
-    """Routed gated experts whose output rows the caller sums (``ops.residual_add_norm``): the ``top`` largest of the router's
-    32-bit logits (+ bias), weighted by the softmax over these alone.  Weight names: ``router``, ``router.b``, ``e<i>.gate`` /
-    ``.up`` / ``.down``."""
+    """Routed experts whose output rows the caller sums (``ops.residual_add_norm``, ``ops.stream_norm2``).  Scores of the router's
+    32-bit logits (+ bias), of which each token's ``top`` largest choose: "softmax" over the chosen ones alone, or "sigmoid" of each,
+    not normalised.  ``act`` "silu_gated" (weights ``e<i>.gate`` / ``.up`` / ``.down``) or "relu_squared" (no gate).
+    ``weigh_input`` (relu_squared): the score scales what an expert reads instead of what it gives.  Other weight names:
+    ``router``, with ``bias`` also ``router.b``."""
 
-    def __init__(self, width: int, experts: int, top: int, ff: int, dtype, device=None, generator=None):
+    def __init__(self, width: int, experts: int, top: int, ff: int, dtype, device=None, generator=None, act: str = "silu_gated",
+                 scores: str = "softmax", bias: bool = True, weigh_input: bool = False):
         if not 0 < top <= min(experts, 16) or experts > 256:
             raise ValueError(f"{top} of {experts} experts: at most 16 of at most 256")
-        self.top, self.ff = top, ff
-        step = 64 if width % 128 == 0 else 8           # columns of zeros bring a small expert to a tile of the grouped products
+        if act not in ("silu_gated", "relu_squared") or scores not in ("softmax", "sigmoid") or (weigh_input and act == "silu_gated"):
+            raise ValueError(f"experts with act {act!r}, scores {scores!r}, weigh_input {weigh_input} are not built")
+        self.top, self.ff, self.act, self.scores, self.weigh_input = top, ff, act, scores, weigh_input
+        self.ups = 2 if act == "silu_gated" else 1     # row blocks of an expert's first product
+        # columns of zeros bring a small expert to a tile of the grouped products
+        step = (64 if self.ups == 2 else 128) if width % 128 == 0 else 8
         pad = -(-ff // step) * step
         self.router = _init_weight(experts, width, dtype, device, generator, std=width ** -0.5)
-        self.router_b = torch.zeros(experts, dtype=torch.float32, device=device)
-        self.gate_up = _init_weight(experts * 2 * pad, width, dtype, device, generator, std=width ** -0.5).view(experts, 2, pad, width)
+        self.router_b = torch.zeros(experts, dtype=torch.float32, device=device) if bias else None
+        self.up = _init_weight(experts * self.ups * pad, width, dtype, device, generator, std=width ** -0.5).view(experts, self.ups, pad, width)
         self.down = _init_weight(experts * width, pad, dtype, device, generator, std=ff ** -0.5).view(experts, width, pad)
-        self.gate_up[:, :, ff:].zero_()
+        self.up[:, :, ff:].zero_()
         self.down[:, :, ff:].zero_()
 
     def named_weights(self, p: str) -> Iterable[tuple[str, torch.Tensor]]:
         yield p + "router", self.router
-        yield p + "router.b", self.router_b
+        if self.router_b is not None:
+            yield p + "router.b", self.router_b
         for i in range(self.router.shape[0]):
-            yield f"{p}e{i}.gate", self.gate_up[i, 0, :self.ff]
-            yield f"{p}e{i}.up", self.gate_up[i, 1, :self.ff]
+            if self.ups == 2:
+                yield f"{p}e{i}.gate", self.up[i, 0, :self.ff]
+            yield f"{p}e{i}.up", self.up[i, self.ups - 1, :self.ff]
             yield f"{p}e{i}.down", self.down[i, :, :self.ff]
 
     def __call__(self, h: torch.Tensor) -> ops.ExpertRows:
         logits = ops.moe_router_logits(h, self.router)
-        ids, weights, _ = ops.moe_route(logits, self.top, True, want_counts=False, bias=self.router_b)
-        return ops.moe_expert_rows(h, ids, weights, self.gate_up.flatten(1, 2), self.down)
+        sig = self.scores == "sigmoid"
+        ids, weights, _ = ops.moe_route(logits, self.top, not sig, want_counts=False, bias=self.router_b, sigmoid=sig)
+        return ops.moe_expert_rows(h, ids, weights, self.up.flatten(1, 2), self.down, self.act, self.weigh_input)

@@ -1036,10 +1036,11 @@ def int8_linear_silu_mul(x: torch.Tensor, wq: torch.Tensor, w_scale: torch.Tenso
 
 # --------------------------------------------------------------------------- N4: fused sparse MoE
 def moe_route(router_logits: torch.Tensor, top_k: int, norm_topk_prob: bool, round_to: Optional[torch.dtype] = None,
-              want_counts: bool = True, bias: Optional[torch.Tensor] = None):
+              want_counts: bool = True, bias: Optional[torch.Tensor] = None, sigmoid: bool = False):
     """-> (topk_ids int32 [T, k], topk_weights fp32 [T, k], expert_counts int32 [E] or None).  ``want_counts=False``:
     no per-expert counting and no launch to zero the counters (``fused_moe``: the grouping counts the ids itself).
-    ``bias`` (fp32 [E]) is added to the logits.  ``norm_topk_prob``: a softmax over the chosen logits only."""
+    ``bias`` (fp32 [E]) is added to the logits.  ``norm_topk_prob``: a softmax over the chosen logits only (``sigmoid``: each
+    logit's sigmoid instead of the softmax, divided by the chosen ones' sum)."""
     _gpu(router_logits, bias)
     t, e = router_logits.shape
     _head_vectors(e, bias)
@@ -1047,7 +1048,7 @@ def moe_route(router_logits: torch.Tensor, top_k: int, norm_topk_prob: bool, rou
     w = torch.empty(t, top_k, dtype=torch.float32, device=router_logits.device)
     counts = torch.empty(e, dtype=torch.int32, device=router_logits.device) if want_counts else None
     check("mi_moe_route", lib.mi_moe_route(_p(ids), _p(w), _p(counts), _p(router_logits), _p(bias), t, e, router_logits.stride(0),
-                                           int(top_k), 1 if norm_topk_prob else 0, _dt(router_logits.dtype),
+                                           int(top_k), 1 if norm_topk_prob else 0, int(sigmoid), _dt(router_logits.dtype),
                                            -1 if round_to is None else _dt(round_to), _stream()))
     return ids, w, counts
 
@@ -1084,10 +1085,10 @@ def fused_moe(x: torch.Tensor, router_logits: torch.Tensor, w_gate_up: torch.Ten
     part = torch.empty(max_rows, h, dtype=x.dtype, device=dev)
     dt = _dt(x.dtype)
     check("mi_moe_expert_gemm", lib.mi_moe_expert_gemm(
-        _p(act), _p(x), _p(w_gate_up), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, 1, i, h, top_k,
+        _p(act), _p(x), _p(w_gate_up), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, _C.MI_MOE_GATED, None, i, h, top_k,
         x.stride(0), act.stride(0), w_gate_up.stride(0), rpt, dt, _stream()))
     check("mi_moe_expert_gemm", lib.mi_moe_expert_gemm(
-        _p(part), _p(act), _p(w_down), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, 0, h, i, top_k,
+        _p(part), _p(act), _p(w_down), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, _C.MI_MOE_PLAIN, None, h, i, top_k,
         act.stride(0), part.stride(0), w_down.stride(0), rpt, dt, _stream()))
     out = torch.empty_like(x)
     if callable(shared_out):      # the caller computed it beside this path (another stream): join here
@@ -1409,10 +1410,27 @@ def _delta_args(proj, conv_w, a_log, dt_bias, norm_w, state, ring, slots, query_
 
 # ------------------------------------------------- layers with mixer and feed-forward side by side
 class ExpertRows:
-    """Output rows of routed experts, one per (token, choice), and how they sum up: ``residual_add_norm`` does it."""
+    """Output rows of routed experts, one per (token, choice), and how they sum up: ``residual_add_norm`` does it.  ``weights``
+    None: every row counts once (``top`` choices a token)."""
 
-    def __init__(self, part: torch.Tensor, weights: torch.Tensor, row_of_pair: Optional[torch.Tensor]):
+    def __init__(self, part: torch.Tensor, weights: Optional[torch.Tensor], row_of_pair: Optional[torch.Tensor], top: Optional[int] = None):
         self.part, self.weights, self.row_of_pair = part, weights, row_of_pair
+        self.top = weights.shape[1] if weights is not None else top
+
+    def check(self, rows: int, width: int, dtype) -> int:
+        """row stride of ``part``, after a look at the sizes"""
+        _gpu(self.part, self.row_of_pair, self.weights)
+        ps, pw = _rows(self.part)
+        ww = self.weights
+        if pw != width or self.part.dtype != dtype or (ww is not None and (ww.shape[0] != rows or ww.dtype != torch.float32
+                                                                           or not ww.is_contiguous())):
+            raise ValueError("expert rows of another shape or dtype")
+        if self.row_of_pair is None and self.part.shape[0] < rows * self.top:
+            raise ValueError("one row per pair expected")
+        if self.row_of_pair is not None and self.row_of_pair.numel() < rows * self.top:
+            raise ValueError("a row per pair expected")
+        _i32(self.row_of_pair)
+        return ps
 
 
 def residual_add_norm(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials"], w_pre: Optional[torch.Tensor], eps: float,
@@ -1442,15 +1460,10 @@ def residual_add_norm(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials"],
         split = 1 if y.dtype == torch.float32 and h.dtype != torch.float32 else 0
     top, rp, ww, ps, prt = 0, None, None, 0, None
     if experts is not None:
-        prt, rp, ww = experts.part, experts.row_of_pair, experts.weights
-        _gpu(prt, rp, ww)
-        ps, pw = _rows(prt)
-        top = ww.shape[1]
-        if pw != width or prt.dtype != h.dtype or ww.shape[0] != rows or ww.dtype != torch.float32 or not ww.is_contiguous():
-            raise ValueError("expert rows of another shape or dtype")
-        if rp is None and prt.shape[0] < rows * top:
-            raise ValueError("one row per pair expected")
-        _i32(rp)
+        prt, rp, ww, top = experts.part, experts.row_of_pair, experts.weights, experts.top
+        if ww is None:
+            raise ValueError("residual_add_norm takes weighted experts' rows")
+        ps = experts.check(rows, width, h.dtype)
     check("mi_residual_add_norm", lib.mi_residual_add_norm(
         _p(x), _p(src), split, _p(prt), _p(rp), _p(ww), top, _p(w_pre), float(w_shift), _p(h), int(start), float(eps), rows, width, xs,
         ys, hs, ps, _dt(h.dtype), _stream()))
@@ -1583,39 +1596,47 @@ def moe_router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     return torch.mm(h, weight.t(), out_dtype=torch.float32)
 
 
-def moe_expert_rows(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor,
-                    w_down: torch.Tensor) -> ExpertRows:
-    """Gated (silu) experts on the rows routed to them, not yet summed: grouped matrix-core products where the sizes allow,
-    the any-size kernel (fp32, odd sizes) elsewhere."""
-    _gpu(x, ids, weights, w_gate_up, w_down)
+def moe_expert_rows(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
+                    act: str = "silu_gated", weigh_input: bool = False) -> ExpertRows:
+    """Experts on the rows routed to them, not yet summed: grouped matrix-core products where the sizes allow, the any-size
+    kernel (fp32, odd sizes) elsewhere.  ``act`` "silu_gated": ``w_up`` holds gate, then up rows; "relu_squared": up rows only.
+    ``weigh_input`` (relu_squared): the weights scale what an expert reads, the rows then sum up as they are."""
+    _gpu(x, ids, weights, w_up, w_down)
     _i32(ids)
     t, h = x.shape
     top = ids.shape[1]
-    e, two_i, k = w_gate_up.shape
-    i = two_i // 2
+    gated = act == "silu_gated"
+    if act not in ("silu_gated", "relu_squared") or (gated and weigh_input):
+        raise ValueError(f"moe_expert_rows: act {act!r}, weigh_input {weigh_input} is not built")
+    form = _C.MI_MOE_GATED if gated else _C.MI_MOE_RELU_SQUARED
+    pw = weights if weigh_input else None
+    if tuple(weights.shape) != (t, top) or weights.dtype != torch.float32 or not weights.is_contiguous():
+        raise ValueError("moe_expert_rows: one fp32 weight per choice")
+    e, ups, k = w_up.shape
+    i = ups // 2 if gated else ups
     xs = _rows(x)[0]
-    if k != h or tuple(w_down.shape) != (e, h, i) or not w_gate_up.is_contiguous() or not w_down.is_contiguous() or w_gate_up.dtype != x.dtype:
+    if k != h or tuple(w_down.shape) != (e, h, i) or not w_up.is_contiguous() or not w_down.is_contiguous() or w_up.dtype != x.dtype:
         raise ValueError("moe_expert_rows: expert weights do not fit")
     dt, dev = _dt(x.dtype), x.device
     if x.dtype == torch.bfloat16 and h % 8 == 0 and i % 8 == 0 and xs % 8 == 0:
-        guard = h % 128 or i % 64
+        guard = h % 128 or i % (64 if gated else 128)
         rpt = int(lib.mi_moe_rows_per_tile(t, top, e))
         rpt = min(rpt, 64) if guard else rpt
         max_rows = int(lib.mi_moe_max_rows(t, top, e, rpt))
         sorted_pairs, row_of_pair, tile_expert, num_tiles = _moe_align(ids, e, max_rows, rpt)
-        act = torch.empty(max_rows, i, dtype=x.dtype, device=dev)
+        mid = torch.empty(max_rows, i, dtype=x.dtype, device=dev)
         part = torch.empty(max_rows, h, dtype=x.dtype, device=dev)
-        for out, a, w, gated, n, kk in ((act, x, w_gate_up, 1, i, h), (part, act, w_down, 0, h, i)):
+        for out, a, w, f, s, n, kk in ((mid, x, w_up, form, pw, i, h), (part, mid, w_down, _C.MI_MOE_PLAIN, None, h, i)):
             check("mi_moe_expert_gemm", lib.mi_moe_expert_gemm(
-                _p(out), _p(a), _p(w), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, gated, n, kk, top, a.stride(0),
+                _p(out), _p(a), _p(w), _p(sorted_pairs), _p(tile_expert), _p(num_tiles), max_rows // rpt, f, _p(s), n, kk, top, a.stride(0),
                 out.stride(0), w.stride(0), rpt, dt, _stream()))
-        return ExpertRows(part, weights, row_of_pair)
-    act = torch.empty(t * top, i, dtype=x.dtype, device=dev)
+        return ExpertRows(part, None if weigh_input else weights, row_of_pair, top)
+    mid = torch.empty(t * top, i, dtype=x.dtype, device=dev)
     part = torch.empty(t * top, h, dtype=x.dtype, device=dev)
-    for out, a, w, gated, n, kk in ((act, x, w_gate_up, 1, i, h), (part, act, w_down, 0, h, i)):
-        check("mi_moe_pair_gemm", lib.mi_moe_pair_gemm(_p(out), _p(a), _p(w), _p(ids), t * top, e, gated, n, kk, top, a.stride(0),
+    for out, a, w, f, s, n, kk in ((mid, x, w_up, form, pw, i, h), (part, mid, w_down, _C.MI_MOE_PLAIN, None, h, i)):
+        check("mi_moe_pair_gemm", lib.mi_moe_pair_gemm(_p(out), _p(a), _p(w), _p(ids), t * top, e, f, _p(s), n, kk, top, a.stride(0),
                                                        out.stride(0), w.stride(0), dt, _stream()))
-    return ExpertRows(part, weights, None)
+    return ExpertRows(part, None if weigh_input else weights, None, top)
 
 
 # ------------------------------------------------- a filter in front of every sublayer, heads that mix their softmax weights
@@ -1865,3 +1886,150 @@ def talking_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
     check("mi_talking_prefill", lib.mi_talking_prefill(ctypes.byref(a), _p(ctx_start), ctx_rows, n, rows, max_query_len, _p(ws), need,
                                                        _stream()))
     return out
+
+
+# ------------------------------------------------- state-space layers, attention whose values are its keys
+def stream_norm2(x: torch.Tensor, y: Union[torch.Tensor, "SplitKPartials", None], w1: torch.Tensor, w2: Optional[torch.Tensor], eps: float,
+                 h1: torch.Tensor, h2: Optional[torch.Tensor] = None, w_shift: float = 0.0, mult: float = 1.0,
+                 experts: Optional[ExpertRows] = None, table: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
+                 add_row: Optional[torch.Tensor] = None) -> None:
+    """``x += mult * (y + the experts' rows)`` in place (x fp32 [T, W]; ``y`` None: x starts from zero), then ``x += table[ids] +
+    add_row`` where given, then ``h1`` / ``h2`` = x / rms(x) * (w1 / w2 + w_shift).  ``y`` as in ``residual_add_norm``."""
+    part = isinstance(y, SplitKPartials)
+    if part:
+        y._live()
+        if y.bias is not None:
+            raise ValueError("stream_norm2 takes partials of a linear without bias")
+    src = y.part if part else y
+    _gpu(x, src, w1, w2, h1, h2, table, ids, add_row)
+    xs, width = _rows(x)
+    rows = x.shape[0]
+    if x.dtype != torch.float32 or (w2 is None) != (h2 is None) or (y is None and (table is None or experts is not None)):
+        raise ValueError("stream_norm2: an fp32 stream that starts from the table or takes a layer's output; one output per norm")
+    strides = []
+    for h, w in ((h1, w1), (h2, w2)):
+        if h is None:
+            strides.append(0)
+            continue
+        hs, hw = _rows(h)
+        if hw != width or h.shape[0] < rows or w.numel() != width or not w.dtype == h.dtype == h1.dtype:
+            raise ValueError("stream_norm2: norm rows and weights of the stream's width")
+        strides.append(hs)
+    split, ys = 0, 0
+    if part:
+        if (y.m, y.n) != (rows, width):
+            raise ValueError("partials of another shape")
+        split, ys = y.split, width
+    elif y is not None:
+        ys, yw = _rows(y)
+        if y.shape[0] != rows or yw != width or y.dtype not in (h1.dtype, torch.float32):
+            raise ValueError("layer output of another shape or dtype")
+        split = 1 if y.dtype == torch.float32 and h1.dtype != torch.float32 else 0
+    prt, rp, ww, top, ps = None, None, None, 0, 0
+    if experts is not None:
+        prt, rp, ww, top = experts.part, experts.row_of_pair, experts.weights, experts.top
+        ps = experts.check(rows, width, h1.dtype)
+    if table is not None:
+        _i64(ids)
+        if not table.is_contiguous() or table.shape[1] != width or table.dtype != h1.dtype or ids is None or ids.numel() < rows:
+            raise ValueError("stream_norm2: an embedding table of the stream's width, an id per row")
+    if add_row is not None and (add_row.numel() != width or add_row.dtype != h1.dtype or not add_row.is_contiguous()):
+        raise ValueError("stream_norm2: a row of the stream's width")
+    check("mi_stream_norm2", lib.mi_stream_norm2(
+        _p(x), _p(src), split, _p(prt), _p(rp), _p(ww), top, float(mult), _p(table), _p(ids) if table is not None else None,
+        table.shape[0] if table is not None else 0, _p(add_row), _p(w1), _p(w2), float(w_shift), _p(h1), _p(h2), float(eps), rows, width, xs,
+        ys, ps, strides[0], strides[1], _dt(h1.dtype), _stream()))
+
+
+def _step_requests(slots, query_start_loc, seq_lens, req0: int, num_reqs: int, what: str) -> None:
+    _i32(slots, query_start_loc, seq_lens)
+    if req0 < 0 or min(seq_lens.shape[0], slots.shape[0], query_start_loc.shape[0] - 1) < req0 + num_reqs:
+        raise ValueError(f"{what}: request range outside the metadata")
+
+
+def conv_rope_cache(x: torch.Tensor, conv_w: torch.Tensor, ring: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor,
+                    v_cache: torch.Tensor, inv_freq: Optional[torch.Tensor], slots: torch.Tensor, query_start_loc: torch.Tensor,
+                    seq_lens: torch.Tensor, slot_mapping: torch.Tensor, num_q_heads: int, dim: int, eps: float, req0: int, num_reqs: int,
+                    max_query_len: int, update_ring: bool = True) -> torch.Tensor:
+    """Rows q | k of requests [req0, req0 + num_reqs): causal filter per channel, value row = the filtered k, rotary on neighbouring
+    pairs, unweighted norm per head, K / V cache write; q to ``q_out``, heads laid out as in the cache.  ``ring`` [slots, taps,
+    channels]; ``inv_freq`` fp32 [rotary dimensions / 2] (None: no rotation)."""
+    _gpu(x, conv_w, ring, q_out, k_cache, v_cache, inv_freq, slots, query_start_loc, seq_lens, slot_mapping)
+    _step_requests(slots, query_start_loc, seq_lens, req0, num_reqs, "conv_rope_cache")
+    _i64(slot_mapping)
+    xs, cols = _rows(x)
+    qs, qc = _rows(q_out)
+    _, bs, g, hd = k_cache.shape
+    cb, ct, chs = _cache_strides(k_cache, v_cache)
+    ch, taps = (num_q_heads + g) * dim, conv_w.shape[1]
+    if cols != ch or tuple(conv_w.shape) != (ch, taps) or tuple(ring.shape[1:]) != (taps, ch) or qc != num_q_heads * hd or hd < dim:
+        raise ValueError("conv_rope_cache: sizes do not fit")
+    if q_out.shape[0] < x.shape[0] or slot_mapping.numel() < x.shape[0]:
+        raise ValueError("conv_rope_cache: one output row and one slot per row")
+    if not conv_w.is_contiguous() or not ring.is_contiguous() or any(t.dtype != x.dtype for t in (conv_w, ring, q_out, k_cache)):
+        raise TypeError("conv_rope_cache: one dtype, contiguous filter and ring")
+    pairs = 0
+    if inv_freq is not None:
+        pairs = inv_freq.numel()
+        _head_vectors(pairs, inv_freq)
+    a = _C.ConvRopeCacheArgs(_p(x), _p(conv_w), _p(ring), _p(q_out), _p(k_cache), _p(v_cache), _p(inv_freq), _p(slots), _p(query_start_loc),
+                             _p(seq_lens), _p(slot_mapping), xs, qs, cb, ct, chs, req0, num_reqs, max_query_len, num_q_heads, g, dim, hd, bs,
+                             2 * pairs, taps, int(update_ring), float(eps))
+    check("mi_conv_rope_cache", lib.mi_conv_rope_cache(ctypes.byref(a), _dt(x.dtype), _stream()))
+    return q_out
+
+
+def state_space(xbc: torch.Tensor, z: torch.Tensor, dt: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, dt_bias: torch.Tensor,
+                a_log: torch.Tensor, d: torch.Tensor, norm_w: torch.Tensor, state: torch.Tensor, ring: torch.Tensor, slots: torch.Tensor,
+                query_start_loc: torch.Tensor, seq_lens: torch.Tensor, groups: int, norm_groups: int, eps: float, out: torch.Tensor,
+                req0: int, num_reqs: int, row0: int, rows: int, max_query_len: int, chunked: bool = True) -> torch.Tensor:
+    """State-space recurrence of requests [req0, req0 + num_reqs), which own rows [row0, row0 + rows).  ``xbc``, ``z`` and ``dt``
+    are column blocks of one matrix; ``state`` fp32 [slots, H, N, V]; ``ring`` [slots, taps, channels].  ``chunked``: 64 tokens at a
+    time (fp32 and sizes outside that form go token by token)."""
+    _gpu(xbc, z, dt, conv_w, conv_b, dt_bias, a_log, d, norm_w, state, ring, slots, query_start_loc, seq_lens, out)
+    _step_requests(slots, query_start_loc, seq_lens, req0, num_reqs, "state_space")
+    ps, ch = _rows(xbc)
+    os_, oc = _rows(out)
+    _, hh, n, v = state.shape
+    taps = ring.shape[1]
+    if _rows(z) != (ps, hh * v) or _rows(dt) != (ps, hh):
+        raise ValueError("state_space: x | B | C, z and dt are column blocks of one matrix")
+    if ch != hh * v + 2 * groups * n or hh % groups or (hh * v) % norm_groups or oc != hh * v or norm_w.numel() != hh * v:
+        raise ValueError("state_space: sizes do not fit")
+    if tuple(conv_w.shape) != (ch, taps) or conv_b.numel() != ch or ring.shape[2] != ch or any(t.numel() != hh for t in (dt_bias, a_log, d)):
+        raise ValueError("state_space: sizes do not fit")
+    if any(t.dtype != torch.float32 for t in (state, dt_bias, a_log, d)):
+        raise TypeError("state_space: state, step bias, A_log and D are fp32")
+    if any(t.dtype != xbc.dtype for t in (z, dt, conv_w, conv_b, norm_w, ring, out)):
+        raise TypeError("state_space: one activation dtype")
+    if not all(t.is_contiguous() for t in (state, ring, conv_w, conv_b, norm_w, dt_bias, a_log, d)):
+        raise ValueError("state_space: contiguous state and weights")
+    if min(xbc.shape[0], z.shape[0], dt.shape[0], out.shape[0]) < row0 + rows:
+        raise ValueError("state_space: rows outside the tensors")
+    ad = _dt(xbc.dtype)
+    need = lib.mi_state_space_workspace_bytes(rows, num_reqs, hh, groups, n, v, 1, ad) if chunked else 0
+    chunked = need > 0
+    if not chunked:
+        need = lib.mi_state_space_workspace_bytes(rows, num_reqs, hh, groups, n, v, 0, ad)
+    ws = torch.empty(max(need, 1), dtype=torch.uint8, device=xbc.device)
+    a = _C.StateSpaceArgs(_p(xbc), _p(z), _p(dt), _p(conv_w), _p(conv_b), _p(norm_w), _p(dt_bias), _p(a_log), _p(d), _p(state), _p(ring),
+                          _p(slots), _p(query_start_loc), _p(seq_lens), _p(out), ps, os_, req0, num_reqs, hh, groups, n, v, taps, norm_groups,
+                          float(eps))
+    check("mi_state_space", lib.mi_state_space(ctypes.byref(a), row0, rows, max_query_len, int(chunked), _p(ws), need, ad, _stream()))
+    return out
+
+
+def soft_cap_argmax(logits: torch.Tensor, cap: float, ids: Optional[torch.Tensor] = None, greedy: bool = True) -> Optional[torch.Tensor]:
+    """``logits`` = cap tanh(logits / cap) in place; with ``greedy`` also the first index of every row's maximum."""
+    _gpu(logits, ids)
+    stride, vocab = _rows(logits)
+    t = logits.shape[0]
+    if greedy and ids is None:
+        ids = torch.empty(t, dtype=torch.int64, device=logits.device)
+    if not greedy:
+        ids = None
+    _i64(ids)
+    if ids is not None and ids.numel() < t:
+        raise ValueError("soft_cap_argmax: an id per row")
+    check("mi_soft_cap_argmax", lib.mi_soft_cap_argmax(_p(logits), _p(ids), float(cap), t, vocab, stride, _dt(logits.dtype), _stream()))
+    return ids

@@ -18,6 +18,7 @@ ARCHITECTURES = {
     "Qwen2_5OmniTalkerForConditionalGeneration": ("talker", "TalkerConfig", "Qwen2_5OmniTalkerForConditionalGeneration"),
     "Dogulorn": ("dogulorn", "DogulornConfig", "DogulornForCausalLM"),
     "Bodopel": ("bodopel", "BodopelConfig", "BodopelForCausalLM"),
+    "Lifuzen": ("lifuzen", "LifuzenConfig", "LifuzenForCausalLM"),
     "Pupopel": ("pupopel", "PupopelConfig", "PupopelForCausalLM"),
 }
 DEFAULT_ARCHITECTURE = "Qwen2_5OmniTalkerForConditionalGeneration"

@@ -42,6 +42,8 @@ class TokenDecoder:
     has_postprocess = False
     prefer_model_sampler = False
     head: torch.Tensor
+    logit_softcap: Optional[float] = None      # logits are cap tanh(logits / cap)
+    unread_weights: frozenset = frozenset()    # names a checkpoint may hold although nothing reads them
 
     def __init__(self, cfg: Any, dtype, device):
         from .distributed import get_tensor_model_parallel_world_size
@@ -71,9 +73,15 @@ class TokenDecoder:
         return []
 
     def compute_logits(self, hidden_states: torch.Tensor) -> torch.Tensor:
-        return tuned_linear(hidden_states, self.head)
+        logits = tuned_linear(hidden_states, self.head)
+        if self.logit_softcap is not None:
+            ops.soft_cap_argmax(logits, self.logit_softcap, greedy=False)
+        return logits
 
     def compute_logits_and_greedy(self, hidden_states: torch.Tensor, ids: Optional[torch.Tensor] = None):
+        if self.logit_softcap is not None:
+            logits = tuned_linear(hidden_states, self.head)
+            return logits, ops.soft_cap_argmax(logits, self.logit_softcap, ids)
         logits = self.compute_logits(hidden_states)
         return logits, ops.mask_logits_argmax(logits, ids=ids)
 
@@ -82,6 +90,8 @@ class TokenDecoder:
         loaded: set[str] = set()
         for name, w in (weights.items() if isinstance(weights, dict) else weights):
             dst = params.get(name)
+            if dst is None and name in self.unread_weights:
+                continue
             if dst is None:
                 raise KeyError(f"checkpoint tensor maps to no parameter: {name!r}")
             want = tuple(dst.shape) if dst.dim() < 3 else (dst.shape[0], dst.shape[1] * dst.shape[2])
