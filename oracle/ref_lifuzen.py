@@ -86,11 +86,11 @@ def mamba_mixer(h, w, m, eps):
 
 
 # ------------------------------------------------------------------------------------------ attention whose values are its keys
-def rotate(x, dims, base):
-    """x [T, heads, D]: neighbours 2i, 2i + 1 of the first ``dims`` turned by position * base^(-2i / dims)"""
+def rotate(x, dims, base, first=0):
+    """x [T, heads, D], positions from ``first`` on: neighbours 2i, 2i + 1 of the first ``dims`` turned by position * base^(-2i / dims)"""
     out = x.clone()
     for i in range(dims // 2):
-        a = torch.arange(x.shape[0], dtype=x.dtype)[:, None] * (float(base) ** (-2.0 * i / dims))
+        a = torch.arange(first, first + x.shape[0], dtype=x.dtype)[:, None] * (float(base) ** (-2.0 * i / dims))
         u, v = x[:, :, 2 * i], x[:, :, 2 * i + 1]
         out[:, :, 2 * i] = u * torch.cos(a) - v * torch.sin(a)
         out[:, :, 2 * i + 1] = v * torch.cos(a) + u * torch.sin(a)

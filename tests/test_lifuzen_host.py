@@ -1,0 +1,281 @@
+"""CPU: configuration, weights map, layer runs, argument checks of the Lifuzen path, and the restatement itself."""
+import copy
+import ctypes
+import json
+
+import pytest
+import torch
+
+import lifuzen_models as lm
+from oracle import ref_lifuzen as ref
+
+
+def build(cfg, dtype=torch.float32):
+    from vllm_omni_amd.lifuzen import LifuzenConfig, LifuzenForCausalLM
+
+    c = LifuzenConfig.from_dict(cfg)
+    return c, LifuzenForCausalLM(c, dtype, "cpu"), lm.random_weights(cfg)
+
+
+def test_registry_picks_the_model(tmp_path):
+    from vllm_omni_amd.lifuzen import LifuzenConfig, LifuzenForCausalLM
+    from vllm_omni_amd.registry import config_from_dir, config_from_hf, model_class_for
+
+    cfg = lm.CONFIGS["mixed"]
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    c = config_from_dir(str(tmp_path))
+    assert isinstance(c, LifuzenConfig) and model_class_for(c) is LifuzenForCausalLM
+    assert config_from_hf(c) is c and config_from_hf(cfg) == c and LifuzenConfig.from_json(str(tmp_path)) == c
+
+
+def test_every_size_and_constant_comes_from_the_configuration():
+    c, m, _ = build(lm.CONFIGS["mixed"])
+    a, s = c.layers[2].mixer, c.layers[3].mixer
+    assert (a.heads, a.kv_heads, a.dim, a.conv, a.scale, a.rot_dims, a.rot_base, a.sink) == (4, 4, 64, 3, 0.3, 64, 77.0, 0.0)
+    assert (s.heads, s.groups, s.state, s.vdim, s.conv, s.norm_groups) == (4, 1, 40, 64, 3, 4)
+    assert (s.inner, s.channels) == (256, 336)
+    e = c.layers[3].mlp
+    assert (e.experts, e.top, e.ff) == (9, 3, 24) and c.layers[1].mlp is None
+    assert (c.vocab_size, c.hidden_size, c.rms_norm_eps, c.residual_mult, c.logit_softcap) == (131, 96, 1e-5, 0.6, 6.0)
+    assert (c.loop.start, c.loop.stop, c.loop.times) == (1, 4, 3) and m.logit_softcap == 6.0
+    freq = m.layers[2].mixer.inv_freq
+    assert freq.dtype == torch.float32 and torch.allclose(freq, 77.0 ** (-torch.arange(0, 64, 2) / 64), rtol=1e-6)
+
+
+@pytest.mark.parametrize("name", list(lm.CONFIGS))
+def test_layer_runs_and_their_memory(name):
+    """every pass of a looped layer has a cache, a state and a ring of its own"""
+    cfg = lm.CONFIGS[name]
+    c, m, _ = build(cfg)
+    assert c.runs == ref.layer_runs(cfg) == m.runs
+    assert [t for _, t in c.runs if t is not None] == list(range(c.loop.times if c.loop else 0))
+    kinds = [cfg["layers"][i]["type"] for i, _ in c.runs]
+    specs = m.kv_cache_specs(16)
+    assert list(specs) == [r for r, k in enumerate(kinds) if k == "attention"]
+    for r, s in specs.items():
+        mx = cfg["layers"][c.runs[r][0]]["mixer"]
+        assert (s.num_kv_heads, s.num_q_heads) == (mx["kv_heads"], mx["heads"]) and s.head_dim >= mx["dim"]
+    states = [torch.zeros(3, *s.shape, dtype=s.dtype) for s in m.state_specs()]
+    assert len(states) == sum(2 if k == "mamba2" else 1 for k in kinds) and m.is_recurrent
+    m.bind_states(states)
+    assert [t.data_ptr() for mem in m.memory for t in mem.states] == [t.data_ptr() for t in states]
+    for mem, (i, _) in zip(m.memory, c.runs):
+        mx = cfg["layers"][i]["mixer"]
+        if cfg["layers"][i]["type"] == "mamba2":
+            assert mem.states[0].shape == (3, mx["heads"], mx["state"], mx["vdim"]) and mem.states[0].dtype == torch.float32
+        assert mem.states[-1].shape[1] == mx["conv"]
+
+
+@pytest.mark.parametrize("change,match", [
+    (lambda d: d["layers"][0].update(type="mamba"), "unknown mixer type"),
+    (lambda d: d["layers"][0]["mlp"].update(kind="dense"), "unknown feed-forward kind"),
+    (lambda d: d["layers"][0]["mixer"].update(vdim=40), "values are the keys"),
+    (lambda d: d["loop"].update(stop=9), "does not fit"),
+    (lambda d: d["loop"].update(times=0), "does not fit"),
+    (lambda d: d.update(logit_softcap=-1.0), "soft cap"),
+    (lambda d: d.update(layers=[]), "at least one layer"),
+])
+def test_configurations_that_do_not_exist_are_refused(change, match):
+    from vllm_omni_amd.lifuzen import LifuzenConfig
+
+    d = copy.deepcopy(lm.CONFIGS["mixed"])
+    change(d)
+    with pytest.raises(ValueError, match=match):
+        LifuzenConfig.from_dict(d)
+
+
+@pytest.mark.parametrize("layer,change,match", [
+    (0, lambda m: m.update(heads=7), "multiple"),
+    (0, lambda m: m.update(scale=0.0), "scale"),
+    (0, lambda m: m.update(conv=0), "tap"),
+    (0, lambda m: m["rot"].update(dims=50), "pairs"),
+    (0, lambda m: m["rot"].update(dims=7), "pairs"),
+    (1, lambda m: m.update(groups=4), "multiple"),
+    (1, lambda m: m.update(norm_groups=7), "multiple"),
+    (1, lambda m: m.update(conv=0), "tap"),
+])
+def test_sizes_that_do_not_fit_are_refused(layer, change, match):
+    from vllm_omni_amd.lifuzen import LifuzenConfig, LifuzenForCausalLM
+
+    d = copy.deepcopy(lm.CONFIGS["mixed"])
+    change(d["layers"][layer]["mixer"])
+    with pytest.raises(ValueError, match=match):
+        LifuzenForCausalLM(LifuzenConfig.from_dict(d), torch.float32, "cpu")
+
+
+@pytest.mark.parametrize("kw", [dict(top=7), dict(top=0), dict(experts=300), dict(act="gelu"), dict(scores="tanh"),
+                                dict(act="silu_gated", weigh_input=True)])
+def test_experts_that_are_not_built_are_refused(kw):
+    from vllm_omni_amd.moe import RoutedExperts
+
+    with pytest.raises(ValueError):
+        RoutedExperts(**{**dict(width=64, experts=6, top=2, ff=32, dtype=torch.float32, device="cpu"), **kw})
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("name", list(lm.CONFIGS))
+def test_weights_map_one_to_one(name, dtype):
+    """every checkpoint tensor has a place of its own; what the recurrence computes in 32-bit is stored in 32-bit; padding is zero"""
+    cfg = lm.CONFIGS[name]
+    _, m, w = build(cfg, dtype)
+    assert m.load_weights(w) == set(w)
+    params = dict(m.named_weights())
+    assert set(params) == set(w)
+    for n, t in w.items():
+        keep = torch.float32 if n.rsplit(".", 1)[-1] in ("dt_bias", "A_log", "D") else dtype
+        assert params[n].dtype == keep and torch.equal(params[n].reshape(t.shape).float(), t.to(keep).float()), n
+    assert m.head is m.embed
+    for i, layer in enumerate(m.layers):
+        p = f"l{i}."
+        if cfg["layers"][i]["type"] == "attention":
+            assert int(layer.mixer.o.count_nonzero()) == int(w[p + "mix.o"].count_nonzero())
+            assert int(layer.mixer.proj.weight.count_nonzero()) == sum(int(w[p + "mix." + x].count_nonzero()) for x in "qk")
+        if layer.experts:
+            n = cfg["layers"][i]["mlp"]["router"]["experts"]
+            for name_, t in (("up", layer.experts.up), ("down", layer.experts.down)):
+                assert int(t.count_nonzero()) == sum(int(w[f"{p}mlp.e{e}.{name_}"].count_nonzero()) for e in range(n))
+    with pytest.raises(KeyError):
+        m.load_weights({"l0.mix.v": torch.zeros(1)})
+    with pytest.raises(ValueError):
+        m.load_weights({"embed": torch.zeros(3, 3)})
+
+
+def test_a_norm_that_nothing_reads_may_be_there():
+    cfg = lm.CONFIGS["mixed"]
+    _, m, w = build(cfg)
+    assert "l1.norm2" not in w and m.load_weights({**w, "l1.norm2": torch.zeros(96)}) == set(w)
+    with pytest.raises(KeyError):
+        m.load_weights({"l9.norm2": torch.zeros(96)})
+
+
+def test_models_outside_the_envelope_say_so():
+    from vllm_omni_amd.lifuzen import LifuzenForCausalLM
+    from vllm_omni_amd.model_runner import GPUARModelRunner
+
+    c, m, _ = build(lm.CONFIGS["flat"])
+    with pytest.raises(ValueError, match="bfloat16 or float32"):
+        LifuzenForCausalLM(c, torch.float16, "cpu")
+    with pytest.raises(ValueError):
+        m.quantize_int8()
+    r = GPUARModelRunner(c, "cpu", torch.float32, max_num_reqs=2, max_model_len=64, max_num_batched_tokens=16, block_size=16,
+                         engine_output_type="text", enable_prefix_caching=True)
+    r.load_model()
+    with pytest.raises(ValueError, match="prefix caching"):
+        r.initialize_kv_cache(8)
+
+
+def test_argument_validation_without_gpu():
+    from vllm_omni_amd import _C
+
+    lib = _C.lib
+    buf = (ctypes.c_char * 4096)()
+    p = (ctypes.addressof(buf) + 15) & ~15
+    bad, no, ws, bf = _C.MI_ERR_INVALID_ARG, _C.MI_ERR_UNSUPPORTED, _C.MI_ERR_WORKSPACE, _C.MI_DTYPE_BF16
+
+    def norm2(**k):
+        return lib.mi_stream_norm2(p, k.get("y", p), 0, k.get("part"), None, None, k.get("top", 0), 1.0, k.get("table"), k.get("ids"), 10, None, p,
+                                   k.get("w2"), 1.0, p, k.get("h2"), 1e-6, 2, 8, 8, k.get("ys", 8), 8, 8, 8, k.get("dt", bf), None)
+
+    assert norm2(y=None) == bad and norm2(ys=7) == bad and norm2(part=p) == bad and norm2(table=p) == bad and norm2(w2=p) == bad
+    assert norm2(dt=_C.MI_DTYPE_F16) == no
+    assert lib.mi_soft_cap_argmax(p, None, 0.0, 2, 8, 8, bf, None) == bad and lib.mi_soft_cap_argmax(p, None, 1.0, 2, 8, 7, bf, None) == bad
+    assert lib.mi_soft_cap_argmax(p, None, 1.0, 2, 8, 8, _C.MI_DTYPE_F16, None) == no
+
+    base = {n: p for n, t in _C.ConvRopeCacheArgs._fields_ if t is ctypes.c_void_p}
+    base.update(x_stride=192, q_stride=256, cache_block_stride=2048, cache_token_stride=128, cache_head_stride=64, num_reqs=1, max_query_len=1,
+                heads=4, kv_heads=2, dim=32, head_dim=64, block_size=16, rot_dims=16, taps=4)
+    cr = lambda **kw: lib.mi_conv_rope_cache(ctypes.byref(_C.ConvRopeCacheArgs(**{**base, **kw})), bf, None)   # noqa: E731
+    for kw in (dict(ring=None), dict(inv_freq=None), dict(rot_dims=15), dict(rot_dims=34), dict(head_dim=24), dict(taps=0), dict(x_stride=191),
+               dict(q_stride=255), dict(heads=0)):
+        assert cr(**kw) == bad, kw
+    assert cr(dim=1100, head_dim=1100, x_stride=8000, q_stride=8000, rot_dims=0) == no
+
+    sp = {n: p for n, t in _C.StateSpaceArgs._fields_ if t is ctypes.c_void_p}
+    sp.update(stride=512, out_stride=128, num_reqs=1, heads=4, groups=2, state_dim=32, vdim=32, taps=4, norm_groups=2, eps=1e-6)
+    ss = lambda chunked=0, size=1 << 30, dt=bf, **kw: lib.mi_state_space(ctypes.byref(_C.StateSpaceArgs(**{**sp, **kw})), 0, 2, 2, chunked, p,   # noqa: E731
+                                                                        size, dt, None)
+    for kw in (dict(state=None), dict(conv_b=None), dict(groups=3), dict(norm_groups=3), dict(taps=0), dict(stride=255), dict(out_stride=127)):
+        assert ss(**kw) == bad and ss(chunked=1, **kw) == bad, kw
+    assert ss(chunked=1, dt=_C.MI_DTYPE_F32) == no and ss(chunked=1, state_dim=300, stride=4096) == no and ss(dt=_C.MI_DTYPE_F16) == no
+    for chunked in (0, 1):
+        need = lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 32, 32, chunked, bf)
+        assert need > 0 and ss(chunked, need - 1) == ws
+    assert lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 32, 32, 1, _C.MI_DTYPE_F32) == 0
+
+    def experts(form, weights, pair=False):
+        if pair:
+            return lib.mi_moe_pair_gemm(p, p, p, p, 4, 2, form, weights, 8, 16, 2, 16, 8, 100, bf, None)
+        return lib.mi_moe_expert_gemm(p, p, p, p, p, p, 1, form, weights, 64, 64, 2, 64, 64, 4096, 32, bf, None)
+
+    for pair in (False, True):
+        assert experts(3, None, pair) == bad and experts(-1, None, pair) == bad
+        assert experts(_C.MI_MOE_GATED, p, pair) == bad and experts(_C.MI_MOE_PLAIN, p, pair) == bad
+
+
+# ------------------------------------------------------------------------------------------------ the restatement itself
+def test_state_space_is_decayed_attention():
+    """y_t = sum_{s <= t} exp(sum of log decays in (s, t]) dt_s (C_t . B_s) x_s + D x_t"""
+    g = torch.Generator().manual_seed(1)
+    T, H, G, N, V = 9, 4, 2, 5, 3
+    x, B, C = (torch.randn(*s, generator=g, dtype=torch.float64) for s in ((T, H, V), (T, G, N), (T, G, N)))
+    dt, a_log, D = torch.rand(T, H, generator=g, dtype=torch.float64), torch.randn(H, generator=g, dtype=torch.float64), torch.randn(H, dtype=torch.float64)
+    y, _ = ref.state_space(x, B, C, dt, a_log, D)
+    cum = (-torch.exp(a_log) * dt).cumsum(0)
+    for h in range(H):
+        w = torch.exp(cum[:, None, h] - cum[None, :, h]) * dt[None, :, h] * (C[:, h // 2] @ B[:, h // 2].T)
+        assert torch.allclose(y[:, h], w.tril() @ x[:, h] + D[h] * x[:, h])
+
+
+def test_a_filter_starts_from_zeros():
+    y = ref.short_conv(torch.ones(4, 1), torch.tensor([[1000.0, 100.0, 10.0]]))
+    assert y[:, 0].tolist() == [10.0, 110.0, 1110.0, 1110.0]
+
+
+def test_sink_is_a_key_of_score_zero_without_a_value():
+    g = torch.Generator().manual_seed(2)
+    q, k, v = torch.randn(6, 2, 4, generator=g), torch.randn(6, 1, 4, generator=g), torch.randn(6, 1, 4, generator=g)
+    got = ref.sink_attention(q, k, v, 3.0)
+    for i in range(6):
+        for h in range(2):
+            s = torch.cat([k[:i + 1, 0] @ q[i, h] * 3.0, torch.zeros(1)])
+            p = torch.softmax(s, -1)[:-1]
+            assert torch.allclose(got[i, h], p @ v[:i + 1, 0], atol=1e-6)
+
+
+def test_rotation_depends_on_the_distance_only():
+    g = torch.Generator().manual_seed(3)
+    q, k = torch.randn(1, 1, 10, generator=g, dtype=torch.float64), torch.randn(1, 1, 10, generator=g, dtype=torch.float64)
+    dot = lambda a, b: float((ref.rotate(q, 6, 100.0, a) * ref.rotate(k, 6, 100.0, b)).sum())   # noqa: E731
+    assert abs(dot(7, 3) - dot(104, 100)) < 1e-9 and abs(dot(7, 3) - dot(7, 4)) > 1e-3
+    assert torch.equal(ref.rotate(q, 6, 100.0, 9)[..., 6:], q[..., 6:])
+
+
+def test_parts_of_the_gated_row_are_normed_apart():
+    g = torch.Generator().manual_seed(4)
+    y, z = torch.randn(2, 12, generator=g), torch.randn(2, 12, generator=g)
+    got = ref.gated_group_norm(y, z, torch.ones(12), 3, 0.0).view(2, 3, 4)
+    assert torch.allclose(got.pow(2).mean(-1), torch.ones(2, 3), atol=1e-5)
+
+
+def test_a_pass_adds_the_embedding_output_but_the_first():
+    """a model of layers that add nothing: the stream is the embedding, once per pass, and the passes' vectors"""
+    cfg = lm.model([(mamba_, None) for mamba_ in (lm.mamba(2, 1, 4, 4, 2, 1), lm.mamba(1, 1, 4, 4, 2, 1))], (0, 2, 3), vocab=11, width=16)
+    w = {k: torch.zeros_like(v) if k.endswith(".o") else v for k, v in lm.random_weights(cfg).items()}
+    _, st = ref.forward(cfg, w, [1, 2, 3])
+    x, steps = w["embed"][[1, 2, 3]].double(), w["loop.step"].double().cumsum(0)
+    for r, s in enumerate(st):
+        assert torch.allclose(s, x * (r // 2 + 1) + steps[r // 2])
+
+
+def test_experts_read_their_weighted_input():
+    """squared relu: a weight on the input is its square on the output"""
+    g = torch.Generator().manual_seed(5)
+    h = torch.randn(4, 8, generator=g, dtype=torch.float64)
+    w = {"router": torch.randn(3, 8, generator=g, dtype=torch.float64)}
+    for e in range(3):
+        w[f"e{e}.up"], w[f"e{e}.down"] = torch.randn(5, 8, generator=g, dtype=torch.float64), torch.randn(8, 5, generator=g, dtype=torch.float64)
+    got = ref.routed_experts(h, lambda n: w[n], 2)
+    s = torch.sigmoid(h @ w["router"].T)
+    for t in range(4):
+        want = sum(s[t, e] ** 2 * (torch.relu(h[t] @ w[f"e{e}.up"].T) ** 2 @ w[f"e{e}.down"].T) for e in s[t].topk(2).indices.tolist())
+        assert torch.allclose(got[t], want)

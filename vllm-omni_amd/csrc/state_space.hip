@@ -720,7 +720,7 @@ extern "C" int mi_state_space(const mi_state_space_args* a, int32_t row0, int32_
     if (rc == MI_OK) rc = launch_scan<false>(p, k, nreq, s);
   }
   if (rc != MI_OK) return rc;
-  if (max_query_len > 1) {
+  if (chunked || max_query_len > 1) {      // (a step of one row has left it there itself)
     rc = dtype == MI_DTYPE_BF16 ? launch_conv_update<uint16_t>(p.in, nreq, s) : launch_conv_update<float>(p.in, nreq, s);
     if (rc != MI_OK) return rc;
   }
