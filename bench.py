@@ -102,6 +102,15 @@ def parse_args():
     ap.add_argument("--bodopel-batches", default="32,256", help="decode batch sizes")
     ap.add_argument("--bodopel-ctx", type=int, default=4096, help="context of the decode cases")
     ap.add_argument("--bodopel-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
+    ap.add_argument("--lifuzen", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the Lifuzen stack beside the Pupopel "
+                         "and talker stacks of equal size (tools/bench_lifuzen.py; one JSON line per case)")
+    ap.add_argument("--lifuzen-size", default="2k,4k")
+    ap.add_argument("--lifuzen-mode", default="decode,prefill")
+    ap.add_argument("--lifuzen-models", default="lifuzen,pupopel,talker")
+    ap.add_argument("--lifuzen-batches", default="32,256", help="decode batch sizes")
+    ap.add_argument("--lifuzen-ctx", type=int, default=4096, help="context of the decode cases")
+    ap.add_argument("--lifuzen-prompts", default="8192;2048,2048,2048,2048", help="prompt lengths of a prefill step; several steps with ';'")
     a = ap.parse_args()
     if a.pmc_child:   # a few steps of the same workload, nothing else: the parent reads the counters of the decode launches
         a.steps, a.warmup, a.no_cpu_baseline, a.roofline_steps, a.traffic = 2, 1, True, 0, "none"
@@ -603,10 +612,11 @@ def time_allreduce(dev, rows: int, cols: int, calls: int = 50) -> dict:
 
 def main():
     a = parse_args()
-    if a.dogulorn or a.pupopel or a.bodopel:
+    stack = next((n for n in ("lifuzen", "bodopel", "pupopel", "dogulorn") if getattr(a, n)), None)
+    if stack:
         sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "tools"))
         sys.modules.setdefault("bench", sys.modules[__name__])
-        return importlib.import_module("bench_bodopel" if a.bodopel else "bench_pupopel" if a.pupopel else "bench_dogulorn").run(a)
+        return importlib.import_module(f"bench_{stack}").run(a)
     launched = "WORLD_SIZE" in os.environ
     if a.gpus > 1 and not launched:
         # no launcher around us: become one.  Nothing has touched the GPU yet (device_count() does not).

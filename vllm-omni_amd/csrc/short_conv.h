@@ -26,6 +26,18 @@ __device__ __forceinline__ const T* conv_input(const ConvInputs& p, const T* x_r
   return pos >= b ? src : x_row;
 }
 
+// four taps of 8 neighbouring channels, the one for the row itself first
+template <typename T>
+__device__ __forceinline__ void conv_taps4(const T* w, float (&wt)[4][8]) {
+#pragma unroll
+  for (int m = 0; m < 4; ++m) {
+    float v[8];
+    Io<T>::template ldv<8>(w + 8 * m, v);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) wt[3 - j % 4][2 * m + j / 4] = v[j];
+  }
+}
+
 // the last rows of every request's portion into its ring (a one-row portion's is there already: the same values again)
 template <typename T>
 __global__ __launch_bounds__(256) void conv_inputs_update_kernel(const ConvInputs p) {

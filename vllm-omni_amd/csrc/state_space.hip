@@ -149,22 +149,32 @@ __global__ __launch_bounds__(256) void state_step_kernel(const SsmParams p) {
 }
 
 // ------------------------------------------------------------------------------------------------ chunks
-// Workspace of one chunk (bf16): C [G][64][Np], B [G][64][Np], Bt [G][Np][64], Xt [H][Vp][64], then fp32 [H][3][64]: dt, and the log
-// decays summed over the token's 16 tokens up to it (lead) and behind it (trail).  Rows past the portion's end are zeros.
-// Within 32 neighbours along the contiguous dimension the order is that of the matrix cores' accumulators, so that an accumulator
-// pair IS an operand: place 8 q + 4 t + r holds index 16 t + 4 q + r.
+// Workspace of one chunk (bf16): C [G][64][Np], B [G][64][Np], Bt [G][Np][64], Xt [H][Vp][64], then fp32 [H][5][64] (ChunkVec below).
+// Rows past the portion's end are zeros.  Within 32 neighbours along the contiguous dimension the order is that of the matrix
+// cores' accumulators, so that an accumulator pair IS an operand: place 8 q + 4 t + r holds index 16 t + 4 q + r.
 struct SsmLayout {
   int G, H, Np, Vp;
   __host__ __device__ int64_t c() const { return 0; }
   __host__ __device__ int64_t b() const { return (int64_t)G * kC * Np; }
   __host__ __device__ int64_t bt() const { return 2 * (int64_t)G * kC * Np; }
   __host__ __device__ int64_t xt() const { return 3 * (int64_t)G * kC * Np; }
-  __host__ __device__ int64_t dt() const { return xt() + (int64_t)H * Vp * kC; }                    // (in bf16 units)
-  __host__ __device__ int64_t size() const { return dt() + (int64_t)H * 3 * kC * 2; }
+  __host__ __device__ int64_t vec() const { return xt() + (int64_t)H * Vp * kC; }                    // (in bf16 units)
+  __host__ __device__ int64_t size() const { return vec() + (int64_t)H * 5 * kC * 2; }
+};
+
+// numbers of a token of a chunk, per head.  ln a summed over the token's own 16 tokens up to it is `lead`; no sum that runs over more
+// is ever taken off another, so that decays of any strength may stand beside each other.
+enum ChunkVec {
+  kDt,       // dt
+  kTail,     // dt e^(ln a summed over the rest of its 16 tokens)
+  kLead,
+  kFrom0,    // e^(ln a summed from the chunk's start up to it)
+  kToEnd,    // dt e^(ln a summed from behind it to the chunk's end)
 };
 
 struct SsmChunks {
   uint16_t* ws;
+  float* y;              // read-outs [chunks][64][H][Vp]
   float* seg_state;      // [requests][nseg][H][N][V]: end state of each segment but the last; the last place: what the request started from
   float* seg_log;        // [requests][nseg][H]: ln of a segment's decay
   SsmLayout lay;
@@ -172,43 +182,52 @@ struct SsmChunks {
   int vec;               // the step's rows may be read 16 bytes at a time
 };
 
-__device__ __forceinline__ int64_t chunk_base(const SsmParams& p, int r) {
-  return (p.in.qsl[r] - p.in.qsl[p.in.req0]) / kC + (r - p.in.req0);
+template <typename P>
+__device__ __forceinline__ int64_t chunk_base(const P& p, int r) {
+  return (p.qsl[r] - p.qsl[p.req0]) / kC + (r - p.req0);
 }
 
-constexpr int kPrepCh = 64;     // channels of a prep workgroup
+constexpr int kPrepCh = 64;     // channels of a prep workgroup: two waves, a thread has 8 channels of four neighbouring tokens
 
-// blockIdx.y: first the filters' (kind, head or group, 64 channels) blocks, then four heads' step sizes each
-__global__ __launch_bounds__(256) void ssm_prep_kernel(const SsmParams p, const SsmChunks k) {
+// blockIdx.y: first the filters' (kind, head or group, 64 channels) blocks, then two heads' token numbers each
+__global__ __launch_bounds__(128) void ssm_prep_kernel(const SsmParams p, const SsmChunks k) {
   scalar_cache_acquire();
-  __shared__ __attribute__((aligned(16))) uint16_t tile[kPrepCh][kC + 8];      // [channel][token in operand order]
+  // [channel 8 a + j in row 8 j + a][token in operand order]
+  __shared__ __attribute__((aligned(16))) uint16_t tile[kPrepCh][kC + 8];
   using E = Elem<bf16_tag>;
   const int r = p.in.req0 + blockIdx.z, ck = blockIdx.x, tid = threadIdx.x;
   const int s0 = p.in.qsl[r], L = p.in.qsl[r + 1] - s0, i0 = ck * kC;
   if (i0 >= L) return;
   const int start = p.in.seq_lens[r] - L, len = min(kC, L - i0);
-  uint16_t* ws = k.ws + (chunk_base(p, r) + ck) * k.lay.size();
+  uint16_t* ws = k.ws + (chunk_base(p.in, r) + ck) * k.lay.size();
   const int Np = k.lay.Np, Vp = k.lay.Vp;
   const int bx = (Vp + kPrepCh - 1) / kPrepCh, bn = (Np + kPrepCh - 1) / kPrepCh;
   int y = blockIdx.y;
   if (y >= p.H * bx + 2 * p.G * bn) {                       // a wave per head, a lane per token
-    const int h = (y - p.H * bx - 2 * p.G * bn) * 4 + (tid >> 6), lane = tid & 63;
+    const int h = (y - p.H * bx - 2 * p.G * bn) * 2 + (tid >> 6), lane = tid & 63;
     if (h >= p.H) return;
-    float* out = reinterpret_cast<float*>(ws + k.lay.dt()) + (int64_t)h * 3 * kC;
+    float* out = reinterpret_cast<float*>(ws + k.lay.vec()) + (int64_t)h * 5 * kC + lane;
     const int64_t row = s0 + i0 + min(lane, len - 1);
     const float raw = E::from_bits(reinterpret_cast<const uint16_t*>(p.dt)[row * p.in.ld + h]);
     const float dt = lane < len ? softplus_f(raw + p.dt_bias[h]) : 0.f, lg = -expf(p.a_log[h]) * dt;
-    float lead = lg, trail = lg;      // sums over the 16-token tile: no differences of sums across tiles, whatever their size
+    float lead = lg, tail = lg;       // sums over the token's 16 up to it, and from it on
 #pragma unroll
     for (int o = 1; o < 16; o <<= 1) {
-      const float a = __shfl_up(lead, o, 64), b = __shfl_down(trail, o, 64);
+      const float a = __shfl_up(lead, o, 64), b = __shfl_down(tail, o, 64);
       lead += (lane & 15) >= o ? a : 0.f;
-      trail += (lane & 15) + o < 16 ? b : 0.f;
+      tail += (lane & 15) + o < 16 ? b : 0.f;
     }
-    trail = __shfl_down(trail, 1, 64);
-    out[lane] = dt;
-    out[kC + lane] = lead;
-    out[2 * kC + lane] = (lane & 15) == 15 ? 0.f : trail;
+    const float next = __shfl_down(tail, 1, 64);
+    const float t0 = __shfl(lead, 15, 64), t1 = __shfl(lead, 31, 64), t2 = __shfl(lead, 47, 64), t3 = __shfl(lead, 63, 64);
+    const int t = lane >> 4;
+    const float behind = (lane & 15) == 15 ? 0.f : next;
+    const float before = t == 0 ? 0.f : t == 1 ? t0 : t == 2 ? t0 + t1 : t0 + t1 + t2;
+    const float after = t == 3 ? 0.f : t == 2 ? t3 : t == 1 ? t2 + t3 : t1 + t2 + t3;
+    out[kDt * kC] = dt;
+    out[kTail * kC] = dt * expf(behind);
+    out[kLead * kC] = lead;
+    out[kFrom0 * kC] = expf(before + lead);
+    out[kToEnd * kC] = dt * expf(behind + after);
     return;
   }
   int unit, blk, kind, width, real, ch0;
@@ -219,65 +238,63 @@ __global__ __launch_bounds__(256) void ssm_prep_kernel(const SsmParams p, const 
     kind = 1 + y / (p.G * bn), y %= p.G * bn;
     unit = y / bn, blk = y % bn, width = Np, real = p.N, ch0 = p.H * p.V + ((kind - 1) * p.G + unit) * p.N;
   }
-  // a thread: 8 channels of two neighbouring tokens
-  const int c = blk * kPrepCh + (tid & 7) * 8, t = (tid >> 3) * 2;
+  const int c = blk * kPrepCh + (tid & 7) * 8, t = (tid >> 3) * 4;
   const int taps = p.in.taps, CH = p.in.channels;
   const uint16_t* X = reinterpret_cast<const uint16_t*>(p.in.x);
   const uint16_t* W = reinterpret_cast<const uint16_t*>(p.in.w);
   const uint16_t* ring = reinterpret_cast<const uint16_t*>(p.in.ring) + (int64_t)p.in.slots[r] * taps * CH;
   const int live = min(8, real - c);                        // <= 0: padding channels only
-  float acc[2][8];
-  auto load = [&](const uint16_t* src, float (&v)[8]) {     // src: channel c of a row
-    if (k.vec) {
-      Io<uint16_t>::ldv<8>(src, v);
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = Io<uint16_t>::ld(src + min(j, live - 1));
-    }
-  };
-  auto input = [&](int i, float (&v)[8]) {                  // token i of the portion (negative: before it), zeros before the start
-    const int pos = start + i;
-    const uint16_t* src = i >= 0 ? X + (int64_t)(s0 + min(i, L - 1)) * p.in.ld : ring + (int64_t)(max(pos, 0) % taps) * CH;
-    load(src + ch0 + c, v);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = pos >= 0 ? v[j] : 0.f;
+  float acc[4][8];
+  auto source = [&](int i) {                                // token i of the portion (negative: before it)
+    return (i >= 0 ? X + (int64_t)(s0 + min(i, L - 1)) * p.in.ld : ring + (int64_t)(max(start + i, 0) % taps) * CH) + ch0 + c;
   };
   if (live > 0) {
-    float bias[8];
-    load(reinterpret_cast<const uint16_t*>(p.conv_b) + ch0 + c, bias);
+    if (k.vec && taps == 4) {
+      uint4 raw[7];
+      float wt[4][8], bias[8], v[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) acc[0][j] = acc[1][j] = bias[j];
-    auto weight = [&](int b, int j) { return Io<uint16_t>::ld(W + (int64_t)(ch0 + c + min(j, live - 1)) * taps + taps - 1 - b); };
-    if (taps == 4) {
-      float v[5][8];
+      for (int b = 0; b < 7; ++b) raw[b] = *reinterpret_cast<const uint4*>(source(i0 + t + 3 - b));
+      conv_taps4<uint16_t>(W + (int64_t)(ch0 + c) * 4, wt);
+      Io<uint16_t>::ldv<8>(reinterpret_cast<const uint16_t*>(p.conv_b) + ch0 + c, bias);
 #pragma unroll
-      for (int b = 0; b < 5; ++b) input(i0 + t + 1 - b, v[b]);
+      for (int u = 0; u < 4; ++u)
 #pragma unroll
-      for (int b = 0; b < 4; ++b)
+        for (int j = 0; j < 8; ++j) acc[u][j] = bias[j];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const float wt = weight(b, j);
-          acc[1][j] += wt * v[b][j], acc[0][j] += wt * v[b + 1][j];
-        }
-    } else {
-      for (int b = 0; b < taps; ++b) {
-        float v0[8], v1[8];
-        input(i0 + t - b, v0);
-        input(i0 + t + 1 - b, v1);
+      for (int b = 0; b < 7; ++b) {                         // the input of token t + 3 - b: tap u - (3 - b) of token t + u
+        Io<uint16_t>::ldv<8>(reinterpret_cast<const uint16_t*>(&raw[b]), v);
+        const bool there = start + i0 + t + 3 - b >= 0;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const float wt = weight(b, j);
-          acc[0][j] += wt * v0[j], acc[1][j] += wt * v1[j];
-        }
+        for (int u = 0; u < 4; ++u)
+          if (u - (3 - b) >= 0 && u - (3 - b) < 4)
+#pragma unroll
+            for (int j = 0; j < 8; ++j) acc[u][j] += wt[u - (3 - b)][j] * (there ? v[j] : 0.f);
       }
+    } else {
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[u][j] = Io<uint16_t>::ld(reinterpret_cast<const uint16_t*>(p.conv_b) + ch0 + c + min(j, live - 1));
+      for (int b = 0; b < taps; ++b)
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int i = i0 + t + u - b;
+          if (start + i < 0) continue;
+          const uint16_t* src = source(i);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const int jj = min(j, live - 1);
+            acc[u][j] += Io<uint16_t>::ld(W + (int64_t)(ch0 + c + jj) * taps + taps - 1 - b) * Io<uint16_t>::ld(src + jj);
+          }
+        }
     }
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < 4; ++u)
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[u][j] = j < live && t + u < len ? silu_f(acc[u][j]) : 0.f;
   } else {
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < 4; ++u)
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[u][j] = 0.f;
   }
@@ -286,21 +303,24 @@ __global__ __launch_bounds__(256) void ssm_prep_kernel(const SsmParams p, const 
     const int at = (c & ~31) + ((c & 15) >> 2) * 8 + ((c >> 4) & 1) * 4;
     if (c < Np)
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
+      for (int u = 0; u < 4; ++u) {
         *reinterpret_cast<uint2*>(rows + (int64_t)u * Np + at) = make_uint2(E::pack(acc[u][0], acc[u][1]), E::pack(acc[u][2], acc[u][3]));
         *reinterpret_cast<uint2*>(rows + (int64_t)u * Np + at + 8) = make_uint2(E::pack(acc[u][4], acc[u][5]), E::pack(acc[u][6], acc[u][7]));
       }
     if (kind == 2) return;
   }
-  const int at = (t & ~31) + ((t & 15) >> 2) * 8 + ((t >> 4) & 1) * 4 + (t & 3);      // t is even: its neighbour is the next place
+  const int at = (t & ~31) + ((t & 15) >> 2) * 8 + ((t >> 4) & 1) * 4;      // four neighbours stay together
 #pragma unroll
-  for (int j = 0; j < 8; ++j) *reinterpret_cast<uint32_t*>(&tile[(tid & 7) * 8 + j][at]) = E::pack(acc[0][j], acc[1][j]);
+  for (int j = 0; j < 8; ++j)
+    *reinterpret_cast<uint2*>(&tile[8 * j + (tid & 7)][at]) = make_uint2(E::pack(acc[0][j], acc[1][j]), E::pack(acc[2][j], acc[3][j]));
   __syncthreads();
   uint16_t* cols = ws + (kind == 0 ? k.lay.xt() : k.lay.bt()) + (int64_t)unit * width * kC;
-  for (int n = tid; n < kPrepCh * 8; n += 256) {
+#pragma unroll
+  for (int n = tid; n < kPrepCh * 8; n += 128) {
     const int cc = n >> 3, piece = (n & 7) * 8;
     if (blk * kPrepCh + cc < width)
-      *reinterpret_cast<uint4*>(cols + (int64_t)(blk * kPrepCh + cc) * kC + piece) = *reinterpret_cast<const uint4*>(&tile[cc][piece]);
+      *reinterpret_cast<uint4*>(cols + (int64_t)(blk * kPrepCh + cc) * kC + piece) =
+          *reinterpret_cast<const uint4*>(&tile[8 * (cc & 7) + (cc >> 3)][piece]);
   }
 }
 
@@ -323,19 +343,16 @@ __device__ __forceinline__ Terms split8(const f32x4_t& a, const f32x4_t& b) {
   split2(b[2], b[3], t.hi.w, t.mid.w, t.lo.w);
   return t;
 }
-__device__ __forceinline__ f32x4_t exp4(const f32x4_t& v) {
-  f32x4_t e;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) e[i] = fast_exp2(v[i] * kLog2e);
-  return e;
-}
-
 // NT: 32-wide tiles of the state's rows.  A wave has 16 columns of a head's S; the four waves of a workgroup form a quarter of P
-// each and share it through LDS (two buffers: one barrier a chunk).  ENDS: only the end state of a segment.
+// each and share it through LDS (two buffers, formed a chunk ahead: one barrier a chunk that nobody waits long at).  ENDS: only the
+// end state of a segment.  The chain of chunks is the critical path and its loads must not be: registers are loaded for the next
+// chunk as soon as this one's products have read them, every load and store unconditional, so that the number in flight is known at
+// every wait (waves past the last column do the last tile's work once more; past the last chunk the loads fetch it again).
 template <int NT, bool ENDS>
-__global__ __launch_bounds__(256, NT <= 4 ? 2 : 1) void ssm_scan_kernel(const SsmParams p, const SsmChunks k, int vgroups) {
+__global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, const SsmChunks k, int vgroups) {
   scalar_cache_acquire();
   constexpr int Np = 32 * NT;
+  constexpr bool AHEAD = NT <= 4;          // (a state of 256 rows leaves no registers for the operands of P)
   __shared__ uint4 sP[ENDS ? 1 : 2][ENDS ? 1 : 6 * 3 * 64];      // fragments (row tile 0..3, 32 columns up to it), three terms
   // the heads of a group, and the column groups of a head, on one XCD (workgroups go to the 8 XCDs in turn)
   const int work = p.H * vgroups, each = (work + 7) / 8;
@@ -348,9 +365,8 @@ __global__ __launch_bounds__(256, NT <= 4 ? 2 : 1) void ssm_scan_kernel(const Ss
   if (ENDS ? seg >= segs - 1 : seg >= segs) return;
   const int first = seg * k.seg_chunks, nck = min(k.seg_chunks, all - first);
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, kg = lane >> 4;
-  const int grp = h / (p.H / p.G), vt = vg * 4 + wave, v = vt * 16 + lr;
-  const bool active = vt * 16 < p.V;                        // (a wave without columns still forms its part of P)
-  if (ENDS && !active) return;
+  const SsmLayout& lay = k.lay;
+  const int grp = h / (p.H / p.G), vt = min(vg * 4 + wave, lay.Vp / 16 - 1), v = vt * 16 + lr;
   float* S = p.state + ((int64_t)p.in.slots[r] * p.H + h) * p.N * p.V;
   auto seg_at = [&](int n) { return k.seg_state + (((int64_t)(r - p.in.req0) * k.nseg + n) * p.H + h) * p.N * p.V; };
   auto log_at = [&](int n) { return k.seg_log + ((int64_t)(r - p.in.req0) * k.nseg + n) * p.H + h; };
@@ -375,165 +391,193 @@ __global__ __launch_bounds__(256, NT <= 4 ? 2 : 1) void ssm_scan_kernel(const Ss
         if (d < p.N && v < p.V) dst[(int64_t)d * p.V + v] = st[n][i];
       }
   };
-  if (active) {
-    if (segs == 1) {
+  if (segs == 1) {
+    if (start > 0) add_state(S, 0.f);
+  } else if constexpr (ENDS) {
+    // the first segment starts from the request's state and leaves a copy of it: the pass behind this one overwrites it
+    if (seg == 0) {
       if (start > 0) add_state(S, 0.f);
-    } else if constexpr (ENDS) {
-      // the first segment starts from the request's state and leaves a copy of it: the pass behind this one overwrites it
-      if (seg == 0) {
-        if (start > 0) add_state(S, 0.f);
-        put_state(seg_at(k.nseg - 1));
-      }
-    } else if (seg == 0) {
-      add_state(seg_at(k.nseg - 1), 0.f);
-    } else {
-      for (int n = 0; n < seg; ++n) add_state(seg_at(n), n ? fast_exp2(*log_at(n) * kLog2e) : 0.f);
+      put_state(seg_at(k.nseg - 1));
     }
+  } else if (seg == 0) {
+    add_state(seg_at(k.nseg - 1), 0.f);
+  } else {
+    for (int n = 0; n < seg; ++n) add_state(seg_at(n), n ? fast_exp2(*log_at(n) * kLog2e) : 0.f);
   }
-  const SsmLayout& lay = k.lay;
-  const uint16_t* base = k.ws + (chunk_base(p, r) + first) * lay.size();
+  const int64_t chunk0 = chunk_base(p.in, r) + first;
+  const uint16_t* base = k.ws + chunk0 * lay.size();
   const int64_t gofs = (int64_t)grp * kC * Np;
-  const float skip = p.d[h];
-  float seg_sum = 0.f;
-  float* yb = p.y + (int64_t)(s0 - p.row0 + first * kC) * p.H * p.V + (int64_t)h * p.V + v;
-  for (int ck = 0; ck < nck; ++ck, base += lay.size()) {
-    const float* dt = reinterpret_cast<const float*>(base + lay.dt()) + (int64_t)h * 3 * kC;
-    const float* lead = dt + kC;
-    const float* trail = lead + kC;
-    float tot[4];                                           // log decay of each 16 tokens
+  auto chunk = [&](int c) { return base + min(c, nck - 1) * lay.size(); };
+  auto numbers = [&](const uint16_t* b, int which) { return reinterpret_cast<const float*>(b + lay.vec()) + ((int64_t)h * 5 + which) * kC; };
+  auto ld4 = [](const uint16_t* a) { return *reinterpret_cast<const uint4*>(a); };
+  auto ldf4 = [](const float* a) { return *reinterpret_cast<const f32x4_t*>(a); };
+
+  // ---- S <- e^(G_C) S + sum_j B_j (weight_j x_j)^T
+  uint4 tf[2 * NT][2], xf[2];
+  f32x4_t wx[4];
+  float decay;
+  auto load_t = [&](int c) {
+    const uint16_t* b = chunk(c);
 #pragma unroll
-    for (int t = 0; t < 4; ++t) tot[t] = lead[16 * t + 15];
-    const float t01 = tot[0] + tot[1], t12 = tot[1] + tot[2], t23 = tot[2] + tot[3], t012 = t01 + tot[2], t123 = t12 + tot[3];
-    const float whole = t01 + t23;
-    // operands of this wave's columns
-    uint4 xf[2];
+    for (int t = 0; t < 2; ++t) xf[t] = ld4(b + lay.xt() + ((int64_t)h * lay.Vp + v) * kC + 32 * t + 8 * kg);
+    const float* w = numbers(b, kToEnd);
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
-      xf[t] = *reinterpret_cast<const uint4*>(base + lay.xt() + ((int64_t)h * lay.Vp + (active ? vt * 16 : 0) + lr) * kC + 32 * t + 8 * kg);
-    if constexpr (!ENDS) {
-      // ---- P of row tile `wave`, as P^T: rows j, columns i
-      uint4 cf[NT];
-      const uint16_t* crow = base + lay.c() + gofs + (int64_t)(16 * wave + lr) * Np + 8 * kg;
+    for (int t = 0; t < 4; ++t) wx[t] = ldf4(w + 16 * t + 4 * kg);
+    decay = numbers(b, kFrom0)[kC - 1];
+    const uint16_t* bt = b + lay.bt() + gofs + (int64_t)lr * kC + 8 * kg;
 #pragma unroll
-      for (int n = 0; n < NT; ++n) cf[n] = *reinterpret_cast<const uint4*>(crow + 32 * n);
-      const float li = lead[16 * wave + lr];
-      uint4* dst = sP[ck & 1] + (wave < 2 ? wave : 2 * wave - 2) * 3 * 64 + lane;      // tiles before: 0, 1, 2, 4
+    for (int n = 0; n < 2 * NT; ++n)
 #pragma unroll
-      for (int tp = 0; tp < 2; ++tp) {
-        if (2 * tp > wave) continue;
-        f32x4_t pr[2];
+      for (int t = 0; t < 2; ++t) tf[n][t] = ld4(bt + (int64_t)16 * n * kC + 32 * t);
+  };
+  auto update = [&]() {
+    using E = Elem<bf16_tag>;
+    Terms xw[2];
 #pragma unroll
-        for (int q = 0; q < 2; ++q) {
-          const int tj = 2 * tp + q;
-          f32x4_t a = {};
-          if (tj <= wave) {
-            const uint16_t* brow = base + lay.b() + gofs + (int64_t)(16 * tj + lr) * Np + 8 * kg;
+    for (int t = 0; t < 2; ++t) {
+      f32x4_t a = wx[2 * t], b = wx[2 * t + 1];
+      a[0] *= E::lo(xf[t].x), a[1] *= E::hi(xf[t].x), a[2] *= E::lo(xf[t].y), a[3] *= E::hi(xf[t].y);
+      b[0] *= E::lo(xf[t].z), b[1] *= E::hi(xf[t].z), b[2] *= E::lo(xf[t].w), b[3] *= E::hi(xf[t].w);
+      xw[t] = split8(a, b);
+    }
 #pragma unroll
-            for (int n = 0; n < NT; ++n) a = mfma16<bf16_tag>(*reinterpret_cast<const uint4*>(brow + 32 * n), cf[n], a);
-            const f32x4_t dj = *reinterpret_cast<const f32x4_t*>(dt + 16 * tj + 4 * kg);
-            const int gap = wave - tj;
-            if (gap == 0) {
-              const f32x4_t lj = *reinterpret_cast<const f32x4_t*>(lead + 16 * tj + 4 * kg);
-              const f32x4_t e = exp4(f32x4_t{li - lj[0], li - lj[1], li - lj[2], li - lj[3]});
+    for (int n = 0; n < 2 * NT; ++n) st[n] *= decay;
 #pragma unroll
-              for (int i = 0; i < 4; ++i) {
-                const int j = 4 * kg + i;
-                a[i] = j <= lr ? a[i] * e[i] * dj[i] + (j == lr ? skip : 0.f) : 0.f;
-              }
-            } else {
-              const f32x4_t tr = *reinterpret_cast<const f32x4_t*>(trail + 16 * tj + 4 * kg);
-              const float mid = gap == 1 ? 0.f : gap == 3 ? t12 : tj == 0 ? tot[1] : tot[2];
-              const float ref = li + mid;
-              a *= exp4(f32x4_t{ref + tr[0], ref + tr[1], ref + tr[2], ref + tr[3]}) * dj;
-            }
+    for (int t = 0; t < 2; ++t) {
+#pragma unroll
+      for (int n = 0; n < 2 * NT; ++n) st[n] = mfma16<bf16_tag>(tf[n][t], xw[t].lo, st[n]);
+#pragma unroll
+      for (int n = 0; n < 2 * NT; ++n) st[n] = mfma16<bf16_tag>(tf[n][t], xw[t].mid, st[n]);
+#pragma unroll
+      for (int n = 0; n < 2 * NT; ++n) st[n] = mfma16<bf16_tag>(tf[n][t], xw[t].hi, st[n]);
+    }
+  };
+  if constexpr (ENDS) {
+    float seg_sum = 0.f;
+    load_t(0);
+    for (int ck = 0; ck < nck; ++ck) {
+      const float* lead = numbers(chunk(ck), kLead);
+      seg_sum += (lead[15] + lead[31]) + (lead[47] + lead[63]);
+      update();
+      load_t(ck + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    put_state(seg_at(seg));
+    if (tid == 0 && vg == 0) *log_at(seg) = seg_sum;
+  } else {
+    // ---- P of row tile `wave`, as P^T (rows j, columns i): an accumulator pair is an operand of P X
+    uint4 bf[4][NT], cw[NT];
+    f32x4_t pw[4], pl;
+    float li, m1, m2;
+    auto load_p = [&](int c) {
+      const uint16_t* b = chunk(c);
+      const float* lead = numbers(b, kLead);
+      li = lead[16 * wave + lr], m1 = lead[31], m2 = lead[47];
+      pl = ldf4(lead + 16 * wave + 4 * kg);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) pw[t] = ldf4(numbers(b, t < wave ? kTail : kDt) + 16 * t + 4 * kg);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) cw[n] = ld4(b + lay.c() + gofs + (int64_t)(16 * wave + lr) * Np + 32 * n + 8 * kg);
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) bf[t][n] = ld4(b + lay.b() + gofs + (int64_t)(16 * t + lr) * Np + 32 * n + 8 * kg);
+    };
+    const float skip = p.d[h];
+    auto form_p = [&](int c) {
+      f32x4_t a[4] = {};
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int t = 0; t < 4; ++t) a[t] = mfma16<bf16_tag>(bf[t][n], cw[n], a[t]);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        if (t < wave) {           // between the tiles: those of wave - 1 .. t + 1
+          const float mid = wave - t == 1 ? 0.f : wave - t == 3 ? m1 + m2 : t == 0 ? m1 : m2;
+          a[t] *= pw[t] * fast_exp2((li + mid) * kLog2e);
+        } else if (t == wave) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int j = 4 * kg + i;
+            const float e = a[t][i] * pw[t][i] * fast_exp2(fminf(li - pl[i], 0.f) * kLog2e);
+            a[t][i] = j < lr ? e : j == lr ? e + skip : 0.f;
           }
-          pr[q] = a;
+        } else {
+          a[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         }
-        const Terms t = split8(pr[0], pr[1]);
-        dst[(3 * tp + 0) * 64] = t.hi;
-        dst[(3 * tp + 1) * 64] = t.mid;
-        dst[(3 * tp + 2) * 64] = t.lo;
       }
-      // ---- C S0
+      uint4* dst = sP[c & 1] + (wave < 2 ? wave : 2 * wave - 2) * 3 * 64 + lane;      // fragments in front: 0, 1, 2, 4
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        if (t == 1 && wave < 2) continue;
+        const Terms f = split8(a[2 * t], a[2 * t + 1]);
+        dst[(3 * t + 0) * 64] = f.hi;
+        dst[(3 * t + 1) * 64] = f.mid;
+        dst[(3 * t + 2) * 64] = f.lo;
+      }
+    };
+    uint4 cf[4][NT];
+    f32x4_t eq[4];
+    auto load_c = [&](int c) {
+      const uint16_t* b = chunk(c);
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int t = 0; t < 4; ++t) cf[t][n] = ld4(b + lay.c() + gofs + (int64_t)(16 * t + lr) * Np + 32 * n + 8 * kg);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) eq[t] = ldf4(numbers(b, kFrom0) + 16 * t + 4 * kg);
+    };
+    load_p(0);
+    load_c(0);
+    load_t(0);
+    __builtin_amdgcn_sched_barrier(0);
+    form_p(0);
+    if constexpr (AHEAD) load_p(1);
+    __builtin_amdgcn_sched_barrier(0);
+    float* yr = k.y + ((chunk0 * kC + 4 * kg) * p.H + h) * lay.Vp + v;
+    const int64_t ys = (int64_t)p.H * lay.Vp;
+    for (int ck = 0; ck < nck; ++ck, yr += kC * ys) {
+      // ---- e^(G_i) C S0
       f32x4_t acc[4] = {};
 #pragma unroll
       for (int n = 0; n < NT; ++n) {
         const Terms t = split8(st[2 * n], st[2 * n + 1]);
 #pragma unroll
-        for (int it = 0; it < 4; ++it) {
-          const uint4 a = *reinterpret_cast<const uint4*>(base + lay.c() + gofs + (int64_t)(16 * it + lr) * Np + 32 * n + 8 * kg);
-          acc[it] = mfma16<bf16_tag>(a, t.lo, acc[it]);
-          acc[it] = mfma16<bf16_tag>(a, t.mid, acc[it]);
-          acc[it] = mfma16<bf16_tag>(a, t.hi, acc[it]);
-        }
+        for (int it = 0; it < 4; ++it) acc[it] = mfma16<bf16_tag>(cf[it][n], t.lo, acc[it]);
+#pragma unroll
+        for (int it = 0; it < 4; ++it) acc[it] = mfma16<bf16_tag>(cf[it][n], t.mid, acc[it]);
+#pragma unroll
+        for (int it = 0; it < 4; ++it) acc[it] = mfma16<bf16_tag>(cf[it][n], t.hi, acc[it]);
       }
 #pragma unroll
-      for (int it = 0; it < 4; ++it) {
-        const f32x4_t le = *reinterpret_cast<const f32x4_t*>(lead + 16 * it + 4 * kg);
-        const float before = it == 0 ? 0.f : it == 1 ? tot[0] : it == 2 ? t01 : t012;
-        acc[it] *= exp4(f32x4_t{before + le[0], before + le[1], before + le[2], before + le[3]});
-      }
-      // the parts of P are there; nobody still reads the other buffer's
+      for (int it = 0; it < 4; ++it) acc[it] *= eq[it];
+      load_c(ck + 1);
+      __builtin_amdgcn_sched_barrier(0);
+      // every part of this chunk's P is there; nobody still reads the other buffer's
       asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
       const uint4* src = sP[ck & 1] + lane;
-      const int len = min(kC, L - (first + ck) * kC);
 #pragma unroll
-      for (int it = 0; it < 4; ++it) {
+      for (int it = 0; it < 4; ++it)
 #pragma unroll
-        for (int tp = 0; tp <= it / 2; ++tp) {
-          const uint4* f = src + ((it < 2 ? it : 2 * it - 2) + tp) * 3 * 64;
-          acc[it] = mfma16<bf16_tag>(f[128], xf[tp], acc[it]);
-          acc[it] = mfma16<bf16_tag>(f[64], xf[tp], acc[it]);
-          acc[it] = mfma16<bf16_tag>(f[0], xf[tp], acc[it]);
+        for (int t = 0; t <= it / 2; ++t) {
+          const uint4* f = src + ((it < 2 ? it : 2 * it - 2) + t) * 3 * 64;
+          acc[it] = mfma16<bf16_tag>(f[128], xf[t], acc[it]);
+          acc[it] = mfma16<bf16_tag>(f[64], xf[t], acc[it]);
+          acc[it] = mfma16<bf16_tag>(f[0], xf[t], acc[it]);
         }
-        if (v < p.V)
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (16 * it + 4 * kg + i < len) yb[((int64_t)ck * kC + 16 * it + 4 * kg + i) * p.H * p.V] = acc[it][i];
-      }
+      for (int it = 0; it < 4; ++it)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) yr[(16 * it + i) * ys] = acc[it][i];
+      update();
+      load_t(ck + 1);
+      __builtin_amdgcn_sched_barrier(0);
+      if constexpr (!AHEAD) load_p(ck + 1);
+      form_p(ck + 1);
+      if constexpr (AHEAD) load_p(ck + 2);
+      __builtin_amdgcn_sched_barrier(0);
     }
-    // ---- S
-    const float decay = fast_exp2(whole * kLog2e);
-    seg_sum += whole;
-    Terms xw[2];
-#pragma unroll
-    for (int t = 0; t < 2; ++t) {
-      f32x4_t a[2];
-#pragma unroll
-      for (int q = 0; q < 2; ++q) {
-        const int tj = 2 * t + q;
-        const f32x4_t dj = *reinterpret_cast<const f32x4_t*>(dt + 16 * tj + 4 * kg);
-        const f32x4_t tr = *reinterpret_cast<const f32x4_t*>(trail + 16 * tj + 4 * kg);
-        const float after = tj == 0 ? t123 : tj == 1 ? t23 : tj == 2 ? tot[3] : 0.f;
-        a[q] = dj * exp4(f32x4_t{after + tr[0], after + tr[1], after + tr[2], after + tr[3]});
-      }
-      const uint32_t xs[4] = {xf[t].x, xf[t].y, xf[t].z, xf[t].w};
-      using E = Elem<bf16_tag>;
-#pragma unroll
-      for (int q = 0; q < 2; ++q) {
-        a[q][0] *= E::lo(xs[2 * q]), a[q][1] *= E::hi(xs[2 * q]);
-        a[q][2] *= E::lo(xs[2 * q + 1]), a[q][3] *= E::hi(xs[2 * q + 1]);
-      }
-      xw[t] = split8(a[0], a[1]);
-    }
-    const uint16_t* bt = base + lay.bt() + gofs + (int64_t)lr * kC + 8 * kg;
-#pragma unroll
-    for (int n = 0; n < 2 * NT; ++n) {
-      st[n] *= decay;
-#pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        const uint4 a = *reinterpret_cast<const uint4*>(bt + (int64_t)16 * n * kC + 32 * t);
-        st[n] = mfma16<bf16_tag>(a, xw[t].lo, st[n]);
-        st[n] = mfma16<bf16_tag>(a, xw[t].mid, st[n]);
-        st[n] = mfma16<bf16_tag>(a, xw[t].hi, st[n]);
-      }
-    }
-  }
-  if constexpr (ENDS) {
-    put_state(seg_at(seg));
-    if (tid == 0 && vg == 0) *log_at(seg) = seg_sum;
-  } else if (active && seg == segs - 1) {
-    put_state(S);
+    if (seg == segs - 1) put_state(S);
   }
 }
 
@@ -542,9 +586,11 @@ struct SsmFinish {
   void* out;                // [rows][ld_out]
   const void* z;            // [rows][ld]
   const void* norm_w;       // [H V]
-  const float* y;           // [rows - row0][H V]
+  const float* y;           // the step's [rows - row0][H V], or (chunked) [chunks][64][H][Vp]
+  const int32_t* qsl;
   int64_t ld_out, ld;
-  int row0, inner, part;    // part: columns normed together
+  int req0, nreq, row0, H, V, pitch;      // pitch: a head's columns in y
+  int part, chunked;        // part: columns normed together
   float eps;
 };
 
@@ -554,7 +600,12 @@ __global__ __launch_bounds__(256) void ssm_finish_kernel(const SsmFinish p) {
   __shared__ float smem[16];
   const int64_t row = p.row0 + blockIdx.x;
   const int c0 = blockIdx.y * p.part;
-  const float* y = p.y + (int64_t)blockIdx.x * p.inner + c0;
+  int64_t at = blockIdx.x;
+  if (p.chunked) {
+    const int r = p.req0 + row_request(p.qsl + p.req0, p.nreq, (int)row), i = (int)row - p.qsl[r];
+    at = chunk_base(p, r) * kC + i;       // (a request's chunks follow each other)
+  }
+  const float* y = p.y + at * p.H * p.pitch;
   const T* z = reinterpret_cast<const T*>(p.z) + row * p.ld + c0;
   float x[MAXC][VEC];
   float ss = 0.f;
@@ -563,7 +614,7 @@ __global__ __launch_bounds__(256) void ssm_finish_kernel(const SsmFinish p) {
     const int c = (threadIdx.x + k * blockDim.x) * VEC;
     if (c >= p.part) continue;
     float g[VEC];
-    Io<float>::ldv<VEC>(y + c, x[k]);
+    Io<float>::ldv<VEC>(y + (int64_t)((c0 + c) / p.V) * p.pitch + (c0 + c) % p.V, x[k]);
     Io<T>::template ldv<VEC>(z + c, g);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
@@ -589,7 +640,7 @@ __global__ __launch_bounds__(256) void ssm_finish_kernel(const SsmFinish p) {
 template <typename T>
 int finish(const SsmFinish& f, int rows, int parts, hipStream_t s) {
   const int al = 16 / sizeof(T), n = f.part;
-  const bool vec = n % 8 == 0 && f.ld_out % al == 0 && f.ld % al == 0 && aligned16(f.out) && aligned16(f.z) && aligned16(f.norm_w);
+  const bool vec = n % 8 == 0 && f.V % 8 == 0 && f.ld_out % al == 0 && f.ld % al == 0 && aligned16(f.out) && aligned16(f.z) && aligned16(f.norm_w);
   const int per = vec ? 8 : 1;
   const dim3 grid(rows, parts), block(n <= 64 * per ? 64 : n <= 128 * per ? 128 : 256);
 #define MI_SF(VEC, MAXC) hipLaunchKernelGGL((ssm_finish_kernel<T, VEC, MAXC>), grid, block, 0, s, f)
@@ -666,11 +717,11 @@ using namespace mi;
 extern "C" int64_t mi_state_space_workspace_bytes(int32_t rows, int32_t num_reqs, int32_t heads, int32_t groups, int32_t state_dim,
                                                   int32_t vdim, int32_t chunked, int dtype) {
   if (rows < 0 || num_reqs < 0 || heads <= 0 || groups <= 0 || state_dim <= 0 || vdim <= 0) return 0;
-  const int64_t y = align256((int64_t)rows * heads * vdim * 4);
-  if (!chunked) return y;
+  if (!chunked) return align256((int64_t)rows * heads * vdim * 4);
   SsmLayout lay;
   if (dtype != MI_DTYPE_BF16 || !ssm_layout(groups, heads, state_dim, vdim, &lay)) return 0;
-  return y + align256(((int64_t)rows / kC + num_reqs) * lay.size() * 2) +
+  const int64_t chunks = (int64_t)rows / kC + num_reqs;
+  return align256(chunks * kC * heads * lay.Vp * 4) + align256(chunks * lay.size() * 2) +
          (int64_t)num_reqs * kMaxSegments * heads * ((int64_t)state_dim * vdim + 1) * 4;
 }
 
@@ -695,26 +746,29 @@ extern "C" int mi_state_space(const mi_state_space_args* a, int32_t row0, int32_
   const SsmParams p{{a->xbc, a->conv_w, a->ring, a->slots, a->query_start_loc, a->seq_lens, a->stride, a->req0, a->taps, ch},
                     a->conv_b, a->dt, a->dt_bias, a->a_log, a->d, a->state, y, row0, H, G, N, V};
   int rc;
+  SsmChunks k{};
   if (!chunked) {
     rc = dtype == MI_DTYPE_BF16 ? step<uint16_t>(p, nreq, s) : step<float>(p, nreq, s);
   } else {
-    SsmChunks k{};
+    const int64_t held = (int64_t)rows / kC + nreq;
     ssm_layout(G, H, N, V, &k.lay);
-    k.ws = (uint16_t*)((char*)workspace + align256((int64_t)rows * inner * 4));
-    k.seg_state = (float*)((char*)k.ws + align256(((int64_t)rows / kC + nreq) * k.lay.size() * 2));
+    k.y = y;
+    k.ws = (uint16_t*)((char*)workspace + align256(held * kC * H * k.lay.Vp * 4));
+    k.seg_state = (float*)((char*)k.ws + align256(held * k.lay.size() * 2));
     k.seg_log = k.seg_state + (int64_t)nreq * kMaxSegments * H * N * V;
-    k.vec = N % 8 == 0 && V % 8 == 0 && a->stride % 8 == 0 && aligned16(a->xbc) && aligned16(a->ring) && aligned16(a->conv_b);
+    k.vec = N % 8 == 0 && V % 8 == 0 && a->stride % 8 == 0 && aligned16(a->xbc) && aligned16(a->ring) && aligned16(a->conv_b) &&
+            aligned16(a->conv_w);
     const int chunks = (max_query_len + kC - 1) / kC;
     const int64_t groups = (int64_t)nreq * H * ((V + 63) / 64);
-    int n = (int)(512 / groups);                           // segments: about two workgroups a CU
+    int n = (int)(256 / groups);                           // segments: a workgroup a CU
     if (n > chunks / 4) n = chunks / 4;
     if (n > kMaxSegments) n = kMaxSegments;
     if (n < 1) n = 1;
     k.seg_chunks = (chunks + n - 1) / n;
     k.nseg = (chunks + k.seg_chunks - 1) / k.seg_chunks;
-    const int blocks = H * ((k.lay.Vp + kPrepCh - 1) / kPrepCh) + 2 * G * ((k.lay.Np + kPrepCh - 1) / kPrepCh) + (H + 3) / 4;
+    const int blocks = H * ((k.lay.Vp + kPrepCh - 1) / kPrepCh) + 2 * G * ((k.lay.Np + kPrepCh - 1) / kPrepCh) + (H + 1) / 2;
     if (blocks > 65535) return MI_ERR_UNSUPPORTED;
-    hipLaunchKernelGGL(ssm_prep_kernel, dim3(chunks, blocks, nreq), dim3(256), 0, s, p, k);
+    hipLaunchKernelGGL(ssm_prep_kernel, dim3(chunks, blocks, nreq), dim3(128), 0, s, p, k);
     rc = launch_status();
     if (rc == MI_OK && k.nseg > 1) rc = launch_scan<true>(p, k, nreq, s);
     if (rc == MI_OK) rc = launch_scan<false>(p, k, nreq, s);
@@ -724,6 +778,7 @@ extern "C" int mi_state_space(const mi_state_space_args* a, int32_t row0, int32_
     rc = dtype == MI_DTYPE_BF16 ? launch_conv_update<uint16_t>(p.in, nreq, s) : launch_conv_update<float>(p.in, nreq, s);
     if (rc != MI_OK) return rc;
   }
-  const SsmFinish f{a->out, a->z, a->norm_w, y, a->out_stride, a->stride, row0, inner, inner / a->norm_groups, a->eps};
+  const SsmFinish f{a->out, a->z, a->norm_w, y, a->query_start_loc, a->out_stride, a->stride, a->req0, nreq, row0, H, V,
+                    chunked ? k.lay.Vp : V, inner / a->norm_groups, chunked, a->eps};
   return dtype == MI_DTYPE_BF16 ? finish<uint16_t>(f, rows, a->norm_groups, s) : finish<float>(f, rows, a->norm_groups, s);
 }
