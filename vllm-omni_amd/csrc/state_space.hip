@@ -150,8 +150,9 @@ __global__ __launch_bounds__(256) void state_step_kernel(const SsmParams p) {
 
 // ------------------------------------------------------------------------------------------------ chunks
 // Workspace of one chunk (bf16): C [G][64][Np], B [G][64][Np], Bt [G][Np][64], Xt [H][Vp][64], then fp32 [H][5][64] (ChunkVec below).
-// Rows past the portion's end are zeros.  Within 32 neighbours along the contiguous dimension the order is that of the matrix
-// cores' accumulators, so that an accumulator pair IS an operand: place 8 q + 4 t + r holds index 16 t + 4 q + r.
+// Rows past the portion's end are zeros.  A matrix lies in fragments of 16 rows x 32 columns as the matrix cores take them, a lane's
+// eight values after the other's: one contiguous KB a load (a lane per row would be 64 cache accesses).  Lane 16 q + row, value 4 t +
+// r holds column 16 t + 4 q + r: the order of an accumulator pair, which so IS an operand.
 struct SsmLayout {
   int G, H, Np, Vp;
   __host__ __device__ int64_t c() const { return 0; }
@@ -192,8 +193,8 @@ constexpr int kPrepCh = 64;     // channels of a prep workgroup: two waves, a th
 // blockIdx.y: first the filters' (kind, head or group, 64 channels) blocks, then two heads' token numbers each
 __global__ __launch_bounds__(128) void ssm_prep_kernel(const SsmParams p, const SsmChunks k) {
   scalar_cache_acquire();
-  // [channel 8 a + j in row 8 j + a][token in operand order]
-  __shared__ __attribute__((aligned(16))) uint16_t tile[kPrepCh][kC + 8];
+  // fragments [token tile][channel half] of the rows, then [channel tile][token half] of the columns, in units of 16 bytes
+  __shared__ uint4 frag[2][8 * 64];
   using E = Elem<bf16_tag>;
   const int r = p.in.req0 + blockIdx.z, ck = blockIdx.x, tid = threadIdx.x;
   const int s0 = p.in.qsl[r], L = p.in.qsl[r + 1] - s0, i0 = ck * kC;
@@ -298,29 +299,43 @@ __global__ __launch_bounds__(128) void ssm_prep_kernel(const SsmParams p, const 
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[u][j] = 0.f;
   }
+  // units are spread over the banks: the low bits of a place take in the bits that the writing threads differ in
+  auto place = [](int u) { return u ^ ((u >> 3) & 1) ^ (((u >> 5) & 1) << 1) ^ (((u >> 4) & 1) << 2); };
+  const int a = tid & 7, q = tid >> 3;
   if (kind != 0) {                                          // rows: 8 neighbours fall into two pieces of 4
-    uint16_t* rows = ws + (kind == 1 ? k.lay.b() : k.lay.c()) + ((int64_t)unit * kC + t) * Np;
-    const int at = (c & ~31) + ((c & 15) >> 2) * 8 + ((c >> 4) & 1) * 4;
-    if (c < Np)
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        *reinterpret_cast<uint2*>(rows + (int64_t)u * Np + at) = make_uint2(E::pack(acc[u][0], acc[u][1]), E::pack(acc[u][2], acc[u][3]));
-        *reinterpret_cast<uint2*>(rows + (int64_t)u * Np + at + 8) = make_uint2(E::pack(acc[u][4], acc[u][5]), E::pack(acc[u][6], acc[u][7]));
-      }
-    if (kind == 2) return;
+    for (int u = 0; u < 4; ++u) {
+      const int unit0 = ((t >> 4) * 2 + (a >> 2)) * 64 + 2 * (a & 1) * 16 + (t & 15) + u;
+      uint2* d0 = reinterpret_cast<uint2*>(&frag[0][place(unit0)]) + ((a >> 1) & 1);
+      uint2* d1 = reinterpret_cast<uint2*>(&frag[0][place(unit0 + 16)]) + ((a >> 1) & 1);
+      *d0 = make_uint2(E::pack(acc[u][0], acc[u][1]), E::pack(acc[u][2], acc[u][3]));
+      *d1 = make_uint2(E::pack(acc[u][4], acc[u][5]), E::pack(acc[u][6], acc[u][7]));
+    }
   }
-  const int at = (t & ~31) + ((t & 15) >> 2) * 8 + ((t >> 4) & 1) * 4;      // four neighbours stay together
+  if (kind != 2) {
 #pragma unroll
-  for (int j = 0; j < 8; ++j)
-    *reinterpret_cast<uint2*>(&tile[8 * j + (tid & 7)][at]) = make_uint2(E::pack(acc[0][j], acc[1][j]), E::pack(acc[2][j], acc[3][j]));
+    for (int j = 0; j < 8; ++j) {
+      const int u = ((a >> 1) * 2 + (q >> 3)) * 64 + (q & 3) * 16 + 8 * (a & 1) + j;
+      *(reinterpret_cast<uint2*>(&frag[1][place(u)]) + ((q >> 2) & 1)) =
+          make_uint2(E::pack(acc[0][j], acc[1][j]), E::pack(acc[2][j], acc[3][j]));
+    }
+  }
   __syncthreads();
-  uint16_t* cols = ws + (kind == 0 ? k.lay.xt() : k.lay.bt()) + (int64_t)unit * width * kC;
+  if (kind != 0) {
+    uint4* dst = reinterpret_cast<uint4*>(ws + (kind == 1 ? k.lay.b() : k.lay.c()) + (int64_t)unit * kC * Np);
 #pragma unroll
-  for (int n = tid; n < kPrepCh * 8; n += 128) {
-    const int cc = n >> 3, piece = (n & 7) * 8;
-    if (blk * kPrepCh + cc < width)
-      *reinterpret_cast<uint4*>(cols + (int64_t)(blk * kPrepCh + cc) * kC + piece) =
-          *reinterpret_cast<const uint4*>(&tile[8 * (cc & 7) + (cc >> 3)][piece]);
+    for (int m = 0; m < 4; ++m) {
+      const int u = tid + 128 * m, f = u >> 6;              // fragment (token tile f / 2, half f % 2)
+      if (blk * kPrepCh + 32 * (f & 1) < Np) dst[((f >> 1) * (Np / 32) + blk * 2 + (f & 1)) * 64 + (u & 63)] = frag[0][place(u)];
+    }
+  }
+  if (kind != 2) {
+    uint4* dst = reinterpret_cast<uint4*>(ws + (kind == 0 ? k.lay.xt() : k.lay.bt()) + ((int64_t)unit * width + blk * kPrepCh) * kC);
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      const int u = tid + 128 * m;                          // fragment (channel tile f / 2, token half f % 2)
+      if (blk * kPrepCh + 16 * (u >> 7) < width) dst[u] = frag[1][place(u)];
+    }
   }
 }
 
@@ -353,7 +368,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
   scalar_cache_acquire();
   constexpr int Np = 32 * NT;
   constexpr bool AHEAD = NT <= 4;          // (a state of 256 rows leaves no registers for the operands of P)
-  __shared__ uint4 sP[ENDS ? 1 : 2][ENDS ? 1 : 6 * 3 * 64];      // fragments (row tile 0..3, 32 columns up to it), three terms
+  __shared__ uint4 sP[ENDS ? 1 : 2][ENDS ? 1 : 4 * 2 * 3 * 64];      // fragments (row tile, 32 columns), three terms each
   // the heads of a group, and the column groups of a head, on one XCD (workgroups go to the 8 XCDs in turn)
   const int work = p.H * vgroups, each = (work + 7) / 8;
   const int item = (blockIdx.x & 7) * each + (blockIdx.x >> 3);
@@ -409,7 +424,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
   const int64_t gofs = (int64_t)grp * kC * Np;
   auto chunk = [&](int c) { return base + min(c, nck - 1) * lay.size(); };
   auto numbers = [&](const uint16_t* b, int which) { return reinterpret_cast<const float*>(b + lay.vec()) + ((int64_t)h * 5 + which) * kC; };
-  auto ld4 = [](const uint16_t* a) { return *reinterpret_cast<const uint4*>(a); };
+  auto ld4 = [&](const uint16_t* a) { return reinterpret_cast<const uint4*>(a)[lane]; };      // a fragment
   auto ldf4 = [](const float* a) { return *reinterpret_cast<const f32x4_t*>(a); };
 
   // ---- S <- e^(G_C) S + sum_j B_j (weight_j x_j)^T
@@ -419,16 +434,16 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
   auto load_t = [&](int c) {
     const uint16_t* b = chunk(c);
 #pragma unroll
-    for (int t = 0; t < 2; ++t) xf[t] = ld4(b + lay.xt() + ((int64_t)h * lay.Vp + v) * kC + 32 * t + 8 * kg);
+    for (int t = 0; t < 2; ++t) xf[t] = ld4(b + lay.xt() + ((int64_t)h * lay.Vp + vt * 16) * kC + t * 512);
     const float* w = numbers(b, kToEnd);
 #pragma unroll
     for (int t = 0; t < 4; ++t) wx[t] = ldf4(w + 16 * t + 4 * kg);
     decay = numbers(b, kFrom0)[kC - 1];
-    const uint16_t* bt = b + lay.bt() + gofs + (int64_t)lr * kC + 8 * kg;
+    const uint16_t* bt = b + lay.bt() + gofs;
 #pragma unroll
     for (int n = 0; n < 2 * NT; ++n)
 #pragma unroll
-      for (int t = 0; t < 2; ++t) tf[n][t] = ld4(bt + (int64_t)16 * n * kC + 32 * t);
+      for (int t = 0; t < 2; ++t) tf[n][t] = ld4(bt + (2 * n + t) * 512);
   };
   auto update = [&]() {
     using E = Elem<bf16_tag>;
@@ -477,11 +492,11 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
 #pragma unroll
       for (int t = 0; t < 4; ++t) pw[t] = ldf4(numbers(b, t < wave ? kTail : kDt) + 16 * t + 4 * kg);
 #pragma unroll
-      for (int n = 0; n < NT; ++n) cw[n] = ld4(b + lay.c() + gofs + (int64_t)(16 * wave + lr) * Np + 32 * n + 8 * kg);
+      for (int n = 0; n < NT; ++n) cw[n] = ld4(b + lay.c() + gofs + (wave * NT + n) * 512);
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int n = 0; n < NT; ++n) bf[t][n] = ld4(b + lay.b() + gofs + (int64_t)(16 * t + lr) * Np + 32 * n + 8 * kg);
+        for (int n = 0; n < NT; ++n) bf[t][n] = ld4(b + lay.b() + gofs + (t * NT + n) * 512);
     };
     const float skip = p.d[h];
     auto form_p = [&](int c) {
@@ -490,26 +505,21 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
       for (int n = 0; n < NT; ++n)
 #pragma unroll
         for (int t = 0; t < 4; ++t) a[t] = mfma16<bf16_tag>(bf[t][n], cw[n], a[t]);
+      // no branches: what lies behind the diagonal is dropped by selects
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        if (t < wave) {           // between the tiles: those of wave - 1 .. t + 1
-          const float mid = wave - t == 1 ? 0.f : wave - t == 3 ? m1 + m2 : t == 0 ? m1 : m2;
-          a[t] *= pw[t] * fast_exp2((li + mid) * kLog2e);
-        } else if (t == wave) {
+        const float mid = wave - t <= 1 ? 0.f : wave - t == 3 ? m1 + m2 : t == 0 ? m1 : m2;      // the tiles between
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int j = 4 * kg + i;
-            const float e = a[t][i] * pw[t][i] * fast_exp2(fminf(li - pl[i], 0.f) * kLog2e);
-            a[t][i] = j < lr ? e : j == lr ? e + skip : 0.f;
-          }
-        } else {
-          a[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int i = 0; i < 4; ++i) {
+          const int below = 16 * (wave - t) + lr - (4 * kg + i);      // row - column
+          const float e = a[t][i] * pw[t][i] * fast_exp2((t == wave ? li - pl[i] : li + mid) * kLog2e);
+          a[t][i] = below > 0 ? e : 0.f;
+          if (below == 0) a[t][i] = e + skip;
         }
       }
-      uint4* dst = sP[c & 1] + (wave < 2 ? wave : 2 * wave - 2) * 3 * 64 + lane;      // fragments in front: 0, 1, 2, 4
+      uint4* dst = sP[c & 1] + wave * 6 * 64 + lane;
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
-        if (t == 1 && wave < 2) continue;
         const Terms f = split8(a[2 * t], a[2 * t + 1]);
         dst[(3 * t + 0) * 64] = f.hi;
         dst[(3 * t + 1) * 64] = f.mid;
@@ -523,7 +533,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
 #pragma unroll
       for (int n = 0; n < NT; ++n)
 #pragma unroll
-        for (int t = 0; t < 4; ++t) cf[t][n] = ld4(b + lay.c() + gofs + (int64_t)(16 * t + lr) * Np + 32 * n + 8 * kg);
+        for (int t = 0; t < 4; ++t) cf[t][n] = ld4(b + lay.c() + gofs + (t * NT + n) * 512);
 #pragma unroll
       for (int t = 0; t < 4; ++t) eq[t] = ldf4(numbers(b, kFrom0) + 16 * t + 4 * kg);
     };
@@ -537,6 +547,15 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
     float* yr = k.y + ((chunk0 * kC + 4 * kg) * p.H + h) * lay.Vp + v;
     const int64_t ys = (int64_t)p.H * lay.Vp;
     for (int ck = 0; ck < nck; ++ck, yr += kC * ys) {
+      // every part of this chunk's P is there; nobody still reads the other buffer's
+      asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+      const uint4* src = sP[ck & 1] + lane;
+      uint4 pf[6][3];                     // row tiles 0..3 of the first 32 columns, 2 and 3 of the others
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+#pragma unroll
+        for (int z = 0; z < 3; ++z) pf[q][z] = src[(q * 6 + z) * 64];
+      __builtin_amdgcn_sched_barrier(0);
       // ---- e^(G_i) C S0
       f32x4_t acc[4] = {};
 #pragma unroll
@@ -553,18 +572,18 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
       for (int it = 0; it < 4; ++it) acc[it] *= eq[it];
       load_c(ck + 1);
       __builtin_amdgcn_sched_barrier(0);
-      // every part of this chunk's P is there; nobody still reads the other buffer's
-      asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-      const uint4* src = sP[ck & 1] + lane;
 #pragma unroll
-      for (int it = 0; it < 4; ++it)
+      for (int q = 4; q < 6; ++q)
 #pragma unroll
-        for (int t = 0; t <= it / 2; ++t) {
-          const uint4* f = src + ((it < 2 ? it : 2 * it - 2) + t) * 3 * 64;
-          acc[it] = mfma16<bf16_tag>(f[128], xf[t], acc[it]);
-          acc[it] = mfma16<bf16_tag>(f[64], xf[t], acc[it]);
-          acc[it] = mfma16<bf16_tag>(f[0], xf[t], acc[it]);
-        }
+        for (int z = 0; z < 3; ++z) pf[q][z] = src[((q - 2) * 6 + 3 + z) * 64];
+#pragma unroll
+      for (int z = 2; z >= 0; --z)
+#pragma unroll
+        for (int it = 0; it < 4; ++it) acc[it] = mfma16<bf16_tag>(pf[it][z], xf[0], acc[it]);
+#pragma unroll
+      for (int z = 2; z >= 0; --z)
+#pragma unroll
+        for (int it = 2; it < 4; ++it) acc[it] = mfma16<bf16_tag>(pf[it + 2][z], xf[1], acc[it]);
 #pragma unroll
       for (int it = 0; it < 4; ++it)
 #pragma unroll
