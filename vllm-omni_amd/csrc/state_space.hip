@@ -343,12 +343,16 @@ __global__ __launch_bounds__(128) void ssm_prep_kernel(const SsmParams p, const 
 struct Terms {
   uint4 hi, mid, lo;
 };
+// (cut off, not rounded: 8 + 8 + 8 bits, and a pair of upper halves is one instruction)
 __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& mid, uint32_t& lo) {
-  using E = Elem<bf16_tag>;
-  hi = E::pack(a, b);
-  const float a1 = a - E::lo(hi), b1 = b - E::hi(hi);
-  mid = E::pack(a1, b1);
-  lo = E::pack(a1 - E::lo(mid), b1 - E::hi(mid));
+  auto bits = [](float x) { return __builtin_bit_cast(uint32_t, x); };
+  auto cut = [&](float x) { return __builtin_bit_cast(float, bits(x) & 0xffff0000u); };
+  auto upper = [&](float x, float y) { return __builtin_amdgcn_perm(bits(y), bits(x), 0x07060302); };
+  hi = upper(a, b);
+  a -= cut(a), b -= cut(b);
+  mid = upper(a, b);
+  a -= cut(a), b -= cut(b);
+  lo = upper(a, b);
 }
 __device__ __forceinline__ Terms split8(const f32x4_t& a, const f32x4_t& b) {
   Terms t;
@@ -374,9 +378,10 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
   const int item = (blockIdx.x & 7) * each + (blockIdx.x >> 3);
   if ((int)(blockIdx.x >> 3) >= each || item >= work) return;
   const int h = item / vgroups, vg = item % vgroups, r = p.in.req0 + blockIdx.y, seg = blockIdx.z;
-  const int s0 = p.in.qsl[r], L = p.in.qsl[r + 1] - s0;
+  // (scalars, so that the operands' addresses are)
+  const int s0 = __builtin_amdgcn_readfirstlane(p.in.qsl[r]), L = __builtin_amdgcn_readfirstlane(p.in.qsl[r + 1]) - s0;
   if (L <= 0) return;
-  const int start = p.in.seq_lens[r] - L, all = (L + kC - 1) / kC, segs = (all + k.seg_chunks - 1) / k.seg_chunks;
+  const int start = __builtin_amdgcn_readfirstlane(p.in.seq_lens[r]) - L, all = (L + kC - 1) / kC, segs = (all + k.seg_chunks - 1) / k.seg_chunks;
   if (ENDS ? seg >= segs - 1 : seg >= segs) return;
   const int first = seg * k.seg_chunks, nck = min(k.seg_chunks, all - first);
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, kg = lane >> 4;
@@ -419,13 +424,14 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
   } else {
     for (int n = 0; n < seg; ++n) add_state(seg_at(n), n ? fast_exp2(*log_at(n) * kLog2e) : 0.f);
   }
-  const int64_t chunk0 = chunk_base(p.in, r) + first;
+  const int64_t chunk0 = (s0 - __builtin_amdgcn_readfirstlane(p.in.qsl[p.in.req0])) / kC + (r - p.in.req0) + first;
   const uint16_t* base = k.ws + chunk0 * lay.size();
   const int64_t gofs = (int64_t)grp * kC * Np;
   auto chunk = [&](int c) { return base + min(c, nck - 1) * lay.size(); };
   auto numbers = [&](const uint16_t* b, int which) { return reinterpret_cast<const float*>(b + lay.vec()) + ((int64_t)h * 5 + which) * kC; };
-  auto ld4 = [&](const uint16_t* a) { return reinterpret_cast<const uint4*>(a)[lane]; };      // a fragment
-  auto ldf4 = [](const float* a) { return *reinterpret_cast<const f32x4_t*>(a); };
+  const uint32_t lofs = lane * 16, kofs = kg * 16;
+  auto ld4 = [&](const uint16_t* a) { return *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(a) + lofs); };      // a fragment
+  auto ldf4 = [&](const float* a) { return *reinterpret_cast<const f32x4_t*>(reinterpret_cast<const char*>(a) + kofs); };      // values 4 kg ..
 
   // ---- S <- e^(G_C) S + sum_j B_j (weight_j x_j)^T
   uint4 tf[2 * NT][2], xf[2];
@@ -437,7 +443,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
     for (int t = 0; t < 2; ++t) xf[t] = ld4(b + lay.xt() + ((int64_t)h * lay.Vp + vt * 16) * kC + t * 512);
     const float* w = numbers(b, kToEnd);
 #pragma unroll
-    for (int t = 0; t < 4; ++t) wx[t] = ldf4(w + 16 * t + 4 * kg);
+    for (int t = 0; t < 4; ++t) wx[t] = ldf4(w + 16 * t);
     decay = numbers(b, kFrom0)[kC - 1];
     const uint16_t* bt = b + lay.bt() + gofs;
 #pragma unroll
@@ -488,9 +494,9 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
       const uint16_t* b = chunk(c);
       const float* lead = numbers(b, kLead);
       li = lead[16 * wave + lr], m1 = lead[31], m2 = lead[47];
-      pl = ldf4(lead + 16 * wave + 4 * kg);
+      pl = ldf4(lead + 16 * wave);
 #pragma unroll
-      for (int t = 0; t < 4; ++t) pw[t] = ldf4(numbers(b, t < wave ? kTail : kDt) + 16 * t + 4 * kg);
+      for (int t = 0; t < 4; ++t) pw[t] = ldf4(numbers(b, t < wave ? kTail : kDt) + 16 * t);
 #pragma unroll
       for (int n = 0; n < NT; ++n) cw[n] = ld4(b + lay.c() + gofs + (wave * NT + n) * 512);
 #pragma unroll
@@ -535,7 +541,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
 #pragma unroll
         for (int t = 0; t < 4; ++t) cf[t][n] = ld4(b + lay.c() + gofs + (t * NT + n) * 512);
 #pragma unroll
-      for (int t = 0; t < 4; ++t) eq[t] = ldf4(numbers(b, kFrom0) + 16 * t + 4 * kg);
+      for (int t = 0; t < 4; ++t) eq[t] = ldf4(numbers(b, kFrom0) + 16 * t);
     };
     load_p(0);
     load_c(0);
@@ -544,8 +550,9 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
     form_p(0);
     if constexpr (AHEAD) load_p(1);
     __builtin_amdgcn_sched_barrier(0);
-    float* yr = k.y + ((chunk0 * kC + 4 * kg) * p.H + h) * lay.Vp + v;
     const int64_t ys = (int64_t)p.H * lay.Vp;
+    float* yr = k.y + chunk0 * kC * ys + (int64_t)h * lay.Vp + vt * 16;
+    const uint32_t yofs = (uint32_t)(4 * kg * ys + lr) * 4;
     for (int ck = 0; ck < nck; ++ck, yr += kC * ys) {
       // every part of this chunk's P is there; nobody still reads the other buffer's
       asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
@@ -587,7 +594,7 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmParams p, con
 #pragma unroll
       for (int it = 0; it < 4; ++it)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) yr[(16 * it + i) * ys] = acc[it][i];
+        for (int i = 0; i < 4; ++i) *reinterpret_cast<float*>(reinterpret_cast<char*>(yr + (16 * it + i) * ys) + yofs) = acc[it][i];
       update();
       load_t(ck + 1);
       __builtin_amdgcn_sched_barrier(0);
