@@ -31,7 +31,7 @@ CONFIGS = {
     "odd": model([(attn(3, 1, 21, 6, 2), moe(5, 1, 21)), (mamba(3, 3, 19, 13, 1, 1), moe(7, 2, 33)), (mamba(5, 1, 33, 21, 2, 5), None)], (0, 3, 2),
                  vocab=89, width=100, mult=1.0, cap=2.5),
     # a real layer's head sizes, the loop at the end and once only, many experts, parts of the norm that cross heads
-    "wide": model([(mamba(8, 2, 128, 64, 4, 2), moe(40, 4, 64)), (attn(16, 2, 128, 64, 4, base=50000.0), moe(8, 8, 128)),
+    "wide": model([(mamba(8, 2, 128, 64, 4, 2), moe(40, 4, 64)), (attn(16, 2, 128, 64, 4, base=20000.0), moe(8, 8, 128)),
                    (mamba(4, 2, 64, 128, 4, 8), moe(16, 2, 128)), (attn(8, 8, 64, 16, 4), None)], (2, 4, 1), vocab=200, width=256, mult=0.4),
     # heads past the matrix-core attention's sizes, long filters, a state of many rows, a loop over the first layer
     "tall": model([(mamba(3, 1, 200, 80, 6, 1), moe(3, 2, 64)), (attn(2, 1, 160, 160, 6), moe(4, 1, 48)), (mamba(1, 1, 72, 144, 4, 2), None)],

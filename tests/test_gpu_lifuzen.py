@@ -135,7 +135,7 @@ def test_mixed_batches_pages_and_slots_used_again(dev, dtype, wait):
 def test_the_first_tokens_and_one_far_back(dev, dtype):
     """one early token changed: the rows behind it move as the plain forward says, the rows in front of it not at all, in prompts
     and in decoding, at page and chunk borders"""
-    cfg = lm.model([(lm.attn(6, 2, 48, 24, 4, 0.5), lm.moe(5, 2, 40)), (lm.mamba(4, 2, 32, 32, 4, 2), None)], (0, 2, 2))
+    cfg = lm.model([(lm.attn(6, 2, 48, 24, 4, 0.5), lm.moe(5, 2, 40)), (lm.mamba(4, 2, 40, 32, 4, 1), None)], (0, 2, 2))
     w = weights(cfg, dtype, 9)
     a = lm.random_tokens(cfg, 130, 5)
     e = engine(cfg, w, dtype, tokens=1024)

@@ -17,7 +17,7 @@ def test_stream_norm2(dev, dtype, width):
     """the multiplied add, a pass's vector and the embedding output, experts' rows (weighted or not), both norms, a stream that starts"""
     from vllm_omni_amd import ops
 
-    rows, top, eps, mult = 5, 3, 3e-2, 0.3             # eps of the order of the rows' mean square: a misplaced one shows
+    rows, top, eps, mult = 5, 3, 3e-2, 0.45            # eps of the order of the rows' mean square: a misplaced one shows
     x, y = rnd(rows, width, std=0.2, seed=1), rnd(rows, width, dtype=dtype, std=0.3, seed=2)
     w1, w2, step = (rnd(width, dtype=dtype, std=0.3, seed=3 + i) for i in range(3))
     table, ids = rnd(30, width, dtype=dtype, std=0.2, seed=6), torch.tensor([3, 29, 0, 30, -1])
@@ -129,7 +129,7 @@ class ConvRopeCase:
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("sizes", [(6, 2, 64, 64, 32, 4), (3, 1, 21, 64, 6, 2), (4, 4, 48, 64, 20, 4), (2, 2, 128, 128, 128, 4), (3, 1, 96, 128, 0, 1),
+@pytest.mark.parametrize("sizes", [(6, 1, 64, 64, 32, 4), (3, 1, 21, 64, 6, 2), (4, 4, 48, 64, 20, 4), (2, 2, 128, 128, 128, 4), (3, 1, 96, 128, 0, 1),
                                    (40, 8, 40, 64, 40, 3), (2, 1, 160, 160, 160, 6), (5, 5, 33, 40, 32, 4), (1, 1, 300, 304, 100, 4)],
                          ids=lambda s: "x".join(map(str, s)))
 def test_conv_rope_cache(dev, dtype, sizes):
@@ -299,7 +299,7 @@ def state_tol(dtype):
     return dict(rtol=4e-3, atol=4e-3) if dtype == torch.bfloat16 else dict(rtol=1e-4, atol=1e-4)
 
 
-SSM = [(4, 2, 32, 32, 4, 2), (6, 2, 24, 40, 4, 3), (3, 3, 19, 13, 1, 1), (5, 1, 33, 21, 2, 5), (8, 2, 128, 64, 4, 2), (2, 1, 64, 128, 4, 8),
+SSM = [(4, 2, 32, 48, 4, 1), (6, 2, 24, 40, 4, 3), (3, 3, 19, 13, 1, 1), (5, 1, 33, 21, 2, 5), (8, 2, 128, 64, 4, 2), (2, 1, 64, 128, 4, 8),
        (2, 2, 200, 80, 6, 1), (1, 1, 72, 144, 4, 2), (3, 1, 256, 16, 3, 1), (2, 1, 300, 20, 4, 2), (2, 1, 16, 256, 4, 16)]
 
 
@@ -388,7 +388,7 @@ def test_one_early_token_reaches_the_end(dev):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("t,width,experts,top,ff", [(7, 96, 6, 2, 40), (70, 128, 8, 3, 128), (33, 100, 5, 1, 21), (300, 320, 9, 4, 96),
                                                     (90, 256, 40, 4, 64), (20, 128, 130, 16, 16), (3, 200, 4, 4, 24),
-                                                    (1500, 72, 20, 2, 16), (1400, 256, 4, 2, 256), (1, 192, 12, 1, 72)])
+                                                    (1500, 72, 20, 2, 16), (1400, 256, 4, 2, 256), (1, 176, 11, 1, 72)])
 def test_routed_experts(dev, dtype, t, width, experts, top, ff):
     """sigmoid scores that scale what an expert reads, squared relu, no gate; widely spread router logits"""
     from vllm_omni_amd import ops

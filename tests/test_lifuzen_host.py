@@ -191,16 +191,16 @@ def test_argument_validation_without_gpu():
     assert cr(dim=1100, head_dim=1100, x_stride=8000, q_stride=8000, rot_dims=0) == no
 
     sp = {n: p for n, t in _C.StateSpaceArgs._fields_ if t is ctypes.c_void_p}
-    sp.update(stride=512, out_stride=128, num_reqs=1, heads=4, groups=2, state_dim=32, vdim=32, taps=4, norm_groups=2, eps=1e-6)
+    sp.update(stride=512, out_stride=160, num_reqs=1, heads=4, groups=2, state_dim=24, vdim=40, taps=4, norm_groups=4, eps=1e-6)
     ss = lambda chunked=0, size=1 << 30, dt=bf, **kw: lib.mi_state_space(ctypes.byref(_C.StateSpaceArgs(**{**sp, **kw})), 0, 2, 2, chunked, p,   # noqa: E731
                                                                         size, dt, None)
-    for kw in (dict(state=None), dict(conv_b=None), dict(groups=3), dict(norm_groups=3), dict(taps=0), dict(stride=255), dict(out_stride=127)):
+    for kw in (dict(state=None), dict(conv_b=None), dict(groups=3), dict(norm_groups=3), dict(taps=0), dict(stride=255), dict(out_stride=159)):
         assert ss(**kw) == bad and ss(chunked=1, **kw) == bad, kw
     assert ss(chunked=1, dt=_C.MI_DTYPE_F32) == no and ss(chunked=1, state_dim=300, stride=4096) == no and ss(dt=_C.MI_DTYPE_F16) == no
     for chunked in (0, 1):
-        need = lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 32, 32, chunked, bf)
+        need = lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 24, 40, chunked, bf)
         assert need > 0 and ss(chunked, need - 1) == ws
-    assert lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 32, 32, 1, _C.MI_DTYPE_F32) == 0
+    assert lib.mi_state_space_workspace_bytes(2, 1, 4, 2, 24, 40, 1, _C.MI_DTYPE_F32) == 0
 
     def experts(form, weights, pair=False):
         if pair:

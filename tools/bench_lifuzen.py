@@ -24,7 +24,7 @@ def lifuzen_config(s):
                                            "rot": {"base": 500000.0, "dims": DIM // 2}}}
     moe = {"kind": "moe", "router": {"experts": 64, "top": 8}, "expert": {"ff": s["ff"] // 8}}
     cfg = config_from_hf({"architecture": "Lifuzen", "vocab": VOCAB, "width": s["width"], "norm": {"eps": 1e-6}, "residual_mult": 0.5,
-                          "logit_softcap": 30.0, "layers": [dict(m, mlp=moe) for m in (ssm, attn) * 3],
+                          "logit_softcap": 25.0, "layers": [dict(m, mlp=moe) for m in (ssm, attn) * 3],
                           "loop": {"start": 2, "stop": 4, "times": 2}})
     assert len(cfg.runs) == LAYERS
     return cfg

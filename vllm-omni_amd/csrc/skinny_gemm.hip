@@ -1042,8 +1042,9 @@ int launch_grouped_skinny(const GroupedGemmArgs& a, hipStream_t s) {
     if (chain > n_tiles || n_tiles % chain) chain = 1;
   }
   p.chain = chain;
-  const dim3 grid(n_tiles / chain, a.max_tiles);
   const int rpt = a.rows_per_tile;
+  p.by_xcd = rpt >= 128;      // prefill chunks: a row tile's rows outweigh its expert's weights
+  const dim3 grid(n_tiles / chain, (a.max_tiles + 7) / 8 * 8);
   if (a.dtype == MI_DTYPE_BF16)
     return gated ? launch_grouped_rows<bf16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<bf16_tag, false>(p, grid, rpt, s);
   return gated ? launch_grouped_rows<f16_tag, true>(p, grid, rpt, s) : launch_grouped_rows<f16_tag, false>(p, grid, rpt, s);

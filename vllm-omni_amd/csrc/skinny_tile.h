@@ -58,7 +58,9 @@ struct SkinnyParams {
   // GATED: 0 = silu(gate) * up; > 0 = the clamped form g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit)
   float glu_alpha = 0.f, glu_limit = 0.f;
   int32_t relu_squared = 0;    // not GATED, S == 1: the output is relu(sum)^2
-  // GROUPED (sparse-MoE expert GEMMs, fused_moe.hip): grid.y = one tile of `rpt` token rows that share one expert
+  // GROUPED (sparse-MoE expert GEMMs, fused_moe.hip): grid.y = one tile of `rpt` token rows that share one expert; by_xcd: tiles
+  // dealt to the XCDs in ranges instead
+  int32_t by_xcd = 0;
   const int32_t* row_map;      // [max_rows] pair index per row or -1
   const int32_t* tile_expert;  // [max_tiles]
   const int32_t* num_tiles;    // [1]
@@ -217,12 +219,23 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
   const int tid = threadIdx.x, lane = tid & 63;
   const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const uint16_t* wbase = p.w;
-  int m0 = 0, wg = wg_linear;
+  int m0 = 0, wg = wg_linear, row_tile = 0;
   if constexpr (GROUPED) {
     // the maps were written by the alignment kernel just before this launch: keep their reads off a stale scalar cache
     scalar_cache_acquire();
-    if ((int)blockIdx.y >= p.num_tiles[0]) return;   // whole workgroup, before any barrier
-    wbase += (int64_t)p.tile_expert[blockIdx.y] * p.w_expert_stride;
+    if (p.by_xcd) {
+      // workgroup ids go round-robin over the 8 XCDs: hand every XCD a contiguous range of the (row tile, weight tiles) that are
+      // live, so that the weight tiles of a row tile read its rows through one L2 (the grid holds a multiple of 8 workgroups)
+      const int nx = gridDim.x, work = p.num_tiles[0] * nx, each = (work + 7) >> 3;
+      const int id = blockIdx.y * nx + blockIdx.x, slot = id >> 3, item = (id & 7) * each + slot;
+      if (slot >= each || item >= work) return;      // whole workgroup, before any barrier
+      row_tile = item / nx;
+      wg = item - row_tile * nx;
+    } else {
+      row_tile = blockIdx.y;
+      if (row_tile >= p.num_tiles[0]) return;        // whole workgroup, before any barrier
+    }
+    wbase += (int64_t)p.tile_expert[row_tile] * p.w_expert_stride;
   } else {
     // More rows than one image holds (16 MT): RB row blocks per (tile, slice).  Workgroup ids go round-robin over the 8
     // XCDs, so the row blocks of one work item are dealt 8 ids apart: id = 8 RB q + 8 rb + j <-> item u = 8 q + j, row
@@ -256,7 +269,7 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
       if (q < XI) {
         int m = m0 + row < p.M ? m0 + row : p.M - 1;   // rows past M repeat the last one; never stored
         if constexpr (GROUPED) {   // row of the tile -> row of the source matrix (padding rows read some valid row)
-          const int R = blockIdx.y * p.rpt + (row < p.rpt ? row : 0);
+          const int R = row_tile * p.rpt + (row < p.rpt ? row : 0);
           if (p.gather_div > 0) {
             const int pr = p.row_map[R];
             m = (pr < 0 ? 0 : pr) / p.gather_div;
@@ -387,7 +400,7 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
     for (int j = 0; j < MTW; ++j) {
       int m = m0 + 16 * (mh * MTW + j) + r16;
       if (m >= p.M) continue;
-      if constexpr (GROUPED) m += blockIdx.y * p.rpt;
+      if constexpr (GROUPED) m += row_tile * p.rpt;
       float v[4], gq[4], uq[4];
       finish_quad<Tag>(p, acc[0][j], m, n, zero4, gq);
       finish_quad<Tag>(p, acc[1][j], m, p.N + n, zero4, uq);
@@ -416,7 +429,7 @@ __device__ __forceinline__ void skinny_tile(const SkinnyParams& p, const int wg_
     for (int j = 0; j < MTW; ++j) {
       int m = m0 + 16 * (mh * MTW + j) + r16;
       if (m >= p.M) continue;
-      if constexpr (GROUPED) m += blockIdx.y * p.rpt;
+      if constexpr (GROUPED) m += row_tile * p.rpt;
       if (!slabs) {
         float v[4];
         if constexpr (GROUPED) {
