@@ -1033,7 +1033,8 @@ int launch_grouped_skinny(const GroupedGemmArgs& a, hipStream_t s) {
     if (e && atoi(e) > 0) {
       chain = atoi(e);
     } else {
-      for (int c = n_tiles; c >= 1; --c)
+      // (tall row tiles: few, so that a row tile's workgroups run at the same time and share its rows in their XCD's L2)
+      for (int c = a.rows_per_tile >= 128 && n_tiles > 4 ? 4 : n_tiles; c >= 1; --c)
         if (n_tiles % c == 0 && (int64_t)(n_tiles / c) * a.max_tiles >= 512) {
           chain = c;
           break;
