@@ -424,36 +424,59 @@ __global__ __launch_bounds__(256) void stream_norm2_kernel(const StreamParams p)
   const bool known = id >= 0 && id < p.vocab;   // an id outside the table reads as a zero row
   const T* er = reinterpret_cast<const T*>(p.table) + (known ? id : 0) * p.width;
   float* xr = p.x + row * p.x_stride;
-  float x[MAXC][VEC];
+  float x[MAXC][VEC] = {};
+  // slabs and experts' rows four at a time: their loads are on their way together (past the last one: it again, times zero)
+  if (p.split) {
+    const float* yp = reinterpret_cast<const float*>(p.y) + row * p.y_stride;
+    for (int s0 = 0; s0 < p.split; s0 += 4)
+#pragma unroll
+      for (int k = 0; k < MAXC; ++k) {
+        const int c = (threadIdx.x + k * 256) * VEC;
+        if (c >= p.width) continue;
+        float t[4][VEC];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) Io<float>::ldv<VEC>(yp + c + (int64_t)min(s0 + u, p.split - 1) * p.rows * p.y_stride, t[u]);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) x[k][j] += s0 + u < p.split ? t[u][j] : 0.f;
+      }
+  } else if (p.y) {
+#pragma unroll
+    for (int k = 0; k < MAXC; ++k) {
+      const int c = (threadIdx.x + k * 256) * VEC;
+      if (c < p.width) Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.y) + row * p.y_stride + c, x[k]);
+    }
+  }
+  for (int j0 = 0; j0 < p.top; j0 += 4) {
+    const T* src[4];
+    float w[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int64_t pair = row * p.top + min(j0 + u, p.top - 1);
+      src[u] = reinterpret_cast<const T*>(p.part) + (p.row_of_pair ? p.row_of_pair[pair] : pair) * p.part_stride;
+      w[u] = j0 + u >= p.top ? 0.f : p.weights ? p.weights[pair] : 1.f;
+    }
+#pragma unroll
+    for (int k = 0; k < MAXC; ++k) {
+      const int c = (threadIdx.x + k * 256) * VEC;
+      if (c >= p.width) continue;
+      float t[4][VEC];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) Io<T>::template ldv<VEC>(src[u] + c, t[u]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) x[k][j] += w[u] != 0.f ? w[u] * t[u][j] : 0.f;
+    }
+  }
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < MAXC; ++k) {
     const int c = (threadIdx.x + k * 256) * VEC;
     if (c >= p.width) continue;
     float t[VEC];
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) x[k][j] = 0.f;
     if (p.y) {
-      if (p.split) {
-        const float* yp = reinterpret_cast<const float*>(p.y) + row * p.y_stride + c;
-        for (int s = 0; s < p.split; ++s) {
-          Io<float>::ldv<VEC>(yp + (int64_t)s * p.rows * p.y_stride, t);
-#pragma unroll
-          for (int j = 0; j < VEC; ++j) x[k][j] += t[j];
-        }
-      } else {
-        Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.y) + row * p.y_stride + c, x[k]);
-      }
-      if (p.part) {
-        for (int j0 = 0; j0 < p.top; ++j0) {
-          const int64_t pair = row * p.top + j0;
-          const int64_t pr = p.row_of_pair ? p.row_of_pair[pair] : pair;
-          const float w = p.weights ? p.weights[pair] : 1.f;
-          Io<T>::template ldv<VEC>(reinterpret_cast<const T*>(p.part) + pr * p.part_stride + c, t);
-#pragma unroll
-          for (int j = 0; j < VEC; ++j) x[k][j] += w * t[j];
-        }
-      }
       Io<float>::ldv<VEC>(xr + c, t);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) x[k][j] = t[j] + p.mult * x[k][j];
